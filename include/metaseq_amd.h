@@ -266,6 +266,13 @@ int msa_greedy_select_f16(const void* logits, int64_t ld_logits, int B, int V, f
                           int force_eos_all, int eos_idx, int64_t* tok, int64_t tok_stride,
                           float* score, int64_t score_stride, const int32_t* len_dev,
                           void* stream);
+/* the same over fp32 logits */
+int msa_greedy_select_f32(const void* logits, int64_t ld_logits, int B, int V, float temperature,
+                          const int32_t* banned_host, int n_banned, const int32_t* stop_host,
+                          int n_stop, uint8_t* finished, const uint8_t* row_mode,
+                          int force_eos_all, int eos_idx, int64_t* tok, int64_t tok_stride,
+                          float* score, int64_t score_stride, const int32_t* len_dev,
+                          void* stream);
 
 /* One step of nucleus (top-p) sampling over fp16 logits[B, V], with the same bookkeeping as
  * msa_greedy_select_f16 (masks, row_mode, finished rows, token / score write-back) plus the
@@ -308,6 +315,17 @@ int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B, int V, flo
                         float alpha_frequency_src, const float* penalty_rows,
                         float* lprobs_out, int64_t ld_lprobs, int64_t* tok, int64_t tok_stride,
                         float* score, int64_t score_stride, void* stream);
+/* the same over fp32 logits */
+int msa_sample_topp_f32(const void* logits, int64_t ld_logits, int B, int V, float temperature,
+                        const float* temperature_rows, const int32_t* banned_host, int n_banned,
+                        const int32_t* stop_host, int n_stop, uint8_t* finished,
+                        const uint8_t* row_mode, int force_eos_all, int eos_idx,
+                        const float* topp_rows, float topp_all, const float* noise,
+                        int64_t* counts, const int64_t* counts_src, float alpha_presence,
+                        float alpha_frequency, float alpha_presence_src,
+                        float alpha_frequency_src, const float* penalty_rows,
+                        float* lprobs_out, int64_t ld_lprobs, int64_t* tok, int64_t tok_stride,
+                        float* score, int64_t score_stride, void* stream);
 
 /* fp32 log-softmax of n_outer x n_inner fp16 logits rows of V ids:
  *   out[o*out_outer_stride + i*ld_out + v] = z[v] - max z - log(sum(exp(z - max z))),
@@ -318,12 +336,19 @@ int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B, int V, flo
 int msa_log_softmax_f16(const void* logits, int64_t in_outer_stride, int64_t ld_logits,
                         int n_outer, int n_inner, int V, float temperature, float* out,
                         int64_t out_outer_stride, int64_t ld_out, void* stream);
+/* the same over fp32 logits */
+int msa_log_softmax_f32(const void* logits, int64_t in_outer_stride, int64_t ld_logits,
+                        int n_outer, int n_inner, int V, float temperature, float* out,
+                        int64_t out_outer_stride, int64_t ld_out, void* stream);
 
 /* Log-probabilities of given target ids under fp16 logits rows:
  *   out[r] = logits[r, target[r]]/temperature - logsumexp_fp32(logits[r,:]/temperature).
  * Replaces the prompt scoring gather of SequenceGenerator._generate
  * (metaseq/sequence_generator.py:235-258). */
 int msa_target_logprob_f16(const void* logits, int64_t ld_logits, int64_t rows, int V,
+                           float temperature, const int64_t* target, float* out, void* stream);
+/* the same over fp32 logits */
+int msa_target_logprob_f32(const void* logits, int64_t ld_logits, int64_t rows, int V,
                            float temperature, const int64_t* target, float* out, void* stream);
 
 /* Vocabulary projection fused with the greedy selection (M <= 64 rows, packed activations):

@@ -1,4 +1,5 @@
-"""ctypes binding of libmetaseq_amd.so (the C ABI declared in include/metaseq_amd.h).
+"""ctypes binding of libmetaseq_amd.so and libmetaseq_hybrid.so (the C ABIs declared in
+include/metaseq_amd.h and include/metaseq_hybrid.h).
 
 There is no fallback: if the library is missing or a call fails, an exception is raised.
 Shape / argument errors surface as ValueError, capacity overruns as ValueError, HIP
@@ -102,11 +103,127 @@ SIGNATURES = {
     "msa_decoder_step": [_P, ctypes.POINTER(StepArgs), _P],
     "msa_probe_stream_read": [_P, c_int64, _P],
 }
+for _n in ("msa_greedy_select", "msa_sample_topp", "msa_log_softmax", "msa_target_logprob"):
+    SIGNATURES[_n + "_f32"] = SIGNATURES[_n + "_f16"]  # the same over fp32 logits
 OTHER_SYMBOLS = ["msa_last_error", "msa_version", "msa_lm_head_select_workspace_bytes",
                  "msa_decoder_destroy", "msa_decoder_step_workspace_bytes",
                  "msa_attention_split_workspace_bytes"]
 
+# ---- the hybrid library (include/metaseq_hybrid.h) -----------------------------------------
+HYBRID_LIB_PATH = os.path.join(_HERE, "csrc", "libmetaseq_hybrid.so")
+MSA_BF16, MSA_F32 = 0, 1
+MSA_GLU_NONE, MSA_GLU_GELU, MSA_GLU_CLAMPED = -1, 0, 1
+MSA_MIX_LATENT, MSA_MIX_RGLRU, MSA_MIX_DELTA = 0, 1, 2
+MSA_FF_NONE, MSA_FF_DENSE, MSA_FF_MOE = 0, 1, 2
+_I32P = ctypes.POINTER(c_int32)
+
+
+def _struct(name, doc, *groups):
+    """A ctypes structure from (type, "field field ...") groups."""
+    fields = [(n, t) for t, names in groups for n in names.split()]
+    return type(name, (ctypes.Structure,), {"_fields_": fields, "__doc__": doc})
+
+
+Batch = _struct("Batch", "msa_batch", (c_int, "M nseg max_count key_bound"),
+                (c_void_p, "tok_slot tok_pos tok_off seg_start seg_slot seg_pos"),
+                (_I32P, "host_start host_slot host_pos"))
+GroupLinearArgs = _struct(
+    "GroupLinearArgs", "msa_group_linear_args", (c_int, "dtype"), (c_void_p, "x"),
+    (c_int64, "ldx"), (c_int, "x_group x_groups x_mb"), (c_void_p, "W y"), (c_int64, "ldy"),
+    (c_int, "y_group y_mb y_f32 y_row0 N K groups glu"), (c_float, "limit"), (c_int64, "M"),
+    (c_void_p, "perm tile_group tile_row n_tiles group_end"),
+    (c_int, "rows_per_x max_tiles tile_rows"))
+TailArgs = _struct("TailArgs", "msa_tail_args", (c_int, "dtype M D Dp S top h_mb"),
+                   (c_float, "eps"), (c_void_p, "part gate pair_w pair_y inverse w_post w_next x h"))
+HybridLayer = _struct(
+    "HybridLayer", "msa_hybrid_layer", (c_int, "kind heads hd q_rank qp kv_rank rp kv_from"),
+    (c_float, "scale"), (c_void_p, "w_in w_q w_kv w_absorb w_v wq_norm wkv_norm"),
+    (c_int, "kv_heads dim dp vdim vp channels blocks taps"),
+    (c_void_p, "conv_w conv_b in_bias y_bias gate_bias lam decay_rate dt_bias o_norm w_gates w_out"),
+    (c_int, "n_in ko"), (c_void_p, "norm1 norm1b norm2 norm2b"),
+    (c_int, "ff_kind ff experts top n_groups keep ff_expert ff_shared"),
+    (c_float, "router_scale limit_expert limit_shared"), (c_void_p, "w_ff_in"),
+    (c_int, "n_ff_in"), (c_void_p, "w_ff_down w_e_in w_e_down"))
+HybridConfigC = _struct("HybridConfigC", "msa_hybrid_config",
+                        (c_int, "dtype layers D Dp vocab Vp"), (c_float, "eps embed_scale"),
+                        (c_void_p, "embed inv_freq final_norm head"))
+HybridState = _struct("HybridState", "msa_hybrid_state", (c_void_p, "latent conv rec"))
+HybridStepArgs = _struct(
+    "HybridStepArgs", "msa_hybrid_step_args", (Batch, "batch"), (c_void_p, "tokens"),
+    (ctypes.POINTER(HybridState), "state"), (c_int, "capacity"), (c_void_p, "rows"),
+    (c_int, "n_rows"), (c_void_p, "logits probe workspace"), (c_int64, "workspace_bytes"))
+
+_BP = ctypes.POINTER(Batch)
+HYBRID_SIGNATURES = {
+    "msa_linear_bf16": [_P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_float, c_uint, _P],
+    "msa_linear_f32": [_P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_float, _P],
+    "msa_linear_partial_bf16": [_P, _P, _P, c_int64, c_int, c_int, c_int, c_uint, _P],
+    "msa_linear_bf16_splits": [c_int64, c_int, c_int, c_int],
+    "msa_group_linear": [ctypes.POINTER(GroupLinearArgs), _P],
+    "msa_moe_route": [_P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, _P, _P, _P, _P],
+    "msa_moe_plan": [_P, c_int, c_int, c_int, _P, _P, _P, _P, _P, _P, c_int, _P],
+    "msa_embed_rmsnorm": [c_int, _P, _P, c_int, _P, c_int, c_float, _P, c_int, c_int, c_float, _P,
+                          _P, _P, c_int, _P],
+    "msa_residual_rmsnorm_tail": [ctypes.POINTER(TailArgs), _P],
+    "msa_short_conv": [c_int, _P, c_int64, c_int, c_int, _P, _P, _P, c_int, _P, c_int64, _P, _BP,
+                       _P],
+    "msa_conv_state": [c_int, _P, c_int64, c_int, c_int, _P, _BP, _P],
+    "msa_rglru_chunks": [c_int],
+    "msa_rglru_scan": [c_int, _P, _P, _P, _P, c_int64, _P, c_int64, _P, c_int, _P, _P, _P, c_int64,
+                       c_int, _BP, _P],
+    "msa_delta_scan": [c_int, _P, c_int64, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int,
+                       _P, _P, _BP, _P],
+    "msa_delta_output": [c_int, _P, _P, c_int64, _P, c_int, c_int, c_int, c_float, _P, c_int64,
+                         c_int, c_int, _P],
+    "msa_latent_norm": [c_int, _P, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_int, _P,
+                        c_float, _P, c_int, _P, c_int, _BP, _P],
+    "msa_latent_attention_splits": [c_int, c_int, c_int, c_int, c_int],
+    "msa_latent_attention": [c_int, _P, _P, c_int, c_int, c_int, c_float, _P, _P, c_int, _P, _P,
+                             c_int, _P],
+    "msa_flash_attention_bf16": [_P, c_int64, _P, c_int64, _P, c_int64, c_int, c_int, c_int, c_int,
+                                 c_int, c_int, c_float, _P],
+    "msa_zero_columns": [c_int, _P, c_int64, c_int64, c_int, c_int, c_int, _P],
+    "msa_gather_rows": [c_int, _P, c_int, _P, c_int, c_int, _P, c_int, _P],
+    "msa_step_positions": [_P, _P, c_int64, c_int64, c_int, _P, _P],
+    "msa_advance_active": [_P, _P, c_int, _P],
+    "msa_hybrid_create": [ctypes.POINTER(HybridConfigC), ctypes.POINTER(HybridLayer),
+                          ctypes.POINTER(c_void_p)],
+    "msa_hybrid_step": [_P, ctypes.POINTER(HybridStepArgs), _P],
+}
+HYBRID_OTHER_SYMBOLS = ["msa_hybrid_destroy", "msa_hybrid_workspace_bytes"]
+
 _lib = None
+_hybrid_lib = None
+
+
+def _open(path):
+    if not os.path.exists(path):
+        raise RuntimeError(
+            "metaseq_amd: %s is missing - build it with `python -m metaseq_amd.csrc.build` "
+            "(there is no non-HIP fallback)" % path)
+    lib = ctypes.CDLL(path)
+    lib.msa_last_error.argtypes = []
+    lib.msa_last_error.restype = c_char_p
+    lib.msa_version.argtypes = []
+    lib.msa_version.restype = c_int
+    return lib
+
+
+def load_hybrid():
+    """Loads the hybrid decoders' library once; raises if it has not been built."""
+    global _hybrid_lib
+    if _hybrid_lib is None:
+        lib = _open(HYBRID_LIB_PATH)
+        for name, args in HYBRID_SIGNATURES.items():
+            fn = getattr(lib, name)
+            fn.argtypes = args
+            fn.restype = c_int
+        lib.msa_hybrid_destroy.argtypes = [_P]
+        lib.msa_hybrid_destroy.restype = None
+        lib.msa_hybrid_workspace_bytes.argtypes = [_P, ctypes.POINTER(HybridStepArgs)]
+        lib.msa_hybrid_workspace_bytes.restype = c_int64
+        _hybrid_lib = lib
+    return _hybrid_lib
 
 
 def load():
@@ -114,19 +231,11 @@ def load():
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(LIB_PATH):
-        raise RuntimeError(
-            "metaseq_amd: %s is missing - build it with `python -m metaseq_amd.csrc.build` "
-            "(there is no non-HIP fallback)" % LIB_PATH)
-    lib = ctypes.CDLL(LIB_PATH)
+    lib = _open(LIB_PATH)
     for name, args in SIGNATURES.items():
         fn = getattr(lib, name)
         fn.argtypes = args
         fn.restype = c_int
-    lib.msa_last_error.argtypes = []
-    lib.msa_last_error.restype = c_char_p
-    lib.msa_version.argtypes = []
-    lib.msa_version.restype = c_int
     lib.msa_lm_head_select_workspace_bytes.argtypes = [c_int]
     lib.msa_lm_head_select_workspace_bytes.restype = c_int64
     lib.msa_decoder_destroy.argtypes = [_P]
@@ -147,6 +256,13 @@ def check(rc, lib=None):
     if rc == -3:
         raise RuntimeError("metaseq_amd HIP failure: " + msg)
     raise ValueError("metaseq_amd: " + msg)
+
+
+def for_logits(lib, name, logits):
+    """The entry point ``name`` for logits of this dtype (fp16 or fp32)."""
+    import torch
+
+    return getattr(lib, name + {torch.float16: "_f16", torch.float32: "_f32"}[logits.dtype])
 
 
 def ptr(t):

@@ -24,7 +24,9 @@ Only tensors are read from files: `torch.load(..., weights_only=True)` executes 
 pickle, so a file whose "cfg" entry holds arbitrary Python objects is refused by the loader;
 re-save such a file as {"model": state_dict} with the reference's own tools first.
 """
+import json
 import logging
+import os
 import re
 from collections import OrderedDict
 from typing import Dict, List
@@ -300,3 +302,43 @@ def find_model_parts(names: List[str]) -> List[str]:
     if [r for r, _ in numbered] != list(range(len(numbered))):
         raise ValueError("model parts are not numbered 0..%d" % (len(numbered) - 1))
     return [n for _, n in numbered]
+
+
+# ---------------------------------------------------------------- safetensors files
+_SAFETENSORS_DTYPES = {"BF16": torch.bfloat16, "F16": torch.float16, "F32": torch.float32,
+                       "F64": torch.float64, "I8": torch.int8, "U8": torch.uint8,
+                       "I16": torch.int16, "I32": torch.int32, "I64": torch.int64,
+                       "BOOL": torch.bool}
+
+
+def read_safetensors(path: str) -> "OrderedDict[str, torch.Tensor]":
+    """name -> tensor of a safetensors file (an 8-byte little-endian length, that many bytes of
+    JSON: name -> dtype, shape, data_offsets, then the data).  The tensors are views of the
+    memory-mapped file, copy-on-write."""
+    size = os.path.getsize(path)
+    with open(path, "rb") as f:
+        n = int.from_bytes(f.read(8), "little")
+        if n > size - 8:
+            raise ValueError("%s is not a safetensors file" % path)
+        header = json.loads(f.read(n))
+    base, out = 8 + n, OrderedDict()
+    # the file's pages stay untouched: the mapping is private, and read-only by use
+    data = torch.from_file(path, shared=False, size=size, dtype=torch.uint8)
+    for name, info in header.items():
+        if name == "__metadata__":
+            continue
+        if info["dtype"] not in _SAFETENSORS_DTYPES:
+            raise ValueError("%s: %s has dtype %s" % (path, name, info["dtype"]))
+        dtype = _SAFETENSORS_DTYPES[info["dtype"]]
+        lo, hi = info["data_offsets"]
+        shape = tuple(info["shape"])
+        count = 1
+        for d in shape:
+            count *= d
+        if lo < 0 or hi > size - base or hi - lo != count * dtype.itemsize:
+            raise ValueError("%s: %s does not fit its data" % (path, name))
+        piece = data[base + lo:base + hi]
+        if (base + lo) % dtype.itemsize:
+            piece = piece.clone()
+        out[name] = piece.view(dtype).view(shape)
+    return out

@@ -1,9 +1,13 @@
 """Flat model configuration with the attribute names the reference's decoder reads from
 its args namespace (metaseq/models/transformer_decoder.py:73-117,
 metaseq/modules/transformer_decoder_layer.py:44-98), and the OPT size table
-(metaseq/launcher/opt_job_constants.py:32-45)."""
-from dataclasses import dataclass, replace
+(metaseq/launcher/opt_job_constants.py:32-45).  Below them: configurations of hybrid decoders,
+whose layers each choose their own mixer and feed-forward."""
+import logging
+from dataclasses import MISSING, dataclass, fields, replace
+from typing import List, Optional, Union
 
+logger = logging.getLogger(__name__)
 
 # head sizes the attention kernels are instantiated for (lanes per key row = head_dim / 8)
 SUPPORTED_HEAD_DIMS = (64, 128)
@@ -101,3 +105,210 @@ def config_from_state_dict(state, heads: int = 0, **overrides) -> OPTConfig:
     cfg = OPTConfig(layers, dim, heads, decoder_ffn_embed_dim=ffn, vocab_size=vocab,
                     max_target_positions=positions - padding_idx - 1, padding_idx=padding_idx)
     return replace(cfg, **overrides)
+
+
+# ---------------------------------------------------------------- hybrid decoders
+@dataclass
+class LatentAttentionSpec:
+    """Attention over a cached latent vector per position: per-head keys and values are linear
+    images of it.  ``kv_from``: the layer whose latents are used instead of own ones."""
+    heads: int
+    dim: int          # query / key size per head
+    vdim: int         # value size per head
+    kv_rank: int
+    q_rank: int
+    scale: float
+    kv_from: Optional[int] = None
+
+
+@dataclass
+class RGLRUSpec:
+    """Gated linear recurrent unit behind a short causal convolution; the gates are
+    block-diagonal."""
+    width: int
+    blocks: int
+    conv: int         # taps
+
+
+@dataclass
+class DeltaSpec:
+    """Gated delta rule with one decay per head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+
+@dataclass
+class DenseSpec:
+    ff: int
+
+
+@dataclass
+class ExpertSpec:
+    ff: int
+    limit: float
+
+
+@dataclass
+class RouterSpec:
+    experts: int
+    top: int
+    scale: float = 1.0
+    groups: int = 1   # experts form this many equal groups,
+    keep: int = 1     # of which the best ``keep`` are eligible
+
+
+@dataclass
+class MoESpec:
+    router: RouterSpec
+    expert: ExpertSpec
+    shared: Optional[ExpertSpec] = None
+
+
+@dataclass
+class HybridLayerSpec:
+    mixer: Union[LatentAttentionSpec, RGLRUSpec, DeltaSpec]
+    mlp: Union[DenseSpec, MoESpec, None] = None
+
+
+def _take(section, where, spec, rename=None, **extra):
+    """Builds ``spec`` from a dictionary of a config.json; keys nobody reads are reported."""
+    section = dict(section)
+    values = {}
+    for f in fields(spec):
+        key = (rename or {}).get(f.name, f.name)
+        if f.name in extra:
+            values[f.name] = extra[f.name]
+        elif section.get(key) is not None:
+            values[f.name] = section[key]
+        elif f.default is MISSING:
+            raise ValueError("config.json: %s lacks %r" % (where, key))
+        section.pop(key, None)
+    unused = sorted(set(section) - set(extra))
+    if unused:
+        logger.warning("config.json: %s: unknown keys %s are ignored", where, ", ".join(unused))
+    return spec(**values)
+
+
+@dataclass
+class HybridConfig:
+    """A decoder whose layers each choose a mixer and a feed-forward, with RMS norms before and
+    after every sublayer, fixed sinusoidal positions and an untied vocabulary projection."""
+    width: int
+    vocab_size: int
+    layers: List[HybridLayerSpec]
+    norm_eps: float = 1e-6
+    embed_scale: float = 1.0
+    max_target_positions: int = 1 << 17
+    padding_idx: int = 1
+    eos_idx: int = 2
+
+    def __post_init__(self):
+        if not self.layers:
+            raise ValueError("a hybrid decoder needs at least one layer")
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if isinstance(m, LatentAttentionSpec) and m.kv_from is not None:
+                j = m.kv_from
+                src = self.layers[j].mixer if 0 <= j < i else None
+                if not isinstance(src, LatentAttentionSpec) or src.kv_from is not None:
+                    raise ValueError("layer %d takes its latents from layer %s, which owns none"
+                                     % (i, j))
+                if src.kv_rank != m.kv_rank:
+                    raise ValueError("layer %d and the layer it takes its latents from differ in "
+                                     "kv_rank" % i)
+            if isinstance(m, DeltaSpec) and m.heads % m.kv_heads:
+                raise ValueError("layer %d: heads must be a multiple of kv_heads" % i)
+            if isinstance(m, RGLRUSpec) and m.width % m.blocks:
+                raise ValueError("layer %d: width must be a multiple of blocks" % i)
+            if isinstance(layer.mlp, MoESpec):
+                r = layer.mlp.router
+                if r.experts % r.groups or not 1 <= r.keep <= r.groups \
+                        or r.top > r.experts // r.groups * r.keep:
+                    raise ValueError("layer %d: %d experts in %d groups, %d kept, top %d"
+                                     % (i, r.experts, r.groups, r.keep, r.top))
+
+    MIXERS = {"latent_attention": LatentAttentionSpec, "rglru": RGLRUSpec, "delta": DeltaSpec}
+
+    @classmethod
+    def from_json(cls, obj):
+        """The configuration of a config.json (already parsed)."""
+        layers = []
+        for i, entry in enumerate(obj["layers"]):
+            where = "layer %d" % i
+            kind = entry["type"]
+            if kind not in cls.MIXERS:
+                raise NotImplementedError("config.json: %s: unknown mixer %r" % (where, kind))
+            mixer = _take(entry["mixer"], where + " mixer", cls.MIXERS[kind])
+            mlp = entry.get("mlp")
+            if mlp is not None:
+                mlp = cls._mlp(dict(mlp), where + " mlp")
+            layers.append(HybridLayerSpec(mixer, mlp))
+        special = {k: obj[k] for k in ("padding_idx", "eos_idx", "max_target_positions")
+                   if k in obj}
+        return cls(width=obj["width"], vocab_size=obj["vocab"], layers=layers,
+                   norm_eps=obj["norm"]["eps"], embed_scale=obj["embedding"]["scale"], **special)
+
+    @staticmethod
+    def _mlp(mlp, where):
+        kind = mlp.pop("kind")
+        if kind == "dense":
+            return _take(mlp, where, DenseSpec)
+        if kind != "moe":
+            raise NotImplementedError("config.json: %s: unknown kind %r" % (where, kind))
+        router = dict(mlp.pop("router"))
+        groups = router.pop("groups", None) or {"count": 1, "keep": 1}
+        expert, shared = mlp.pop("expert"), mlp.pop("shared", None)
+        if mlp:
+            logger.warning("config.json: %s: unknown keys %s are ignored", where,
+                           ", ".join(sorted(mlp)))
+        return MoESpec(
+            _take(router, where + " router", RouterSpec, groups=groups["count"],
+                  keep=groups["keep"]),
+            _take(expert, where + " expert", ExpertSpec),
+            _take(shared, where + " shared expert", ExpertSpec) if shared else None)
+
+    def tensor_shapes(self):
+        """name -> shape of every tensor of a checkpoint of this model."""
+        D, out = self.width, {}
+        out["embed"] = (self.vocab_size, D)
+        for i, layer in enumerate(self.layers):
+            pre, m = "l%d." % i, layer.mixer
+            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if layer.mlp else ()):
+                out[pre + n] = (D,)
+
+            def put(section, **shapes):
+                for name, shape in shapes.items():
+                    out[pre + section + "." + name.replace("_dot_", ".")] = shape
+
+            if isinstance(m, LatentAttentionSpec):
+                put("mix", dq=(m.q_rank, D), dq_dot_norm=(m.q_rank,),
+                    uq=(m.heads * m.dim, m.q_rank), uk=(m.heads * m.dim, m.kv_rank),
+                    uv=(m.heads * m.vdim, m.kv_rank), o=(D, m.heads * m.vdim))
+                if m.kv_from is None:
+                    put("mix", dkv=(m.kv_rank, D), dkv_dot_norm=(m.kv_rank,))
+            elif isinstance(m, RGLRUSpec):
+                W, nb, bs = m.width, m.blocks, m.width // m.blocks
+                put("mix", y=(W, D), y_dot_b=(W,), x=(W, D), x_dot_b=(W,), conv=(W, m.conv),
+                    conv_dot_b=(W,), ra=(nb, bs, bs), ra_dot_b=(nb, bs), ri=(nb, bs, bs),
+                    ri_dot_b=(nb, bs), lam=(W,), o=(D, W))
+            else:
+                qk, v = m.kv_heads * m.dim, m.heads * m.vdim
+                put("mix", q=(qk, D), q_dot_conv=(qk, m.conv), k=(qk, D), k_dot_conv=(qk, m.conv),
+                    v=(v, D), v_dot_conv=(v, m.conv), b=(m.heads, D), a=(m.heads, D),
+                    A_log=(m.heads,), dt_bias=(m.heads,), norm=(m.vdim,), g=(v, D), o=(D, v))
+            if isinstance(layer.mlp, DenseSpec):
+                F = layer.mlp.ff
+                put("mlp", gate=(F, D), up=(F, D), down=(D, F))
+            elif layer.mlp is not None:
+                r, e, s = layer.mlp.router, layer.mlp.expert, layer.mlp.shared
+                put("mlp", router=(r.experts, D))
+                for x in range(r.experts):
+                    put("mlp.e%d" % x, gate=(e.ff, D), up=(e.ff, D), down=(D, e.ff))
+                if s is not None:
+                    put("mlp.shared", gate=(s.ff, D), up=(s.ff, D), down=(D, s.ff), sg=(1, D))
+        out["final.norm"] = (D,)
+        out["head"] = (self.vocab_size, D)
+        return out

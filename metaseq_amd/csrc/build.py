@@ -1,6 +1,10 @@
-"""Builds libmetaseq_amd.so for gfx950 with hipcc (no GPU needed: hipcc cross-compiles).
+"""Builds the shared libraries for gfx950 with hipcc (no GPU needed: hipcc cross-compiles).
 
-Usage: python -m metaseq_amd.csrc.build [--force]
+    core    libmetaseq_amd.so     OPT decoder, selection and sampling (include/metaseq_amd.h)
+    hybrid  libmetaseq_hybrid.so  hybrid decoders: latent attention, recurrent layers, routed
+                                  feed-forwards (include/metaseq_hybrid.h)
+
+Usage: python -m metaseq_amd.csrc.build [core|hybrid ...]
 """
 import os
 import subprocess
@@ -8,19 +12,28 @@ import sys
 from concurrent.futures import ThreadPoolExecutor
 
 HERE = os.path.dirname(os.path.abspath(__file__))
-LIB = os.path.join(HERE, "libmetaseq_amd.so")
-SOURCES = ["capi.hip", "layernorm.hip", "embed.hip", "gemm.hip", "attention.hip", "attention_prefill.hip",
-           "sampling.hip", "probe.hip", "decoder_step.hip"]
+LIBS = {"core": os.path.join(HERE, "libmetaseq_amd.so"),
+        "hybrid": os.path.join(HERE, "libmetaseq_hybrid.so")}
+LIB = LIBS["core"]
+SOURCES = {
+    "core": ["capi.hip", "layernorm.hip", "embed.hip", "gemm.hip", "attention.hip",
+             "attention_prefill.hip", "sampling.hip", "probe.hip", "decoder_step.hip"],
+    "hybrid": ["capi.hip", "gemm_bf16.hip", "group_linear.hip", "moe.hip", "rmsnorm.hip",
+               "recurrent.hip", "latent_attention.hip", "hybrid_step.hip"],
+}
+HEADERS = ["common.h", "gemm_kernels.h", os.path.join("..", "..", "include", "metaseq_amd.h"),
+           os.path.join("..", "..", "include", "metaseq_hybrid.h")]
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-fPIC", "-std=c++17", "-Wall", "-Wno-unused-function",
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
 ]
 
 
-# per-source extras.  The prefill attention kernel keeps its MFMA results in ordinary vector
-# registers (its softmax reads every score; by default hipcc parks them in the accumulator bank
+# per-source extras.  The flash-style attention kernels keep their MFMA results in ordinary vector
+# registers (their softmax reads every score; by default hipcc parks them in the accumulator bank
 # and copies each one out)
-EXTRA_FLAGS = {"attention_prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
+EXTRA_FLAGS = {"attention_prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+               "latent_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
 
 
 def _hipcc():
@@ -30,17 +43,19 @@ def _hipcc():
     raise RuntimeError("hipcc not found")
 
 
-def needs_build():
-    if not os.path.exists(LIB):
+def needs_build(component="core"):
+    lib = LIBS[component]
+    if not os.path.exists(lib):
         return True
-    t = os.path.getmtime(LIB)
-    deps = SOURCES + ["common.h", os.path.join("..", "..", "include", "metaseq_amd.h")]
-    return any(os.path.getmtime(os.path.join(HERE, d)) > t for d in deps)
+    t = os.path.getmtime(lib)
+    return any(os.path.getmtime(os.path.join(HERE, d)) > t for d in SOURCES[component] + HEADERS)
 
 
-def build(force=True, verbose=True):
-    """Compiles every kernel source and links the shared library in-tree."""
-    if not force and not needs_build():
+def build(force=True, verbose=True, components=("core", "hybrid")):
+    """Compiles the sources of the named components and links their shared libraries in-tree.
+    Without ``force`` a component whose library is newer than its sources is left alone."""
+    components = [c for c in components if force or needs_build(c)]
+    if not components:
         return LIB
     hipcc = _hipcc()
     objdir = os.path.join(HERE, "build")
@@ -58,16 +73,22 @@ def build(force=True, verbose=True):
             print(err, file=sys.stderr)
         return obj
 
-    with ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
-        objs = list(ex.map(compile_one, SOURCES))
-    cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB] + objs
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError("link failed:\n" + r.stderr)
-    if verbose:
-        print("built", LIB)
+    sources = sorted({src for c in components for src in SOURCES[c]})
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as ex:
+        objs = dict(zip(sources, ex.map(compile_one, sources)))
+    for c in components:
+        # linked under another name and moved into place: a reader never sees half a library
+        part = LIBS[c] + ".part"
+        cmd = ([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-Wl,-Bsymbolic", "-o", part]
+               + [objs[src] for src in SOURCES[c]])
+        r = subprocess.run(cmd, capture_output=True, text=True)
+        if r.returncode != 0:
+            raise RuntimeError("link failed:\n" + r.stderr)
+        os.replace(part, LIBS[c])
+        if verbose:
+            print("built", LIBS[c])
     return LIB
 
 
 if __name__ == "__main__":
-    build(force=True)
+    build(force=True, components=sys.argv[1:] or ("core", "hybrid"))

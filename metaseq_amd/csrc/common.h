@@ -6,11 +6,16 @@
 #include <stdio.h>
 
 #include "../../include/metaseq_amd.h"
+#include "../../include/metaseq_hybrid.h"
 
 typedef _Float16 half_t;
 typedef _Float16 half2_t __attribute__((ext_vector_type(2)));
 typedef _Float16 half4_t __attribute__((ext_vector_type(4)));
 typedef _Float16 half8_t __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16_t;
+typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float float4_t __attribute__((ext_vector_type(4)));
 typedef float float16_t __attribute__((ext_vector_type(16)));
 
@@ -76,6 +81,23 @@ __host__ __device__ __forceinline__ int64_t packed_act_offset(int m, int k, int 
 
 // round-to-nearest-even fp32 -> fp16 -> fp32 (a "materialise in fp16" point)
 __device__ __forceinline__ float round_h(float v) { return (float)(half_t)v; }
+
+// 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), with (1 + tanh(t)) / 2 = 1 / (1 + exp(-2 t))
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z / (1.f + expf(-2.f * t));
+}
+__device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z)); }
+
+// Gated activations of a (gate, up) pair.  GELU: gelu_tanh(g) u.  CLAMPED: g' = min(g, limit),
+// u' = clamp(u, -limit, limit): g' sigmoid(1.702 g') (u' + 1).
+
+__device__ __forceinline__ float glu_act(int kind, float g, float u, float limit) {
+  if (kind == MSA_GLU_GELU) return gelu_tanh(g) * u;
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * sigmoidf(1.702f * g) * (u + 1.f);
+}
 
 // (max, sum of exp(z - max)) pairs merge associatively: one pass over a row suffices
 __device__ __forceinline__ void lse_merge(float& m, float& s, float om, float os) {

@@ -1,0 +1,482 @@
+// Recurrent mixers over flat batches of segments: the short causal convolution, the gated linear
+// recurrent unit and the gated delta rule.  All state is fp32 and lives per cache slot; a segment
+// whose first position is 0 starts from zero whatever the slot held before.
+#include <math.h>
+
+#include "common.h"
+
+namespace {
+
+template <typename T>
+struct Vec8 {
+  typedef T type __attribute__((ext_vector_type(8), aligned(16)));
+};
+
+__device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
+__device__ __forceinline__ float softplus(float v) {
+  return v > 20.f ? v : log1pf(expf(v));
+}
+
+// ---- short convolution ----------------------------------------------------------------------
+constexpr int SC_TOK = 16;     // tokens per workgroup
+constexpr int SC_MAX_TAPS = 8;
+
+// A thread owns 8 channels and walks SC_TOK tokens.  STEP: one token per segment; the thread also
+// shifts the state.
+template <typename T, bool STEP>
+__global__ __launch_bounds__(256) void short_conv_kernel(
+    const T* __restrict__ in, int64_t ld_in, int C, int taps, const float* __restrict__ in_bias,
+    const float* __restrict__ weight, const float* __restrict__ bias, int act, T* __restrict__ out,
+    int64_t ld_out, T* __restrict__ state, const int32_t* __restrict__ tok_slot,
+    const int32_t* __restrict__ tok_pos, const int32_t* __restrict__ tok_off, int M) {
+  typedef typename Vec8<T>::type v8;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (c >= C) return;
+  const int m0 = blockIdx.y * (STEP ? 1 : SC_TOK), m1 = min(M, m0 + (STEP ? 1 : SC_TOK));
+  float ib[8], b[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    ib[i] = in_bias ? in_bias[c + i] : 0.f;
+    b[i] = bias ? bias[c + i] : 0.f;
+  }
+  for (int m = m0; m < m1; ++m) {
+    const int pos = tok_pos[m], off = tok_off[m];
+    T* st = state + ((int64_t)tok_slot[m] * (taps - 1)) * C + c;
+    float a[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) a[i] = b[i];
+    for (int lag = taps - 1; lag >= 0; --lag) {
+      if (pos - lag < 0) continue;  // before the start (or an inactive token)
+      const v8 v = lag <= off ? *reinterpret_cast<const v8*>(in + (int64_t)(m - lag) * ld_in + c)
+                              : *reinterpret_cast<const v8*>(st + (int64_t)(taps - 1 - (lag - off)) * C);
+      const float* w = weight + (int64_t)(taps - 1 - lag) * C + c;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] = fmaf((float)v[i] + ib[i], w[i], a[i]);
+      if (STEP && lag < taps - 1)  // the state row in front of the one this lag came from
+        *reinterpret_cast<v8*>(st + (int64_t)(taps - 2 - lag) * C) = v;
+    }
+    v8 o;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] = (T)(act ? silu(a[i]) : a[i]);
+    *reinterpret_cast<v8*>(out + (int64_t)m * ld_out + c) = o;
+  }
+}
+
+// state after the segment: row j holds the input of position end - (taps - 1) + j
+template <typename T>
+__global__ __launch_bounds__(256) void conv_state_kernel(
+    const T* __restrict__ in, int64_t ld_in, int C, int taps, T* __restrict__ state,
+    const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
+    const int32_t* __restrict__ seg_pos) {
+  const int c = blockIdx.x * 256 + threadIdx.x, s = blockIdx.y;
+  if (c >= C || seg_pos[s] < 0) return;
+  const int first = seg_start[s], n = seg_start[s + 1] - first;
+  T* st = state + (int64_t)seg_slot[s] * (taps - 1) * C + c;
+  // rows move towards the front only, so they can be written in increasing order
+  for (int j = 0; j < taps - 1; ++j) {
+    const int t = n - (taps - 1) + j;  // offset in the segment; negative: in the old state
+    st[(int64_t)j * C] = t >= 0 ? in[(int64_t)(first + t) * ld_in + c]
+                                : st[(int64_t)(t + taps - 1) * C];
+  }
+}
+
+// ---- gated linear recurrent unit ------------------------------------------------------------
+constexpr int RG_CHUNK = 32;
+
+// log a and the input term of one (token, channel)
+__device__ __forceinline__ void rglru_terms(float gr, float gi, float rate, float u, float& a, float& b) {
+  const float log_a = -8.f * sigmoidf(gr) * rate;
+  a = expf(log_a);
+  b = sqrtf(-expm1f(2.f * log_a)) * sigmoidf(gi) * u;
+}
+
+// pass 1: a and b of every token in place of the gates, and the chunk's (product of a, end state
+// from zero)
+template <typename T>
+__global__ __launch_bounds__(256) void rglru_local_kernel(
+    float* __restrict__ gates, const float* __restrict__ gate_bias, const float* __restrict__ lam,
+    const T* __restrict__ u, int64_t ld_u, int C, float* __restrict__ carry, int chunks,
+    const int32_t* __restrict__ seg_start) {
+  const int c = blockIdx.x * 256 + threadIdx.x, ch = blockIdx.y, s = blockIdx.z;
+  if (c >= C) return;
+  const int first = seg_start[s] + ch * RG_CHUNK, end = min(seg_start[s + 1], first + RG_CHUNK);
+  if (first >= end) return;
+  const float rate = softplus(lam[c]), br = gate_bias[c], bi = gate_bias[C + c];
+  float A = 1.f, S = 0.f;
+  for (int m = first; m < end; ++m) {
+    float* g = gates + (int64_t)m * 2 * C + c;
+    float a, b;
+    rglru_terms(g[0] + br, g[C] + bi, rate, (float)u[(int64_t)m * ld_u + c], a, b);
+    g[0] = a, g[C] = b;
+    A *= a;
+    S = fmaf(a, S, b);
+  }
+  float* k = carry + (((int64_t)s * chunks + ch) * 2) * C + c;
+  k[0] = A, k[C] = S;
+}
+
+// pass 2: the state in front of the chunk from the slot's state and the carries of the chunks
+// before it, then the outputs.  DIRECT: no pass 1, one chunk covers the segment.
+template <typename T, bool DIRECT>
+__global__ __launch_bounds__(256) void rglru_output_kernel(
+    const float* __restrict__ gates, const float* __restrict__ gate_bias,
+    const float* __restrict__ lam, const T* __restrict__ u, int64_t ld_u, const T* __restrict__ y,
+    int64_t ld_y, const float* __restrict__ y_bias, int C, float* __restrict__ state,
+    const float* __restrict__ carry, int chunks, T* __restrict__ out, int64_t ld_out, int out_mb,
+    const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
+    const int32_t* __restrict__ seg_pos) {
+  const int c = blockIdx.x * 256 + threadIdx.x, ch = blockIdx.y, s = blockIdx.z;
+  if (c >= C) return;
+  const int n = seg_start[s + 1] - seg_start[s];
+  const int first = seg_start[s] + (DIRECT ? 0 : ch * RG_CHUNK);
+  const int end = DIRECT ? seg_start[s + 1] : min(seg_start[s + 1], first + RG_CHUNK);
+  if (first >= end) return;
+  const int pos = seg_pos[s];
+  float* slot = state + (int64_t)seg_slot[s] * C + c;
+  float S = pos > 0 ? *slot : 0.f;
+  if (!DIRECT) {
+    const float* k = carry + (int64_t)s * chunks * 2 * C + c;
+    for (int j = 0; j < ch; ++j) S = fmaf(k[(int64_t)j * 2 * C], S, k[(int64_t)j * 2 * C + C]);
+  }
+  float rate = 0.f, br = 0.f, bi = 0.f;
+  if (DIRECT) rate = softplus(lam[c]), br = gate_bias[c], bi = gate_bias[C + c];
+  const float yb = y_bias[c];
+  for (int m = first; m < end; ++m) {
+    const float* g = gates + (int64_t)m * 2 * C + c;
+    float a = g[0], b = g[C];
+    if (DIRECT) rglru_terms(g[0] + br, g[C] + bi, rate, (float)u[(int64_t)m * ld_u + c], a, b);
+    S = fmaf(a, S, b);
+    const float o = S * gelu_tanh((float)y[(int64_t)m * ld_y + c] + yb);
+    out[out_mb > 0 ? packed_act_offset(m, c, out_mb) : (int64_t)m * ld_out + c] = (T)o;
+  }
+  // the state is read by every chunk of the segment in this launch: only with one chunk may the
+  // same launch write it (rglru_state_kernel otherwise)
+  if ((DIRECT || n <= RG_CHUNK) && pos >= 0) *slot = S;
+}
+
+__global__ __launch_bounds__(256) void rglru_state_kernel(
+    int C, float* __restrict__ state, const float* __restrict__ carry, int chunks,
+    const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
+    const int32_t* __restrict__ seg_pos) {
+  const int c = blockIdx.x * 256 + threadIdx.x, s = blockIdx.y;
+  if (c >= C || seg_pos[s] < 0) return;
+  const int n = seg_start[s + 1] - seg_start[s], used = (n + RG_CHUNK - 1) / RG_CHUNK;
+  if (used <= 1) return;
+  float* slot = state + (int64_t)seg_slot[s] * C + c;
+  float S = seg_pos[s] > 0 ? *slot : 0.f;
+  const float* k = carry + (int64_t)s * chunks * 2 * C + c;
+  for (int j = 0; j < used; ++j) S = fmaf(k[(int64_t)j * 2 * C], S, k[(int64_t)j * 2 * C + C]);
+  *slot = S;
+}
+
+// ---- gated delta rule -------------------------------------------------------------------------
+// Every column of a head's state evolves by itself (given k and q), so a workgroup owns one
+// segment, one head and 16 of its columns: a wave holds 4 columns, 16 lanes each, and a lane R
+// consecutive rows in registers, through all tokens of the segment.  With S the state before the
+// token's decay, one pass over it yields both products the token needs:
+//   u = beta (v - g S^T k),   o = S_new^T q = g S^T q + u (k . q),   S_new = g S + k u^T.
+// Tokens are taken DR_TOK at a time: the next chunk's rows are fetched into registers while the
+// current chunk runs out of LDS, where k and q arrive as unit vectors.
+constexpr int DR_TOK = 16;
+
+__device__ __forceinline__ float row16_sum(float v) {
+  v += dpp_move<0xB1, 0xf>(0.f, v);
+  v += dpp_move<0x4E, 0xf>(0.f, v);
+  v += dpp_move<0x124, 0xf>(0.f, v);
+  v += dpp_move<0x128, 0xf>(0.f, v);
+  return v;
+}
+
+template <typename T, int R>
+__global__ __launch_bounds__(256) void delta_scan_kernel(
+    const T* __restrict__ qkv, int64_t ld, const float* __restrict__ ba, int ldba,
+    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias, int heads, int kv_heads,
+    float q_scale, int vp, float* __restrict__ state, float* __restrict__ o,
+    const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
+    const int32_t* __restrict__ seg_pos) {
+  constexpr int DP = 16 * R;
+  __shared__ __attribute__((aligned(16))) float lk[DR_TOK][DP], lq[DR_TOK][DP];
+  __shared__ float lv[DR_TOK][16], lo[DR_TOK][16], lg[DR_TOK], lb[DR_TOK], lkq[DR_TOK];
+  const int s = blockIdx.z, h = blockIdx.y, col0 = blockIdx.x * 16;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int first = seg_start[s], n = seg_start[s + 1] - first, pos = seg_pos[s];
+  const int hk = h / (heads / kv_heads);
+  const int q_at = hk * DP, k_at = kv_heads * DP + hk * DP, v_at = 2 * kv_heads * DP + h * vp + col0;
+  if (pos < 0) {
+    for (int i = tid; i < n * 16; i += 256)
+      o[(int64_t)(first + i / 16) * heads * vp + h * vp + col0 + i % 16] = 0.f;
+    return;
+  }
+  const int cl = wave * 4 + (lane >> 4), rl = lane & 15;  // column of the 16, row group
+  float* st = state + (((int64_t)seg_slot[s] * heads + h) * vp + col0 + cl) * DP + rl * R;
+  float S[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) S[i] = pos > 0 ? st[i] : 0.f;
+  const float rate = decay_rate[h], dtb = dt_bias[h];
+
+  // staging: vector x = tid / 8 (tokens 0 .. 15 of q, then of k), elements 2R * (tid % 8) ..
+  constexpr int EV = 2 * R;
+  const int sv = tid >> 3, stok = sv & 15, sel = (tid & 7) * EV;
+  const bool is_k = sv >= 16;
+  T raw[EV];
+  float rv = 0.f, rb = 0.f, rg = 0.f;
+  auto fetch = [&](int t0) {
+    const int t = min(t0 + stok, n - 1);
+    const T* p = qkv + (int64_t)(first + t) * ld + (is_k ? k_at : q_at) + sel;
+    typedef T t4 __attribute__((ext_vector_type(4), aligned(8)));
+#pragma unroll
+    for (int i = 0; i < EV; i += 4) {
+      const t4 x = *reinterpret_cast<const t4*>(p + i);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) raw[i + j] = x[j];
+    }
+    const int tv = min(t0 + (tid >> 4), n - 1);
+    rv = (float)qkv[(int64_t)(first + tv) * ld + v_at + (tid & 15)];
+    if (tid < DR_TOK) {
+      const float* z = ba + (int64_t)(first + min(t0 + tid, n - 1)) * ldba;
+      rb = z[h];
+      rg = z[heads + h];
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < n; t0 += DR_TOK) {
+    const int nt = min(DR_TOK, n - t0);
+    {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < EV; ++i) ss += (float)raw[i] * (float)raw[i];
+      ss += __shfl_xor(ss, 1, MSA_WAVE);
+      ss += __shfl_xor(ss, 2, MSA_WAVE);
+      ss += __shfl_xor(ss, 4, MSA_WAVE);
+      const float f = (is_k ? 1.f : q_scale) / sqrtf(ss + 1e-6f);
+      float* dst = (is_k ? lk[stok] : lq[stok]) + sel;
+#pragma unroll
+      for (int i = 0; i < EV; ++i) dst[i] = (float)raw[i] * f;
+      lv[tid >> 4][tid & 15] = rv;
+      if (tid < DR_TOK) {
+        lb[tid] = sigmoidf(rb);
+        lg[tid] = expf(-rate * softplus(rg + dtb));
+      }
+    }
+    __syncthreads();
+    {
+      const int t = tid >> 4, r = tid & 15;
+      float d = 0.f;
+#pragma unroll
+      for (int i = 0; i < R; ++i) d = fmaf(lk[t][r * R + i], lq[t][r * R + i], d);
+      d = row16_sum(d);
+      if (r == 0) lkq[t] = d;
+    }
+    if (t0 + DR_TOK < n) fetch(t0 + DR_TOK);
+    __syncthreads();
+    for (int t = 0; t < nt; ++t) {
+      float k[R], d1 = 0.f, d2 = 0.f, e1 = 0.f, e2 = 0.f;
+#pragma unroll
+      for (int i = 0; i < R; ++i) k[i] = lk[t][rl * R + i];
+#pragma unroll
+      for (int i = 0; i < R; i += 2) {
+        d1 = fmaf(S[i], k[i], d1);
+        e1 = fmaf(S[i + 1], k[i + 1], e1);
+        d2 = fmaf(S[i], lq[t][rl * R + i], d2);
+        e2 = fmaf(S[i + 1], lq[t][rl * R + i + 1], e2);
+      }
+      d1 = row16_sum(d1 + e1);
+      d2 = row16_sum(d2 + e2);
+      const float g = lg[t];
+      const float u = lb[t] * (lv[t][cl] - g * d1);
+#pragma unroll
+      for (int i = 0; i < R; ++i) S[i] = fmaf(k[i], u, g * S[i]);
+      if (rl == 0) lo[t][cl] = fmaf(u, lkq[t], g * d2);
+    }
+    __syncthreads();
+    if (tid < nt * 16)
+      o[(int64_t)(first + t0 + (tid >> 4)) * heads * vp + h * vp + col0 + (tid & 15)] =
+          lo[tid >> 4][tid & 15];
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) st[i] = S[i];
+}
+
+// one wave per (token, head)
+template <typename T>
+__global__ __launch_bounds__(256) void delta_output_kernel(
+    const float* __restrict__ o, const T* __restrict__ gate, int64_t ld_gate,
+    const float* __restrict__ w, int heads, int vdim, int vp, float eps, T* __restrict__ out,
+    int64_t ld_out, int out_mb, int M) {
+  const int64_t idx = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (idx >= (int64_t)M * heads) return;
+  const int lane = threadIdx.x & 63;
+  const int m = (int)(idx / heads), h = (int)(idx % heads);
+  const float* row = o + idx * vp;
+  float v[8], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = lane + 64 * i;
+    v[i] = c < vp ? row[c] : 0.f;
+    ss += v[i] * v[i];
+  }
+  ss = wave_sum(ss);
+  const float r = 1.f / sqrtf(ss / (float)vdim + eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = lane + 64 * i;
+    if (c < vp) {
+      const int at = h * vp + c;
+      const float y = v[i] * r * w[c] * silu((float)gate[(int64_t)m * ld_gate + at]);
+      out[out_mb > 0 ? packed_act_offset(m, at, out_mb) : (int64_t)m * ld_out + at] = (T)y;
+    }
+  }
+}
+
+template <typename T>
+void run_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
+               const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vp, float* state,
+               float* o, const msa_batch* b, hipStream_t s) {
+  const dim3 grid(vp / 16, heads, b->nseg);
+  const float q_scale = (float)pow((double)dim, -0.5);
+#define DR_CASE(RR)                                                                                 \
+  case 16 * RR:                                                                                     \
+    hipLaunchKernelGGL((delta_scan_kernel<T, RR>), grid, dim3(256), 0, s, (const T*)qkv, ld, ba,    \
+                       ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vp, state, o,           \
+                       b->seg_start, b->seg_slot, b->seg_pos);                                      \
+    break;
+  switch (dp) {
+    DR_CASE(2)
+    DR_CASE(4)
+    DR_CASE(6)
+    DR_CASE(8)
+    DR_CASE(12)
+    DR_CASE(16)
+  }
+#undef DR_CASE
+}
+
+}  // namespace
+
+extern "C" int msa_short_conv(int dtype, const void* in, int64_t ld_in, int C, int taps,
+                              const float* in_bias, const float* weight, const float* bias, int silu,
+                              void* out, int64_t ld_out, void* state, const msa_batch* b,
+                              void* stream) {
+  const char* name = "msa_short_conv";
+  MSA_REQUIRE(in && weight && out && b && (state || taps == 1), MSA_ERR_INVALID_ARG,
+              "%s: null pointer", name);
+  MSA_REQUIRE(C > 0 && C % 8 == 0 && ld_in % 8 == 0 && ld_out % 8 == 0 && taps >= 1 &&
+                  taps <= SC_MAX_TAPS && b->M > 0 && b->M <= 65535 * SC_TOK,
+              MSA_ERR_INVALID_ARG, "%s: C=%d taps=%d (at most %d) M=%d", name, C, taps, SC_MAX_TAPS,
+              b->M);
+  const bool step = b->max_count == 1 && b->M <= 65535;
+  const dim3 grid((C / 8 + 255) / 256, step ? b->M : (b->M + SC_TOK - 1) / SC_TOK);
+#define SC_RUN(T, STEP)                                                                             \
+  hipLaunchKernelGGL((short_conv_kernel<T, STEP>), grid, dim3(256), 0, (hipStream_t)stream,         \
+                     (const T*)in, ld_in, C, taps, in_bias, weight, bias, silu, (T*)out, ld_out,    \
+                     (T*)state, b->tok_slot, b->tok_pos, b->tok_off, b->M)
+  if (dtype == MSA_BF16) {
+    if (step) SC_RUN(bf16_t, true);
+    else SC_RUN(bf16_t, false);
+  } else {
+    if (step) SC_RUN(float, true);
+    else SC_RUN(float, false);
+  }
+#undef SC_RUN
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_conv_state(int dtype, const void* in, int64_t ld_in, int C, int taps, void* state,
+                              const msa_batch* b, void* stream) {
+  const char* name = "msa_conv_state";
+  MSA_REQUIRE(in && b && (state || taps == 1), MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  if (taps == 1 || (b->max_count == 1 && b->M <= 65535)) return MSA_OK;  // nothing, or done
+  MSA_REQUIRE(b->nseg <= 65535, MSA_ERR_INVALID_ARG, "%s: too many segments", name);
+  const dim3 grid((C + 255) / 256, b->nseg);
+  if (dtype == MSA_BF16)
+    hipLaunchKernelGGL(conv_state_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream,
+                       (const bf16_t*)in, ld_in, C, taps, (bf16_t*)state, b->seg_start, b->seg_slot,
+                       b->seg_pos);
+  else
+    hipLaunchKernelGGL(conv_state_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream,
+                       (const float*)in, ld_in, C, taps, (float*)state, b->seg_start, b->seg_slot,
+                       b->seg_pos);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_rglru_chunks(int max_count) { return (max_count + RG_CHUNK - 1) / RG_CHUNK; }
+
+extern "C" int msa_rglru_scan(int dtype, float* gates, const float* gate_bias, const float* lam,
+                              const void* u, int64_t ld_u, const void* y, int64_t ld_y,
+                              const float* y_bias, int C, float* state, float* carry, void* out,
+                              int64_t ld_out, int out_mb, const msa_batch* b, void* stream) {
+  const char* name = "msa_rglru_scan";
+  MSA_REQUIRE(gates && gate_bias && lam && u && y && y_bias && state && out && b, MSA_ERR_INVALID_ARG,
+              "%s: null pointer", name);
+  const int chunks = msa_rglru_chunks(b->max_count);
+  MSA_REQUIRE(C > 0 && b->nseg > 0 && b->nseg <= 65535 && chunks >= 1 && chunks <= 65535 &&
+                  (chunks == 1 || carry),
+              MSA_ERR_INVALID_ARG, "%s: C=%d nseg=%d chunks=%d", name, C, b->nseg, chunks);
+  hipStream_t s = (hipStream_t)stream;
+  const dim3 grid((C + 255) / 256, chunks, b->nseg);
+#define RG_RUN(T)                                                                                   \
+  if (chunks == 1) {                                                                                \
+    hipLaunchKernelGGL((rglru_output_kernel<T, true>), grid, dim3(256), 0, s, gates, gate_bias, lam, \
+                       (const T*)u, ld_u, (const T*)y, ld_y, y_bias, C, state, carry, chunks,       \
+                       (T*)out, ld_out, out_mb, b->seg_start, b->seg_slot, b->seg_pos);             \
+  } else {                                                                                          \
+    hipLaunchKernelGGL((rglru_local_kernel<T>), grid, dim3(256), 0, s, gates, gate_bias, lam,       \
+                       (const T*)u, ld_u, C, carry, chunks, b->seg_start);                          \
+    hipLaunchKernelGGL((rglru_output_kernel<T, false>), grid, dim3(256), 0, s, gates, gate_bias,    \
+                       lam, (const T*)u, ld_u, (const T*)y, ld_y, y_bias, C, state, carry, chunks,  \
+                       (T*)out, ld_out, out_mb, b->seg_start, b->seg_slot, b->seg_pos);             \
+    hipLaunchKernelGGL(rglru_state_kernel, dim3((C + 255) / 256, b->nseg), dim3(256), 0, s, C,      \
+                       state, carry, chunks, b->seg_start, b->seg_slot, b->seg_pos);                \
+  }
+  if (dtype == MSA_BF16) {
+    RG_RUN(bf16_t)
+  } else {
+    RG_RUN(float)
+  }
+#undef RG_RUN
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
+                              const float* decay_rate, const float* dt_bias, int heads, int kv_heads,
+                              int dim, int dp, int vp, float* state, float* o, const msa_batch* b,
+                              void* stream) {
+  const char* name = "msa_delta_scan";
+  MSA_REQUIRE(qkv && ba && decay_rate && dt_bias && state && o && b, MSA_ERR_INVALID_ARG,
+              "%s: null pointer", name);
+  MSA_REQUIRE((dp == 32 || dp == 64 || dp == 96 || dp == 128 || dp == 192 || dp == 256) && dim <= dp &&
+                  vp > 0 && vp % 16 == 0 && kv_heads > 0 && heads % kv_heads == 0 &&
+                  ldba >= 2 * heads && ld % 8 == 0 && heads <= 65535 && b->nseg > 0 &&
+                  b->nseg <= 65535,
+              MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
+              kv_heads, dim, dp, vp);
+  if (dtype == MSA_BF16)
+    run_delta<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o,
+                      b, (hipStream_t)stream);
+  else
+    run_delta<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
+                     (hipStream_t)stream);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_delta_output(int dtype, const float* o, const void* gate, int64_t ld_gate,
+                                const float* w, int heads, int vdim, int vp, float eps, void* out,
+                                int64_t ld_out, int out_mb, int M, void* stream) {
+  const char* name = "msa_delta_output";
+  MSA_REQUIRE(o && gate && w && out && M > 0 && heads > 0 && vp > 0 && vp <= 512 && vdim <= vp,
+              MSA_ERR_INVALID_ARG, "%s: bad arguments (vp=%d)", name, vp);
+  const dim3 grid((unsigned)(((int64_t)M * heads + 3) / 4));
+  if (dtype == MSA_BF16)
+    hipLaunchKernelGGL(delta_output_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, o,
+                       (const bf16_t*)gate, ld_gate, w, heads, vdim, vp, eps, (bf16_t*)out, ld_out,
+                       out_mb, M);
+  else
+    hipLaunchKernelGGL(delta_output_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, o,
+                       (const float*)gate, ld_gate, w, heads, vdim, vp, eps, (float*)out, ld_out, 0, M);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}

@@ -1,0 +1,345 @@
+// RMS norms of hybrid decoders with what surrounds them fused in: the embedding with sinusoidal
+// positions, the tail of a sublayer (split-K sums, the combination of routed experts, post-norm,
+// residual add, next pre-norm), the latent norms with the cache append, and small row utilities.
+// One workgroup per token; a row lives in registers (NV float4 per thread).
+#include <math.h>
+
+#include "common.h"
+
+namespace {
+
+constexpr int RN_THREADS = 256;
+
+// one activation element group: 4 consecutive columns of row m
+template <typename T>
+__device__ __forceinline__ void store_act4(void* h, int64_t m, int64_t ld, int mb, int c, float4_t v) {
+  if constexpr (sizeof(T) == 4) {
+    *reinterpret_cast<float4_t*>((float*)h + m * ld + c) = v;
+  } else {
+    bf16_t* p = (bf16_t*)h + (mb > 0 ? packed_act_offset((int)m, c, mb) : m * ld + c);
+    *reinterpret_cast<bf16x4_t*>(p) = bf16x4_t{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+  }
+}
+
+__device__ __forceinline__ float dot4(float4_t v) {
+  return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+}
+
+// x (registers) -> h = x / rms(x) * w
+template <typename T, int NV>
+__device__ __forceinline__ void norm_out(const float4_t (&x)[NV], int64_t m, int D, int Dp, float eps,
+                                         const float* w, void* h, int mb, float* red) {
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) ss += dot4(x[i]);
+  ss = block_sum(ss, red);
+  const float r = 1.f / sqrtf(ss / (float)D + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    if (c < Dp) {
+      const float4_t wv = *reinterpret_cast<const float4_t*>(w + c);
+      store_act4<T>(h, m, Dp, mb, c, x[i] * r * wv);
+    }
+  }
+}
+
+template <typename T, int NV>
+__global__ __launch_bounds__(RN_THREADS) void embed_kernel(
+    const int64_t* __restrict__ tokens, const int32_t* __restrict__ tok_pos,
+    const bf16_t* __restrict__ table, int vocab, float scale, const double* __restrict__ inv_freq,
+    int D, int Dp, float eps, float* __restrict__ x, const float* __restrict__ w, void* h, int mb) {
+  __shared__ float red[16];
+  const int64_t m = blockIdx.x;
+  int64_t t = tokens[m];
+  t = t < 0 ? 0 : (t >= vocab ? vocab - 1 : t);
+  const double pos = (double)max(tok_pos[m], 0);
+  float4_t v[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    v[i] = float4_t{0.f, 0.f, 0.f, 0.f};
+    if (c >= Dp) continue;
+    const bf16x4_t e = *reinterpret_cast<const bf16x4_t*>(table + t * Dp + c);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      float p = 0.f;
+      if (c + j < D) {
+        // the angle in turns, reduced to [-1/2, 1/2] in double; sin / cos of pi * (2 turns)
+        double turns = pos * inv_freq[(c + j) >> 1] * 0.15915494309189535;
+        turns -= rint(turns);
+        const float a = 2.f * (float)turns;
+        p = (j & 1) ? cospif(a) : sinpif(a);
+      }
+      v[i][j] = (float)e[j] * scale + p;
+    }
+    *reinterpret_cast<float4_t*>(x + m * Dp + c) = v[i];
+  }
+  if (w) norm_out<T, NV>(v, m, D, Dp, eps, w, h, mb, red);
+}
+
+template <typename T, int NV>
+__global__ __launch_bounds__(RN_THREADS) void tail_kernel(msa_tail_args a) {
+  __shared__ float red[16];
+  const int64_t m = blockIdx.x;
+  const int D = a.D, Dp = a.Dp;
+  float4_t b[NV], x[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    b[i] = x[i] = float4_t{0.f, 0.f, 0.f, 0.f};
+    if (c < Dp) x[i] = *reinterpret_cast<const float4_t*>(a.x + m * Dp + c);
+  }
+  if (a.part) {
+    for (int s = 0; s < a.S; ++s) {
+      const float* p = a.part + ((int64_t)s * a.M + m) * Dp;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + i * RN_THREADS) * 4;
+        if (c < Dp) b[i] += *reinterpret_cast<const float4_t*>(p + c);
+      }
+    }
+    if (a.gate) {
+      const float g = a.gate[m];
+#pragma unroll
+      for (int i = 0; i < NV; ++i) b[i] = b[i] * g;
+    }
+  }
+  if (a.pair_y) {
+    for (int k = 0; k < a.top; ++k) {
+      const float w = a.pair_w[m * a.top + k];
+      const T* p = (const T*)a.pair_y + (int64_t)a.inverse[m * a.top + k] * Dp;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + i * RN_THREADS) * 4;
+        if (c < Dp) {
+          typedef T t4 __attribute__((ext_vector_type(4)));
+          const t4 y = *reinterpret_cast<const t4*>(p + c);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) b[i][j] += w * (float)y[j];
+        }
+      }
+    }
+  }
+  float r = 1.f;
+  if (a.w_post) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss += dot4(b[i]);
+    ss = block_sum(ss, red);
+    r = 1.f / sqrtf(ss / (float)D + a.eps);
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    if (c < Dp) {
+      if (a.w_post) {
+        const float4_t wv = *reinterpret_cast<const float4_t*>(a.w_post + c);
+        b[i] = b[i] * r * wv;
+      }
+      x[i] += b[i];
+      *reinterpret_cast<float4_t*>(a.x + m * Dp + c) = x[i];
+    }
+  }
+  if (a.w_next) norm_out<T, NV>(x, m, D, Dp, a.eps, a.w_next, a.h, a.h_mb, red);
+}
+
+// Down-projected latents: one workgroup per token, the two norms by different halves of it.
+template <typename T>
+__global__ __launch_bounds__(RN_THREADS) void latent_norm_kernel(
+    const float* __restrict__ part, int S, int N, int M, int q_rank, int qp,
+    const float* __restrict__ wq, int kv_rank, int rp, const float* __restrict__ wkv, float eps,
+    void* cq, int cq_mb, T* latent, int capacity, const int32_t* __restrict__ tok_slot,
+    const int32_t* __restrict__ tok_pos) {
+  __shared__ float red[16];
+  __shared__ float row[4096];  // summed latents of this token (N <= 4096)
+  const int64_t m = blockIdx.x;
+  float sq = 0.f, skv = 0.f;
+  for (int c = threadIdx.x; c < qp + rp; c += RN_THREADS) {
+    float v = part[m * N + c];
+    for (int s = 1; s < S; ++s) v += part[((int64_t)s * M + m) * N + c];
+    row[c] = v;
+    if (c < qp) sq += v * v;
+    else skv += v * v;
+  }
+  sq = block_sum(sq, red);
+  const float rq = 1.f / sqrtf(sq / (float)q_rank + eps);
+  for (int c = threadIdx.x * 4; c < qp; c += RN_THREADS * 4) {
+    const float4_t v = *reinterpret_cast<const float4_t*>(row + c);
+    store_act4<T>(cq, m, qp, cq_mb, c, v * rq * *reinterpret_cast<const float4_t*>(wq + c));
+  }
+  if (!latent) return;
+  skv = block_sum(skv, red);
+  const float rkv = 1.f / sqrtf(skv / (float)kv_rank + eps);
+  const int pos = tok_pos[m];
+  if (pos < 0 || pos >= capacity) return;
+  T* dst = latent + ((int64_t)tok_slot[m] * capacity + pos) * rp;
+  for (int c = threadIdx.x * 4; c < rp; c += RN_THREADS * 4) {
+    const float4_t v = *reinterpret_cast<const float4_t*>(row + qp + c);
+    store_act4<T>(dst, 0, rp, 0, c, v * rkv * *reinterpret_cast<const float4_t*>(wkv + c));
+  }
+}
+
+template <typename T>
+__global__ void zero_columns_kernel(T* y, int64_t M, int64_t ld, int mb, int c0, int c1) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  const int w = c1 - c0;
+  if (i >= M * w) return;
+  const int64_t m = i / w;
+  const int c = c0 + (int)(i - m * w);
+  y[mb > 0 ? packed_act_offset((int)m, c, mb) : m * ld + c] = (T)0.f;
+}
+
+// 8 elements (16 or 32 bytes) per thread; rows past n of a packed destination stay as they are
+template <typename T>
+__global__ void gather_rows_kernel(const T* src, int src_mb, const int32_t* rows, int n, int K, T* dst,
+                                   int dst_mb) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  const int q = K / 8;
+  if (i >= (int64_t)n * q) return;
+  const int r = (int)(i / q), c = (int)(i % q) * 8;
+  const int64_t m = rows[r];
+  typedef T t8 __attribute__((ext_vector_type(8), aligned(16)));
+  const T* s = src + (src_mb > 0 ? packed_act_offset((int)m, c, src_mb) : m * K + c);
+  T* d = dst + (dst_mb > 0 ? packed_act_offset(r, c, dst_mb) : (int64_t)r * K + c);
+  *reinterpret_cast<t8*>(d) = *reinterpret_cast<const t8*>(s);
+}
+
+__global__ void step_positions_kernel(const int32_t* lens, const int64_t* tokens, int64_t stride,
+                                      int64_t pad, int B, int32_t* step_pos) {
+  const int b = blockIdx.x * 256 + threadIdx.x;
+  if (b < B) step_pos[b] = lens[b] >= 0 && tokens[b * stride] != pad ? lens[b] : -1;
+}
+
+__global__ void advance_active_kernel(int32_t* lens, const int32_t* step_pos, int B) {
+  const int b = blockIdx.x * 256 + threadIdx.x;
+  if (b < B && step_pos[b] >= 0) lens[b] = step_pos[b] + 1;
+}
+
+int vectors_per_thread(int Dp) {  // 1, 2, 4, 8 or 16; 0: too wide
+  const int q = (Dp / 4 + RN_THREADS - 1) / RN_THREADS;
+  for (int v = 1; v <= 16; v *= 2)
+    if (q <= v) return v;
+  return 0;
+}
+
+#define RN_DISPATCH(KERNEL, T, nv, ...)                                                         \
+  do {                                                                                          \
+    if (nv == 1) hipLaunchKernelGGL((KERNEL<T, 1>), __VA_ARGS__);                               \
+    else if (nv == 2) hipLaunchKernelGGL((KERNEL<T, 2>), __VA_ARGS__);                          \
+    else if (nv == 4) hipLaunchKernelGGL((KERNEL<T, 4>), __VA_ARGS__);                          \
+    else if (nv == 8) hipLaunchKernelGGL((KERNEL<T, 8>), __VA_ARGS__);                          \
+    else hipLaunchKernelGGL((KERNEL<T, 16>), __VA_ARGS__);                                      \
+  } while (0)
+
+}  // namespace
+
+extern "C" int msa_embed_rmsnorm(int dtype, const int64_t* tokens, const int32_t* tok_pos, int M,
+                                 const void* table, int vocab, float scale, const double* inv_freq,
+                                 int D, int Dp, float eps, float* x, const float* w, void* h, int h_mb,
+                                 void* stream) {
+  const char* name = "msa_embed_rmsnorm";
+  MSA_REQUIRE(tokens && tok_pos && table && inv_freq && x && (!w || h), MSA_ERR_INVALID_ARG,
+              "%s: null pointer", name);
+  const int nv = vectors_per_thread(Dp);
+  MSA_REQUIRE(M > 0 && vocab > 0 && D > 0 && D <= Dp && Dp % 4 == 0 && nv > 0, MSA_ERR_INVALID_ARG,
+              "%s: M=%d vocab=%d D=%d Dp=%d", name, M, vocab, D, Dp);
+  if (dtype == MSA_BF16)
+    RN_DISPATCH(embed_kernel, bf16_t, nv, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream, tokens,
+                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, h_mb);
+  else
+    RN_DISPATCH(embed_kernel, float, nv, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream, tokens,
+                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, 0);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_residual_rmsnorm_tail(const msa_tail_args* a, void* stream) {
+  const char* name = "msa_residual_rmsnorm_tail";
+  MSA_REQUIRE(a && a->x && (a->part || a->pair_y) && (!a->w_next || a->h), MSA_ERR_INVALID_ARG,
+              "%s: null pointer", name);
+  MSA_REQUIRE(!a->pair_y || (a->pair_w && a->inverse && a->top > 0), MSA_ERR_INVALID_ARG,
+              "%s: routed terms without weights", name);
+  const int nv = vectors_per_thread(a->Dp);
+  MSA_REQUIRE(a->M > 0 && a->D > 0 && a->D <= a->Dp && a->Dp % 4 == 0 && nv > 0 &&
+                  (!a->part || a->S > 0),
+              MSA_ERR_INVALID_ARG, "%s: M=%d D=%d Dp=%d S=%d", name, a->M, a->D, a->Dp, a->S);
+  if (a->dtype == MSA_BF16)
+    RN_DISPATCH(tail_kernel, bf16_t, nv, dim3(a->M), dim3(RN_THREADS), 0, (hipStream_t)stream, *a);
+  else
+    RN_DISPATCH(tail_kernel, float, nv, dim3(a->M), dim3(RN_THREADS), 0, (hipStream_t)stream, *a);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_latent_norm(int dtype, const float* part, int S, int N, int M, int q_rank, int qp,
+                               const float* wq, int kv_rank, int rp, const float* wkv, float eps,
+                               void* cq, int cq_mb, void* latent, int capacity, const msa_batch* b,
+                               void* stream) {
+  const char* name = "msa_latent_norm";
+  MSA_REQUIRE(part && wq && cq && b && (!latent || wkv), MSA_ERR_INVALID_ARG, "%s: null pointer",
+              name);
+  const int r = latent ? rp : 0;
+  MSA_REQUIRE(M > 0 && S > 0 && qp % 4 == 0 && r % 4 == 0 && qp + r <= N && qp + r <= 4096,
+              MSA_ERR_INVALID_ARG, "%s: M=%d S=%d N=%d, latents of %d and %d (at most 4096 together)",
+              name, M, S, N, qp, r);
+  if (dtype == MSA_BF16)
+    hipLaunchKernelGGL(latent_norm_kernel<bf16_t>, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream,
+                       part, S, N, M, q_rank, qp, wq, kv_rank, r, wkv, eps, cq, cq_mb,
+                       (bf16_t*)latent, capacity, b->tok_slot, b->tok_pos);
+  else
+    hipLaunchKernelGGL(latent_norm_kernel<float>, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream,
+                       part, S, N, M, q_rank, qp, wq, kv_rank, r, wkv, eps, cq, 0, (float*)latent,
+                       capacity, b->tok_slot, b->tok_pos);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_zero_columns(int dtype, void* y, int64_t M, int64_t ld, int mb, int c0, int c1,
+                                void* stream) {
+  MSA_REQUIRE(y && M >= 0 && c0 >= 0 && c1 <= ld, MSA_ERR_INVALID_ARG, "msa_zero_columns: bad range");
+  if (M == 0 || c1 <= c0) return MSA_OK;
+  const dim3 grid((unsigned)((M * (c1 - c0) + 255) / 256));
+  if (dtype == MSA_BF16)
+    hipLaunchKernelGGL(zero_columns_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream,
+                       (bf16_t*)y, M, ld, mb, c0, c1);
+  else
+    hipLaunchKernelGGL(zero_columns_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (float*)y,
+                       M, ld, 0, c0, c1);
+  MSA_CHECK_LAUNCH("msa_zero_columns");
+  return MSA_OK;
+}
+
+extern "C" int msa_gather_rows(int dtype, const void* src, int src_mb, const int32_t* rows, int n, int K,
+                               void* dst, int dst_mb, void* stream) {
+  MSA_REQUIRE(src && rows && dst && n >= 0 && K > 0 && K % 8 == 0, MSA_ERR_INVALID_ARG,
+              "msa_gather_rows: bad arguments");
+  if (n == 0) return MSA_OK;
+  const dim3 grid((unsigned)(((int64_t)n * (K / 8) + 255) / 256));
+  if (dtype == MSA_BF16)
+    hipLaunchKernelGGL(gather_rows_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream,
+                       (const bf16_t*)src, src_mb, rows, n, K, (bf16_t*)dst, dst_mb);
+  else
+    hipLaunchKernelGGL(gather_rows_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream,
+                       (const float*)src, 0, rows, n, K, (float*)dst, 0);
+  MSA_CHECK_LAUNCH("msa_gather_rows");
+  return MSA_OK;
+}
+
+extern "C" int msa_step_positions(const int32_t* lens, const int64_t* tokens, int64_t tok_stride,
+                                  int64_t pad, int B, int32_t* step_pos, void* stream) {
+  MSA_REQUIRE(lens && tokens && step_pos && B > 0, MSA_ERR_INVALID_ARG,
+              "msa_step_positions: bad arguments");
+  hipLaunchKernelGGL(step_positions_kernel, dim3((B + 255) / 256), dim3(256), 0, (hipStream_t)stream,
+                     lens, tokens, tok_stride, pad, B, step_pos);
+  MSA_CHECK_LAUNCH("msa_step_positions");
+  return MSA_OK;
+}
+
+extern "C" int msa_advance_active(int32_t* lens, const int32_t* step_pos, int B, void* stream) {
+  MSA_REQUIRE(lens && step_pos && B > 0, MSA_ERR_INVALID_ARG, "msa_advance_active: bad arguments");
+  hipLaunchKernelGGL(advance_active_kernel, dim3((B + 255) / 256), dim3(256), 0, (hipStream_t)stream,
+                     lens, step_pos, B);
+  MSA_CHECK_LAUNCH("msa_advance_active");
+  return MSA_OK;
+}

@@ -1,5 +1,5 @@
-// Per-row vocabulary reductions of the greedy generation loop: fp32 log-sum-exp over fp16
-// logits, masked arg-max with lowest-index tie-break, and target log-probability gather.
+// Per-row vocabulary reductions of the greedy generation loop: fp32 log-sum-exp over fp16 or fp32
+// logits (LT), masked arg-max with lowest-index tie-break, and target log-probability gather.
 // One workgroup per logits row; the row (V * 2 bytes) is read twice from cache/HBM.
 #include <atomic>
 #include <math.h>
@@ -15,15 +15,21 @@ struct RowStats {
   float lse;  // log(sum(exp(z - max)))   (so log_softmax(z) = z - max - lse)
 };
 
-// visits every element of a logits row as z = logit (/ temperature), 8 halves per load where the
+// visits every element of a logits row as z = logit (/ temperature), 8 values per load where the
 // row is 16-byte aligned
-template <typename F>
-__device__ __forceinline__ void for_each_z(const half_t* __restrict__ row, int V, float temp,
+template <typename LT>
+struct Logits8 {
+  typedef LT type __attribute__((ext_vector_type(8), aligned(16)));
+};
+
+template <typename LT, typename F>
+__device__ __forceinline__ void for_each_z(const LT* __restrict__ row, int V, float temp,
                                            bool scale, F f) {
+  typedef typename Logits8<LT>::type lt8;
   if ((reinterpret_cast<uintptr_t>(row) & 15) == 0) {
     const int nv = V >> 3;
     for (int c = threadIdx.x; c < nv; c += blockDim.x) {
-      const half8_t v = *reinterpret_cast<const half8_t*>(row + (c << 3));
+      const lt8 v = *reinterpret_cast<const lt8*>(row + (c << 3));
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         float z = (float)v[i];
@@ -45,7 +51,8 @@ __device__ __forceinline__ void for_each_z(const half_t* __restrict__ row, int V
   }
 }
 
-__device__ __forceinline__ RowStats row_logsumexp(const half_t* __restrict__ row, int V,
+template <typename LT>
+__device__ __forceinline__ RowStats row_logsumexp(const LT* __restrict__ row, int V,
                                                   float temp, bool scale, float* red) {
   float mx = -INFINITY;
   bool nan = false;
@@ -64,8 +71,9 @@ __device__ __forceinline__ RowStats row_logsumexp(const half_t* __restrict__ row
   return r;
 }
 
+template <typename LT>
 __global__ __launch_bounds__(SM_THREADS) void greedy_select_kernel(
-    const half_t* __restrict__ logits, int64_t ld, int V, float temperature, bool scale,
+    const LT* __restrict__ logits, int64_t ld, int V, float temperature, bool scale,
     IdList banned, IdList stop, uint8_t* __restrict__ finished,
     const uint8_t* __restrict__ row_mode, int force_eos_all, int eos,
     int64_t* __restrict__ tok, int64_t tok_stride, float* __restrict__ score,
@@ -73,7 +81,7 @@ __global__ __launch_bounds__(SM_THREADS) void greedy_select_kernel(
   __shared__ float wm[16], ws[16], wbest[16], wnan[16];
   __shared__ int widx[16];
   const int b = blockIdx.x;
-  const half_t* row = logits + (int64_t)b * ld;
+  const LT* row = logits + (int64_t)b * ld;
   const unsigned rm = row_mode ? row_mode[b] : 0u;
   const bool only_eos = force_eos_all || (finished && finished[b]) || (rm & MSA_ROW_ONLY_EOS);
   const bool ban_early = rm & MSA_ROW_BAN_EARLY;  // eos and the stop ids are not eligible
@@ -99,10 +107,11 @@ __global__ __launch_bounds__(SM_THREADS) void greedy_select_kernel(
     const int nv = V >> 3;
     constexpr int UNR = 4;  // chunks requested together: one memory round trip per UNR chunks
     for (int c0 = threadIdx.x; c0 < nv; c0 += blockDim.x * UNR) {
-      half8_t vv[UNR];
+      typedef typename Logits8<LT>::type lt8;
+      lt8 vv[UNR];
 #pragma unroll
       for (int u = 0; u < UNR; ++u)
-        vv[u] = *reinterpret_cast<const half8_t*>(row + (min(c0 + u * (int)blockDim.x, nv - 1) << 3));
+        vv[u] = *reinterpret_cast<const lt8*>(row + (min(c0 + u * (int)blockDim.x, nv - 1) << 3));
 #pragma unroll
       for (int u = 0; u < UNR; ++u) {
         const int c = c0 + u * blockDim.x;
@@ -186,12 +195,13 @@ __global__ __launch_bounds__(SM_THREADS) void greedy_select_kernel(
   }
 }
 
+template <typename LT>
 __global__ __launch_bounds__(SM_THREADS) void target_logprob_kernel(
-    const half_t* __restrict__ logits, int64_t ld, int V, float temperature, bool scale,
+    const LT* __restrict__ logits, int64_t ld, int V, float temperature, bool scale,
     const int64_t* __restrict__ target, float* __restrict__ out) {
   __shared__ float red[16];
   const int64_t r = blockIdx.x;
-  const half_t* row = logits + r * ld;
+  const LT* row = logits + r * ld;
   const RowStats st = row_logsumexp(row, V, temperature, scale, red);
   if (threadIdx.x == 0) {
     int64_t t = target[r];
@@ -271,15 +281,17 @@ __global__ __launch_bounds__(256) void select_combine_kernel(
 
 // fp32 log-softmax of fp16 logits rows; row (o, i) is read at o * in_outer + i * ld and written
 // at o * out_outer + i * ld_out
+template <typename LT>
 __global__ __launch_bounds__(SM_THREADS) void log_softmax_kernel(
-    const half_t* __restrict__ logits, int64_t in_outer, int64_t ld, int n_inner, int V,
+    const LT* __restrict__ logits, int64_t in_outer, int64_t ld, int n_inner, int V,
     float temperature, bool scale, float* __restrict__ out, int64_t out_outer, int64_t ld_out) {
   __shared__ float red[16];
   const int o = blockIdx.x / n_inner, i = blockIdx.x % n_inner;
-  const half_t* row = logits + o * in_outer + i * ld;
+  const LT* row = logits + o * in_outer + i * ld;
   float* orow = out + o * out_outer + i * ld_out;
   const RowStats st = row_logsumexp(row, V, temperature, scale, red);
-  for_each_z(row, V, temperature, scale, [&](int id, float z) { orow[id] = (z - st.max) - st.lse; });
+  for_each_z(row, V, temperature, scale, [&](int id, float z) { orow[id] = (z - st.max) - st.lse;
+             });
 }
 
 // ---- nucleus (top-p) sampling --------------------------------------------------------------
@@ -332,8 +344,9 @@ __device__ __forceinline__ void argbest(float& v, int& i, float ov, int oi) {
   }
 }
 
+template <typename LT>
 __global__ __launch_bounds__(SP_THREADS) void sample_topp_kernel(
-    const half_t* __restrict__ logits, int64_t ld, int V, float temperature_all,
+    const LT* __restrict__ logits, int64_t ld, int V, float temperature_all,
     const float* __restrict__ temperature_rows, IdList banned, IdList stop,
     uint8_t* __restrict__ finished, const uint8_t* __restrict__ row_mode, int force_eos_all,
     int eos, const float* __restrict__ topp_rows, float topp_all,
@@ -360,7 +373,7 @@ __global__ __launch_bounds__(SP_THREADS) void sample_topp_kernel(
   __shared__ unsigned tcnt[SP_TIE_BLOCKS];
   __shared__ unsigned long long tmask[SP_THREADS / 64];
   const int b = blockIdx.x;
-  const half_t* row = logits + (int64_t)b * ld;
+  const LT* row = logits + (int64_t)b * ld;
   const unsigned rm = row_mode ? row_mode[b] : 0u;
   if (rm & MSA_ROW_SKIP) return;  // the whole workgroup: this row is not part of the call
   const bool only_eos = force_eos_all || (finished && finished[b]) || (rm & MSA_ROW_ONLY_EOS);
@@ -520,7 +533,8 @@ __global__ __launch_bounds__(SP_THREADS) void sample_topp_kernel(
     const long long n_ties = Tfx ? (long long)(tie_mass / Tfx) : 0;
     // the i-th tied id (from 0) has above + i * T before it
     long long n_in = n_ties;
-    if (Tfx && P != ~0ull && above < P) n_in = min(n_ties, (long long)((P - above + Tfx - 1) / Tfx));
+    if (Tfx && P != ~0ull && above < P) n_in = min(n_ties, (long long)((P - above + Tfx - 1) /
+        Tfx));
     if (n_in < n_ties && V <= SP_TIE_BLOCKS * SP_THREADS) {
       // The smallest id bound below which exactly n_in tied ids lie.  Ids in increasing order
       // are (round k of the loop, wave, lane) in lexicographic order: count the tied ids of
@@ -687,13 +701,14 @@ __global__ __launch_bounds__(SP_THREADS) void sample_topp_kernel(
 }
 
 // Raises sample_topp_kernel's dynamic LDS limit, once per device.
+template <typename LT>
 bool allow_cache_lds(int bytes) {
   static std::atomic<uint64_t> done{0};
   int dev = -1;
   if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return false;
   const uint64_t bit = 1ull << dev;
   if (done.load(std::memory_order_acquire) & bit) return true;
-  if (hipFuncSetAttribute((const void*)sample_topp_kernel,
+  if (hipFuncSetAttribute((const void*)sample_topp_kernel<LT>,
                           hipFuncAttributeMaxDynamicSharedMemorySize, bytes) != hipSuccess) {
     (void)hipGetLastError();
     return false;
@@ -713,67 +728,64 @@ int msa_launch_select_combine(const SelectPartial* partials, int n_parts, int B,
   return 0;
 }
 
-extern "C" int msa_greedy_select_f16(const void* logits, int64_t ld_logits, int B, int V,
-                                     float temperature, const int32_t* banned_host, int n_banned,
-                                     const int32_t* stop_host, int n_stop, uint8_t* finished,
-                                     const uint8_t* row_mode, int force_eos_all, int eos_idx,
-                                     int64_t* tok,
-                                     int64_t tok_stride, float* score, int64_t score_stride,
-                                     const int32_t* len_dev, void* stream) {
-  MSA_REQUIRE(logits && tok && score, MSA_ERR_INVALID_ARG, "msa_greedy_select_f16: null pointer");
+namespace {
+
+template <typename LT>
+int greedy_select_impl(const char* name, const void* logits, int64_t ld_logits, int B, int V, float
+                       temperature, const int32_t* banned_host, int n_banned, const int32_t*
+                       stop_host, int n_stop, uint8_t* finished, const uint8_t* row_mode, int
+                       force_eos_all, int eos_idx, int64_t* tok, int64_t tok_stride, float* score,
+                       int64_t score_stride, const int32_t* len_dev, void* stream) {
+  MSA_REQUIRE(logits && tok && score, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
   MSA_REQUIRE(B > 0 && V > 0 && ld_logits >= V, MSA_ERR_INVALID_ARG,
-              "msa_greedy_select_f16: bad shape B=%d V=%d ld=%lld", B, V, (long long)ld_logits);
+              "%s: bad shape B=%d V=%d ld=%lld", name, B, V, (long long)ld_logits);
   MSA_REQUIRE(n_banned >= 0 && n_banned <= 16 && (n_banned == 0 || banned_host),
-              MSA_ERR_INVALID_ARG, "msa_greedy_select_f16: n_banned=%d (0..16)", n_banned);
+              MSA_ERR_INVALID_ARG, "%s: n_banned=%d (0..16)", name, n_banned);
   MSA_REQUIRE(n_stop >= 0 && n_stop <= 16 && (n_stop == 0 || stop_host), MSA_ERR_INVALID_ARG,
-              "msa_greedy_select_f16: n_stop=%d (0..16)", n_stop);
+              "%s: n_stop=%d (0..16)", name, n_stop);
   MSA_REQUIRE(eos_idx >= 0 && eos_idx < V, MSA_ERR_INVALID_ARG,
-              "msa_greedy_select_f16: eos_idx=%d outside the vocabulary", eos_idx);
-  MSA_REQUIRE(temperature >= 0.f, MSA_ERR_INVALID_ARG, "msa_greedy_select_f16: temperature < 0");
+              "%s: eos_idx=%d outside the vocabulary", name, eos_idx);
+  MSA_REQUIRE(temperature >= 0.f, MSA_ERR_INVALID_ARG, "%s: temperature < 0", name);
   const bool scale = temperature > 0.f && temperature != 1.0f;
   IdList banned{}, stop{};
   banned.n = n_banned;
   for (int i = 0; i < n_banned; ++i) banned.id[i] = banned_host[i];
   stop.n = n_stop;
   for (int i = 0; i < n_stop; ++i) stop.id[i] = stop_host[i];
-  hipLaunchKernelGGL(greedy_select_kernel, dim3(B), dim3(SM_THREADS), 0, (hipStream_t)stream,
-                     (const half_t*)logits, ld_logits, V, temperature, scale, banned, stop,
+  hipLaunchKernelGGL(greedy_select_kernel<LT>, dim3(B), dim3(SM_THREADS), 0, (hipStream_t)stream,
+                     (const LT*)logits, ld_logits, V, temperature, scale, banned, stop,
                      finished, row_mode, force_eos_all, eos_idx, tok, tok_stride, score,
                      score_stride, len_dev);
-  MSA_CHECK_LAUNCH("msa_greedy_select_f16");
+  MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }
 
-extern "C" int msa_target_logprob_f16(const void* logits, int64_t ld_logits, int64_t rows, int V,
-                                      float temperature, const int64_t* target, float* out,
-                                      void* stream) {
-  MSA_REQUIRE(logits && target && out, MSA_ERR_INVALID_ARG, "msa_target_logprob_f16: null pointer");
+template <typename LT>
+int target_logprob_impl(const char* name, const void* logits, int64_t ld_logits, int64_t rows, int
+                        V, float temperature, const int64_t* target, float* out, void* stream) {
+  MSA_REQUIRE(logits && target && out, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
   MSA_REQUIRE(rows >= 0 && rows < (1ll << 31) && V > 0 && ld_logits >= V, MSA_ERR_INVALID_ARG,
-              "msa_target_logprob_f16: bad shape rows=%lld V=%d ld=%lld", (long long)rows, V,
+              "%s: bad shape rows=%lld V=%d ld=%lld", name, (long long)rows, V,
               (long long)ld_logits);
   if (rows == 0) return MSA_OK;
   const bool scale = temperature > 0.f && temperature != 1.0f;
-  hipLaunchKernelGGL(target_logprob_kernel, dim3((unsigned)rows), dim3(SM_THREADS), 0,
-                     (hipStream_t)stream, (const half_t*)logits, ld_logits, V, temperature, scale,
+  hipLaunchKernelGGL(target_logprob_kernel<LT>, dim3((unsigned)rows), dim3(SM_THREADS), 0,
+                     (hipStream_t)stream, (const LT*)logits, ld_logits, V, temperature, scale,
                      target, out);
-  MSA_CHECK_LAUNCH("msa_target_logprob_f16");
+  MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }
 
-extern "C" int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B, int V,
-                                   float temperature, const float* temperature_rows,
-                                   const int32_t* banned_host, int n_banned,
-                                   const int32_t* stop_host, int n_stop, uint8_t* finished,
-                                   const uint8_t* row_mode, int force_eos_all, int eos_idx,
-                                   const float* topp_rows, float topp_all, const float* noise,
-                                   int64_t* counts, const int64_t* counts_src,
-                                   float alpha_presence, float alpha_frequency,
-                                   float alpha_presence_src, float alpha_frequency_src,
-                                   const float* penalty_rows, float* lprobs_out,
-                                   int64_t ld_lprobs, int64_t* tok,
-                                   int64_t tok_stride, float* score, int64_t score_stride,
-                                   void* stream) {
-  const char* name = "msa_sample_topp_f16";
+template <typename LT>
+int sample_topp_impl(const char* name, const void* logits, int64_t ld_logits, int B, int V, float
+                     temperature, const float* temperature_rows, const int32_t* banned_host, int
+                     n_banned, const int32_t* stop_host, int n_stop, uint8_t* finished, const
+                     uint8_t* row_mode, int force_eos_all, int eos_idx, const float* topp_rows,
+                     float topp_all, const float* noise, int64_t* counts, const int64_t*
+                     counts_src, float alpha_presence, float alpha_frequency, float
+                     alpha_presence_src, float alpha_frequency_src, const float* penalty_rows,
+                     float* lprobs_out, int64_t ld_lprobs, int64_t* tok, int64_t tok_stride, float*
+                     score, int64_t score_stride, void* stream) {
   MSA_REQUIRE(logits && tok && score, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
   MSA_REQUIRE(B > 0 && V > 0 && ld_logits >= V, MSA_ERR_INVALID_ARG,
               "%s: bad shape B=%d V=%d ld=%lld", name, B, V, (long long)ld_logits);
@@ -802,9 +814,9 @@ extern "C" int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B,
   // as many ids' values as the CU's LDS holds beside the kernel's own 3 KB stay in LDS
   // between the passes (none if the limit cannot be raised)
   int cap = min(V, SP_CACHE_IDS);
-  if (cap * 4 > 48 * 1024 && !allow_cache_lds(SP_CACHE_IDS * 4)) cap = 48 * 1024 / 4;
-  hipLaunchKernelGGL(sample_topp_kernel, dim3(B), dim3(SP_THREADS), (size_t)cap * 4,
-                     (hipStream_t)stream, (const half_t*)logits, ld_logits, V, temperature,
+  if (cap * 4 > 48 * 1024 && !allow_cache_lds<LT>(SP_CACHE_IDS * 4)) cap = 48 * 1024 / 4;
+  hipLaunchKernelGGL(sample_topp_kernel<LT>, dim3(B), dim3(SP_THREADS), (size_t)cap * 4,
+                     (hipStream_t)stream, (const LT*)logits, ld_logits, V, temperature,
                      temperature_rows, banned, stop, finished, row_mode, force_eos_all, eos_idx,
                      topp_rows, topp_all, noise, pen, lprobs_out, ld_lprobs, tok, tok_stride,
                      score, score_stride, cap);
@@ -812,11 +824,10 @@ extern "C" int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B,
   return MSA_OK;
 }
 
-extern "C" int msa_log_softmax_f16(const void* logits, int64_t in_outer_stride, int64_t ld_logits,
-                                   int n_outer, int n_inner, int V, float temperature,
-                                   float* out, int64_t out_outer_stride, int64_t ld_out,
-                                   void* stream) {
-  const char* name = "msa_log_softmax_f16";
+template <typename LT>
+int log_softmax_impl(const char* name, const void* logits, int64_t in_outer_stride, int64_t
+                     ld_logits, int n_outer, int n_inner, int V, float temperature, float* out,
+                     int64_t out_outer_stride, int64_t ld_out, void* stream) {
   MSA_REQUIRE(logits && out, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
   MSA_REQUIRE(n_outer >= 0 && n_inner >= 0 && V > 0 && ld_logits >= V && ld_out >= V &&
                   (int64_t)n_outer * n_inner < (1ll << 31),
@@ -825,9 +836,103 @@ extern "C" int msa_log_softmax_f16(const void* logits, int64_t in_outer_stride, 
   MSA_REQUIRE(temperature >= 0.f, MSA_ERR_INVALID_ARG, "%s: temperature < 0", name);
   if (n_outer == 0 || n_inner == 0) return MSA_OK;
   const bool scale = temperature > 0.f && temperature != 1.0f;
-  hipLaunchKernelGGL(log_softmax_kernel, dim3((unsigned)(n_outer * n_inner)), dim3(SM_THREADS), 0,
-                     (hipStream_t)stream, (const half_t*)logits, in_outer_stride, ld_logits,
+  hipLaunchKernelGGL(log_softmax_kernel<LT>, dim3((unsigned)(n_outer * n_inner)), dim3(SM_THREADS),
+                     0,
+                     (hipStream_t)stream, (const LT*)logits, in_outer_stride, ld_logits,
                      n_inner, V, temperature, scale, out, out_outer_stride, ld_out);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
+}
+
+}  // namespace
+
+extern "C" int msa_greedy_select_f16(const void* logits, int64_t ld_logits, int B, int V, float
+                                    temperature, const int32_t* banned_host, int n_banned, const
+                                    int32_t* stop_host, int n_stop, uint8_t* finished, const
+                                    uint8_t* row_mode, int force_eos_all, int eos_idx, int64_t*
+                                    tok, int64_t tok_stride, float* score, int64_t score_stride,
+                                    const int32_t* len_dev, void* stream) {
+  return greedy_select_impl<half_t>("msa_greedy_select_f16", logits, ld_logits, B, V, temperature,
+                                    banned_host, n_banned, stop_host, n_stop, finished, row_mode,
+                                    force_eos_all, eos_idx, tok, tok_stride, score, score_stride,
+                                    len_dev, stream);
+}
+
+extern "C" int msa_greedy_select_f32(const void* logits, int64_t ld_logits, int B, int V, float
+                                    temperature, const int32_t* banned_host, int n_banned, const
+                                    int32_t* stop_host, int n_stop, uint8_t* finished, const
+                                    uint8_t* row_mode, int force_eos_all, int eos_idx, int64_t*
+                                    tok, int64_t tok_stride, float* score, int64_t score_stride,
+                                    const int32_t* len_dev, void* stream) {
+  return greedy_select_impl<float>("msa_greedy_select_f32", logits, ld_logits, B, V, temperature,
+                                   banned_host, n_banned, stop_host, n_stop, finished, row_mode,
+                                   force_eos_all, eos_idx, tok, tok_stride, score, score_stride,
+                                   len_dev, stream);
+}
+
+extern "C" int msa_target_logprob_f16(const void* logits, int64_t ld_logits, int64_t rows, int V,
+                                    float temperature, const int64_t* target, float* out, void*
+                                    stream) {
+  return target_logprob_impl<half_t>("msa_target_logprob_f16", logits, ld_logits, rows, V,
+                                    temperature, target, out, stream);
+}
+
+extern "C" int msa_target_logprob_f32(const void* logits, int64_t ld_logits, int64_t rows, int V,
+                                    float temperature, const int64_t* target, float* out, void*
+                                    stream) {
+  return target_logprob_impl<float>("msa_target_logprob_f32", logits, ld_logits, rows, V,
+                                    temperature, target, out, stream);
+}
+
+extern "C" int msa_sample_topp_f16(const void* logits, int64_t ld_logits, int B, int V, float
+                                   temperature, const float* temperature_rows, const int32_t*
+                                   banned_host, int n_banned, const int32_t* stop_host, int n_stop,
+                                   uint8_t* finished, const uint8_t* row_mode, int force_eos_all,
+                                   int eos_idx, const float* topp_rows, float topp_all, const
+                                   float* noise, int64_t* counts, const int64_t* counts_src, float
+                                   alpha_presence, float alpha_frequency, float alpha_presence_src,
+                                   float alpha_frequency_src, const float* penalty_rows, float*
+                                   lprobs_out, int64_t ld_lprobs, int64_t* tok, int64_t tok_stride,
+                                   float* score, int64_t score_stride, void* stream) {
+  return sample_topp_impl<half_t>("msa_sample_topp_f16", logits, ld_logits, B, V, temperature,
+                                  temperature_rows, banned_host, n_banned, stop_host, n_stop,
+                                  finished, row_mode, force_eos_all, eos_idx, topp_rows, topp_all,
+                                  noise, counts, counts_src, alpha_presence, alpha_frequency,
+                                  alpha_presence_src, alpha_frequency_src, penalty_rows,
+                                  lprobs_out, ld_lprobs, tok, tok_stride, score, score_stride,
+                                  stream);
+}
+
+extern "C" int msa_sample_topp_f32(const void* logits, int64_t ld_logits, int B, int V, float
+                                   temperature, const float* temperature_rows, const int32_t*
+                                   banned_host, int n_banned, const int32_t* stop_host, int n_stop,
+                                   uint8_t* finished, const uint8_t* row_mode, int force_eos_all,
+                                   int eos_idx, const float* topp_rows, float topp_all, const
+                                   float* noise, int64_t* counts, const int64_t* counts_src, float
+                                   alpha_presence, float alpha_frequency, float alpha_presence_src,
+                                   float alpha_frequency_src, const float* penalty_rows, float*
+                                   lprobs_out, int64_t ld_lprobs, int64_t* tok, int64_t tok_stride,
+                                   float* score, int64_t score_stride, void* stream) {
+  return sample_topp_impl<float>("msa_sample_topp_f32", logits, ld_logits, B, V, temperature,
+                                 temperature_rows, banned_host, n_banned, stop_host, n_stop,
+                                 finished, row_mode, force_eos_all, eos_idx, topp_rows, topp_all,
+                                 noise, counts, counts_src, alpha_presence, alpha_frequency,
+                                 alpha_presence_src, alpha_frequency_src, penalty_rows, lprobs_out,
+                                 ld_lprobs, tok, tok_stride, score, score_stride, stream);
+}
+
+extern "C" int msa_log_softmax_f16(const void* logits, int64_t in_outer_stride, int64_t ld_logits,
+                                   int n_outer, int n_inner, int V, float temperature, float* out,
+                                   int64_t out_outer_stride, int64_t ld_out, void* stream) {
+  return log_softmax_impl<half_t>("msa_log_softmax_f16", logits, in_outer_stride, ld_logits,
+                                  n_outer, n_inner, V, temperature, out, out_outer_stride, ld_out,
+                                  stream);
+}
+
+extern "C" int msa_log_softmax_f32(const void* logits, int64_t in_outer_stride, int64_t ld_logits,
+                                   int n_outer, int n_inner, int V, float temperature, float* out,
+                                   int64_t out_outer_stride, int64_t ld_out, void* stream) {
+  return log_softmax_impl<float>("msa_log_softmax_f32", logits, in_outer_stride, ld_logits,
+                                 n_outer, n_inner, V, temperature, out, out_outer_stride, ld_out,
+                                 stream);
 }

@@ -1,4 +1,5 @@
-"""Preallocated contiguous per-layer KV cache.
+"""Preallocated contiguous per-layer caches: keys and values, and the latents and recurrent states
+of hybrid decoders (``HybridCache``).
 
 The reference grows its cache by ``torch.cat`` every step and every layer
 (metaseq/modules/multihead_attention.py:449-479), re-copying the whole history.  Here each
@@ -56,6 +57,11 @@ class KVCache:
             self.layers[i] = new
         self.capacity = new_capacity
 
+    def copy_row(self, src, dst, n):
+        """Row ``dst`` takes the first ``n`` positions of row ``src``."""
+        for layer in self.layers:
+            layer[:, dst, :, :n].copy_(layer[:, src, :, :n])
+
     def bytes(self):
         return sum(t.numel() * 2 for t in self.layers)
 
@@ -79,3 +85,68 @@ class _RowsView:
 
     def v(self, i):
         return self._cache.layers[i][1][self._b0:self._b1]
+
+
+class HybridCache:
+    """What the layers of a hybrid decoder keep per slot (a row of a batch, or a serving slot):
+
+    * attention layers that own a latent: ``latent`` [slots, capacity, rank], activation format;
+    * recurrent layers: ``conv`` [slots, taps - 1, channels], the short convolution's last inputs
+      (activation format), and ``rec``, the fp32 recurrent state.
+
+    ``lens`` (int32 [slots] on the device): positions each slot holds, negative = empty slot;
+    ``host_lens``: the same on the host where the caller of the slot interface knows it.  Nothing
+    has to be cleared when a slot is given to a new sequence: a segment that starts at position 0
+    ignores what the slot held.  Lives in the caller's ``incremental_state`` like ``KVCache``."""
+
+    has_pads = False
+    ragged = True
+
+    def __init__(self, layout, slots, capacity, dtype, device):
+        """``layout``: per layer {"latent": rank} and / or {"conv": (taps - 1, channels), "rec":
+        shape} (what the layer keeps; an empty dict: nothing)."""
+        self.layout, self.batch, self.capacity = layout, int(slots), int(capacity)
+        self.dtype, self.device = dtype, device
+        self.length = 0
+        self.lens = torch.full((self.batch,), -1, dtype=torch.int32, device=device)
+        self.host_lens = [-1] * self.batch
+        self.layers = []
+        for keep in layout:
+            t = {}
+            if "latent" in keep:
+                t["latent"] = torch.zeros(self.batch, self.capacity, keep["latent"], dtype=dtype,
+                                          device=device)
+            if "rec" in keep:
+                t["rec"] = torch.zeros((self.batch,) + tuple(keep["rec"]), dtype=torch.float32,
+                                       device=device)
+            if keep.get("conv", (0,))[0] > 0:
+                t["conv"] = torch.zeros((self.batch,) + tuple(keep["conv"]), dtype=dtype,
+                                        device=device)
+            self.layers.append(t)
+
+    def grow(self, new_capacity):
+        """Re-allocates the latents to ``new_capacity`` positions per slot."""
+        new_capacity = int(new_capacity)
+        if new_capacity <= self.capacity:
+            return
+        for t in self.layers:
+            if "latent" in t:
+                old = t["latent"]
+                new = torch.zeros(self.batch, new_capacity, old.shape[2], dtype=self.dtype,
+                                  device=self.device)
+                new[:, :self.capacity].copy_(old)
+                t["latent"] = new
+        self.capacity = new_capacity
+
+    def copy_row(self, src, dst, n):
+        """Slot ``dst`` becomes slot ``src``, which holds ``n`` positions."""
+        for t in self.layers:
+            for name, x in t.items():
+                if name == "latent":
+                    x[dst, :n].copy_(x[src, :n])
+                else:
+                    x[dst].copy_(x[src])
+        self.host_lens[dst] = n
+
+    def bytes(self):
+        return sum(x.numel() * x.element_size() for t in self.layers for x in t.values())

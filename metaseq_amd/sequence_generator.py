@@ -137,7 +137,7 @@ class SequenceGenerator(nn.Module):
         col = 0 if len_dev is not None else step
         tok = tokens[:, col]
         sc = scores[:, col]
-        check(lib.msa_greedy_select_f16(
+        check(_capi.for_logits(lib, "msa_greedy_select", logits2d)(
             ptr(logits2d), logits2d.stride(0), B, V, float(self.temperature), arr, len(banned),
             stop, len(self.stop), ptr(finished), None, int(step >= max_len - 1), self.eos,
             ptr(tok), tokens.stride(0), ptr(sc), scores.stride(0), ptr(len_dev),
@@ -226,9 +226,9 @@ class SequenceGenerator(nn.Module):
                 target = torch.zeros(BB, T, dtype=torch.long, device=dev)
                 target[:, :-1] = tokens[:, 1:start_step]
                 lp = torch.empty(BB, T, dtype=torch.float32, device=dev)
-                check(lib.msa_target_logprob_f16(ptr(flat), flat.stride(0), BB * T, V,
-                                                 float(self.temperature), ptr(target), ptr(lp),
-                                                 stream))
+                check(_capi.for_logits(lib, "msa_target_logprob", flat)(
+                    ptr(flat), flat.stride(0), BB * T, V, float(self.temperature), ptr(target),
+                    ptr(lp), stream))
                 scores[:, 1:start_step] = lp[:, :-1]
             # scores after each row's own prompt are reset (:262-266)
             col = torch.arange(max_len, device=dev).unsqueeze(0)
@@ -236,7 +236,7 @@ class SequenceGenerator(nn.Module):
             if all_lprobs is not None and start_step > 1:
                 # the distributions of the prompt positions (:247-250), fp32 rows written in place
                 dst = all_lprobs[:, 1]
-                check(lib.msa_log_softmax_f16(ptr(flat), T * flat.stride(0), flat.stride(0), BB,
+                check(_capi.for_logits(lib, "msa_log_softmax", flat)(ptr(flat), T * flat.stride(0), flat.stride(0), BB,
                                               start_step - 1, V, float(self.temperature), ptr(dst),
                                               all_lprobs.stride(0), all_lprobs.stride(1), stream))
             # the row that predicts each sample's first free token (:262-267)
@@ -255,7 +255,8 @@ class SequenceGenerator(nn.Module):
             gs = self._general_state(src_tokens, BB, V, dev) if general else None
             st = None
             if (self.use_graph and all_lprobs is None and cache is not None and BB <= 64
-                    and not cache.has_pads and not general):
+                    and not cache.has_pads and not general
+                    and hasattr(decoder, "decode_step_static")):
                 st = self.static_state(decoder, cache, tokens, scores, finished, step_logits)
             fused = (not general and all_lprobs is None and st is None and BB <= 128
                      and hasattr(decoder, "forward_select"))
@@ -380,7 +381,7 @@ class SequenceGenerator(nn.Module):
                      else gs["noise"].exponential_())
         topp_rows = gs["topp"] if (self.sampling and self.lambda_decay > 0) else None
         tok, sc = tokens[:, step], scores[:, step]
-        check(lib.msa_sample_topp_f16(
+        check(_capi.for_logits(lib, "msa_sample_topp", step_logits)(
             ptr(step_logits), step_logits.stride(0), BB, V, float(self.temperature), None, ba,
             len(banned), sa, len(self.stop), ptr(finished), None, int(step >= max_len - 1),
             self.eos, ptr(topp_rows), float(self.sampling_topp) if self.sampling else 0.0,

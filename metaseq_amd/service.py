@@ -28,9 +28,9 @@ from typing import Any, Dict, List, Optional
 
 def upload(values, dtype, device):
     """A short host list as a device tensor, stream-ordered through pinned memory (see
-    ``transformer_decoder.upload``): the serving loop must not wait for the step in flight
+    ``decoder_base.upload``): the serving loop must not wait for the step in flight
     every time it hands the GPU a few indices."""
-    from .transformer_decoder import upload as _upload
+    from .decoder_base import upload as _upload
     return _upload(values, dtype, device)
 
 # options that must agree within a run-to-completion batch (metaseq/service/workers.py:13-23)
@@ -519,7 +519,8 @@ class ContinuousBatcher(_Front):
             torch, dev, slots = self._torch, self.device, len(self.batch.rows)
             V = len(self.dict)
             self._topp = torch.zeros(slots, dtype=torch.float32, device=dev)
-            self._logits = torch.empty(slots, V, dtype=torch.float16, device=dev)
+            self._logits = torch.empty(
+                slots, V, dtype=getattr(self.decoder, "logits_dtype", torch.float16), device=dev)
             self._noise = torch.empty(slots, V, dtype=torch.float32, device=dev)
             self._since = torch.zeros(slots, 1, dtype=torch.float32, device=dev)
 

@@ -7,19 +7,20 @@ from typing import Dict, Optional
 import torch
 from torch import nn
 
-from .config import OPTConfig
-from .transformer_decoder import TransformerDecoder
+from .decoder_base import IncrementalDecoder
 
 
 class TransformerLanguageModel(nn.Module):
-    def __init__(self, decoder: TransformerDecoder):
+    def __init__(self, decoder: IncrementalDecoder):
         super().__init__()
         self.decoder = decoder
 
     @classmethod
-    def build_model(cls, cfg: OPTConfig, state_dict: Optional[Dict[str, torch.Tensor]] = None,
-                    device="cuda"):
-        return cls(TransformerDecoder(cfg, state_dict, device=device))
+    def build_model(cls, cfg, state_dict: Optional[Dict[str, torch.Tensor]] = None,
+                    device="cuda", **kwargs):
+        """``cfg``: the configuration of a registered architecture; ``kwargs`` go to its decoder."""
+        from .registry import decoder_class
+        return cls(decoder_class(cfg)(cfg, state_dict, device=device, **kwargs))
 
     def forward(self, src_tokens, **kwargs):
         """metaseq/models/base_model.py:152-168."""
