@@ -7,12 +7,13 @@ from .hybrid_decoder import HybridDecoder
 from .kv_cache import HybridCache, KVCache
 from .registry import load_model
 from .sequence_generator import SequenceGenerator
-from .synthetic import iter_random_state_dict, random_prompts, random_state_dict
+from .synthetic import (iter_random_state_dict, random_hybrid_state_dict, random_prompts,
+                        random_state_dict)
 from .transformer_decoder import ModelParallelTransformerDecoder, TransformerDecoder
 from .transformer_lm import TransformerLanguageModel
 
 __all__ = [
     "OPTConfig", "HybridConfig", "HybridDecoder", "HybridCache", "load_model", "opt_config", "config_from_state_dict", "Dictionary", "GeneratorInterface", "KVCache", "SequenceGenerator", "random_prompts",
-    "random_state_dict", "iter_random_state_dict", "TransformerDecoder", "ModelParallelTransformerDecoder",
+    "random_state_dict", "random_hybrid_state_dict", "iter_random_state_dict", "TransformerDecoder", "ModelParallelTransformerDecoder",
     "TransformerLanguageModel",
 ]

@@ -11,7 +11,7 @@ from typing import Dict, Iterator, Tuple
 
 import torch
 
-from .config import OPTConfig
+from .config import HybridConfig, OPTConfig
 
 
 def iter_random_state_dict(cfg: OPTConfig, seed: int = 1234, dtype=torch.float16,
@@ -70,3 +70,33 @@ def random_prompts(cfg: OPTConfig, batch: int, prompt_len: int, seed: int = 4321
     ids = torch.randint(4, cfg.vocab_size, (batch, prompt_len), generator=gen, dtype=torch.long)
     eos = torch.full((batch, 1), cfg.eos_idx, dtype=torch.long)
     return torch.cat([eos, ids], dim=1).to(device)
+
+
+def random_hybrid_state_dict(cfg: HybridConfig, seed: int = 1234, dtype=torch.bfloat16,
+                             device="cpu") -> Dict[str, torch.Tensor]:
+    """Seeded random weights of a hybrid decoder by checkpoint name, drawn in the order of
+    ``tensor_shapes``: matrices ~ N(0, 1 / fan-in), norm weights around 1, convolution taps of
+    order 1, decays spread over short and long memories."""
+    device = torch.device(device)
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    out = {}
+    for name, shape in cfg.tensor_shapes().items():
+        t = torch.empty(*shape, dtype=torch.float32, device=device)
+        last = name.rsplit(".", 1)[-1]
+        if last.startswith("norm"):
+            t.normal_(1.0, 0.1, generator=gen)
+        elif last == "embed":
+            t.normal_(0.0, 1.0, generator=gen)
+        elif last == "lam":                 # softplus(lam) 8 r: from slow to fast decays
+            t.uniform_(-7.0, 0.0, generator=gen)
+        elif last in ("A_log", "dt_bias"):
+            t.uniform_(-3.0, 0.5, generator=gen)
+        elif last == "conv":
+            t.normal_(0.0, shape[-1] ** -0.5, generator=gen)
+        elif last == "b" and len(shape) < 3 and not name.endswith("mix.b"):
+            t.normal_(0.0, 0.3, generator=gen)
+        else:
+            t.normal_(0.0, shape[-1] ** -0.5, generator=gen)
+        out[name] = t.to(dtype)
+    return out

@@ -29,7 +29,8 @@ def sinusoid(positions, width, dtype=torch.float64):
 
 
 def causal_conv(x, w, bias=None):
-    """x [T, C], w [C, taps]; the last tap weighs the current position, zeros before the start."""
+    """x [T, C], w [C, taps]; the last tap weighs the current position; a position in front of the
+    sequence counts as 0."""
     T, taps = x.shape[0], w.shape[1]
     out = torch.zeros_like(x)
     for t in range(T):

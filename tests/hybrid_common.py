@@ -1,0 +1,113 @@
+"""Small hybrid configurations, their weights and comparisons with the plain oracle."""
+import torch
+
+from metaseq_amd import HybridConfig, HybridDecoder, random_hybrid_state_dict
+from oracle import hybrid_oracle as O
+
+# error of the logits: root mean square over the vocabulary of the mean-free difference, over the
+# root mean square of all logits: the most any row may have, and the median row
+LIMIT = {torch.float32: 2e-5, torch.bfloat16: 6e-2}
+MEDIAN = {torch.float32: 5e-6, torch.bfloat16: 2e-2}
+
+
+def latent(heads=3, dim=24, vdim=40, kv_rank=80, q_rank=56, scale=0.3, kv_from=None):
+    m = dict(heads=heads, dim=dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank, scale=scale)
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return "latent_attention", m
+
+
+def rglru(width=96, blocks=3, conv=3):
+    return "rglru", dict(width=width, blocks=blocks, conv=conv)
+
+
+def delta(heads=6, kv_heads=2, dim=20, vdim=24, conv=4):
+    return "delta", dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=conv)
+
+
+def dense(ff=136):
+    return dict(kind="dense", ff=ff)
+
+
+def moe(experts=10, top=3, scale=1.5, groups=(5, 2), ff=40, limit=1.5, shared=(72, 0.8)):
+    router = dict(experts=experts, top=top, scale=scale)
+    if groups:
+        router["groups"] = dict(count=groups[0], keep=groups[1])
+    out = dict(kind="moe", router=router, expert=dict(ff=ff, limit=limit))
+    if shared:
+        out["shared"] = dict(ff=shared[0], limit=shared[1])
+    return out
+
+
+def config(layers, width=72, vocab=101, eps=1e-5, scale=2.0):
+    """A config.json dictionary; ``layers``: ((type, mixer), mlp) pairs."""
+    return dict(architecture="Sinulorn", width=width, vocab=vocab, norm=dict(eps=eps),
+                embedding=dict(scale=scale),
+                layers=[dict(type=t, mixer=m, mlp=f) for (t, m), f in layers])
+
+
+def mixed(dtype=torch.float32, width=72):
+    """Every mechanism once, a borrowed latent, an expert layer without groups, a layer without a
+    feed-forward.  With random weights some token's choice of experts is always so close that bf16
+    rounding decides it (and the recurrences carry the other choice on), so in bf16 every
+    expert is chosen; the choice itself is tested in fp32 and row by row."""
+    pick = {} if dtype == torch.float32 else dict(experts=4, top=4, groups=(2, 2))
+    flat = dict(pick, groups=None)
+    return config([(delta(), dense()), (latent(), moe(**pick)), (rglru(), None),
+                   (latent(heads=2, dim=36, vdim=16, q_rank=40, kv_from=1), moe(**flat)),
+                   (delta(heads=4, kv_heads=4, dim=40, vdim=16, conv=2), moe(shared=None, **pick)),
+                   (rglru(width=80, blocks=2, conv=5), dense(100))], width=width)
+
+
+def no_specials(state):
+    """Logits of the special ids 0 .. 3 are never the largest (a record ends at one)."""
+    state["head"][:4] = 0
+
+
+class Case:
+    """A model and its oracle; the oracle sees the weights the product loads (rounded to bf16)."""
+
+    def __init__(self, cfg, seed=1, dtype=torch.float32, tweak=None, device="cuda"):
+        self.json, self.dtype = cfg, dtype
+        self.cfg = HybridConfig.from_json(cfg)
+        self.state = random_hybrid_state_dict(self.cfg, seed)
+        if tweak is not None:
+            tweak(self.state)
+        self.W = {k: v.double() for k, v in self.state.items()}
+        self.decoder = HybridDecoder(self.cfg, self.state, device=device, dtype=dtype)
+
+    def tokens(self, n, seed=0):
+        g = torch.Generator().manual_seed(seed)
+        return torch.randint(4, self.cfg.vocab_size, (n,), generator=g)
+
+    def want(self, tokens, layers=False):
+        return O.forward(torch.as_tensor(tokens), self.W, self.json, layers)
+
+    def run(self, tokens, portions=None, slot=0, cache=None):
+        """Logits of every position, the tokens cut into ``portions`` (the last one repeats)."""
+        n = len(tokens)
+        cache = cache or self.decoder.new_slot_cache(slot + 1, n)
+        out, at, k = [], 0, 0
+        while at < n:
+            step = n if portions is None else portions[min(k, len(portions) - 1)]
+            piece = torch.as_tensor(tokens[at:at + step]).to(self.decoder.device)
+            out.append(self.decoder.extend(cache, [(slot, piece)], want_all=True))
+            at, k = at + step, k + 1
+        return torch.cat(out)
+
+    def check(self, got, want, what="", close_calls=0.0):
+        """Every row within the limit, but for a share of ``close_calls`` of them."""
+        got, want = got.double().cpu(), want.double().cpu()
+        assert got.shape == want.shape, (what, got.shape, want.shape)
+        assert torch.isfinite(got).all(), what
+        d = got - want
+        d = d - d.mean(dim=-1, keepdim=True)
+        rows = d.pow(2).mean(dim=-1).sqrt() / want.pow(2).mean().sqrt()
+        worst = float(rows.max())
+        print("%s %s: worst row error %.2e at %d of %d" % (what, self.dtype, worst,
+                                                           int(rows.argmax()), rows.numel()),
+              flush=True)
+        over = float((rows > LIMIT[self.dtype]).double().mean())
+        assert over <= close_calls, (what, worst, over)
+        assert float(rows.median()) <= MEDIAN[self.dtype], (what, float(rows.median()))
+        return worst

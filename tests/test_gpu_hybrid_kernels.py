@@ -1,0 +1,266 @@
+"""Kernels of the hybrid library one by one against plain PyTorch on the CPU."""
+import ctypes
+
+import pytest
+import torch
+
+from metaseq_amd import _capi
+from metaseq_amd._capi import check, ptr
+from metaseq_amd.hybrid_decoder import pack_tiles
+from oracle import hybrid_oracle as O
+
+pytestmark = pytest.mark.gpu
+BF16, F32 = torch.bfloat16, torch.float32
+
+
+def gen(seed):
+    return torch.Generator().manual_seed(seed)
+
+
+def pack_rows(x):
+    """[M, K] bf16 -> the packed activation layout of at most 128 rows."""
+    M, K = x.shape
+    MB = (M + 15) // 16 if M <= 64 else 8
+    full = torch.zeros(MB * 16, K, dtype=x.dtype)
+    full[:M] = x
+    return full.view(MB, 16, K // 32, 4, 8).permute(2, 0, 3, 1, 4).contiguous()
+
+
+def unpack_rows(p, M, K):
+    MB = (M + 15) // 16 if M <= 64 else 8
+    return p.view(K // 32, MB, 4, 16, 8).permute(1, 3, 0, 2, 4).reshape(MB * 16, K)[:M]
+
+
+def close(got, want, tol, what):
+    err = float((got.double().cpu() - want.double()).abs().max() / want.double().abs().max())
+    print(what, "%.2e" % err, flush=True)
+    assert err <= tol, (what, err)
+
+
+def glu(kind, g, u, limit):
+    if kind == _capi.MSA_GLU_GELU:
+        return O.gelu_tanh(g) * u
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return g * torch.sigmoid(1.702 * g) * (u + 1)
+
+
+# rows x features x reduction: every kernel of the bf16 products (packed streaming up to 128 rows,
+# 128 x 128 tiles, four-wave tiles of three widths, ragged bottoms)
+SHAPES = [(1, 64, 128), (5, 208, 192), (17, 96, 256), (33, 4096, 512), (64, 272, 128),
+          (100, 1040, 320), (128, 512, 1024), (129, 48, 128), (200, 272, 192), (300, 1600, 256),
+          (700, 4112, 256), (1024, 8192, 128), (1100, 16384, 192)]
+
+
+@pytest.mark.parametrize("M,N,K", SHAPES)
+def test_linear_bf16(M, N, K):
+    lib = _capi.load_hybrid()
+    print("linear_bf16", M, N, K, flush=True)
+    g = gen(M + N)
+    x = torch.randn(M, K, generator=g).to(BF16)
+    w = (torch.randn(N, K, generator=g) * K ** -0.5).to(BF16)
+    ref = x.double() @ w.double().T
+    wp = pack_tiles(w).cuda()
+    packed = M <= 128
+    xd = (pack_rows(x) if packed else x).cuda()
+    flags = _capi.MSA_IN_PACKED if packed else 0
+    for n32 in sorted({N, N - 16, N // 2 // 16 * 16, 0}):
+        y = torch.zeros(M, n32, dtype=BF16, device="cuda")
+        y32 = torch.zeros(M, N - n32, dtype=F32, device="cuda")
+        check(lib.msa_linear_bf16(ptr(xd), ptr(wp), ptr(y), ptr(y32), M, N, K, n32, -1, 0.0, flags,
+                                  _capi.stream_ptr()), lib)
+        if n32:
+            close(y, ref[:, :n32], 6e-3, "bf16 columns of n32=%d" % n32)
+        if n32 < N:
+            close(y32, ref[:, n32:], 1e-5, "fp32 columns of n32=%d" % n32)
+    for kind, n32 in ((_capi.MSA_GLU_GELU, N // 32 * 32), (_capi.MSA_GLU_CLAMPED, N // 64 * 32)):
+        if n32 == 0:
+            continue
+        out_packed = packed and (n32 // 2) % 32 == 0
+        MB = (M + 15) // 16 if M <= 64 else 8
+        y = torch.zeros((MB * 16 if out_packed else M) * (n32 // 2), dtype=BF16, device="cuda")
+        y32 = torch.zeros(M, N - n32, dtype=F32, device="cuda")
+        check(lib.msa_linear_bf16(ptr(xd), ptr(wp), ptr(y), ptr(y32), M, N, K, n32, kind, 0.7,
+                                  flags | (_capi.MSA_OUT_PACKED if out_packed else 0),
+                                  _capi.stream_ptr()), lib)
+        got = unpack_rows(y.cpu(), M, n32 // 2) if out_packed else y.view(M, n32 // 2)
+        close(got, glu(kind, ref[:, 0:n32:2], ref[:, 1:n32:2], 0.7), 6e-3, "glu %d" % kind)
+        if n32 < N:
+            close(y32, ref[:, n32:], 1e-5, "fp32 columns beside glu")
+    for S in {1, lib.msa_linear_bf16_splits(M, N, K, int(packed))}:
+        part = torch.zeros(S, M, N, dtype=F32, device="cuda")
+        check(lib.msa_linear_partial_bf16(ptr(xd), ptr(wp), ptr(part), M, N, K, S, flags,
+                                          _capi.stream_ptr()), lib)
+        close(part.sum(0), ref, 1e-5, "partial sums, S=%d" % S)
+
+
+@pytest.mark.parametrize("M,N,K", [(1, 16, 32), (70, 80, 96), (200, 144, 128)])
+def test_linear_f32(M, N, K):
+    lib = _capi.load_hybrid()
+    g = gen(M)
+    x, w = torch.randn(M, K, generator=g), torch.randn(N, K, generator=g) * K ** -0.5
+    ref = x.double() @ w.double().T
+    n32 = N // 32 * 32
+    if n32 == N:
+        n32 -= 32
+    xd, wd = x.cuda(), w.cuda()
+    for kind in (-1, 0, 1):
+        cols = n32 if kind < 0 else n32 // 2
+        y = torch.zeros(M, cols, device="cuda")
+        y32 = torch.zeros(M, N - n32, device="cuda")
+        check(lib.msa_linear_f32(ptr(xd), ptr(wd), ptr(y), ptr(y32), M, N, K, n32, kind, 0.6,
+                                 _capi.stream_ptr()), lib)
+        if cols:
+            want = ref[:, :n32] if kind < 0 else glu(kind, ref[:, 0:n32:2], ref[:, 1:n32:2], 0.6)
+            close(y, want, 2e-6, "glu %d" % kind)
+        close(y32, ref[:, n32:], 2e-6, "tail")
+
+
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+@pytest.mark.parametrize("M", [1, 16, 20, 64, 150])
+def test_group_linear_dense(M, dtype):
+    """Per-group columns (a head, a diagonal block), also with the groups' inputs shared."""
+    lib = _capi.load_hybrid()
+    for G, N, K, share in ((3, 48, 64, 0), (6, 160, 32, 3), (1, 272, 128, 0)):
+        g = gen(M + G)
+        xg = share or G
+        x = torch.randn(M, xg * K, generator=g).to(dtype)
+        w = (torch.randn(G, N, K, generator=g) * K ** -0.5).to(dtype)
+        ref = torch.stack([x[:, (i % xg) * K:(i % xg + 1) * K].double() @ w[i].double().T
+                           for i in range(G)], dim=1).view(M, G * N)
+        wd = (pack_tiles(w.view(G * N, K)) if dtype == BF16 else w.view(G * N, K)).cuda()
+        xd = x.cuda()
+        for y_f32 in (0, 1):
+            y = torch.zeros(M, G * N, dtype=F32 if y_f32 else dtype, device="cuda")
+            a = _capi.GroupLinearArgs()
+            a.dtype, a.glu = (0 if dtype == BF16 else 1), -1
+            a.x, a.ldx, a.x_group, a.x_groups = ptr(xd), xg * K, K, share
+            a.W, a.y, a.ldy, a.y_group, a.y_f32 = ptr(wd), ptr(y), G * N, N, y_f32
+            a.N, a.K, a.groups, a.M = N, K, G, M
+            check(lib.msa_group_linear(ctypes.byref(a), _capi.stream_ptr()), lib)
+            tol = 2e-6 if dtype == F32 else (1e-5 if y_f32 else 6e-3)
+            close(y, ref, tol, "groups %s" % ((G, N, K, share),))
+
+
+@pytest.mark.parametrize("E,groups,keep,top", [(1, 1, 1, 1), (12, 1, 1, 5), (12, 4, 2, 3),
+                                               (96, 8, 3, 10), (512, 16, 16, 8), (300, 100, 1, 3)])
+def test_route_and_plan(E, groups, keep, top):
+    lib = _capi.load_hybrid()
+    M = 77
+    z = torch.randn(M, E + 5, generator=gen(E)) * 2
+    want_ids, want_w = O.route(z[:, :E].double(), dict(
+        top=top, scale=1.7, groups=dict(count=groups, keep=keep)))
+    zd = z.cuda()
+    ids = torch.zeros(M, top, dtype=torch.int32, device="cuda")
+    w = torch.zeros(M, top, device="cuda")
+    sg = torch.zeros(M, device="cuda")
+    check(lib.msa_moe_route(ptr(zd), E + 5, M, E, groups, keep, top, 1.7, ptr(ids), ptr(w), ptr(sg),
+                            _capi.stream_ptr()), lib)
+    assert torch.equal(ids.cpu().long(), want_ids)
+    close(w, want_w, 1e-5, "weights")
+    close(sg, torch.sigmoid(z[:, E].double()), 1e-6, "shared gate")
+    P = M * top
+    for rows in (16, 64):
+        n_max = P // rows + min(E, P)
+        perm, inv = (torch.full((P,), -1, dtype=torch.int32, device="cuda") for _ in range(2))
+        end = torch.zeros(E, dtype=torch.int32, device="cuda")
+        tg, tr = (torch.full((n_max,), -1, dtype=torch.int32, device="cuda") for _ in range(2))
+        n = torch.zeros(1, dtype=torch.int32, device="cuda")
+        check(lib.msa_moe_plan(ptr(ids), P, E, rows, ptr(perm), ptr(inv), ptr(end), ptr(tg), ptr(tr),
+                               ptr(n), n_max, _capi.stream_ptr()), lib)
+        flat = ids.cpu().view(-1).long()
+        order = torch.sort(flat, stable=True).indices
+        assert torch.equal(perm.cpu().long(), order)
+        assert torch.equal(inv.cpu().long()[order], torch.arange(P))
+        counts = torch.bincount(flat, minlength=E)
+        assert torch.equal(end.cpu().long(), counts.cumsum(0))
+        tiles = [(e, int(counts[:e].sum()) + r) for e in range(E)
+                 for r in range(0, int(counts[e]), rows)]
+        assert int(n) == len(tiles)
+        assert list(zip(tg.cpu().tolist(), tr.cpu().tolist()))[:len(tiles)] == tiles
+
+
+@pytest.mark.parametrize("hd", [32, 64, 96, 128, 192, 256])
+@pytest.mark.parametrize("T,pos0", [(1, 0), (17, 3), (64, 64), (130, 0), (33, 400), (300, 100)])
+def test_flash_attention(hd, T, pos0):
+    lib = _capi.load_hybrid()
+    heads, S = 3, T + pos0
+    g = gen(hd + T)
+    q = torch.randn(T, heads * hd, generator=g).to(BF16)
+    kv = torch.randn(S, 2 * heads * hd, generator=g).to(BF16)
+    scale = 1.5 * hd ** -0.5
+    k, v = (t.double().view(S, heads, hd) for t in kv.split(heads * hd, dim=1))
+    s = torch.einsum("thd,shd->hts", q.double().view(T, heads, hd), k) * scale
+    mask = torch.arange(S).view(1, S) > pos0 + torch.arange(T).view(T, 1)
+    p = torch.softmax(s.masked_fill(mask, float("-inf")), dim=-1)
+    ref = torch.einsum("hts,shd->thd", p, v).reshape(T, heads * hd)
+    out = torch.zeros(T, heads * hd, dtype=BF16, device="cuda")
+    qd, kvd = q.cuda(), kv.cuda()
+    check(lib.msa_flash_attention_bf16(ptr(qd), heads * hd, ptr(kvd), 2 * heads * hd, ptr(out),
+                                       heads * hd, 0, 0, heads, hd, T, pos0, scale,
+                                       _capi.stream_ptr()), lib)
+    close(out, ref, 1e-2, "flash %d" % hd)
+
+
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+@pytest.mark.parametrize("rp", [128, 192, 256, 384, 512, 640])
+def test_latent_attention(rp, dtype):
+    """Rows of several slots at their own positions, an inactive row, and one to eight splits."""
+    lib = _capi.load_hybrid()
+    heads, cap, slots = 19, 700, 3
+    g = gen(rp)
+    pos = [0, 31, 32, 127, 128, 129, 300, 640, 699, -1]
+    slot = [i % slots for i in range(len(pos))]
+    M = len(pos)
+    c = torch.randn(slots, cap, rp, generator=g).to(dtype)
+    q = torch.randn(M, heads, rp, generator=g).to(dtype)
+    scale = 1.5 * rp ** -0.5
+    ref = torch.zeros(M, heads, rp, dtype=torch.float64)
+    for m in range(M):
+        if pos[m] >= 0:
+            rows = c[slot[m], :pos[m] + 1].double()
+            ref[m] = torch.softmax(q[m].double() @ rows.T * scale, dim=-1) @ rows
+    cd, qd = c.cuda(), q.cuda()
+    ts = torch.tensor(slot, dtype=torch.int32, device="cuda")
+    tp = torch.tensor(pos, dtype=torch.int32, device="cuda")
+    for splits in (1, 2, 8):
+        out = torch.full((M, heads, rp), 9.0, dtype=dtype, device="cuda")
+        part = torch.zeros(M, heads, splits, rp + 4, device="cuda")
+        check(lib.msa_latent_attention(0 if dtype == BF16 else 1, ptr(qd), ptr(cd), cap, heads, rp,
+                                       scale, ptr(out), ptr(part), splits, ptr(ts), ptr(tp), M,
+                                       _capi.stream_ptr()), lib)
+        close(out, ref, 1e-2 if dtype == BF16 else 1e-5, "latent %d, %d splits" % (rp, splits))
+
+
+def test_selection_over_fp32_logits():
+    """The fp32 forms of selection, scoring and sampling agree with plain PyTorch, at row strides
+    and vocabulary sizes that are no multiple of 8."""
+    lib = _capi.load()
+    for V, ld in ((101, 112), (1000, 1000), (50001, 50016)):
+        z = torch.randn(5, ld, generator=gen(V)).cuda() * 3
+        lp = torch.log_softmax(z[:, :V].double(), dim=-1)
+        tok = torch.zeros(5, dtype=torch.long, device="cuda")
+        score = torch.zeros(5, device="cuda")
+        ban = (ctypes.c_int32 * 1)(1)
+        none = (ctypes.c_int32 * 1)()
+        check(lib.msa_greedy_select_f32(ptr(z), ld, 5, V, 1.0, ban, 1, none, 0, None, None, 0, 2,
+                                        ptr(tok), 1, ptr(score), 1, None, _capi.stream_ptr()))
+        masked = lp.clone()
+        masked[:, 1] = float("-inf")
+        assert torch.equal(tok, masked.argmax(dim=-1))
+        close(score, masked.max(dim=-1).values.cpu(), 1e-5, "score")
+        target = torch.randint(0, V, (5,), generator=gen(1)).cuda()
+        got = torch.zeros(5, device="cuda")
+        check(lib.msa_target_logprob_f32(ptr(z), ld, 5, V, 1.0, ptr(target), ptr(got),
+                                         _capi.stream_ptr()))
+        close(got, lp.gather(1, target.view(-1, 1)).view(-1).cpu(), 1e-5, "target")
+        rows = torch.zeros(5, V, device="cuda")
+        check(lib.msa_log_softmax_f32(ptr(z), 0, ld, 1, 5, V, 1.0, ptr(rows), 0, V,
+                                      _capi.stream_ptr()))
+        close(rows, lp.cpu(), 1e-5, "log-softmax")
+        noise = torch.empty(5, V, device="cuda").exponential_()
+        check(lib.msa_sample_topp_f32(ptr(z), ld, 5, V, 1.0, None, ban, 1, none, 0, None, None, 0, 2,
+                                      None, 0.999999, ptr(noise), None, None, 0.0, 0.0, 0.0, 0.0,
+                                      None, None, 0, ptr(tok), 1, ptr(score), 1, _capi.stream_ptr()))
+        p = torch.softmax(z[:, :V].double(), dim=-1)
+        p[:, 1] = 0
+        assert torch.equal(tok, (p / noise.double()).argmax(dim=-1))
