@@ -387,6 +387,125 @@ def service_throughput(config, slots, prefill_batch, prefill_wait, seed=1):
     }
 
 
+HYBRID_STACKS = {
+    # four layers each: (mixer, feed-forward)
+    "latent + dense": [("latent", "dense")] * 4,
+    "rglru + dense": [("rglru", "dense")] * 4,
+    "delta + dense": [("delta", "dense")] * 4,
+    "latent + moe": [("latent", "moe")] * 4,
+    "mixed": [("rglru", "dense"), ("latent", "moe"), ("delta", "dense"), ("latent-borrowed", "moe")],
+}
+
+
+def hybrid_config(width, stack, vocab=50272):
+    """A hybrid decoder of a real model's layer sizes at this width: heads of 128, a latent of
+    512, gate blocks of 256, 64 experts of which 8 run, and a dense feed-forward of as many
+    weights as OPT's 4 x width."""
+    from metaseq_amd import HybridConfig
+    heads = width // 128
+
+    def mixer(kind, i):
+        if kind.startswith("latent"):
+            m = dict(heads=heads, dim=128, vdim=128, kv_rank=512, q_rank=3 * width // 8,
+                     scale=128 ** -0.5)
+            if kind.endswith("borrowed"):
+                m["kv_from"] = 1
+            return "latent_attention", m
+        if kind == "rglru":
+            return kind, dict(width=width, blocks=width // 256, conv=4)
+        return kind, dict(heads=heads, kv_heads=heads // 2, dim=128, vdim=128, conv=4)
+
+    def mlp(kind):
+        if kind == "dense":
+            return dict(kind=kind, ff=(8 * width // 3 + 63) // 64 * 64)
+        ff = 11 * width // 32 // 64 * 64
+        return dict(kind=kind, expert=dict(ff=ff, limit=7.0), shared=dict(ff=2 * ff, limit=7.0),
+                    router=dict(experts=64, top=8, scale=2.5, groups=dict(count=8, keep=4)))
+    layers = []
+    for i, (m, f) in enumerate(HYBRID_STACKS[stack]):
+        kind, sizes = mixer(m, i)
+        layers.append(dict(type=kind, mixer=sizes, mlp=mlp(f)))
+    return HybridConfig.from_json(dict(width=width, vocab=vocab, layers=layers,
+                                       norm=dict(eps=1e-6), embedding=dict(scale=1.0)))
+
+
+def hybrid_throughput(width, only=None, prompt=1024, steps=20, warmup=5):
+    """Prefill and decode throughput of hybrid decoders (random weights, bf16) of four layers at
+    one width, beside OPT layers of that width and number of weights (fp16), all driven through
+    the slot interface: a prefill of 8 prompts in one step, decode steps of 1, 32 and 128 rows
+    that each hold the prompt."""
+    import torch
+
+    from metaseq_amd import (OPTConfig, TransformerLanguageModel, random_hybrid_state_dict,
+                             random_state_dict)
+    dev = torch.device("cuda:0")
+
+    def clock(fn, n):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for i in range(n):
+            fn(i)
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t0) / n
+
+    def run(cfg, state):
+        decoder = TransformerLanguageModel.build_model(cfg, state, device=dev).decoder
+        del state
+        out, V = {}, cfg.vocab_size
+        g = torch.Generator().manual_seed(7)
+        prompts = [torch.randint(4, V, (prompt,), generator=g).to(dev) for _ in range(8)]
+        for rows in (1, 32, 128):
+            cache = decoder.new_slot_cache(max(rows, 8) if rows > 1 else 1, prompt + 128)
+            if rows == 32:
+                fn = lambda i: decoder.prefill_slots(cache, list(range(8)), prompts)
+                fn(0)
+                out["prefill_ms"] = clock(fn, 3) * 1e3
+                out["prefill_tokens_per_s"] = 8 * prompt / out["prefill_ms"] * 1e3
+                if rows == 32:
+                    one = lambda i: decoder.prefill_slot(cache, 0, prompts[0])
+                    one(0)
+                    out["prefill_one_prompt_ms"] = clock(one, 3) * 1e3
+            for slot in range(rows):
+                if slot < 8:
+                    decoder.prefill_slot(cache, slot, prompts[slot])
+                else:
+                    decoder.copy_slot(cache, slot % 8, slot, length=prompt)
+            tok = torch.zeros(cache.batch, dtype=torch.long, device=dev)
+            score = torch.zeros(cache.batch, dtype=torch.float32, device=dev)
+            last = torch.randint(4, V, (cache.batch,), generator=g).to(dev)
+            step = lambda i: decoder.decode_slots(cache, last, banned=[1], tok_out=tok,
+                                                  score_out=score)
+            clock(step, warmup)
+            ms = clock(step, steps) * 1e3
+            out["decode_%d_ms" % rows] = ms
+            out["decode_%d_tokens_per_s" % rows] = rows / ms * 1e3
+            del cache
+        del decoder
+        torch.cuda.empty_cache()
+        return {k: round(v, 4) for k, v in out.items()}
+
+    results = {}
+    for stack in HYBRID_STACKS:
+        if only is None or stack == only:
+            cfg = hybrid_config(width, stack)
+            results[stack] = run(cfg, random_hybrid_state_dict(cfg, device=dev))
+            print("hybrid: %s done" % stack, file=sys.stderr, flush=True)
+    if only is None or only == "OPT":
+        cfg = OPTConfig(4, width, width // 128, max_target_positions=2048)
+        results["OPT"] = run(cfg, random_state_dict(cfg, dtype=torch.float16, device=dev))
+    head = "mixed" if "mixed" in results else next(iter(results))
+    return {
+        "metric": "decode tokens/s at 32 rows, four-layer hybrid decoder (%s), width %d, 1xMI355X"
+                  % (head, width),
+        "value": results[head]["decode_32_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": steps, "warmup": warmup, "ms_per_step": results[head]["decode_32_ms"],
+        "higher_is_better": True, "vs_baseline": None, "dtype": "bf16 (OPT: f16)",
+        "data": "synthetic",
+        "config": {"width": width, "prompt": prompt, "layers": 4, "vocab": 50272},
+        "stacks": results,
+    }
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -431,6 +550,11 @@ def main():
                     help="--service: requests that may share one prefill")
     ap.add_argument("--prefill-wait", type=int, default=0,
                     help="--service: steps admissible requests may be held back for company")
+    ap.add_argument("--hybrid", type=int, default=0, metavar="WIDTH",
+                    help="instead of the headline run: prefill and decode throughput of hybrid "
+                         "decoders of this width beside OPT layers of equal size, one JSON line "
+                         "of its own (--hybrid-stack: one stack only)")
+    ap.add_argument("--hybrid-stack", default=None, choices=sorted(HYBRID_STACKS) + ["OPT"])
     ap.add_argument("--torch-eager", action="store_true",
                     help="also time the same decode steps written with stock PyTorch fp16 "
                          "operators on this GPU (reported as torch_eager_same_gpu)")
@@ -445,12 +569,17 @@ def main():
     from metaseq_amd import (Dictionary, SequenceGenerator, TransformerLanguageModel, _capi,
                              opt_config, random_prompts, random_state_dict)
 
-    if not os.path.exists(_capi.LIB_PATH):
+    if not (os.path.exists(_capi.LIB_PATH) and os.path.exists(_capi.HYBRID_LIB_PATH)):
         from metaseq_amd.csrc.build import build
         build(force=True)
     if args.service:
         print(json.dumps(service_throughput(args.config, args.service, args.prefill_batch,
                                             args.prefill_wait)))
+        return
+
+    if args.hybrid:
+        print(json.dumps(hybrid_throughput(args.hybrid, args.hybrid_stack,
+                                           prompt=args.prompt or 1024)))
         return
 
     size, B, P, G = CONFIGS[args.config]

@@ -63,6 +63,7 @@ int msa_linear_bf16_splits(int64_t M, int N, int K, int packed);
  * and `groups` groups.  Routed: the tiles of a msa_moe_plan; row r of group g's sorted rows reads x row
  * perm[r] / rows_per_x (perm NULL: x row r) and writes y row r.  x_mb / y_mb > 0: packed layout with
  * that many row blocks (bf16 only).  y_f32: fp32 output.  glu as above (y has N / 2 columns).
+ * Routed tiles have 16, 32 or 64 rows, or 256 (bf16 row-major, K % 64 == 0, K >= 128).
  * x_groups > 0: group g reads column group g % x_groups.  y_row0 is added to every row of y. */
 typedef struct {
   int dtype;
@@ -142,6 +143,12 @@ int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const float* ba, int 
 int msa_delta_output(int dtype, const float* o, const void* gate, int64_t ld_gate, const float* w,
                      int heads, int vdim, int vp, float eps, void* out, int64_t ld_out, int out_mb,
                      int M, void* stream);
+/* Both in one launch where every segment holds one token. */
+int msa_delta_step(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
+                   const float* decay_rate, const float* dt_bias, int heads, int kv_heads, int dim,
+                   int dp, int vdim, int vp, float* state, const void* gate, int64_t ld_gate,
+                   const float* w, float eps, void* out, int64_t ld_out, int out_mb,
+                   const msa_batch* b, void* stream);
 
 /* Latents: part = fp32 sums [S][M][N] of the down-projections, columns [0, qp) the query latent,
  * [qp, qp + rp) the key/value latent (absent with latent NULL).  Both RMS-normed over their q_rank /

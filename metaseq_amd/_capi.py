@@ -175,6 +175,8 @@ HYBRID_SIGNATURES = {
                        _P, _P, _BP, _P],
     "msa_delta_output": [c_int, _P, _P, c_int64, _P, c_int, c_int, c_int, c_float, _P, c_int64,
                          c_int, c_int, _P],
+    "msa_delta_step": [c_int, _P, c_int64, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int,
+                       c_int, _P, _P, c_int64, _P, c_float, _P, c_int64, c_int, _BP, _P],
     "msa_latent_norm": [c_int, _P, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_int, _P,
                         c_float, _P, c_int, _P, c_int, _BP, _P],
     "msa_latent_attention_splits": [c_int, c_int, c_int, c_int, c_int],

@@ -29,6 +29,9 @@ int msa_launch_prefill_attention(const void* q, const void* Kc, const void* Vc,
                                  int B, int H, int hd, int T, int S0, int S_cap,
                                  hipStream_t stream);
 
+// routed products over 256-row tiles, bf16 (gemm_bf16.hip)
+bool msa_launch_group_quad(const msa_group_linear_args& a, hipStream_t stream);
+
 #define MSA_REQUIRE(cond, code, ...) \
   do {                               \
     if (!(cond)) {                   \
@@ -107,6 +110,12 @@ __device__ __forceinline__ void lse_merge(float& m, float& s, float om, float os
   } else if (om > -INFINITY) {
     s += os * expf(om - m);
   }
+}
+
+// Barrier of a workgroup for data exchanged through LDS: waits for this wave's LDS operations but, other
+// than __syncthreads(), not for its global loads, which stay in flight across it.
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 }
 
 // Cross-lane step of the wave reductions on the data-parallel-primitive path of the vector ALU

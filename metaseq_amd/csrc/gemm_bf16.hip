@@ -13,7 +13,32 @@ void run_linear(const void* x, const void* W, const Epilogue& e, int64_t M, int 
     launch_tiled<false, MODE>(x, W, nullptr, M, N, K, e, s);
 }
 
+template <int MODE>
+bool run_grouped(const msa_group_linear_args& a, const Epilogue& e, hipStream_t s) {
+  static std::atomic<uint64_t> lds_allowed{0};
+  auto kernel = linear_quad_kernel<MODE, 8, false, true>;
+  if (!allow_lds((const void*)kernel, tq_lds_bytes(8), lds_allowed)) return false;
+  const int ncol = (a.N + tq_bn(8) - 1) / tq_bn(8);
+  // the shares of the eight XCDs are rounded up: up to 7 workgroups beyond the tiles
+  const GroupTiles gt{a.perm, a.tile_group, a.tile_row, a.n_tiles, a.group_end, a.rows_per_x};
+  hipLaunchKernelGGL(kernel, dim3(ncol, a.max_tiles + (7 + ncol - 1) / ncol), dim3(TQ_THREADS),
+                     tq_lds_bytes(8), s, (const half_t*)a.x, a.W, (int64_t)0, a.N, a.K, 0, 0, 0, e,
+                     (float*)nullptr, 0, gt);
+  return true;
+}
+
 }  // namespace
+
+// Routed products over 256-row tiles (msa_group_linear).  Returns false if the launch is refused.
+bool msa_launch_group_quad(const msa_group_linear_args& a, hipStream_t s) {
+  Epilogue e{};
+  e.N = e.n32 = a.N;
+  e.yb = (bf16_t*)a.y;
+  e.ldy = (int)a.ldy;
+  e.glu = a.glu;
+  e.limit = a.limit;
+  return a.glu == MSA_GLU_NONE ? run_grouped<MODE_BF>(a, e, s) : run_grouped<MODE_BF_GLU>(a, e, s);
+}
 
 extern "C" int msa_linear_bf16(const void* x, const void* W, void* y, float* y32, int64_t M, int N,
                                int K, int n32, int glu, float limit, unsigned flags, void* stream) {

@@ -1113,13 +1113,24 @@ __device__ __forceinline__ void epilogue8(const Epilogue& e, int64_t m, int n, h
   }
 }
 
+// Row tiles of a grouped product (routed experts): tile t holds rows tile_row[t] .. of group
+// tile_group[t], at most TQ_BM of them and none past group_end; row r of the product reads row
+// perm[r] / rows_per_x of the activations (perm NULL: row r) and multiplies the group's own matrix.
+struct GroupTiles {
+  const int32_t *perm, *tile_group, *tile_row, *n_tiles, *group_end;
+  int rows_per_x;
+};
+
+// GROUPED: the row tiles come from `gt`; every XCD takes a contiguous share of the tiles, columns
+// fastest, so that the column tiles of a row tile run side by side behind one L2.
 // PART: split-K.  Workgroup (bx, by, z) sums over the K range of ``part_stages`` 64-wide stages
 // that starts at stage z * part_stages and stores its fp32 sums, with no epilogue, as slice z of
 // ``part`` ([gridDim.z][M][N]); a later launch adds the slices in slice order.
-template <int MODE, int WF, bool PART = false>
+template <int MODE, int WF, bool PART = false, bool GROUPED = false>
 __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
     const half_t* __restrict__ x, const void* __restrict__ Wp, int64_t M, int N, int K,
-    int rm_a, int rm_b, int rm_r, Epilogue epi, float* __restrict__ part, int part_stages) {
+    int rm_a, int rm_b, int rm_r, Epilogue epi, float* __restrict__ part, int part_stages,
+    GroupTiles gt = GroupTiles{}) {
   extern __shared__ __attribute__((aligned(16))) char tq_lds[];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int lr = lane & 15, lg = lane >> 4;
@@ -1127,7 +1138,18 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
   constexpr int TQ_BN = tq_bn(WF), TQ_WBYTES = tq_wbytes(WF);
   constexpr int WL = WF / 2;  // weight load instructions per wave and step
   int bx = blockIdx.x, by = blockIdx.y;
-  if (rm_a > 0) {
+  int64_t g_first = 0;
+  if constexpr (GROUPED) {
+    const int ncol = gridDim.x, L = by * ncol + bx, total = *gt.n_tiles * ncol;
+    const int per = (total + 7) / 8, t = (L & 7) * per + (L >> 3);
+    if ((L >> 3) >= per || t >= total) return;
+    by = t / ncol;
+    bx = t - by * ncol;
+    const int g = gt.tile_group[by];
+    g_first = gt.tile_row[by];
+    M = min((int64_t)gt.group_end[g], g_first + TQ_BM);
+    Wp = (const char*)Wp + (int64_t)g * N * K * 2;
+  } else if (rm_a > 0) {
     const int ncol = gridDim.x, L = by * ncol + bx, round = L >> 8, i = L & 255;
     if ((round + 1) * rm_r <= (int)gridDim.y) {  // a full round of 256 tiles
       const int xcd = i & 7, k = i >> 3, gx = ncol / rm_a;
@@ -1138,8 +1160,8 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
   // The narrowest form (WF = 2) also serves fewer than 256 rows: it does not move a ragged tile up
   // but repeats the last row in its loads and drops the rows past it in the epilogue.  So does
   // the split-K form of WF = 4 (decode batches of 129 .. 255 rows cut K eight ways over it).
-  constexpr bool CLAMP = WF == 2 || (WF == 4 && PART);
-  const int64_t m_own = (int64_t)by * TQ_BM;  // first row this tile owns
+  constexpr bool CLAMP = WF == 2 || (WF == 4 && PART) || GROUPED;
+  const int64_t m_own = GROUPED ? g_first : (int64_t)by * TQ_BM;  // first row this tile owns
   const int64_t m0 = !CLAMP && m_own + TQ_BM > M ? M - TQ_BM : m_own;
   const int n0 = bx * TQ_BN;
   // the stages this workgroup sums over: all of K, or its slice (the operand bases below move
@@ -1158,8 +1180,8 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     const int64_t r = m0 + wave * 64 + i * 8;
-    xb[i] = (const char*)(x + (CLAMP ? min(r, M - 1) : r) * K + (int64_t)st_first * 64) -
-            (i - 4) * 1024;
+    const int64_t base_row = GROUPED ? 0 : CLAMP ? min(r, M - 1) : r;
+    xb[i] = (const char*)(x + base_row * K + (int64_t)st_first * 64) - (i - 4) * 1024;
   }
 #pragma unroll
   for (int j = 0; j < WL; ++j) {
@@ -1176,7 +1198,12 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int64_t r = m0 + wave * 64 + i * 8;
-      const int64_t d = min(r + (lane >> 3), M - 1) - min(r, M - 1);
+      int64_t d = min(r + (lane >> 3), M - 1);
+      if (GROUPED) {
+        if (gt.perm) d = gt.perm[d] / gt.rows_per_x;
+      } else {
+        d -= min(r, M - 1);
+      }
       xl[i] = (uint32_t)d * (uint32_t)K * 2 + ((i & 1 ? xlane1 : xlane0) - xrow);
     }
   }
@@ -1703,7 +1730,7 @@ void launch_quad_partial_w(const void* x, const void* W, float* part, int64_t M,
   const int nrow = (int)((M + TQ_BM - 1) / TQ_BM);
   Epilogue e{};
   hipLaunchKernelGGL(kernel, dim3(ncol, nrow, S), dim3(TQ_THREADS), tq_lds_bytes(WF), s,
-                     (const half_t*)x, W, M, N, K, 0, 0, 0, e, part, K / 64 / S);
+                     (const half_t*)x, W, M, N, K, 0, 0, 0, e, part, K / 64 / S, GroupTiles{});
 }
 
 // 256 x 64 tiles while their S slices fit the chip in one round; an S beyond that means 256 x 128

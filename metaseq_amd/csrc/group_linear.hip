@@ -7,6 +7,9 @@
 // barrier in the main loop.  Few rows (a decode step): the four waves split K and their sums meet
 // in LDS; many rows: every wave owns its own column tiles.  Loads run one stage ahead of the MFMAs.
 //
+// Routed products with more than 64 rows per expert run on the four-wave 256 x 256 kernel of the dense
+// products instead (gemm_kernels.h).
+//
 // fp32: 64 x 64 tiles through LDS on the vector ALU in full fp32; also the fp32 linear layers.
 #include <math.h>
 
@@ -247,7 +250,7 @@ extern "C" int msa_group_linear(const msa_group_linear_args* args, void* stream)
               "%s: packed activations have no column groups", name);
   const bool routed = a.tile_group != nullptr;
   MSA_REQUIRE(!routed || (a.tile_row && a.n_tiles && a.group_end && a.max_tiles > 0 &&
-                          a.tile_rows > 0 && a.tile_rows <= 64 && (!a.perm || a.rows_per_x > 0)),
+                          a.tile_rows > 0 && (a.tile_rows <= 64 || a.tile_rows == 256) && (!a.perm || a.rows_per_x > 0)),
               MSA_ERR_INVALID_ARG, "%s: incomplete routing tables", name);
   MSA_REQUIRE(routed || !a.perm, MSA_ERR_INVALID_ARG, "%s: a permutation needs tiles", name);
   if (!routed && a.M <= 0) return MSA_OK;
@@ -257,7 +260,13 @@ extern "C" int msa_group_linear(const msa_group_linear_args* args, void* stream)
   if (!routed) a.tile_rows = rows = a.dtype == MSA_F32 ? 64 : a.M <= 16 ? 16 : a.M <= 32 ? 32 : 64;
   const int64_t row_tiles = routed ? a.max_tiles : (a.M + rows - 1) / rows;
   MSA_REQUIRE(row_tiles <= 65535, MSA_ERR_INVALID_ARG, "%s: too many rows", name);
-  if (a.dtype == MSA_F32) {
+  if (rows == 256) {
+    MSA_REQUIRE(a.dtype == MSA_BF16 && a.x_mb == 0 && a.y_mb == 0 && !a.y_f32 && a.ldx == a.K &&
+                    a.K % 64 == 0 && a.K >= 128 && a.y_row0 == 0 && a.M * a.K * 2 < (1ll << 32) &&
+                    (a.glu == MSA_GLU_NONE || a.N % 32 == 0),
+                MSA_ERR_INVALID_ARG, "%s: 256-row tiles of row-major bf16 rows, K=%d", name, a.K);
+    MSA_REQUIRE(msa_launch_group_quad(a, s), MSA_ERR_HIP, "%s: LDS limit", name);
+  } else if (a.dtype == MSA_F32) {
     hipLaunchKernelGGL(linear_f32_kernel, dim3((a.N + 63) / 64, (unsigned)row_tiles,
                                                routed ? 1 : a.groups),
                        dim3(256), 0, s, a, (float*)nullptr, a.N);

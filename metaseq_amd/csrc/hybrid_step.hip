@@ -233,15 +233,23 @@ int Run::delta(int li, const Act& h, Act& out) {
   float* ba = (float*)alloc((int64_t)M * (l.n_in - n32) * 4);
   HY(linear(h, l.w_in, in, false, ba, l.n_in, n32, MSA_GLU_NONE, 0.f));
   void* qkv = alloc((int64_t)M * C * es);
-  float* o = (float*)alloc((int64_t)M * l.heads * l.vp * 4);
+  const bool step = b.max_count == 1;
+  float* o = step ? nullptr : (float*)alloc((int64_t)M * l.heads * l.vp * 4);
   if (!dry) {
     const msa_hybrid_state& st = a->state[li];
     HY(msa_short_conv(d->cfg.dtype, in, n32, C, l.taps, nullptr, l.conv_w, nullptr, 1, qkv, C, st.conv,
                       &b, stream));
     HY(msa_conv_state(d->cfg.dtype, in, n32, C, l.taps, st.conv, &b, stream));
+    const char* gate = in + (int64_t)C * es;
+    if (step) {
+      HY(msa_delta_step(d->cfg.dtype, qkv, C, ba, l.n_in - n32, l.decay_rate, l.dt_bias, l.heads,
+                        l.kv_heads, l.dim, l.dp, l.vdim, l.vp, st.rec, gate, n32, l.o_norm, d->cfg.eps,
+                        out.p, out.ld, mb, &b, stream));
+      return zero_tail(out, l.heads * l.vp);
+    }
     HY(msa_delta_scan(d->cfg.dtype, qkv, C, ba, l.n_in - n32, l.decay_rate, l.dt_bias, l.heads,
                       l.kv_heads, l.dim, l.dp, l.vp, st.rec, o, &b, stream));
-    HY(msa_delta_output(d->cfg.dtype, o, in + (int64_t)C * es, n32, l.o_norm, l.heads, l.vdim, l.vp,
+    HY(msa_delta_output(d->cfg.dtype, o, gate, n32, l.o_norm, l.heads, l.vdim, l.vp,
                         d->cfg.eps, out.p, out.ld, mb, M, stream));
   }
   return zero_tail(out, l.heads * l.vp);
@@ -276,7 +284,8 @@ int Run::feed_forward(int li, Act& h, float* x, const float* next) {
   // the shared expert's hidden layer, the router logits and the shared gate's logit in one product
   HY(linear(h, l.w_ff_in, u.p, true, z, l.n_ff_in, n32, shared ? MSA_GLU_CLAMPED : MSA_GLU_NONE,
             l.limit_shared));
-  const int avg = P / E, tile_rows = f32 ? 64 : avg <= 16 ? 16 : avg <= 32 ? 32 : 64;
+  const int avg = P / E, tile_rows = f32 ? 64 : avg <= 16 ? 16 : avg <= 32 ? 32
+                                                 : avg <= 64 || mb > 0 ? 64 : 256;
   const int max_tiles = P / tile_rows + (E < P ? E : P);
   int32_t* ids = (int32_t*)alloc((int64_t)P * 4);
   float* w = (float*)alloc((int64_t)P * 4);
@@ -472,7 +481,7 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
     } else {
       MSA_REQUIRE(l.kind == MSA_MIX_DELTA && l.heads > 0 && l.kv_heads > 0 &&
                       l.heads % l.kv_heads == 0 && l.conv_w && l.decay_rate && l.dt_bias && l.o_norm &&
-                      l.ko >= l.heads * l.vp &&
+                      l.ko >= l.heads * l.vp && l.vp <= 512 &&
                       l.n_in >= 2 * l.kv_heads * l.dp + 2 * l.heads * l.vp + 2 * l.heads,
                   MSA_ERR_INVALID_ARG, "%s: layer %d: gated delta rule", name, i);
     }
@@ -480,7 +489,7 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
       MSA_REQUIRE(k_ok(l.ff) && l.n_ff_in == 2 * l.ff && l.w_ff_in && l.w_ff_down && l.norm2 && l.norm2b,
                   MSA_ERR_INVALID_ARG, "%s: layer %d: feed-forward", name, i);
     else if (l.ff_kind == MSA_FF_MOE)
-      MSA_REQUIRE(l.experts > 0 && l.top > 0 && l.ff_expert % 32 == 0 && l.ff_expert > 0 && l.w_ff_in &&
+      MSA_REQUIRE(l.experts > 0 && l.top > 0 && k_ok(l.ff_expert) && l.w_ff_in &&
                       l.w_e_in && l.w_e_down && l.norm2 && l.norm2b && l.n_groups > 0 &&
                       (l.ff_shared == 0 || (k_ok(l.ff_shared) && l.w_ff_down)) &&
                       l.n_ff_in >= 2 * l.ff_shared + l.experts + (l.ff_shared > 0 ? 1 : 0),

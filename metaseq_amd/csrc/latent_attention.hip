@@ -3,10 +3,10 @@
 //
 //  * Few new tokens per sequence (decode): the query is multiplied by the key up-projection
 //    first, so that scores are dot products with the latent itself, and the value up-projection is
-//    applied to the weighted sum of latents.  All heads share the latent rows: a wave takes 32
-//    positions at a time into LDS once and uses them twice, row-wise for the scores and through the
-//    transposing LDS read for the weighted sum.  Bound: the latent rows from HBM, once per 16
-//    heads; the workgroups of one token's head blocks and key range run on one XCD.
+//    applied to the weighted sum of latents.  All heads share the latent rows: a workgroup takes
+//    64 positions at a time into LDS once and uses them twice, row-wise for the scores and through
+//    the transposing LDS read for the weighted sum.  Bound: the latent rows from HBM, once per 32
+//    heads; the workgroups of one token's head groups and key range run on one XCD.
 //  * Prompts: keys and values are expanded per head and flash_attention_kernel runs over them.
 #include <math.h>
 
@@ -43,87 +43,101 @@ bool raise_lds(const void* kernel, int bytes, std::atomic<uint64_t>& done) {
   return true;
 }
 
-// keys of one split, a multiple of 128 (four waves x 32)
+// keys of one split, a multiple of the 64-key tile
 __device__ __forceinline__ int split_keys(int n_keys, int splits) {
-  return ((n_keys + splits - 1) / splits + 127) & ~127;
+  return ((n_keys + splits - 1) / splits + 63) & ~63;
 }
 
+constexpr int LA_KEYS = 64, LA_SC = LA_KEYS + 4;  // keys per tile; pitch of a head's scores
 template <int RP>
-constexpr int la_tile_bytes = 32 * (RP * 2 + 16);
+constexpr int la_tile_bytes = LA_KEYS * (RP * 2 + 16);
+template <int RP, int NHB>
+constexpr int la_lds_bytes = la_tile_bytes<RP> + NHB * 16 * LA_SC * 4;
 
 // ---- few new tokens, bf16 --------------------------------------------------------------------
-template <int RP>
-__global__ __launch_bounds__(256) void latent_decode_kernel(
+// A workgroup owns one token, one range of keys and NHB blocks of 16 heads, four waves per block.
+// The four waves share the scores of a 64-key tile (16 keys each) through LDS and then the weighted
+// sum by latent dimensions (RP / 4 each), so that no wave holds more than its share of the
+// accumulators and nothing has to be merged at the end.  The next tile's rows are fetched into
+// registers while a tile is worked on.
+template <int RP, int NHB>
+__global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ latent, int capacity, int heads,
     float scale_log2, bf16_t* __restrict__ out, float* __restrict__ partial, int splits,
     const int32_t* __restrict__ tok_slot, const int32_t* __restrict__ tok_pos, int M) {
-  constexpr int KS = RP / 32, DB = RP / 16, PITCH = RP * 2 + 16, TILE = la_tile_bytes<RP>;
-  constexpr int CH = RP / 8, LD = 32 * CH / 64;  // 16-byte chunks of a row; loads per lane and tile
-  extern __shared__ __attribute__((aligned(16))) char lds[];  // [4][TILE], then float [4][2][16]
-  const int HB = (heads + 15) / 16;
-  // workgroup -> (token, split, head block): the head blocks of one (token, split) on one XCD
+  constexpr int KS = RP / 32, DW = RP / 64, PITCH = RP * 2 + 16, THREADS = 256 * NHB;
+  constexpr int CH = RP / 8, LD = LA_KEYS * CH / THREADS;  // 16-byte chunks of a row; loads per thread
+  extern __shared__ __attribute__((aligned(16))) char lds[];  // tile, then scores [NHB][16][LA_SC]
+  const int HG = (heads + 16 * NHB - 1) / (16 * NHB);
+  // workgroup -> (token, split, head group): the head groups of one (token, split) on one XCD
   const int L = blockIdx.x, xcd = L & 7, seq = L >> 3;
-  const int pair = (seq / HB) * 8 + xcd, hb = seq % HB;
+  const int pair = (seq / HG) * 8 + xcd, hg = seq % HG;
   if (pair >= M * splits) return;
   const int m = pair / splits, split = pair - m * splits;
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int w4 = wave & 3, hb = wave >> 2;
   const int hc = lane & 15, g = lane >> 4;  // head column, lane group
+  const int head = (hg * NHB + hb) * 16 + hc;
   const int n_keys = min(tok_pos[m] + 1, capacity);  // <= 0: inactive
   const int per = split_keys(n_keys, splits);
   const int k_begin = split * per, k_end = min(n_keys, k_begin + per);
   const bf16_t* rows = latent + (int64_t)tok_slot[m] * capacity * RP;
-  char* tile = lds + wave * TILE;
-
-  bf16x8_t qf[KS];
-  {
-    const bf16_t* qr = q + ((int64_t)m * heads + min(hb * 16 + hc, heads - 1)) * RP + g * 8;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8_t*>(qr + ks * 32);
-  }
-  float4_t o[DB];
-#pragma unroll
-  for (int d = 0; d < DB; ++d) o[d] = float4_t{0.f, 0.f, 0.f, 0.f};
-  float mx = -INFINITY, l = 0.f;
 
   half8_t pre[LD];
   auto fetch = [&](int k0) {
 #pragma unroll
     for (int i = 0; i < LD; ++i) {
-      const int c = lane + 64 * i;
+      const int c = tid + THREADS * i;
       const int key = min(k0 + c / CH, n_keys - 1);
       pre[i] = *reinterpret_cast<const half8_t*>(rows + (int64_t)key * RP + (c % CH) * 8);
     }
   };
-  // transposing reads: lane (g, ii) is the source of key row 4 g + ii / 4, columns 4 (ii % 4) ..
-  const char* tr = tile + (4 * g + (hc >> 2)) * PITCH + (hc & 3) * 8;
-  int k0 = k_begin + wave * 32;
-  if (k0 < k_end) fetch(k0);
-  for (; k0 < k_end; k0 += 128) {
+  if (k_begin < k_end) fetch(k_begin);
+  bf16x8_t qf[KS];
+  {
+    const bf16_t* qr = q + ((int64_t)m * heads + min(head, heads - 1)) * RP + g * 8;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8_t*>(qr + ks * 32);
+  }
+  float4_t o[DW];
+#pragma unroll
+  for (int d = 0; d < DW; ++d) o[d] = float4_t{0.f, 0.f, 0.f, 0.f};
+  float mx = -INFINITY, l = 0.f;
+  float* sc = reinterpret_cast<float*>(lds + la_tile_bytes<RP>) + (hb * 16 + hc) * LA_SC;
+  const char* krow = lds + (16 * w4 + hc) * PITCH + g * 16;
+  // transposing reads: lane (g, i) is the source of key row 4 g + i / 4, columns 4 (i % 4) ..
+  const char* tr = lds + (4 * g + (hc >> 2)) * PITCH + w4 * (RP / 2) + (hc & 3) * 8;
+  for (int k0 = k_begin; k0 < k_end; k0 += LA_KEYS) {
+    lds_barrier();  // the previous tile and its scores are consumed
 #pragma unroll
     for (int i = 0; i < LD; ++i) {
-      const int c = lane + 64 * i;
-      *reinterpret_cast<half8_t*>(tile + (c / CH) * PITCH + (c % CH) * 16) = pre[i];
+      const int c = tid + THREADS * i;
+      *reinterpret_cast<half8_t*>(lds + (c / CH) * PITCH + (c % CH) * 16) = pre[i];
     }
-    if (k0 + 128 < k_end) fetch(k0 + 128);
-    __builtin_amdgcn_wave_barrier();
-    float4_t s[2] = {float4_t{0.f, 0.f, 0.f, 0.f}, float4_t{0.f, 0.f, 0.f, 0.f}};
+    if (k0 + LA_KEYS < k_end) fetch(k0 + LA_KEYS);
+    lds_barrier();
+    float4_t s2[2] = {float4_t{0.f, 0.f, 0.f, 0.f}, float4_t{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
+      s2[ks & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          *reinterpret_cast<const bf16x8_t*>(krow + ks * 64), qf[ks], s2[ks & 1], 0, 0, 0);
+    float4_t s = s2[0] + s2[1];
+    // s[r]: this lane's head, key k0 + 16 w4 + 4 g + r
 #pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(tile + (16 * b + hc) * PITCH + ks * 64 +
-                                                              g * 16);
-        s[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[ks], s[b], 0, 0, 0);
-      }
-    // s[b][r]: head hc, key k0 + 16 b + 4 g + r
+    for (int r = 0; r < 4; ++r)
+      s[r] = k0 + 16 * w4 + 4 * g + r < k_end ? s[r] * scale_log2 : -INFINITY;
+    *reinterpret_cast<float4_t*>(sc + 16 * w4 + 4 * g) = s;
+    lds_barrier();
+    // every wave of a head block: the lane's keys 32 t + 4 g + {0 .. 3}, 32 t + 16 + 4 g + {0 .. 3}
+    float4_t e[2][2];
     float tm = -INFINITY;
 #pragma unroll
-    for (int b = 0; b < 2; ++b)
+    for (int t = 0; t < 2; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        s[b][r] = k0 + 16 * b + 4 * g + r < k_end ? s[b][r] * scale_log2 : -INFINITY;
-        tm = fmaxf(tm, s[b][r]);
+      for (int b = 0; b < 2; ++b) {
+        e[t][b] = *reinterpret_cast<const float4_t*>(sc + 32 * t + 16 * b + 4 * g);
+        tm = fmaxf(fmaxf(tm, fmaxf(e[t][b][0], e[t][b][1])), fmaxf(e[t][b][2], e[t][b][3]));
       }
     tm = fmaxf(tm, __shfl_xor(tm, 16, MSA_WAVE));
     tm = fmaxf(tm, __shfl_xor(tm, 32, MSA_WAVE));
@@ -132,69 +146,46 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
       const float f = __builtin_amdgcn_exp2f(mx - mn);
       l *= f;
 #pragma unroll
-      for (int d = 0; d < DB; ++d) o[d] = o[d] * f;
+      for (int d = 0; d < DW; ++d) o[d] = o[d] * f;
       mx = mn;
     }
-    bf16x8_t p;
-    float ts = 0.f;
 #pragma unroll
-    for (int b = 0; b < 2; ++b)
+    for (int t = 0; t < 2; ++t) {
+      bf16x8_t p;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float e = __builtin_amdgcn_exp2f(s[b][r] - mx);
-        ts += e;
-        p[4 * b + r] = (bf16_t)e;
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float v = __builtin_amdgcn_exp2f(e[t][b][r] - mx);
+          l += v;  // this lane group's keys; the groups are summed at the end
+          p[4 * b + r] = (bf16_t)v;
+        }
+#pragma unroll
+      for (int d = 0; d < DW; ++d) {
+        const char* a = tr + 32 * t * PITCH + d * 32;
+        o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(read_column8(a, a + 16 * PITCH), p, o[d], 0,
+                                                       0, 0);
       }
-    l += ts;  // this lane group's keys; the groups are summed at the end
-#pragma unroll
-    for (int d = 0; d < DB; ++d)
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-          read_column8(tr + d * 32, tr + 16 * PITCH + d * 32), p, o[d], 0, 0, 0);
-    __builtin_amdgcn_wave_barrier();
+    }
   }
   l += __shfl_xor(l, 16, MSA_WAVE);
   l += __shfl_xor(l, 32, MSA_WAVE);
-
-  // merge the four waves: o as [16 heads][RP] floats in the wave's tile
-  float* stat = reinterpret_cast<float*>(lds + 4 * TILE);  // [4][2][16]
-  __syncthreads();
-  if (g == 0) {
-    stat[wave * 32 + hc] = mx;
-    stat[wave * 32 + 16 + hc] = l;
-  }
-  float* mine = reinterpret_cast<float*>(tile);
+  if (head >= heads) return;
+  // o[d][r]: dimension w4 RP / 4 + 16 d + 4 g + r
+  const int64_t row = (int64_t)m * heads + head;
+  const int c0 = w4 * (RP / 4) + 4 * g;
+  if (splits > 1) {
+    float* p = partial + (row * splits + split) * (RP + 4);
 #pragma unroll
-  for (int d = 0; d < DB; ++d)
-    *reinterpret_cast<float4_t*>(mine + hc * RP + d * 16 + 4 * g) = o[d];
-  __syncthreads();
-  for (int i = tid; i < 16 * (RP / 4); i += 256) {
-    const int h = i / (RP / 4), c = (i % (RP / 4)) * 4;
-    if (hb * 16 + h >= heads) continue;
-    float M4 = -INFINITY;
+    for (int d = 0; d < DW; ++d) *reinterpret_cast<float4_t*>(p + c0 + 16 * d) = o[d];
+    if (w4 == 0 && g == 0) p[RP] = mx, p[RP + 1] = l;
+  } else {
+    const float inv = l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
-    for (int w = 0; w < 4; ++w) M4 = fmaxf(M4, stat[w * 32 + h]);
-    float Ls = 0.f;
-    float4_t acc = {0.f, 0.f, 0.f, 0.f};
-    if (M4 > -INFINITY) {
-#pragma unroll
-      for (int w = 0; w < 4; ++w) {
-        const float f = __builtin_amdgcn_exp2f(stat[w * 32 + h] - M4);
-        Ls += f * stat[w * 32 + 16 + h];
-        acc += f * *reinterpret_cast<const float4_t*>(
-                       reinterpret_cast<const float*>(lds + w * TILE) + h * RP + c);
-      }
-    }
-    const int64_t row = (int64_t)m * heads + hb * 16 + h;
-    if (splits > 1) {
-      float* p = partial + (row * splits + split) * (RP + 4);
-      *reinterpret_cast<float4_t*>(p + c) = acc;
-      if (c == 0) p[RP] = M4, p[RP + 1] = Ls;
-    } else {
-      const float inv = Ls > 0.f ? 1.f / Ls : 0.f;
-      *reinterpret_cast<bf16x4_t*>(out + row * RP + c) =
-          bf16x4_t{(bf16_t)(acc[0] * inv), (bf16_t)(acc[1] * inv), (bf16_t)(acc[2] * inv),
-                   (bf16_t)(acc[3] * inv)};
-    }
+    for (int d = 0; d < DW; ++d)
+      *reinterpret_cast<bf16x4_t*>(out + row * RP + c0 + 16 * d) =
+          bf16x4_t{(bf16_t)(o[d][0] * inv), (bf16_t)(o[d][1] * inv), (bf16_t)(o[d][2] * inv),
+                   (bf16_t)(o[d][3] * inv)};
   }
 }
 
@@ -359,7 +350,7 @@ __global__ __launch_bounds__(256) void flash_attention_kernel(
   fetch(0);
   park(0);
   if (ntiles > 1) fetch(1);
-  __syncthreads();
+  lds_barrier();
   for (int tile = 0; tile < ntiles; ++tile) {
     const int slot = tile & 1;
     const char* kt = lds + slot * 2 * TILE;
@@ -423,7 +414,7 @@ __global__ __launch_bounds__(256) void flash_attention_kernel(
         }
       l += (t4[0] + t4[1]) + (t4[2] + t4[3]);
     }
-    __syncthreads();
+    lds_barrier();
   }
   l += __shfl_xor(l, 32, MSA_WAVE);
   if (tq < T) {
@@ -443,19 +434,29 @@ __global__ __launch_bounds__(256) void flash_attention_kernel(
   }
 }
 
+template <int RP, int NHB>
+bool run_decode_blocks(const void* q, const void* latent, int capacity, int heads, float scale,
+                       void* out, float* partial, int splits, const int32_t* tok_slot,
+                       const int32_t* tok_pos, int M, hipStream_t s) {
+  static std::atomic<uint64_t> raised{0};
+  constexpr int bytes = la_lds_bytes<RP, NHB>;
+  if (!raise_lds((const void*)latent_decode_kernel<RP, NHB>, bytes, raised)) return false;
+  const int HG = (heads + 16 * NHB - 1) / (16 * NHB);
+  const int64_t groups = ((int64_t)M * splits + 7) / 8 * 8 * HG;
+  hipLaunchKernelGGL((latent_decode_kernel<RP, NHB>), dim3((unsigned)groups), dim3(256 * NHB), bytes,
+                     s, (const bf16_t*)q, (const bf16_t*)latent, capacity, heads, scale * LOG2E,
+                     (bf16_t*)out, partial, splits, tok_slot, tok_pos, M);
+  return true;
+}
+
 template <int RP>
 bool run_decode(const void* q, const void* latent, int capacity, int heads, float scale, void* out,
                 float* partial, int splits, const int32_t* tok_slot, const int32_t* tok_pos, int M,
                 hipStream_t s) {
-  static std::atomic<uint64_t> raised{0};
-  constexpr int bytes = 4 * la_tile_bytes<RP> + 4 * 2 * 16 * 4;
-  if (!raise_lds((const void*)latent_decode_kernel<RP>, bytes, raised)) return false;
-  const int HB = (heads + 15) / 16;
-  const int64_t groups = ((int64_t)M * splits + 7) / 8 * 8 * HB;
-  hipLaunchKernelGGL(latent_decode_kernel<RP>, dim3((unsigned)groups), dim3(256), bytes, s,
-                     (const bf16_t*)q, (const bf16_t*)latent, capacity, heads, scale * LOG2E,
-                     (bf16_t*)out, partial, splits, tok_slot, tok_pos, M);
-  return true;
+  return heads <= 16 ? run_decode_blocks<RP, 1>(q, latent, capacity, heads, scale, out, partial,
+                                                splits, tok_slot, tok_pos, M, s)
+                     : run_decode_blocks<RP, 2>(q, latent, capacity, heads, scale, out, partial,
+                                                splits, tok_slot, tok_pos, M, s);
 }
 
 bool has_decode_kernel(int dtype, int rp) {
@@ -478,10 +479,10 @@ bool run_flash(const void* q, int64_t ldq, const void* kv, int64_t ldkv, void* o
 
 extern "C" int msa_latent_attention_splits(int dtype, int M, int heads, int rp, int key_bound) {
   if (M < 1 || heads < 1 || key_bound < 1) return 1;
-  const int64_t groups = (int64_t)M * (has_decode_kernel(dtype, rp) ? (heads + 15) / 16 : heads);
+  const int64_t groups = (int64_t)M * (has_decode_kernel(dtype, rp) ? (heads + 31) / 32 : heads);
   int s = 1;
-  // about two workgroups per CU, at least 256 keys each
-  while (s < 64 && groups * s < 512 && (int64_t)key_bound >= 512 * s) s *= 2;
+  // about a workgroup per CU, at least 128 keys each
+  while (s < 64 && groups * s < 256 && (int64_t)key_bound >= 256 * s) s *= 2;
   return s;
 }
 

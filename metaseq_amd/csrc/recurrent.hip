@@ -18,12 +18,14 @@ __device__ __forceinline__ float softplus(float v) {
 }
 
 // ---- short convolution ----------------------------------------------------------------------
-constexpr int SC_TOK = 16;     // tokens per workgroup
+constexpr int SC_TOK = 8;      // tokens per workgroup
 constexpr int SC_MAX_TAPS = 8;
 
-// A thread owns 8 channels and walks SC_TOK tokens.  STEP: one token per segment; the thread also
-// shifts the state.
-template <typename T, bool STEP>
+// A thread owns 8 channels of SC_TOK tokens.  STEP: one token per segment; the thread also shifts
+// the state.  TAPS > 0: that many taps, and a tile that lies inside one segment behind its first
+// TAPS - 1 tokens (nearly every tile of a prompt) requests all its input rows at once; the other tiles
+// take every input from the segment or the state, tap by tap.
+template <typename T, bool STEP, int TAPS>
 __global__ __launch_bounds__(256) void short_conv_kernel(
     const T* __restrict__ in, int64_t ld_in, int C, int taps, const float* __restrict__ in_bias,
     const float* __restrict__ weight, const float* __restrict__ bias, int act, T* __restrict__ out,
@@ -38,6 +40,34 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
   for (int i = 0; i < 8; ++i) {
     ib[i] = in_bias ? in_bias[c + i] : 0.f;
     b[i] = bias ? bias[c + i] : 0.f;
+  }
+  if constexpr (!STEP && TAPS > 1) {
+    const int off = tok_off[m0];
+    if (m1 - m0 == SC_TOK && off >= TAPS - 1 && tok_pos[m0] >= 0 &&
+        tok_off[m1 - 1] - off == SC_TOK - 1) {
+      v8 x[SC_TOK + TAPS - 1];
+#pragma unroll
+      for (int t = 0; t < SC_TOK + TAPS - 1; ++t)
+        x[t] = *reinterpret_cast<const v8*>(in + (int64_t)(m0 - (TAPS - 1) + t) * ld_in + c);
+      float w[TAPS][8];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) w[j][i] = weight[(int64_t)j * C + c + i];
+#pragma unroll
+      for (int t = 0; t < SC_TOK; ++t) {
+        v8 o;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          float a = b[i];
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) a = fmaf((float)x[t + j][i] + ib[i], w[j][i], a);
+          o[i] = (T)(act ? silu(a) : a);
+        }
+        *reinterpret_cast<v8*>(out + (int64_t)(m0 + t) * ld_out + c) = o;
+      }
+      return;
+    }
   }
   for (int m = m0; m < m1; ++m) {
     const int pos = tok_pos[m], off = tok_off[m];
@@ -258,7 +288,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
         lg[tid] = expf(-rate * softplus(rg + dtb));
       }
     }
-    __syncthreads();
+    lds_barrier();
     {
       const int t = tid >> 4, r = tid & 15;
       float d = 0.f;
@@ -267,34 +297,151 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       d = row16_sum(d);
       if (r == 0) lkq[t] = d;
     }
-    if (t0 + DR_TOK < n) fetch(t0 + DR_TOK);
-    __syncthreads();
-    for (int t = 0; t < nt; ++t) {
-      float k[R], d1 = 0.f, d2 = 0.f, e1 = 0.f, e2 = 0.f;
+    if (t0 + DR_TOK < n) fetch(t0 + DR_TOK);  // in flight across the barriers
+    lds_barrier();
+    // operands of the current and the next token: one set is fetched while the other is used
+    struct Token {
+      float k[R], q[R], g, beta, v, kq;
+    } a, b;
+    auto read = [&](Token& x, int t) {
+      t = min(t, DR_TOK - 1);
 #pragma unroll
-      for (int i = 0; i < R; ++i) k[i] = lk[t][rl * R + i];
+      for (int i = 0; i < R; ++i) x.k[i] = lk[t][rl * R + i], x.q[i] = lq[t][rl * R + i];
+      x.g = lg[t], x.beta = lb[t], x.v = lv[t][cl], x.kq = lkq[t];
+    };
+    auto advance = [&](const Token& x, int t) {
+      float d1 = 0.f, d2 = 0.f, e1 = 0.f, e2 = 0.f;
 #pragma unroll
       for (int i = 0; i < R; i += 2) {
-        d1 = fmaf(S[i], k[i], d1);
-        e1 = fmaf(S[i + 1], k[i + 1], e1);
-        d2 = fmaf(S[i], lq[t][rl * R + i], d2);
-        e2 = fmaf(S[i + 1], lq[t][rl * R + i + 1], e2);
+        d1 = fmaf(S[i], x.k[i], d1);
+        e1 = fmaf(S[i + 1], x.k[i + 1], e1);
+        d2 = fmaf(S[i], x.q[i], d2);
+        e2 = fmaf(S[i + 1], x.q[i + 1], e2);
       }
       d1 = row16_sum(d1 + e1);
       d2 = row16_sum(d2 + e2);
-      const float g = lg[t];
-      const float u = lb[t] * (lv[t][cl] - g * d1);
+      const float u = x.beta * (x.v - x.g * d1);
 #pragma unroll
-      for (int i = 0; i < R; ++i) S[i] = fmaf(k[i], u, g * S[i]);
-      if (rl == 0) lo[t][cl] = fmaf(u, lkq[t], g * d2);
+      for (int i = 0; i < R; ++i) S[i] = fmaf(x.k[i], u, x.g * S[i]);
+      if (rl == 0) lo[t][cl] = fmaf(u, x.kq, x.g * d2);
+    };
+    read(a, 0);
+    for (int t = 0; t < nt; t += 2) {
+      read(b, t + 1);
+      advance(a, t);
+      read(a, t + 2);
+      if (t + 1 < nt) advance(b, t + 1);
     }
-    __syncthreads();
+    lds_barrier();
     if (tid < nt * 16)
       o[(int64_t)(first + t0 + (tid >> 4)) * heads * vp + h * vp + col0 + (tid & 15)] =
           lo[tid >> 4][tid & 15];
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) st[i] = S[i];
+}
+
+// One token per segment (a decode step): a workgroup owns one segment and one head with all its
+// columns, 4 CG of them per wave and pass, requests the whole pass's state at once and finishes the
+// head's output (norm over the columns, gate) itself.  Lanes and arithmetic as above.
+template <typename T, int R, int CG>
+__global__ __launch_bounds__(256) void delta_step_kernel(
+    const T* __restrict__ qkv, int64_t ld, const float* __restrict__ ba, int ldba,
+    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias, int heads, int kv_heads,
+    float q_scale, int vdim, int vp, float* __restrict__ state, const T* __restrict__ gate,
+    int64_t ld_gate, const float* __restrict__ w, float eps, T* __restrict__ out, int64_t ld_out,
+    int out_mb, const int32_t* __restrict__ seg_slot, const int32_t* __restrict__ seg_pos) {
+  constexpr int DP = 16 * R;
+  __shared__ __attribute__((aligned(16))) float lk[DP], lq[DP];
+  __shared__ float lv[512], lo[512], red[16];
+  const int m = blockIdx.y, h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int pos = seg_pos[m];
+  const int rl = lane & 15, cw = wave * 4 + (lane >> 4);  // row group; column within a group of 16
+  float* st = state + (((int64_t)seg_slot[m] * heads + h) * vp) * DP + rl * R;
+  const int ng = vp / 16;
+  typedef float fr __attribute__((ext_vector_type(2), aligned(8)));
+  float S[CG][R];
+  auto load = [&](int g0) {
+#pragma unroll
+    for (int c = 0; c < CG; ++c) {
+      const fr* p = reinterpret_cast<const fr*>(st + (int64_t)(min(g0 + c, ng - 1) * 16 + cw) * DP);
+#pragma unroll
+      for (int i = 0; i < R / 2; ++i) {
+        const fr v = p[i];
+        S[c][2 * i] = v[0], S[c][2 * i + 1] = v[1];
+      }
+    }
+  };
+  load(0);
+  const T* row = qkv + (int64_t)m * ld;
+  const int hk = h / (heads / kv_heads);
+  if (wave < 2) {  // q and k as unit vectors
+    const T* p = row + (wave == 0 ? hk : kv_heads + hk) * DP;
+    float x[(DP + 63) / 64], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < (DP + 63) / 64; ++i) {
+      const int c = lane + 64 * i;
+      x[i] = c < DP ? (float)p[min(c, DP - 1)] : 0.f;
+      ss += x[i] * x[i];
+    }
+    ss = wave_sum(ss);
+    const float f = (wave == 0 ? q_scale : 1.f) / sqrtf(ss + 1e-6f);
+#pragma unroll
+    for (int i = 0; i < (DP + 63) / 64; ++i)
+      if (lane + 64 * i < DP) (wave == 0 ? lq : lk)[lane + 64 * i] = x[i] * f;
+  } else {
+    for (int c = tid - 128; c < vp; c += 128)
+      lv[c] = (float)row[2 * kv_heads * DP + h * vp + c];
+  }
+  const float* z = ba + (int64_t)m * ldba;
+  const float bt = sigmoidf(z[h]);
+  const float g = expf(-decay_rate[h] * softplus(z[heads + h] + dt_bias[h]));
+  lds_barrier();
+  float k[R], q[R], kq = 0.f;
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    k[i] = lk[rl * R + i], q[i] = lq[rl * R + i];
+    kq = fmaf(k[i], q[i], kq);
+  }
+  kq = row16_sum(kq);
+  for (int g0 = 0; g0 < ng; g0 += CG) {
+    if (g0 > 0) load(g0);
+#pragma unroll
+    for (int c = 0; c < CG; ++c) {
+      if (g0 + c >= ng) break;  // uniform
+      const int col = (g0 + c) * 16 + cw;
+      if (pos <= 0) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) S[c][i] = 0.f;
+      }
+      float d1 = 0.f, d2 = 0.f;
+#pragma unroll
+      for (int i = 0; i < R; ++i) {
+        d1 = fmaf(S[c][i], k[i], d1);
+        d2 = fmaf(S[c][i], q[i], d2);
+      }
+      d1 = row16_sum(d1);
+      d2 = row16_sum(d2);
+      const float u = bt * (lv[col] - g * d1);
+      if (rl == 0) lo[col] = fmaf(u, kq, g * d2);
+      if (pos >= 0) {
+        fr* p = reinterpret_cast<fr*>(st + (int64_t)col * DP);
+#pragma unroll
+        for (int i = 0; i < R / 2; ++i)
+          p[i] = fr{fmaf(k[2 * i], u, g * S[c][2 * i]), fmaf(k[2 * i + 1], u, g * S[c][2 * i + 1])};
+      }
+    }
+  }
+  lds_barrier();
+  float ss = 0.f;
+  for (int c = tid; c < vp; c += 256) ss += lo[c] * lo[c];
+  ss = block_sum(ss, red);
+  const float rms = 1.f / sqrtf(ss / (float)vdim + eps);
+  for (int c = tid; c < vp; c += 256) {
+    const int at = h * vp + c;
+    const float y = lo[c] * rms * w[c] * silu((float)gate[(int64_t)m * ld_gate + at]);
+    out[out_mb > 0 ? packed_act_offset(m, at, out_mb) : (int64_t)m * ld_out + at] = (T)y;
+  }
 }
 
 // one wave per (token, head)
@@ -351,7 +498,61 @@ void run_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const flo
 #undef DR_CASE
 }
 
+template <typename T>
+void run_delta_step(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
+                    const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vdim, int vp,
+                    float* state, const void* gate, int64_t ld_gate, const float* w, float eps,
+                    void* out, int64_t ld_out, int out_mb, const msa_batch* b, hipStream_t s) {
+  const dim3 grid(heads, b->nseg);
+  const float q_scale = (float)pow((double)dim, -0.5);
+#define DR_CASE(RR, CG)                                                                             \
+  case 16 * RR:                                                                                     \
+    hipLaunchKernelGGL((delta_step_kernel<T, RR, CG>), grid, dim3(256), 0, s, (const T*)qkv, ld, ba, \
+                       ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vdim, vp, state,        \
+                       (const T*)gate, ld_gate, w, eps, (T*)out, ld_out, out_mb, b->seg_slot,       \
+                       b->seg_pos);                                                                 \
+    break;
+  switch (dp) {
+    DR_CASE(2, 8)
+    DR_CASE(4, 8)
+    DR_CASE(6, 8)
+    DR_CASE(8, 8)
+    DR_CASE(12, 4)
+    DR_CASE(16, 4)
+  }
+#undef DR_CASE
+}
+
+bool delta_sizes_ok(int heads, int kv_heads, int dim, int dp, int vp, int ldba, int64_t ld,
+                    const msa_batch* b) {
+  return (dp == 32 || dp == 64 || dp == 96 || dp == 128 || dp == 192 || dp == 256) && dim <= dp &&
+         vp > 0 && vp % 16 == 0 && kv_heads > 0 && heads % kv_heads == 0 && ldba >= 2 * heads &&
+         ld % 8 == 0 && heads <= 65535 && b->nseg > 0 && b->nseg <= 65535;
+}
+
 }  // namespace
+
+extern "C" int msa_delta_step(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
+                              const float* decay_rate, const float* dt_bias, int heads, int kv_heads,
+                              int dim, int dp, int vdim, int vp, float* state, const void* gate,
+                              int64_t ld_gate, const float* w, float eps, void* out, int64_t ld_out,
+                              int out_mb, const msa_batch* b, void* stream) {
+  const char* name = "msa_delta_step";
+  MSA_REQUIRE(qkv && ba && decay_rate && dt_bias && state && gate && w && out && b,
+              MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  MSA_REQUIRE(delta_sizes_ok(heads, kv_heads, dim, dp, vp, ldba, ld, b) && vdim <= vp && vp <= 512 &&
+                  b->max_count == 1 && b->M == b->nseg,
+              MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
+              kv_heads, dim, dp, vp);
+  if (dtype == MSA_BF16)
+    run_delta_step<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vdim, vp,
+                           state, gate, ld_gate, w, eps, out, ld_out, out_mb, b, (hipStream_t)stream);
+  else
+    run_delta_step<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vdim, vp,
+                          state, gate, ld_gate, w, eps, out, ld_out, 0, b, (hipStream_t)stream);
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
 
 extern "C" int msa_short_conv(int dtype, const void* in, int64_t ld_in, int C, int taps,
                               const float* in_bias, const float* weight, const float* bias, int silu,
@@ -366,17 +567,21 @@ extern "C" int msa_short_conv(int dtype, const void* in, int64_t ld_in, int C, i
               b->M);
   const bool step = b->max_count == 1 && b->M <= 65535;
   const dim3 grid((C / 8 + 255) / 256, step ? b->M : (b->M + SC_TOK - 1) / SC_TOK);
-#define SC_RUN(T, STEP)                                                                             \
-  hipLaunchKernelGGL((short_conv_kernel<T, STEP>), grid, dim3(256), 0, (hipStream_t)stream,         \
+#define SC_RUN(T, STEP, TAPS)                                                                       \
+  hipLaunchKernelGGL((short_conv_kernel<T, STEP, TAPS>), grid, dim3(256), 0, (hipStream_t)stream,   \
                      (const T*)in, ld_in, C, taps, in_bias, weight, bias, silu, (T*)out, ld_out,    \
                      (T*)state, b->tok_slot, b->tok_pos, b->tok_off, b->M)
-  if (dtype == MSA_BF16) {
-    if (step) SC_RUN(bf16_t, true);
-    else SC_RUN(bf16_t, false);
-  } else {
-    if (step) SC_RUN(float, true);
-    else SC_RUN(float, false);
-  }
+#define SC_TYPE(T)                                                                                  \
+  do {                                                                                              \
+    if (step) SC_RUN(T, true, 0);                                                                   \
+    else if (taps == 2) SC_RUN(T, false, 2);                                                        \
+    else if (taps == 3) SC_RUN(T, false, 3);                                                        \
+    else if (taps == 4) SC_RUN(T, false, 4);                                                        \
+    else SC_RUN(T, false, 0);                                                                       \
+  } while (0)
+  if (dtype == MSA_BF16) SC_TYPE(bf16_t);
+  else SC_TYPE(float);
+#undef SC_TYPE
 #undef SC_RUN
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
@@ -447,10 +652,7 @@ extern "C" int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const floa
   const char* name = "msa_delta_scan";
   MSA_REQUIRE(qkv && ba && decay_rate && dt_bias && state && o && b, MSA_ERR_INVALID_ARG,
               "%s: null pointer", name);
-  MSA_REQUIRE((dp == 32 || dp == 64 || dp == 96 || dp == 128 || dp == 192 || dp == 256) && dim <= dp &&
-                  vp > 0 && vp % 16 == 0 && kv_heads > 0 && heads % kv_heads == 0 &&
-                  ldba >= 2 * heads && ld % 8 == 0 && heads <= 65535 && b->nseg > 0 &&
-                  b->nseg <= 65535,
+  MSA_REQUIRE(delta_sizes_ok(heads, kv_heads, dim, dp, vp, ldba, ld, b),
               MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
               kv_heads, dim, dp, vp);
   if (dtype == MSA_BF16)

@@ -1,14 +1,16 @@
 // RMS norms of hybrid decoders with what surrounds them fused in: the embedding with sinusoidal
 // positions, the tail of a sublayer (split-K sums, the combination of routed experts, post-norm,
 // residual add, next pre-norm), the latent norms with the cache append, and small row utilities.
-// One workgroup per token; a row lives in registers (NV float4 per thread).
+// One workgroup per token; a row lives in registers (NV float4 per thread): 256 threads where there
+// are many tokens, up to 1024 where there are few and the latency of one row counts.
 #include <math.h>
 
 #include "common.h"
 
 namespace {
 
-constexpr int RN_THREADS = 256;
+constexpr int RN_THREADS = 256;       // latent norms; norms of many rows
+constexpr int RN_FEW_ROWS = 1024;     // up to here a row is spread over more threads
 
 // one activation element group: 4 consecutive columns of row m
 template <typename T>
@@ -26,7 +28,7 @@ __device__ __forceinline__ float dot4(float4_t v) {
 }
 
 // x (registers) -> h = x / rms(x) * w
-template <typename T, int NV>
+template <typename T, int NV, int NT>
 __device__ __forceinline__ void norm_out(const float4_t (&x)[NV], int64_t m, int D, int Dp, float eps,
                                          const float* w, void* h, int mb, float* red) {
   float ss = 0.f;
@@ -36,7 +38,7 @@ __device__ __forceinline__ void norm_out(const float4_t (&x)[NV], int64_t m, int
   const float r = 1.f / sqrtf(ss / (float)D + eps);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < Dp) {
       const float4_t wv = *reinterpret_cast<const float4_t*>(w + c);
       store_act4<T>(h, m, Dp, mb, c, x[i] * r * wv);
@@ -44,8 +46,8 @@ __device__ __forceinline__ void norm_out(const float4_t (&x)[NV], int64_t m, int
   }
 }
 
-template <typename T, int NV>
-__global__ __launch_bounds__(RN_THREADS) void embed_kernel(
+template <typename T, int NV, int NT>
+__global__ __launch_bounds__(NT) void embed_kernel(
     const int64_t* __restrict__ tokens, const int32_t* __restrict__ tok_pos,
     const bf16_t* __restrict__ table, int vocab, float scale, const double* __restrict__ inv_freq,
     int D, int Dp, float eps, float* __restrict__ x, const float* __restrict__ w, void* h, int mb) {
@@ -57,7 +59,7 @@ __global__ __launch_bounds__(RN_THREADS) void embed_kernel(
   float4_t v[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     v[i] = float4_t{0.f, 0.f, 0.f, 0.f};
     if (c >= Dp) continue;
     const bf16x4_t e = *reinterpret_cast<const bf16x4_t*>(table + t * Dp + c);
@@ -75,29 +77,39 @@ __global__ __launch_bounds__(RN_THREADS) void embed_kernel(
     }
     *reinterpret_cast<float4_t*>(x + m * Dp + c) = v[i];
   }
-  if (w) norm_out<T, NV>(v, m, D, Dp, eps, w, h, mb, red);
+  if (w) norm_out<T, NV, NT>(v, m, D, Dp, eps, w, h, mb, red);
 }
 
-template <typename T, int NV>
-__global__ __launch_bounds__(RN_THREADS) void tail_kernel(msa_tail_args a) {
+template <typename T, int NV, int NT>
+__global__ __launch_bounds__(NT) void tail_kernel(msa_tail_args a) {
   __shared__ float red[16];
   const int64_t m = blockIdx.x;
   const int D = a.D, Dp = a.Dp;
   float4_t b[NV], x[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     b[i] = x[i] = float4_t{0.f, 0.f, 0.f, 0.f};
     if (c < Dp) x[i] = *reinterpret_cast<const float4_t*>(a.x + m * Dp + c);
   }
   if (a.part) {
-    for (int s = 0; s < a.S; ++s) {
-      const float* p = a.part + ((int64_t)s * a.M + m) * Dp;
+    // four slices at a time, their loads in flight together
+    for (int s0 = 0; s0 < a.S; s0 += 4) {
+      float4_t v[4][NV];
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int c = (threadIdx.x + i * RN_THREADS) * 4;
-        if (c < Dp) b[i] += *reinterpret_cast<const float4_t*>(p + c);
+      for (int s = 0; s < 4; ++s) {
+        const float* p = a.part + ((int64_t)min(s0 + s, a.S - 1) * a.M + m) * Dp;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+          const int c = (threadIdx.x + i * NT) * 4;
+          v[s][i] = c < Dp && s0 + s < a.S ? *reinterpret_cast<const float4_t*>(p + c)
+                                           : float4_t{0.f, 0.f, 0.f, 0.f};
+        }
       }
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+#pragma unroll
+        for (int i = 0; i < NV; ++i) b[i] += v[s][i];
     }
     if (a.gate) {
       const float g = a.gate[m];
@@ -106,20 +118,34 @@ __global__ __launch_bounds__(RN_THREADS) void tail_kernel(msa_tail_args a) {
     }
   }
   if (a.pair_y) {
-    for (int k = 0; k < a.top; ++k) {
-      const float w = a.pair_w[m * a.top + k];
-      const T* p = (const T*)a.pair_y + (int64_t)a.inverse[m * a.top + k] * Dp;
+    typedef T t4 __attribute__((ext_vector_type(4)));
+    constexpr int U = NV <= 2 ? 4 : 1;
+    for (int k0 = 0; k0 < a.top; k0 += U) {
+      t4 y[U][NV];
+      float w[U];
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int c = (threadIdx.x + i * RN_THREADS) * 4;
-        if (c < Dp) {
-          typedef T t4 __attribute__((ext_vector_type(4)));
-          const t4 y = *reinterpret_cast<const t4*>(p + c);
+      for (int k = 0; k < U; ++k) {
+        const int64_t at = m * a.top + min(k0 + k, a.top - 1);
+        w[k] = k0 + k < a.top ? a.pair_w[at] : 0.f;
+        const T* p = (const T*)a.pair_y + (int64_t)a.inverse[at] * Dp;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) b[i][j] += w * (float)y[j];
+        for (int i = 0; i < NV; ++i) {
+          const int c = (threadIdx.x + i * NT) * 4;
+          y[k][i] = *reinterpret_cast<const t4*>(p + (c < Dp ? c : 0));
         }
       }
+#pragma unroll
+      for (int k = 0; k < U; ++k)
+        if (k0 + k < a.top) {  // uniform
+#pragma unroll
+          for (int i = 0; i < NV; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) b[i][j] += w[k] * (float)y[k][i][j];
+        }
     }
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if ((threadIdx.x + i * NT) * 4 >= Dp) b[i] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
   float r = 1.f;
   if (a.w_post) {
@@ -131,7 +157,7 @@ __global__ __launch_bounds__(RN_THREADS) void tail_kernel(msa_tail_args a) {
   }
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
-    const int c = (threadIdx.x + i * RN_THREADS) * 4;
+    const int c = (threadIdx.x + i * NT) * 4;
     if (c < Dp) {
       if (a.w_post) {
         const float4_t wv = *reinterpret_cast<const float4_t*>(a.w_post + c);
@@ -141,7 +167,7 @@ __global__ __launch_bounds__(RN_THREADS) void tail_kernel(msa_tail_args a) {
       *reinterpret_cast<float4_t*>(a.x + m * Dp + c) = x[i];
     }
   }
-  if (a.w_next) norm_out<T, NV>(x, m, D, Dp, a.eps, a.w_next, a.h, a.h_mb, red);
+  if (a.w_next) norm_out<T, NV, NT>(x, m, D, Dp, a.eps, a.w_next, a.h, a.h_mb, red);
 }
 
 // Down-projected latents: one workgroup per token, the two norms by different halves of it.
@@ -156,8 +182,14 @@ __global__ __launch_bounds__(RN_THREADS) void latent_norm_kernel(
   const int64_t m = blockIdx.x;
   float sq = 0.f, skv = 0.f;
   for (int c = threadIdx.x; c < qp + rp; c += RN_THREADS) {
-    float v = part[m * N + c];
-    for (int s = 1; s < S; ++s) v += part[((int64_t)s * M + m) * N + c];
+    float v = 0.f;
+    for (int s0 = 0; s0 < S; s0 += 4) {
+      float p[4];
+#pragma unroll
+      for (int s = 0; s < 4; ++s)
+        p[s] = s0 + s < S ? part[((int64_t)min(s0 + s, S - 1) * M + m) * N + c] : 0.f;
+      v += (p[0] + p[1]) + (p[2] + p[3]);
+    }
     row[c] = v;
     if (c < qp) sq += v * v;
     else skv += v * v;
@@ -216,20 +248,24 @@ __global__ void advance_active_kernel(int32_t* lens, const int32_t* step_pos, in
   if (b < B && step_pos[b] >= 0) lens[b] = step_pos[b] + 1;
 }
 
-int vectors_per_thread(int Dp) {  // 1, 2, 4, 8 or 16; 0: too wide
-  const int q = (Dp / 4 + RN_THREADS - 1) / RN_THREADS;
-  for (int v = 1; v <= 16; v *= 2)
-    if (q <= v) return v;
-  return 0;
-}
+constexpr int RN_MAX_WIDTH = 16384;
 
-#define RN_DISPATCH(KERNEL, T, nv, ...)                                                         \
-  do {                                                                                          \
-    if (nv == 1) hipLaunchKernelGGL((KERNEL<T, 1>), __VA_ARGS__);                               \
-    else if (nv == 2) hipLaunchKernelGGL((KERNEL<T, 2>), __VA_ARGS__);                          \
-    else if (nv == 4) hipLaunchKernelGGL((KERNEL<T, 4>), __VA_ARGS__);                          \
-    else if (nv == 8) hipLaunchKernelGGL((KERNEL<T, 8>), __VA_ARGS__);                          \
-    else hipLaunchKernelGGL((KERNEL<T, 16>), __VA_ARGS__);                                      \
+// one row per workgroup of NT threads with NV float4 each
+#define RN_RUN(KERNEL, T, NV, NT, M, ...) \
+  hipLaunchKernelGGL((KERNEL<T, NV, NT>), dim3(M), dim3(NT), 0, (hipStream_t)stream, __VA_ARGS__)
+#define RN_DISPATCH(KERNEL, T, M, Dp, ...)                                                  \
+  do {                                                                                      \
+    const int q_ = (Dp) / 4;                                                                \
+    if (q_ <= 256) RN_RUN(KERNEL, T, 1, 256, M, __VA_ARGS__);                               \
+    else if ((M) <= RN_FEW_ROWS) {                                                          \
+      if (q_ <= 512) RN_RUN(KERNEL, T, 1, 512, M, __VA_ARGS__);                             \
+      else if (q_ <= 1024) RN_RUN(KERNEL, T, 1, 1024, M, __VA_ARGS__);                      \
+      else if (q_ <= 2048) RN_RUN(KERNEL, T, 2, 1024, M, __VA_ARGS__);                      \
+      else RN_RUN(KERNEL, T, 4, 1024, M, __VA_ARGS__);                                      \
+    } else if (q_ <= 512) RN_RUN(KERNEL, T, 2, 256, M, __VA_ARGS__);                        \
+    else if (q_ <= 1024) RN_RUN(KERNEL, T, 4, 256, M, __VA_ARGS__);                         \
+    else if (q_ <= 2048) RN_RUN(KERNEL, T, 4, 512, M, __VA_ARGS__);                         \
+    else RN_RUN(KERNEL, T, 4, 1024, M, __VA_ARGS__);                                        \
   } while (0)
 
 }  // namespace
@@ -241,14 +277,13 @@ extern "C" int msa_embed_rmsnorm(int dtype, const int64_t* tokens, const int32_t
   const char* name = "msa_embed_rmsnorm";
   MSA_REQUIRE(tokens && tok_pos && table && inv_freq && x && (!w || h), MSA_ERR_INVALID_ARG,
               "%s: null pointer", name);
-  const int nv = vectors_per_thread(Dp);
-  MSA_REQUIRE(M > 0 && vocab > 0 && D > 0 && D <= Dp && Dp % 4 == 0 && nv > 0, MSA_ERR_INVALID_ARG,
+  MSA_REQUIRE(M > 0 && vocab > 0 && D > 0 && D <= Dp && Dp % 4 == 0 && Dp <= RN_MAX_WIDTH, MSA_ERR_INVALID_ARG,
               "%s: M=%d vocab=%d D=%d Dp=%d", name, M, vocab, D, Dp);
   if (dtype == MSA_BF16)
-    RN_DISPATCH(embed_kernel, bf16_t, nv, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream, tokens,
+    RN_DISPATCH(embed_kernel, bf16_t, M, Dp, tokens,
                 tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, h_mb);
   else
-    RN_DISPATCH(embed_kernel, float, nv, dim3(M), dim3(RN_THREADS), 0, (hipStream_t)stream, tokens,
+    RN_DISPATCH(embed_kernel, float, M, Dp, tokens,
                 tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, 0);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
@@ -260,14 +295,13 @@ extern "C" int msa_residual_rmsnorm_tail(const msa_tail_args* a, void* stream) {
               "%s: null pointer", name);
   MSA_REQUIRE(!a->pair_y || (a->pair_w && a->inverse && a->top > 0), MSA_ERR_INVALID_ARG,
               "%s: routed terms without weights", name);
-  const int nv = vectors_per_thread(a->Dp);
-  MSA_REQUIRE(a->M > 0 && a->D > 0 && a->D <= a->Dp && a->Dp % 4 == 0 && nv > 0 &&
+  MSA_REQUIRE(a->M > 0 && a->D > 0 && a->D <= a->Dp && a->Dp % 4 == 0 && a->Dp <= RN_MAX_WIDTH &&
                   (!a->part || a->S > 0),
               MSA_ERR_INVALID_ARG, "%s: M=%d D=%d Dp=%d S=%d", name, a->M, a->D, a->Dp, a->S);
   if (a->dtype == MSA_BF16)
-    RN_DISPATCH(tail_kernel, bf16_t, nv, dim3(a->M), dim3(RN_THREADS), 0, (hipStream_t)stream, *a);
+    RN_DISPATCH(tail_kernel, bf16_t, a->M, a->Dp, *a);
   else
-    RN_DISPATCH(tail_kernel, float, nv, dim3(a->M), dim3(RN_THREADS), 0, (hipStream_t)stream, *a);
+    RN_DISPATCH(tail_kernel, float, a->M, a->Dp, *a);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }

@@ -89,7 +89,7 @@ class _LayerPlan:
             self.ff = _k(f.ff)
             self.n_ff = 2 * self.ff
         elif f is not None:
-            self.ffe = _up(f.expert.ff, 32)
+            self.ffe = _k(f.expert.ff)
             self.ffs = _k(f.shared.ff) if f.shared is not None else 0
             self.n_ff = 2 * self.ffs + _up(f.router.experts + (1 if self.ffs else 0), 16)
 
