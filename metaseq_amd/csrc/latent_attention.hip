@@ -43,9 +43,9 @@ bool raise_lds(const void* kernel, int bytes, std::atomic<uint64_t>& done) {
   return true;
 }
 
-// keys of one split, a multiple of the 64-key tile
+// keys of one split
 __device__ __forceinline__ int split_keys(int n_keys, int splits) {
-  return ((n_keys + splits - 1) / splits + 63) & ~63;
+  return ((n_keys + splits - 1) / splits + 15) & ~15;
 }
 
 constexpr int LA_KEYS = 64, LA_SC = LA_KEYS + 4;  // keys per tile; pitch of a head's scores
@@ -58,8 +58,8 @@ constexpr int la_lds_bytes = la_tile_bytes<RP> + NHB * 16 * LA_SC * 4;
 // A workgroup owns one token, one range of keys and NHB blocks of 16 heads, four waves per block.
 // The four waves share the scores of a 64-key tile (16 keys each) through LDS and then the weighted
 // sum by latent dimensions (RP / 4 each), so that no wave holds more than its share of the
-// accumulators and nothing has to be merged at the end.  The next tile's rows are fetched into
-// registers while a tile is worked on.
+// accumulators and nothing has to be merged at the end.  The rows of the next two tiles are on their way
+// into registers while a tile is worked on.
 template <int RP, int NHB>
 __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ latent, int capacity, int heads,
@@ -84,8 +84,8 @@ __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
   const int k_begin = split * per, k_end = min(n_keys, k_begin + per);
   const bf16_t* rows = latent + (int64_t)tok_slot[m] * capacity * RP;
 
-  half8_t pre[LD];
-  auto fetch = [&](int k0) {
+  half8_t pre0[LD], pre1[LD];
+  auto fetch = [&](half8_t(&pre)[LD], int k0) {
 #pragma unroll
     for (int i = 0; i < LD; ++i) {
       const int c = tid + THREADS * i;
@@ -93,13 +93,20 @@ __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
       pre[i] = *reinterpret_cast<const half8_t*>(rows + (int64_t)key * RP + (c % CH) * 8);
     }
   };
-  if (k_begin < k_end) fetch(k_begin);
   bf16x8_t qf[KS];
   {
     const bf16_t* qr = q + ((int64_t)m * heads + min(head, heads - 1)) * RP + g * 8;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8_t*>(qr + ks * 32);
   }
+  if (k_begin < k_end) {
+    fetch(pre0, k_begin);
+    fetch(pre1, k_begin + LA_KEYS);  // past the end: the last key again
+  }
+  // the queries have arrived here: a wait for them inside the loop would, on every pass, also be
+  // one for the tiles in flight
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) asm volatile("" : "+v"(qf[ks]));
   float4_t o[DW];
 #pragma unroll
   for (int d = 0; d < DW; ++d) o[d] = float4_t{0.f, 0.f, 0.f, 0.f};
@@ -108,20 +115,33 @@ __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
   const char* krow = lds + (16 * w4 + hc) * PITCH + g * 16;
   // transposing reads: lane (g, i) is the source of key row 4 g + i / 4, columns 4 (i % 4) ..
   const char* tr = lds + (4 * g + (hc >> 2)) * PITCH + w4 * (RP / 2) + (hc & 3) * 8;
-  for (int k0 = k_begin; k0 < k_end; k0 += LA_KEYS) {
+  auto tile = [&](half8_t(&pre)[LD], int k0) {
     lds_barrier();  // the previous tile and its scores are consumed
 #pragma unroll
     for (int i = 0; i < LD; ++i) {
       const int c = tid + THREADS * i;
       *reinterpret_cast<half8_t*>(lds + (c / CH) * PITCH + (c % CH) * 16) = pre[i];
     }
-    if (k0 + LA_KEYS < k_end) fetch(k0 + LA_KEYS);
+    // (past the end: the last key again - an unconditional load keeps the count of loads in flight
+    // known, so that the wait for one tile's rows is not a wait for the next one's)
+    fetch(pre, k0 + 2 * LA_KEYS);
     lds_barrier();
     float4_t s2[2] = {float4_t{0.f, 0.f, 0.f, 0.f}, float4_t{0.f, 0.f, 0.f, 0.f}};
+    constexpr int PD = 4;  // key fragments read ahead
+    bf16x8_t ka[PD];
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-      s2[ks & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-          *reinterpret_cast<const bf16x8_t*>(krow + ks * 64), qf[ks], s2[ks & 1], 0, 0, 0);
+    for (int ks = 0; ks < PD; ++ks) ka[ks] = *reinterpret_cast<const bf16x8_t*>(krow + ks * 64);
+    __builtin_amdgcn_sched_group_barrier(0x100, PD, 0);
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bf16x8_t cur = ka[ks % PD];
+      s2[ks & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cur, qf[ks], s2[ks & 1], 0, 0, 0);
+      __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+      if (ks + PD < KS) {
+        ka[ks % PD] = *reinterpret_cast<const bf16x8_t*>(krow + (ks + PD) * 64);
+        __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      }
+    }
     float4_t s = s2[0] + s2[1];
     // s[r]: this lane's head, key k0 + 16 w4 + 4 g + r
 #pragma unroll
@@ -141,7 +161,7 @@ __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
       }
     tm = fmaxf(tm, __shfl_xor(tm, 16, MSA_WAVE));
     tm = fmaxf(tm, __shfl_xor(tm, 32, MSA_WAVE));
-    const float mn = fmaxf(mx, tm);  // finite: the tile's first key is visible
+    const float mn = fmaxf(mx, tm);  // finite: the first tile's first key is visible
     if (__ballot(mn > mx)) {
       const float f = __builtin_amdgcn_exp2f(mx - mn);
       l *= f;
@@ -167,7 +187,13 @@ __global__ __launch_bounds__(256 * NHB) void latent_decode_kernel(
                                                        0, 0);
       }
     }
+  };
+  int k0 = k_begin;
+  for (; k0 + LA_KEYS < k_end; k0 += 2 * LA_KEYS) {
+    tile(pre0, k0);
+    tile(pre1, k0 + LA_KEYS);
   }
+  if (k0 < k_end) tile(pre0, k0);
   l += __shfl_xor(l, 16, MSA_WAVE);
   l += __shfl_xor(l, 32, MSA_WAVE);
   if (head >= heads) return;

@@ -43,12 +43,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
 #pragma unroll
     for (int i = 0; i < RT_EPL; ++i)
       if (lane + 64 * i < E && v[i] > bv) bv = v[i], bi = lane + 64 * i;
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, MSA_WAVE);
-      const int oi = __shfl_xor(bi, o, MSA_WAVE);
-      if (ov > bv || (ov == bv && oi < bi)) bv = ov, bi = oi;
-    }
+    const float best = wave_max(bv);
+    unsigned long long at = __ballot(bv == best);
+    int id = E - 1;  // (a row of NaN: no lane compares equal)
+    for (; at; at &= at - 1)  // one lane, but for ties
+      id = min(id, __builtin_amdgcn_readlane(bi, __builtin_ctzll(at)));
+    bv = best, bi = id;
   };
   float v[RT_EPL];  // candidates
   if (keep < n_groups) {

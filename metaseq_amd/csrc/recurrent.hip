@@ -201,8 +201,9 @@ __global__ __launch_bounds__(256) void rglru_state_kernel(
 
 // ---- gated delta rule -------------------------------------------------------------------------
 // Every column of a head's state evolves by itself (given k and q), so a workgroup owns one
-// segment, one head and 16 of its columns: a wave holds 4 columns, 16 lanes each, and a lane R
-// consecutive rows in registers, through all tokens of the segment.  With S the state before the
+// segment, one head and 256 / LPC of its columns: LPC lanes hold a column, each R consecutive rows of
+// it in registers, through all tokens of the segment.  16 lanes per column spread a single
+// prompt over the chip; 8 need fewer instructions per column where there are segments enough.  With S the state before the
 // token's decay, one pass over it yields both products the token needs:
 //   u = beta (v - g S^T k),   o = S_new^T q = g S^T q + u (k . q),   S_new = g S + k u^T.
 // Tokens are taken DR_TOK at a time: the next chunk's rows are fetched into registers while the
@@ -217,39 +218,48 @@ __device__ __forceinline__ float row16_sum(float v) {
   return v;
 }
 
-template <typename T, int R>
+template <int LPC>
+__device__ __forceinline__ float lanes_sum(float v) {  // over LPC = 8 or 16 neighbouring lanes
+  if constexpr (LPC == 16) return row16_sum(v);
+  v += dpp_move<0xB1, 0xf>(0.f, v);
+  v += dpp_move<0x4E, 0xf>(0.f, v);
+  v += dpp_move<0x141, 0xf>(0.f, v);  // row_half_mirror: the other quad of the eight
+  return v;
+}
+
+template <typename T, int DP, int LPC>
 __global__ __launch_bounds__(256) void delta_scan_kernel(
     const T* __restrict__ qkv, int64_t ld, const float* __restrict__ ba, int ldba,
     const float* __restrict__ decay_rate, const float* __restrict__ dt_bias, int heads, int kv_heads,
     float q_scale, int vp, float* __restrict__ state, float* __restrict__ o,
     const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
     const int32_t* __restrict__ seg_pos) {
-  constexpr int DP = 16 * R;
+  constexpr int R = DP / LPC, CW = 256 / LPC, R16 = DP / 16;
   __shared__ __attribute__((aligned(16))) float lk[DR_TOK][DP], lq[DR_TOK][DP];
-  __shared__ float lv[DR_TOK][16], lo[DR_TOK][16], lg[DR_TOK], lb[DR_TOK], lkq[DR_TOK];
-  const int s = blockIdx.z, h = blockIdx.y, col0 = blockIdx.x * 16;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  __shared__ float lv[DR_TOK][CW], lo[DR_TOK][CW], lg[DR_TOK], lb[DR_TOK], lkq[DR_TOK];
+  const int s = blockIdx.z, h = blockIdx.y, col0 = blockIdx.x * CW;
+  const int tid = threadIdx.x;
   const int first = seg_start[s], n = seg_start[s + 1] - first, pos = seg_pos[s];
   const int hk = h / (heads / kv_heads);
   const int q_at = hk * DP, k_at = kv_heads * DP + hk * DP, v_at = 2 * kv_heads * DP + h * vp + col0;
   if (pos < 0) {
-    for (int i = tid; i < n * 16; i += 256)
-      o[(int64_t)(first + i / 16) * heads * vp + h * vp + col0 + i % 16] = 0.f;
+    for (int i = tid; i < n * CW; i += 256)
+      o[(int64_t)(first + i / CW) * heads * vp + h * vp + col0 + i % CW] = 0.f;
     return;
   }
-  const int cl = wave * 4 + (lane >> 4), rl = lane & 15;  // column of the 16, row group
+  const int cl = tid / LPC, rl = tid % LPC;  // column of the workgroup's, row group
   float* st = state + (((int64_t)seg_slot[s] * heads + h) * vp + col0 + cl) * DP + rl * R;
   float S[R];
 #pragma unroll
   for (int i = 0; i < R; ++i) S[i] = pos > 0 ? st[i] : 0.f;
   const float rate = decay_rate[h], dtb = dt_bias[h];
 
-  // staging: vector x = tid / 8 (tokens 0 .. 15 of q, then of k), elements 2R * (tid % 8) ..
-  constexpr int EV = 2 * R;
+  // staging: vector x = tid / 8 (tokens 0 .. 15 of q, then of k), elements EV * (tid % 8) ..
+  constexpr int EV = DP / 8, VPT = DR_TOK * CW / 256;  // q or k elements, v elements per thread
   const int sv = tid >> 3, stok = sv & 15, sel = (tid & 7) * EV;
   const bool is_k = sv >= 16;
   T raw[EV];
-  float rv = 0.f, rb = 0.f, rg = 0.f;
+  float rv[VPT], rb = 0.f, rg = 0.f;
   auto fetch = [&](int t0) {
     const int t = min(t0 + stok, n - 1);
     const T* p = qkv + (int64_t)(first + t) * ld + (is_k ? k_at : q_at) + sel;
@@ -260,8 +270,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) raw[i + j] = x[j];
     }
-    const int tv = min(t0 + (tid >> 4), n - 1);
-    rv = (float)qkv[(int64_t)(first + tv) * ld + v_at + (tid & 15)];
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int e = tid + 256 * i, tv = min(t0 + e / CW, n - 1);
+      rv[i] = (float)qkv[(int64_t)(first + tv) * ld + v_at + e % CW];
+    }
     if (tid < DR_TOK) {
       const float* z = ba + (int64_t)(first + min(t0 + tid, n - 1)) * ldba;
       rb = z[h];
@@ -282,7 +295,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       float* dst = (is_k ? lk[stok] : lq[stok]) + sel;
 #pragma unroll
       for (int i = 0; i < EV; ++i) dst[i] = (float)raw[i] * f;
-      lv[tid >> 4][tid & 15] = rv;
+#pragma unroll
+      for (int i = 0; i < VPT; ++i) (&lv[0][0])[tid + 256 * i] = rv[i];
       if (tid < DR_TOK) {
         lb[tid] = sigmoidf(rb);
         lg[tid] = expf(-rate * softplus(rg + dtb));
@@ -293,7 +307,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       const int t = tid >> 4, r = tid & 15;
       float d = 0.f;
 #pragma unroll
-      for (int i = 0; i < R; ++i) d = fmaf(lk[t][r * R + i], lq[t][r * R + i], d);
+      for (int i = 0; i < R16; ++i) d = fmaf(lk[t][r * R16 + i], lq[t][r * R16 + i], d);
       d = row16_sum(d);
       if (r == 0) lkq[t] = d;
     }
@@ -318,8 +332,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
         d2 = fmaf(S[i], x.q[i], d2);
         e2 = fmaf(S[i + 1], x.q[i + 1], e2);
       }
-      d1 = row16_sum(d1 + e1);
-      d2 = row16_sum(d2 + e2);
+      d1 = lanes_sum<LPC>(d1 + e1);
+      d2 = lanes_sum<LPC>(d2 + e2);
       const float u = x.beta * (x.v - x.g * d1);
 #pragma unroll
       for (int i = 0; i < R; ++i) S[i] = fmaf(x.k[i], u, x.g * S[i]);
@@ -333,9 +347,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       if (t + 1 < nt) advance(b, t + 1);
     }
     lds_barrier();
-    if (tid < nt * 16)
-      o[(int64_t)(first + t0 + (tid >> 4)) * heads * vp + h * vp + col0 + (tid & 15)] =
-          lo[tid >> 4][tid & 15];
+    for (int e = tid; e < nt * CW; e += 256)
+      o[(int64_t)(first + t0 + e / CW) * heads * vp + h * vp + col0 + e % CW] = (&lo[0][0])[e];
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) st[i] = S[i];
@@ -475,27 +488,39 @@ __global__ __launch_bounds__(256) void delta_output_kernel(
   }
 }
 
-template <typename T>
+template <typename T, int LPC>
 void run_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
                const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vp, float* state,
                float* o, const msa_batch* b, hipStream_t s) {
-  const dim3 grid(vp / 16, heads, b->nseg);
+  const dim3 grid(vp / (256 / LPC), heads, b->nseg);
   const float q_scale = (float)pow((double)dim, -0.5);
-#define DR_CASE(RR)                                                                                 \
-  case 16 * RR:                                                                                     \
-    hipLaunchKernelGGL((delta_scan_kernel<T, RR>), grid, dim3(256), 0, s, (const T*)qkv, ld, ba,    \
-                       ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vp, state, o,           \
+#define DR_CASE(DP)                                                                                 \
+  case DP:                                                                                          \
+    hipLaunchKernelGGL((delta_scan_kernel<T, DP, LPC>), grid, dim3(256), 0, s, (const T*)qkv, ld,   \
+                       ba, ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vp, state, o,       \
                        b->seg_start, b->seg_slot, b->seg_pos);                                      \
     break;
   switch (dp) {
-    DR_CASE(2)
-    DR_CASE(4)
-    DR_CASE(6)
-    DR_CASE(8)
-    DR_CASE(12)
-    DR_CASE(16)
+    DR_CASE(32)
+    DR_CASE(64)
+    DR_CASE(96)
+    DR_CASE(128)
+    DR_CASE(192)
+    DR_CASE(256)
   }
 #undef DR_CASE
+}
+
+template <typename T>
+void pick_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
+                const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vp, float* state,
+                float* o, const msa_batch* b, hipStream_t s) {
+  // eight lanes per column from two waves per SIMD on (of 1024)
+  if (vp % 32 == 0 && (int64_t)b->nseg * heads * (vp / 32) * 4 >= 2048)
+    run_delta<T, 8>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b, s);
+  else
+    run_delta<T, 16>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
+                     s);
 }
 
 template <typename T>
@@ -656,10 +681,10 @@ extern "C" int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const floa
               MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
               kv_heads, dim, dp, vp);
   if (dtype == MSA_BF16)
-    run_delta<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o,
+    pick_delta<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o,
                       b, (hipStream_t)stream);
   else
-    run_delta<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
+    pick_delta<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
                      (hipStream_t)stream);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;

@@ -64,16 +64,16 @@ __global__ __launch_bounds__(NT) void embed_kernel(
     if (c >= Dp) continue;
     const bf16x4_t e = *reinterpret_cast<const bf16x4_t*>(table + t * Dp + c);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      float p = 0.f;
+    for (int j = 0; j < 4; j += 2) {
+      float sn = 0.f, cs = 0.f;
       if (c + j < D) {
-        // the angle in turns, reduced to [-1/2, 1/2] in double; sin / cos of pi * (2 turns)
+        // the angle in turns, reduced to [-1/2, 1/2] in double; sine and cosine of pi * (2 turns)
         double turns = pos * inv_freq[(c + j) >> 1] * 0.15915494309189535;
         turns -= rint(turns);
-        const float a = 2.f * (float)turns;
-        p = (j & 1) ? cospif(a) : sinpif(a);
+        sincospif(2.f * (float)turns, &sn, &cs);
       }
-      v[i][j] = (float)e[j] * scale + p;
+      v[i][j] = (float)e[j] * scale + sn;
+      v[i][j + 1] = (float)e[j + 1] * scale + (c + j + 1 < D ? cs : 0.f);
     }
     *reinterpret_cast<float4_t*>(x + m * Dp + c) = v[i];
   }

@@ -231,6 +231,82 @@ def test_latent_attention(rp, dtype):
         close(out, ref, 1e-2 if dtype == BF16 else 1e-5, "latent %d, %d splits" % (rp, splits))
 
 
+def _batch(segments, M):
+    """A msa_batch of (slot, first position, tokens) segments with its tensors."""
+    start, slot, pos = [0], [], []
+    tok = [[], [], []]
+    for s, p, n in segments:
+        start.append(start[-1] + n)
+        slot.append(s)
+        pos.append(p)
+        tok[0] += [s] * n
+        tok[1] += [p + i if p >= 0 else -1 for i in range(n)]
+        tok[2] += range(n)
+    dev = [torch.tensor(x, dtype=torch.int32, device="cuda") for x in tok + [start, slot, pos]]
+    b = _capi.Batch()
+    b.M, b.nseg, b.max_count = M, len(slot), max(n for _, _, n in segments)
+    (b.tok_slot, b.tok_pos, b.tok_off, b.seg_start, b.seg_slot, b.seg_pos) = map(ptr, dev)
+    host = [(ctypes.c_int32 * len(x))(*x) for x in (start, slot, pos)]
+    b.host_start, b.host_slot, b.host_pos = host
+    return b, (dev, host)
+
+
+@pytest.mark.parametrize("heads,kv_heads,dim,dp,vp,counts", [
+    (4, 2, 30, 32, 48, (5, 1, 40)), (3, 3, 128, 128, 64, (17, 16)), (2, 1, 250, 256, 32, (33,)),
+    (32, 8, 64, 64, 64, (9, 2, 1, 30, 16, 17, 3, 4)),      # eight lanes per column
+    (64, 64, 128, 128, 32, (7, 20, 1, 2, 1, 1, 1, 1)), (32, 16, 96, 96, 64, (5,) * 8)])
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+def test_delta_scan(heads, kv_heads, dim, dp, vp, counts, dtype):
+    """Several segments, one of them continuing its slot's state and (with three or more) one
+    inactive; outputs and the states left behind."""
+    lib = _capi.load_hybrid()
+    print("delta_scan", heads, kv_heads, dim, dp, vp, counts, flush=True)
+    g = gen(heads + dp)
+    M, slots = sum(counts), len(counts) + 1
+    C = 2 * kv_heads * dp + heads * vp
+    qkv = torch.randn(M, C, generator=g)
+    qkv[:, :2 * kv_heads * dp].view(M, 2 * kv_heads, dp)[:, :, dim:] = 0
+    qkv = qkv.to(dtype)
+    ba = torch.randn(M, 2 * heads + 3, generator=g)
+    rate, dtb = torch.rand(heads, generator=g) * 0.3, torch.randn(heads, generator=g)
+    state = torch.randn(slots, heads, vp, dp, generator=g)
+    state[..., dim:] = 0
+    segs = [(slots - 1 - i, 0 if i else 12, n) for i, n in enumerate(counts)]
+    if len(counts) > 2:
+        segs[1] = (segs[1][0], -1, segs[1][2])
+    want, S = torch.zeros(M, heads, vp, dtype=torch.float64), state.double().clone()
+    x = qkv.double()
+    unit = lambda t: t / torch.sqrt((t * t).sum(-1, keepdim=True) + 1e-6)
+    at = 0
+    for slot, pos, n in segs:
+        if pos >= 0:
+            s = S[slot] if pos > 0 else torch.zeros_like(S[slot])       # [heads, vp, dp]
+            for m in range(at, at + n):
+                q = unit(x[m, :kv_heads * dp].view(kv_heads, dp)) * dim ** -0.5
+                k = unit(x[m, kv_heads * dp:2 * kv_heads * dp].view(kv_heads, dp))
+                q, k = (t.repeat_interleave(heads // kv_heads, 0) for t in (q, k))
+                v = x[m, 2 * kv_heads * dp:].view(heads, vp)
+                z = ba[m].double()
+                beta = torch.sigmoid(z[:heads])
+                decay = torch.exp(-rate.double() * torch.nn.functional.softplus(
+                    z[heads:2 * heads] + dtb.double()))
+                s = s * decay.view(-1, 1, 1)
+                u = beta.view(-1, 1) * (v - torch.einsum("hvd,hd->hv", s, k))
+                s = s + u.unsqueeze(2) * k.unsqueeze(1)
+                want[m] = torch.einsum("hvd,hd->hv", s, q)
+            S[slot] = s
+        at += n
+    b, alive = _batch(segs, M)
+    qd, bd, rd, td, sd = (t.cuda() for t in (qkv, ba, rate, dtb, state))
+    o = torch.full((M, heads * vp), 7.0, device="cuda")
+    check(lib.msa_delta_scan(0 if dtype == BF16 else 1, ptr(qd), C, ptr(bd), 2 * heads + 3, ptr(rd),
+                             ptr(td), heads, kv_heads, dim, dp, vp, ptr(sd), ptr(o), ctypes.byref(b),
+                             _capi.stream_ptr()), lib)
+    close(o.view(M, heads, vp), want, 2e-5, "outputs")
+    close(sd, S, 2e-5, "states")
+    del alive
+
+
 def test_selection_over_fp32_logits():
     """The fp32 forms of selection, scoring and sampling agree with plain PyTorch, at row strides
     and vocabulary sizes that are no multiple of 8."""
