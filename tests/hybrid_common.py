@@ -1,4 +1,6 @@
 """Small hybrid configurations, their weights and comparisons with the plain oracle."""
+import json
+
 import torch
 
 from metaseq_amd import HybridConfig, HybridDecoder, random_hybrid_state_dict
@@ -62,6 +64,26 @@ def mixed(dtype=torch.float32, width=72):
 def no_specials(state):
     """Logits of the special ids 0 .. 3 are never the largest (a record ends at one)."""
     state["head"][:4] = 0
+
+
+def write_safetensors(path, tensors):
+    names = {torch.bfloat16: "BF16", torch.float32: "F32", torch.int32: "I32"}
+    header, blob = {"__metadata__": {"format": "pt"}}, b""
+    for k, t in tensors.items():
+        data = t.contiguous().view(torch.uint8).numpy().tobytes() if t.numel() else b""
+        header[k] = dict(dtype=names[t.dtype], shape=list(t.shape),
+                         data_offsets=[len(blob), len(blob) + len(data)])
+        blob += data
+    text = json.dumps(header).encode()
+    with open(path, "wb") as f:
+        f.write(len(text).to_bytes(8, "little") + text + blob)
+
+
+def model_folder(path, cfg, state):
+    """A model folder as the registry reads it."""
+    write_safetensors(path / "model.safetensors", state)
+    (path / "config.json").write_text(json.dumps(cfg))
+    return str(path)
 
 
 class Case:

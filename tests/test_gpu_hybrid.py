@@ -1,11 +1,15 @@
 """Hybrid decoders against the plain oracle: every mechanism alone and together, prompts, portions,
 decoding, batches of unequal requests, re-used slots, single keys that must or must not be seen,
 long memories, and generation through the framework's own entry points."""
+import json
+
+import numpy as np
 import pytest
 import torch
 
 from metaseq_amd import (Dictionary, GeneratorInterface, SequenceGenerator,
                          TransformerLanguageModel)
+from metaseq_amd import generate, trace_run
 from metaseq_amd.service import ContinuousBatcher
 from oracle import hybrid_oracle as O
 from tests import hybrid_common as H
@@ -314,6 +318,52 @@ def test_greedy_generation_through_the_continuous_batcher():
             want = _greedy_oracle(case, [2] + p, 5 + i)[1 + len(p):]
             assert [int(x) for x in record[0]["tokens"]][:5 + i] == want, i
         assert len(sampled.get_nowait()[1]) == 2
+
+
+def test_generate_command(tmp_path, capsys):
+    """A model folder through the command line, as one batch and through slots."""
+    case = H.Case(H.mixed(), seed=37, dtype=F32, tweak=H.no_specials)
+    folder = H.model_folder(tmp_path, case.json, case.state)
+    prompts = [case.tokens(n, seed=n).tolist() for n in (4, 9, 2)]
+    lines = [" ".join(map(str, p)) for p in prompts]
+    for extra in ([], ["--slots", "2"]):
+        rc = generate.main(["--model", folder, "--dtype", "float32", "--max-tokens", "5",
+                            "--min-tokens", "5"] + extra, lines=lines)
+        records = [json.loads(x) for x in capsys.readouterr().out.splitlines() if x[:1] == "{"]
+        assert rc == 0 and len(records) == 3
+        for p, r in zip(prompts, records):
+            assert r["tokens"][:4] == _greedy_oracle(case, [2] + p, 4)[1 + len(p):]
+
+
+@DTYPES
+def test_trace_command(tmp_path, capsys, dtype):
+    """Requests replayed in portions and token by token, their slots given back and used again."""
+    case = H.Case(H.mixed(dtype), seed=39, dtype=dtype)
+    folder = H.model_folder(tmp_path, case.json, case.state)
+    out = tmp_path / "out"
+    out.mkdir()
+    toks = {i: case.tokens(n, seed=n) for i, n in (("a", 70), ("b", 45), ("c", 3))}
+    cuts = {"a": [33, 2, 33, 1, 1], "b": [44, 1], "c": [1, 1, 1]}
+    steps, expect = [], []
+    for r in ("a", "b", "c"):
+        at, want = 0, case.want(toks[r])
+        for k, n in enumerate(cuts[r]):
+            places = [] if k == 1 and r == "a" else sorted({0, n - 1})[::-1]
+            steps.append(dict(step=len(steps), end=[r] if at + n == len(toks[r]) else [],
+                              entries=[dict(id=r, tokens=toks[r][at:at + n].tolist(), want=places)]))
+            expect.append(want[[at + p for p in places]])
+            at += n
+    rc = trace_run.main(["--model", folder, "--dtype", str(dtype).split(".")[1], "--out", str(out),
+                         "--max-tokens", "70"], lines=[json.dumps(s) for s in steps])
+    assert rc == 0
+    done = [x for x in capsys.readouterr().out.splitlines() if x.startswith("done")]
+    assert done == ["done %d" % i for i in range(len(steps))]
+    for s, want in zip(steps, expect):
+        path = out / ("%d.f32" % s["step"])
+        assert path.exists() == bool(len(want))
+        if len(want):
+            got = torch.from_numpy(np.fromfile(path, dtype="<f4")).view(len(want), -1)
+            case.check(got, want, "step %d" % s["step"])
 
 
 def test_errors_are_raised_on_the_host():

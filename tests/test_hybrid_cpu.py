@@ -23,19 +23,6 @@ from tests import hybrid_common as H
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def write_safetensors(path, tensors):
-    names = {torch.bfloat16: "BF16", torch.float32: "F32", torch.int32: "I32"}
-    header, blob = {"__metadata__": {"format": "pt"}}, b""
-    for k, t in tensors.items():
-        data = t.contiguous().view(torch.uint8).numpy().tobytes() if t.numel() else b""
-        header[k] = dict(dtype=names[t.dtype], shape=list(t.shape),
-                         data_offsets=[len(blob), len(blob) + len(data)])
-        blob += data
-    text = json.dumps(header).encode()
-    with open(path, "wb") as f:
-        f.write(len(text).to_bytes(8, "little") + text + blob)
-
-
 # ---------------------------------------------------------------- configuration, registry, files
 def test_config_reads_every_layer_kind():
     cfg = HybridConfig.from_json(H.mixed())
@@ -83,7 +70,7 @@ def test_safetensors_round_trip_and_model_folder(tmp_path):
     c = H.mixed()
     state = random_hybrid_state_dict(HybridConfig.from_json(c), 3)
     state["odd"] = torch.arange(5, dtype=torch.int32)
-    write_safetensors(tmp_path / "model.safetensors", state)
+    H.write_safetensors(tmp_path / "model.safetensors", state)
     got = read_safetensors(str(tmp_path / "model.safetensors"))
     assert list(got) == list(state)
     assert all(torch.equal(got[k], state[k]) and got[k].dtype == state[k].dtype for k in state)
