@@ -1,5 +1,5 @@
-"""MI355X-native OPT incremental-decoding forward path (drop-in for metaseq's
-TransformerDecoder.forward / SequenceGenerator on one gfx950 GPU)."""
+"""MI355X-native incremental decoding: OPT (drop-in for metaseq's TransformerDecoder.forward /
+SequenceGenerator on one gfx950 GPU) and hybrid decoders."""
 from .config import HybridConfig, OPTConfig, config_from_state_dict, opt_config
 from .dictionary import Dictionary
 from .hub_utils import GeneratorInterface
@@ -13,7 +13,9 @@ from .transformer_decoder import ModelParallelTransformerDecoder, TransformerDec
 from .transformer_lm import TransformerLanguageModel
 
 __all__ = [
-    "OPTConfig", "HybridConfig", "HybridDecoder", "HybridCache", "load_model", "opt_config", "config_from_state_dict", "Dictionary", "GeneratorInterface", "KVCache", "SequenceGenerator", "random_prompts",
-    "random_state_dict", "random_hybrid_state_dict", "iter_random_state_dict", "TransformerDecoder", "ModelParallelTransformerDecoder",
+    "OPTConfig", "HybridConfig", "HybridDecoder", "HybridCache", "load_model", "opt_config",
+    "config_from_state_dict", "Dictionary", "GeneratorInterface", "KVCache",
+    "SequenceGenerator", "random_prompts", "random_state_dict", "random_hybrid_state_dict",
+    "iter_random_state_dict", "TransformerDecoder", "ModelParallelTransformerDecoder",
     "TransformerLanguageModel",
 ]

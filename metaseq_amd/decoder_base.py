@@ -109,14 +109,16 @@ class IncrementalDecoder(nn.Module):
         if T > 1:
             lp = torch.empty(T - 1, dtype=torch.float32, device=logits.device)
             target = tokens.long()[1:].contiguous()
-            check(_capi.for_logits(lib, "msa_target_logprob", logits)(ptr(logits), logits.stride(0), T - 1, V,
-                                             float(temperature), ptr(target), ptr(lp), stream))
+            check(_capi.for_logits(lib, "msa_target_logprob", logits)(
+                ptr(logits), logits.stride(0), T - 1, V, float(temperature), ptr(target), ptr(lp),
+                stream))
             if not _lazy:   # (_lazy: the caller reads the device tensor once all is queued)
                 scores[1:] = lp.tolist()
             if prompt_topk > 0 and detail is not None:
                 dist = torch.empty(T - 1, V, dtype=torch.float32, device=logits.device)
-                check(_capi.for_logits(lib, "msa_log_softmax", logits)(ptr(logits), 0, logits.stride(0), 1, T - 1, V,
-                                              float(temperature), ptr(dist), 0, V, stream))
+                check(_capi.for_logits(lib, "msa_log_softmax", logits)(
+                    ptr(logits), 0, logits.stride(0), 1, T - 1, V, float(temperature), ptr(dist),
+                    0, V, stream))
                 values, ids = dist.topk(min(int(prompt_topk), V), dim=-1)
                 detail["prompt_top"] = (values.cpu(), ids.cpu())
                 del dist
@@ -133,9 +135,9 @@ class IncrementalDecoder(nn.Module):
         if R > 1:  # every replica reads its own copy of the row (a few hundred KB)
             last = last.expand(R, V).contiguous()
         if plain:
-            check(_capi.for_logits(lib, "msa_greedy_select", logits)(ptr(last), last.stride(0), R, V, 1.0, ba, len(banned),
-                                            sa, len(stop), None, ptr(row_mode), 0, int(eos),
-                                            ptr(tok_out), 1, ptr(score_out), 1, None, stream))
+            check(_capi.for_logits(lib, "msa_greedy_select", logits)(
+                ptr(last), last.stride(0), R, V, 1.0, ba, len(banned), sa, len(stop), None,
+                ptr(row_mode), 0, int(eos), ptr(tok_out), 1, ptr(score_out), 1, None, stream))
         else:
             pen = penalties or {}
             alphas = [float(a) for a in pen.get("alphas", (0.0, 0.0, 0.0, 0.0))]
@@ -152,9 +154,8 @@ class IncrementalDecoder(nn.Module):
                 ptr(last), last.stride(0), R, V, float(temperature), None, ba, len(banned), sa,
                 len(stop), None, ptr(row_mode), 0, int(eos), None, float(topp), ptr(noise),
                 ptr(pen.get("counts")), ptr(pen.get("counts_src")), alphas[0], alphas[1],
-                alphas[2], alphas[3], None, ptr(lprobs_out),
-                lprobs_out.stride(0) if lprobs_out is not None else 0, ptr(tok_out), 1,
-                ptr(score_out), 1, stream))
+                alphas[2], alphas[3], None, ptr(lprobs_out), lprobs_out.stride(0) if lprobs_out is
+                not None else 0, ptr(tok_out), 1, ptr(score_out), 1, stream))
         return lp if _lazy else scores
 
     def copy_slot(self, cache, src: int, dst: int, length: Optional[int] = None):

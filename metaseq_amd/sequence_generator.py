@@ -236,9 +236,10 @@ class SequenceGenerator(nn.Module):
             if all_lprobs is not None and start_step > 1:
                 # the distributions of the prompt positions (:247-250), fp32 rows written in place
                 dst = all_lprobs[:, 1]
-                check(_capi.for_logits(lib, "msa_log_softmax", flat)(ptr(flat), T * flat.stride(0), flat.stride(0), BB,
-                                              start_step - 1, V, float(self.temperature), ptr(dst),
-                                              all_lprobs.stride(0), all_lprobs.stride(1), stream))
+                check(_capi.for_logits(lib, "msa_log_softmax", flat)(
+                    ptr(flat), T * flat.stride(0), flat.stride(0), BB, start_step - 1, V,
+                    float(self.temperature), ptr(dst), all_lprobs.stride(0), all_lprobs.stride(1),
+                    stream))
             # the row that predicts each sample's first free token (:262-267)
             if int(rep_lengths.max()) >= T:
                 # the reference indexes lprobs[i, prompt_len] out of range in this case: every
