@@ -102,6 +102,97 @@ def delta(h, W, pre, m, eps):
     return o.reshape(T, H * vdim) @ W[pre + "o"].T
 
 
+def rotate_half(x, positions, base, dims):
+    """x [T, heads, dim]: rotates the pairs (i, i + dims / 2) of the first ``dims`` dimensions."""
+    half = dims // 2
+    f = float(base) ** (-2.0 * torch.arange(half, dtype=torch.float64) / max(dims, 1))
+    ang = (positions.double().view(-1, 1) * f).unsqueeze(1)
+    c, s = torch.cos(ang).to(x.dtype), torch.sin(ang).to(x.dtype)
+    out = x.clone()
+    u, v = x[..., :half], x[..., half:dims]
+    out[..., :half] = u * c - v * s
+    out[..., half:dims] = v * c + u * s
+    return out
+
+
+def chunk_mask(T, size):
+    """[T, T]: entry (i, j) says whether position i sees position j: none after it, none of another
+    chunk of ``size`` positions (None: one chunk)."""
+    m = torch.zeros(T, T, dtype=torch.bool)
+    for i in range(T):
+        first = 0 if size is None else i // size * size
+        m[i, first:i + 1] = True
+    return m
+
+
+def grouped_attention(h, W, pre, m):
+    """Rotary attention within chunks, several query heads per key/value head, each head's output
+    scaled by a gate of its own."""
+    T, H, G, dim, vdim = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    lin = lambda n: h @ W[pre + n].T + W[pre + n + ".b"]
+    q, k, v = lin("q").view(T, H, dim), lin("k").view(T, G, dim), lin("v").view(T, G, vdim)
+    if m.get("rot"):
+        at = torch.arange(T)
+        q = rotate_half(q, at, m["rot"]["base"], m["rot"]["dims"])
+        k = rotate_half(k, at, m["rot"]["base"], m["rot"]["dims"])
+    sees = chunk_mask(T, (m.get("mask") or {}).get("size"))
+    gate = torch.sigmoid(h @ W[pre + "g"].T)
+    out = torch.zeros(T, H, vdim, dtype=h.dtype)
+    for i in range(H):
+        g = i // (H // G)
+        s = (q[:, i] @ k[:, g].T * m["scale"]).masked_fill(~sees, float("-inf"))
+        out[:, i] = torch.softmax(s, dim=-1) @ v[:, g] * gate[:, i:i + 1]
+    return out.reshape(T, H * vdim) @ W[pre + "o"].T
+
+
+def channel_delta(h, W, pre, m, eps):
+    """Gated delta rule with one decay per head and key channel and a low-rank sigmoid gate."""
+    T, H, Hk, dim, vdim = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    conv = lambda n: F.silu(causal_conv(h @ W[pre + n].T, W[pre + n + ".conv"]))
+    unit = lambda x: x / torch.sqrt((x * x).sum(dim=-1, keepdim=True) + 1e-6)
+    q = unit(conv("q").view(T, Hk, dim)) * dim ** -0.5
+    k = unit(conv("k").view(T, Hk, dim))
+    v = conv("v").view(T, H, vdim)
+    beta = torch.sigmoid(h @ W[pre + "b"].T)
+    z = (h @ W[pre + "a1"].T) @ W[pre + "a2"].T + W[pre + "dt_bias"]
+    decay = torch.exp(-torch.exp(W[pre + "A_log"]).view(1, H, 1) * F.softplus(z).view(T, H, dim))
+    head = torch.arange(H) // (H // Hk)
+    S = torch.zeros(H, dim, vdim, dtype=h.dtype)
+    o = torch.zeros(T, H, vdim, dtype=h.dtype)
+    for t in range(T):
+        kt, qt = k[t, head], q[t, head]
+        S = decay[t].unsqueeze(2) * S
+        u = beta[t].unsqueeze(1) * (v[t] - torch.einsum("hdv,hd->hv", S, kt))
+        S = S + torch.einsum("hd,hv->hdv", kt, u)
+        o[t] = torch.einsum("hdv,hd->hv", S, qt)
+    gate = torch.sigmoid((h @ W[pre + "g1"].T) @ W[pre + "g2"].T).view(T, H, vdim)
+    o = rms(o, eps, W[pre + "norm"]) * gate
+    return o.reshape(T, H * vdim) @ W[pre + "o"].T
+
+
+def parallel(h, W, pre, m, eps):
+    """Attention and delta rule side by side: the mean of their normed outputs."""
+    left = grouped_attention(h, W, pre + "left.", m["left"])
+    right = channel_delta(h, W, pre + "right.", m["right"], eps)
+    return 0.5 * (rms(left, eps, W[pre + "left.out"]) + rms(right, eps, W[pre + "right.out"]))
+
+
+def relu2_ff(h, W, pre):
+    u = torch.relu(h @ W[pre + "up"].T + W[pre + "up.b"])
+    return (u * u) @ W[pre + "down"].T + W[pre + "down.b"]
+
+
+def layer_runs(cfg):
+    """(layer, pass) in the order of execution; pass is None outside the loop."""
+    loop, n = cfg.get("loop"), len(cfg["layers"])
+    if not loop:
+        return [(i, None) for i in range(n)]
+    inner = range(loop["start"], loop["stop"])
+    return ([(i, None) for i in range(loop["start"])]
+            + [(i, t) for t in range(loop["times"]) for i in inner]
+            + [(i, None) for i in range(loop["stop"], n)])
+
+
 def dense_ff(h, W, pre):
     return (gelu_tanh(h @ W[pre + "gate"].T) * (h @ W[pre + "up"].T)) @ W[pre + "down"].T
 
@@ -147,11 +238,33 @@ def embed(tokens, W, cfg):
     return x + sinusoid(torch.arange(len(tokens)), cfg["width"], x.dtype)
 
 
+def forward_looped(tokens, W, cfg):
+    """Pre-norm layers of parallel mixers, a range of them run several times; (logits, streams)."""
+    eps = cfg["norm"]["eps"]
+    x = first = W["embed"][tokens]
+    layers = []
+    for i, t in layer_runs(cfg):
+        if t is not None and i == cfg["loop"]["start"]:
+            if t > 0:
+                x = x + first
+            x = x + W["loop.step"][t]
+        pre = "l%d." % i
+        layer = cfg["layers"][i]
+        x = x + parallel(rms(x, eps, W[pre + "norm1"]), W, pre + "mix.", layer["mixer"], eps)
+        if layer.get("mlp"):
+            x = x + relu2_ff(rms(x, eps, W[pre + "norm2"]), W, pre + "mlp.")
+        layers.append(x)
+    return rms(x, eps, W["final.norm"]) @ W["embed"].T, layers
+
+
 @torch.no_grad()
 def forward(tokens, W, cfg, return_layers=False):
     """Logits [T, vocab] of one sequence (and the residual stream after every layer)."""
     W = dict(W)
     eps = cfg["norm"]["eps"]
+    if cfg.get("architecture") == "Nomalorn":
+        logits, layers = forward_looped(tokens, W, cfg)
+        return (logits, torch.stack(layers)) if return_layers else logits
     x = embed(tokens, W, cfg)
     latents, layers = {}, []
     for i, layer in enumerate(cfg["layers"]):
