@@ -28,8 +28,11 @@ extern "C" {
 
 enum { MSA_BF16 = 0, MSA_F32 = 1 };
 enum { MSA_GLU_NONE = -1, MSA_GLU_GELU = 0, MSA_GLU_CLAMPED = 1 };
-enum { MSA_MIX_LATENT = 0, MSA_MIX_RGLRU = 1, MSA_MIX_DELTA = 2 };
-enum { MSA_FF_NONE = 0, MSA_FF_DENSE = 1, MSA_FF_MOE = 2 };
+enum { MSA_ACT_NONE = 0, MSA_ACT_RELU2 = 1 };
+enum { MSA_GATE_SILU = 0, MSA_GATE_SIGMOID = 1 };
+enum { MSA_MIX_LATENT = 0, MSA_MIX_RGLRU = 1, MSA_MIX_DELTA = 2, MSA_MIX_PARALLEL = 3 };
+enum { MSA_FF_NONE = 0, MSA_FF_DENSE = 1, MSA_FF_MOE = 2, MSA_FF_RELU2 = 3 };
+#define MSA_OUT2_PACKED 16u /* msa_linear: y2 in the packed layout */
 
 /* A flat batch.  tok_*: per token its cache slot, its position in the slot's sequence (negative: the
  * token is inactive - it changes no cache or state, its outputs mean nothing) and its offset in its
@@ -57,6 +60,24 @@ int msa_linear_f32(const float* x, const float* W, float* y, float* y32, int64_t
 int msa_linear_partial_bf16(const void* x, const void* W, float* part, int64_t M, int N, int K, int S,
                             unsigned flags, void* stream);
 int msa_linear_bf16_splits(int64_t M, int N, int K, int packed);
+
+/* A linear layer with what follows it: z = x W^T + bias ; columns below n32 leave as act(z) in the
+ * activation format, those of them from n2 on into a matrix of their own (y2 [M, n32 - n2]; y2 NULL: all
+ * into y, otherwise y is [M, n2]) ; the columns from n32 on leave as fp32 into y32 [M, N - n32], with
+ * decay_rate as decays exp(-decay_rate[n - n32] softplus(z)).  MSA_ACT_RELU2: max(z, 0)^2.  bias [N] and
+ * decay_rate [N - n32] may be NULL.  n2 and n32 are multiples of 16.  flags (bf16): MSA_IN_PACKED,
+ * MSA_OUT_PACKED (y), MSA_OUT2_PACKED (y2). */
+typedef struct {
+  int dtype;
+  const void *x, *W;
+  int64_t M;
+  int N, K, n32, n2, act;
+  unsigned flags;
+  const float *bias, *decay_rate;
+  void *y, *y2;
+  float* y32;
+} msa_linear_args;
+int msa_linear(const msa_linear_args* a, void* stream);
 
 /* Grouped products: group g multiplies its own columns of x, or its own rows, by its own matrix.
  * Dense (tile_group NULL): y[m, g * y_group + n] = sum_k x[m, g * x_group + k] W_g[n, k] for all M rows
@@ -92,20 +113,26 @@ int msa_moe_plan(const int32_t* ids, int P, int E, int tile_rows, int32_t* perm,
                  int32_t* group_end, int32_t* tile_group, int32_t* tile_row, int32_t* n_tiles,
                  int max_tiles, void* stream);
 
-/* x[m] = table[token] * scale + sinusoid(pos), h = rmsnorm(x) * w (activation format).  table: bf16
- * [vocab, Dp]; inv_freq: double [(D + 1) / 2], the angle per position of column pair i. */
+/* e = table[token] * scale + sinusoid(pos), x = e + step, h = rmsnorm(x) * w (activation format).
+ * table: bf16 [vocab, Dp]; inv_freq: double [(D + 1) / 2], the angle per position of column pair i (NULL:
+ * no sinusoid); step: [Dp] or NULL; e: fp32 [M, Dp], written unless NULL. */
 int msa_embed_rmsnorm(int dtype, const int64_t* tokens, const int32_t* tok_pos, int M,
                       const void* table, int vocab, float scale, const double* inv_freq, int D, int Dp,
-                      float eps, float* x, const float* w, void* h, int h_mb, void* stream);
-/* The tail of a sublayer: b = sum of S slices part[S][M][Dp] (times gate[m]) + sum_k pair_w[m, k] *
- * pair_y[inverse[m, k]] ; x += rmsnorm(b) * w_post (w_post NULL: x += b) ; h = rmsnorm(x) * w_next
- * (w_next NULL: no h).  part or pair_y may be NULL. */
+                      float eps, const float* step, float* e, float* x, const float* w, void* h, int h_mb,
+                      void* stream);
+/* The tail of a sublayer: b = sum of S slices part[S][M][Dp] (times gate[m]) + bias + sum_k pair_w[m, k]
+ * * pair_y[inverse[m, k]] ; x += rmsnorm(b) * w_post (w_post NULL: x += b) ; with part2 (S2 slices) also
+ * x += rmsnorm(part2) * w_post2 ; x is written to probe ; x += add + step (what comes between two layers)
+ * ; h = rmsnorm(x) * w_next (w_next NULL: no h).  part or pair_y may be NULL, and bias [Dp], part2, probe
+ * [M, Dp], add [M, Dp] and step [Dp]. */
 typedef struct {
-  int dtype, M, D, Dp, S, top, h_mb;
+  int dtype, M, D, Dp, S, S2, top, h_mb;
   float eps;
   const float *part, *gate, *pair_w;
   const void* pair_y;
   const int32_t* inverse;
+  const float *bias, *part2, *w_post2, *add, *step;
+  float* probe;
   const float *w_post, *w_next;
   float* x;
   void* h;
@@ -132,23 +159,59 @@ int msa_rglru_scan(int dtype, float* gates, const float* gate_bias, const float*
                    float* state, float* carry, void* out, int64_t ld_out, int out_mb,
                    const msa_batch* b, void* stream);
 
-/* Gated delta rule.  qkv: activations after the convolution, [q: kv_heads x dp | k | v: heads x vp]
- * with stride ld; ba: fp32 [M, ldba], beta logits then decay logits per head; state fp32
- * [slot][head][vp][dp]; o: fp32 [M, heads * vp].  dp is 32, 64, 96, 128, 192 or 256, vp a multiple of
- * 16; dim is the unpadded key size. */
-int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
-                   const float* decay_rate, const float* dt_bias, int heads, int kv_heads, int dim,
-                   int dp, int vp, float* state, float* o, const msa_batch* b, void* stream);
-/* out = rmsnorm over vdim of every head's o, times w, times silu(gate) */
-int msa_delta_output(int dtype, const float* o, const void* gate, int64_t ld_gate, const float* w,
-                     int heads, int vdim, int vp, float eps, void* out, int64_t ld_out, int out_mb,
-                     int M, void* stream);
+/* Gated delta rule.  Per head: S <- g S ; u = beta (v - S^T k) ; S <- S + k u^T ; o = S^T q.  qkv:
+ * activations after the convolution, [q: kv_heads x dp | k | v: heads x vp] with stride ld.  ba: fp32
+ * [M, ldba], beta logits, then decay logits, per head.  With decay (fp32 [M, heads * dp], the decays
+ * themselves) every key channel decays by itself, ba holds beta logits only, and decay_rate and dt_bias are
+ * unused.  State fp32 [slot][head][vp][dp]; o: fp32 [M, heads * vp].  dp is 32, 64, 96, 128, 192 or 256,
+ * vp a multiple of 16; dim is the unpadded key size. */
+typedef struct {
+  int dtype, heads, kv_heads, dim, dp, vdim, vp, gate_act;
+  const void* qkv; int64_t ld;
+  const float* ba; int ldba;
+  const float *decay_rate, *dt_bias, *decay;
+  float* state;
+  float* o;               /* msa_delta_scan writes, msa_delta_output reads */
+  const void* gate; int64_t ld_gate;   /* heads * vp columns, activation format */
+  const float* w; float eps;           /* the output's norm over vdim, weight [vp] */
+  void* out; int64_t ld_out; int out_mb;
+} msa_delta_args;
+int msa_delta_scan(const msa_delta_args* a, const msa_batch* b, void* stream);
+/* out = rmsnorm over vdim of every head's o, times w, times silu(gate) or sigmoid(gate) (gate_act) */
+int msa_delta_output(const msa_delta_args* a, int M, void* stream);
 /* Both in one launch where every segment holds one token. */
-int msa_delta_step(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
-                   const float* decay_rate, const float* dt_bias, int heads, int kv_heads, int dim,
-                   int dp, int vdim, int vp, float* state, const void* gate, int64_t ld_gate,
-                   const float* w, float eps, void* out, int64_t ld_out, int out_mb,
-                   const msa_batch* b, void* stream);
+int msa_delta_step(const msa_delta_args* a, const msa_batch* b, void* stream);
+
+/* Attention of several query heads per key/value head over cached keys and values, causal, and within
+ * chunks of `chunk` positions (0: one chunk): position i sees j <= i of its own chunk.  q, k, v: columns of
+ * the step's rows, all with stride ld (q [M, heads * hd], k [M, kv_heads * hd], v [M, kv_heads * vd]).  A
+ * slot's cache holds `rows` positions, k_cache [slot][kv_heads][rows][hd] and v_cache [slot][kv_heads][rows]
+ * [vd], the position at its distance from the chunk's start: rows is at least min(capacity, chunk).  Keys
+ * of the step's own tokens are read from the step's rows, so what a segment appends may take the place
+ * of an older chunk.  gate: fp32 logits [M, ld_gate] per head or NULL: the output is multiplied by their
+ * sigmoid.  out: activation format, heads * vd columns.  Rotary: dimension i < rot_dims / 2 of a head is
+ * rotated with i + rot_dims / 2 by position * inv_freq[i] (double, device). */
+typedef struct {
+  int dtype, heads, kv_heads, hd, vd, chunk, rot_dims, rows;
+  float scale;
+  const double* inv_freq;
+  void *q, *k, *v; int64_t ld;
+  void *k_cache, *v_cache;
+  const float* gate; int ld_gate;
+  void* out; int64_t ldo; int out_mb;
+  float* partial;         /* splits > 1: [M][heads][splits][vd + 4] */
+  int splits;
+} msa_grouped_args;
+/* rotates q and k in place; where every segment holds one token, also appends keys and values */
+int msa_grouped_rotate(const msa_grouped_args* a, const msa_batch* b, void* stream);
+/* appends the keys and values of every segment's last chunk (nothing where msa_grouped_rotate did) */
+int msa_grouped_append(const msa_grouped_args* a, const msa_batch* b, void* stream);
+int msa_grouped_attention_splits(const msa_grouped_args* a, int M, int key_bound);
+/* The outputs of segments seg0 .. seg1 - 1: all of them of one token each (longest == 1), or of any size up
+ * to `longest`, after msa_grouped_rotate and before msa_grouped_append.  Head sizes: fp32, and bf16 beyond
+ * 256, up to 1024; bf16 64, 128, 192 or 256. */
+int msa_grouped_attention(const msa_grouped_args* a, const msa_batch* b, int seg0, int seg1, int longest,
+                          void* stream);
 
 /* Latents: part = fp32 sums [S][M][N] of the down-projections, columns [0, qp) the query latent,
  * [qp, qp + rp) the key/value latent (absent with latent NULL).  Both RMS-normed over their q_rank /
@@ -184,6 +247,15 @@ int msa_step_positions(const int32_t* lens, const int64_t* tokens, int64_t tok_s
 int msa_advance_active(int32_t* lens, const int32_t* step_pos, int B, void* stream);
 
 /* ---- the step function ----------------------------------------------------------------------- */
+/* the attention side of a parallel mixer */
+typedef struct {
+  int heads, kv_heads, hd, vd, chunk, rot_dims, ko;
+  float scale;
+  const double* inv_freq; /* device, [rot_dims / 2] */
+  const void* w_out;      /* [Dp, ko] */
+  const float* out_norm;  /* [Dp] */
+} msa_attention_layer;
+
 typedef struct {
   int kind; /* MSA_MIX_* */
   /* latent attention */
@@ -199,17 +271,27 @@ typedef struct {
   int kv_heads, dim, dp, vdim, vp, channels, blocks, taps;
   const float *conv_w, *conv_b, *in_bias, *y_bias, *gate_bias, *lam, *decay_rate, *dt_bias, *o_norm;
   const void* w_gates;  /* per block r, then per block i: [2 * blocks][channels / blocks]^2          */
+  /* parallel: grouped attention (att) beside a delta rule with channel decays, the sum of their normed
+   * outputs (out_norm: the delta side's).  w_in's columns, with in_bias per column: attention's q, k, v ;
+   * the delta rule's q, k, v ; lr columns of low-rank inputs ; fp32 from there on: a gate logit per
+   * attention head, a beta logit per delta head.  w_lr [heads * (vp + dp), lr]: the read-out gate's columns,
+   * then the decays' (lr_bias per column, lr_rate [heads * dp]). */
+  msa_attention_layer att;
+  int lr;
+  const void* w_lr;
+  const float *lr_bias, *lr_rate, *out_norm;
   /* all */
   const void* w_out;    /* [Dp, ko]                                                                 */
   int n_in, ko;
-  const float *norm1, *norm1b, *norm2, *norm2b;
+  const float *norm1, *norm1b, *norm2, *norm2b; /* norm1b, norm2b: after the sublayer, or NULL */
   /* feed-forward */
   int ff_kind, ff, experts, top, n_groups, keep, ff_expert, ff_shared; /* padded sizes */
   float router_scale, limit_expert, limit_shared;
-  const void* w_ff_in;  /* dense: (gate, up) row pairs [2 ff, Dp]; moe: shared expert's pairs, then
+  const void* w_ff_in;  /* dense: (gate, up) row pairs [2 ff, Dp]; relu2: [ff, Dp]; moe: shared expert's pairs, then
                            router rows and the shared gate's row as fp32 columns                     */
   int n_ff_in;
-  const void* w_ff_down; /* dense or shared expert (NULL: none) */
+  const float *ff_bias, *ff_down_bias; /* relu2: [ff], [Dp] */
+  const void* w_ff_down; /* dense, relu2 or shared expert (NULL: none) */
   const void *w_e_in, *w_e_down; /* per expert [2 ff_expert, Dp] pairs, [Dp, ff_expert] */
 } msa_hybrid_layer;
 
@@ -217,31 +299,40 @@ typedef struct {
   int dtype, layers, D, Dp, vocab, Vp;
   float eps, embed_scale;
   const void* embed;      /* bf16 [vocab, Dp] */
-  const double* inv_freq; /* device */
+  const double* inv_freq; /* device; NULL: no positions are added to the embedding */
   const float* final_norm;
   const void* head;       /* [Vp, Dp] */
+  /* The layers in the order they run (host arrays, copied; n_runs 0: once each).  A run whose run_pass is
+   * t >= 0 begins pass t of a loop: loop_step[t] is added to the residual stream in front of it, and, for
+   * t > 0, the embedding.  Every run has its own cache and state. */
+  int n_runs;
+  const int32_t *run_layer, *run_pass;
+  const float* loop_step; /* device, [passes][Dp] */
 } msa_hybrid_config;
 
 typedef struct msa_hybrid msa_hybrid;
 int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_layer* layers, msa_hybrid** out);
 void msa_hybrid_destroy(msa_hybrid* d);
 
-/* Per-layer cache pointers: latent [slots][capacity][rp] (attention layers that own one), conv
- * [slots][taps - 1][channels] and rec (rglru: [slots][channels], delta: [slots][heads][vp][dp]). */
+/* Cache pointers per run of a layer: latent [slots][capacity][rp] (attention layers that own one), conv
+ * [slots][taps - 1][channels] and rec (rglru: [slots][channels], delta: [slots][heads][vp][dp]), keys and
+ * values [slots][kv_heads][kv_rows][hd or vd]. */
 typedef struct {
   void *latent, *conv;
   float* rec;
+  void *keys, *values;
+  int kv_rows;
 } msa_hybrid_state;
 
 typedef struct {
   msa_batch batch;
   const int64_t* tokens;   /* [M] */
-  const msa_hybrid_state* state; /* host array, one per layer */
+  const msa_hybrid_state* state; /* host array, one per run */
   int capacity;            /* positions per slot */
   const int32_t* rows;     /* device: rows whose logits are wanted, or NULL = all */
   int n_rows;
   float* logits;           /* [n_rows or M][Vp]; NULL: none */
-  float* probe;            /* [layers][M][Dp]: the residual stream after every layer, or NULL */
+  float* probe;            /* [runs][M][Dp]: the residual stream after every run of a layer, or NULL */
   void* workspace;
   int64_t workspace_bytes;
 } msa_hybrid_step_args;

@@ -113,8 +113,11 @@ OTHER_SYMBOLS = ["msa_last_error", "msa_version", "msa_lm_head_select_workspace_
 HYBRID_LIB_PATH = os.path.join(_HERE, "csrc", "libmetaseq_hybrid.so")
 MSA_BF16, MSA_F32 = 0, 1
 MSA_GLU_NONE, MSA_GLU_GELU, MSA_GLU_CLAMPED = -1, 0, 1
-MSA_MIX_LATENT, MSA_MIX_RGLRU, MSA_MIX_DELTA = 0, 1, 2
-MSA_FF_NONE, MSA_FF_DENSE, MSA_FF_MOE = 0, 1, 2
+MSA_ACT_NONE, MSA_ACT_RELU2 = 0, 1
+MSA_GATE_SILU, MSA_GATE_SIGMOID = 0, 1
+MSA_MIX_LATENT, MSA_MIX_RGLRU, MSA_MIX_DELTA, MSA_MIX_PARALLEL = 0, 1, 2, 3
+MSA_FF_NONE, MSA_FF_DENSE, MSA_FF_MOE, MSA_FF_RELU2 = 0, 1, 2, 3
+MSA_OUT2_PACKED = 16
 _I32P = ctypes.POINTER(c_int32)
 
 
@@ -133,21 +136,42 @@ GroupLinearArgs = _struct(
     (c_int, "y_group y_mb y_f32 y_row0 N K groups glu"), (c_float, "limit"), (c_int64, "M"),
     (c_void_p, "perm tile_group tile_row n_tiles group_end"),
     (c_int, "rows_per_x max_tiles tile_rows"))
-TailArgs = _struct("TailArgs", "msa_tail_args", (c_int, "dtype M D Dp S top h_mb"),
-                   (c_float, "eps"), (c_void_p, "part gate pair_w pair_y inverse w_post w_next x h"))
+LinearArgs = _struct(
+    "LinearArgs", "msa_linear_args", (c_int, "dtype"), (c_void_p, "x W"), (c_int64, "M"),
+    (c_int, "N K n32 n2 act"), (c_uint, "flags"), (c_void_p, "bias decay_rate y y2 y32"))
+TailArgs = _struct("TailArgs", "msa_tail_args", (c_int, "dtype M D Dp S S2 top h_mb"),
+                   (c_float, "eps"), (c_void_p, "part gate pair_w pair_y inverse"),
+                   (c_void_p, "bias part2 w_post2 add step probe w_post w_next x h"))
+DeltaArgs = _struct(
+    "DeltaArgs", "msa_delta_args", (c_int, "dtype heads kv_heads dim dp vdim vp gate_act"),
+    (c_void_p, "qkv"), (c_int64, "ld"), (c_void_p, "ba"), (c_int, "ldba"),
+    (c_void_p, "decay_rate dt_bias decay state o gate"), (c_int64, "ld_gate"), (c_void_p, "w"),
+    (c_float, "eps"), (c_void_p, "out"), (c_int64, "ld_out"), (c_int, "out_mb"))
+GroupedArgs = _struct(
+    "GroupedArgs", "msa_grouped_args", (c_int, "dtype heads kv_heads hd vd chunk rot_dims rows"),
+    (c_float, "scale"), (c_void_p, "inv_freq q k v"), (c_int64, "ld"),
+    (c_void_p, "k_cache v_cache gate"), (c_int, "ld_gate"), (c_void_p, "out"), (c_int64, "ldo"),
+    (c_int, "out_mb"), (c_void_p, "partial"), (c_int, "splits"))
+AttentionLayer = _struct(
+    "AttentionLayer", "msa_attention_layer", (c_int, "heads kv_heads hd vd chunk rot_dims ko"),
+    (c_float, "scale"), (c_void_p, "inv_freq w_out out_norm"))
 HybridLayer = _struct(
     "HybridLayer", "msa_hybrid_layer", (c_int, "kind heads hd q_rank qp kv_rank rp kv_from"),
     (c_float, "scale"), (c_void_p, "w_in w_q w_kv w_absorb w_v wq_norm wkv_norm"),
     (c_int, "kv_heads dim dp vdim vp channels blocks taps"),
-    (c_void_p, "conv_w conv_b in_bias y_bias gate_bias lam decay_rate dt_bias o_norm w_gates w_out"),
+    (c_void_p, "conv_w conv_b in_bias y_bias gate_bias lam decay_rate dt_bias o_norm w_gates"),
+    (AttentionLayer, "att"), (c_int, "lr"), (c_void_p, "w_lr lr_bias lr_rate out_norm w_out"),
     (c_int, "n_in ko"), (c_void_p, "norm1 norm1b norm2 norm2b"),
     (c_int, "ff_kind ff experts top n_groups keep ff_expert ff_shared"),
     (c_float, "router_scale limit_expert limit_shared"), (c_void_p, "w_ff_in"),
-    (c_int, "n_ff_in"), (c_void_p, "w_ff_down w_e_in w_e_down"))
+    (c_int, "n_ff_in"), (c_void_p, "ff_bias ff_down_bias w_ff_down w_e_in w_e_down"))
 HybridConfigC = _struct("HybridConfigC", "msa_hybrid_config",
                         (c_int, "dtype layers D Dp vocab Vp"), (c_float, "eps embed_scale"),
-                        (c_void_p, "embed inv_freq final_norm head"))
-HybridState = _struct("HybridState", "msa_hybrid_state", (c_void_p, "latent conv rec"))
+                        (c_void_p, "embed inv_freq final_norm head"), (c_int, "n_runs"),
+                        (ctypes.POINTER(ctypes.c_int32), "run_layer run_pass"),
+                        (c_void_p, "loop_step"))
+HybridState = _struct("HybridState", "msa_hybrid_state", (c_void_p, "latent conv rec keys values"),
+                      (c_int, "kv_rows"))
 HybridStepArgs = _struct(
     "HybridStepArgs", "msa_hybrid_step_args", (Batch, "batch"), (c_void_p, "tokens"),
     (ctypes.POINTER(HybridState), "state"), (c_int, "capacity"), (c_void_p, "rows"),
@@ -157,13 +181,14 @@ _BP = ctypes.POINTER(Batch)
 HYBRID_SIGNATURES = {
     "msa_linear_bf16": [_P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_float, c_uint, _P],
     "msa_linear_f32": [_P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_float, _P],
+    "msa_linear": [ctypes.POINTER(LinearArgs), _P],
     "msa_linear_partial_bf16": [_P, _P, _P, c_int64, c_int, c_int, c_int, c_uint, _P],
     "msa_linear_bf16_splits": [c_int64, c_int, c_int, c_int],
     "msa_group_linear": [ctypes.POINTER(GroupLinearArgs), _P],
     "msa_moe_route": [_P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, _P, _P, _P, _P],
     "msa_moe_plan": [_P, c_int, c_int, c_int, _P, _P, _P, _P, _P, _P, c_int, _P],
     "msa_embed_rmsnorm": [c_int, _P, _P, c_int, _P, c_int, c_float, _P, c_int, c_int, c_float, _P,
-                          _P, _P, c_int, _P],
+                          _P, _P, _P, _P, c_int, _P],
     "msa_residual_rmsnorm_tail": [ctypes.POINTER(TailArgs), _P],
     "msa_short_conv": [c_int, _P, c_int64, c_int, c_int, _P, _P, _P, c_int, _P, c_int64, _P, _BP,
                        _P],
@@ -171,12 +196,13 @@ HYBRID_SIGNATURES = {
     "msa_rglru_chunks": [c_int],
     "msa_rglru_scan": [c_int, _P, _P, _P, _P, c_int64, _P, c_int64, _P, c_int, _P, _P, _P, c_int64,
                        c_int, _BP, _P],
-    "msa_delta_scan": [c_int, _P, c_int64, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int,
-                       _P, _P, _BP, _P],
-    "msa_delta_output": [c_int, _P, _P, c_int64, _P, c_int, c_int, c_int, c_float, _P, c_int64,
-                         c_int, c_int, _P],
-    "msa_delta_step": [c_int, _P, c_int64, _P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int,
-                       c_int, _P, _P, c_int64, _P, c_float, _P, c_int64, c_int, _BP, _P],
+    "msa_delta_scan": [ctypes.POINTER(DeltaArgs), _BP, _P],
+    "msa_delta_output": [ctypes.POINTER(DeltaArgs), c_int, _P],
+    "msa_delta_step": [ctypes.POINTER(DeltaArgs), _BP, _P],
+    "msa_grouped_rotate": [ctypes.POINTER(GroupedArgs), _BP, _P],
+    "msa_grouped_append": [ctypes.POINTER(GroupedArgs), _BP, _P],
+    "msa_grouped_attention_splits": [ctypes.POINTER(GroupedArgs), c_int, c_int],
+    "msa_grouped_attention": [ctypes.POINTER(GroupedArgs), _BP, c_int, c_int, c_int, _P],
     "msa_latent_norm": [c_int, _P, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_int, _P,
                         c_float, _P, c_int, _P, c_int, _BP, _P],
     "msa_latent_attention_splits": [c_int, c_int, c_int, c_int, c_int],

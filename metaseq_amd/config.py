@@ -141,7 +141,44 @@ class DeltaSpec:
 
 
 @dataclass
+class ChannelDeltaSpec(DeltaSpec):
+    """Gated delta rule with one decay per head and key channel; decays and the read-out's gate
+    come from low-rank projections, whose ranks the weights' shapes give."""
+    decay_rank: Optional[int] = None
+    gate_rank: Optional[int] = None
+
+
+@dataclass
+class GroupedAttentionSpec:
+    """Attention of ``heads`` query heads over ``kv_heads`` cached keys and values, rotary on the
+    first ``rot_dims`` dimensions, within chunks of ``chunk`` positions (None: no chunks), with a
+    gate per head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_base: float = 1.0
+    rot_dims: int = 0
+    chunk: Optional[int] = None
+
+
+@dataclass
+class ParallelSpec:
+    """Two mixers over the same input; the mean of their normed outputs."""
+    left: GroupedAttentionSpec
+    right: ChannelDeltaSpec
+
+
+@dataclass
 class DenseSpec:
+    """Gated feed-forward: gelu_tanh(gate) up."""
+    ff: int
+
+
+@dataclass
+class SquaredReluSpec:
+    """Feed-forward with biases whose activation is the square of relu."""
     ff: int
 
 
@@ -169,8 +206,16 @@ class MoESpec:
 
 @dataclass
 class HybridLayerSpec:
-    mixer: Union[LatentAttentionSpec, RGLRUSpec, DeltaSpec]
-    mlp: Union[DenseSpec, MoESpec, None] = None
+    mixer: Union[LatentAttentionSpec, RGLRUSpec, DeltaSpec, ParallelSpec]
+    mlp: Union[DenseSpec, SquaredReluSpec, MoESpec, None] = None
+
+
+@dataclass
+class LoopSpec:
+    """Layers ``start`` .. ``stop`` - 1 run ``times`` times in a row with the same weights."""
+    start: int
+    stop: int
+    times: int
 
 
 def _take(section, where, spec, rename=None, **extra):
@@ -194,8 +239,10 @@ def _take(section, where, spec, rename=None, **extra):
 
 @dataclass
 class HybridConfig:
-    """A decoder whose layers each choose a mixer and a feed-forward, with RMS norms before and
-    after every sublayer, fixed sinusoidal positions and an untied vocabulary projection."""
+    """A decoder whose layers each choose a mixer and a feed-forward, with RMS norms before every
+    sublayer.  ``post_norms``: norms after them too; ``sinusoidal``: fixed positions added to the
+    embedding; ``tied``: the vocabulary projection is the embedding table; ``loop``: a range of
+    layers that runs several times, each pass with a cache of its own."""
     width: int
     vocab_size: int
     layers: List[HybridLayerSpec]
@@ -204,10 +251,18 @@ class HybridConfig:
     max_target_positions: int = 1 << 17
     padding_idx: int = 1
     eos_idx: int = 2
+    post_norms: bool = True
+    sinusoidal: bool = True
+    tied: bool = False
+    loop: Optional[LoopSpec] = None
 
     def __post_init__(self):
         if not self.layers:
             raise ValueError("a hybrid decoder needs at least one layer")
+        k = self.loop
+        if k is not None and not (0 <= k.start < k.stop <= len(self.layers) and k.times >= 1):
+            raise ValueError("a loop of layers %d .. %d, %d times, in a model of %d layers"
+                             % (k.start, k.stop - 1, k.times, len(self.layers)))
         for i, layer in enumerate(self.layers):
             m = layer.mixer
             if isinstance(m, LatentAttentionSpec) and m.kv_from is not None:
@@ -219,8 +274,17 @@ class HybridConfig:
                 if src.kv_rank != m.kv_rank:
                     raise ValueError("layer %d and the layer it takes its latents from differ in "
                                      "kv_rank" % i)
-            if isinstance(m, DeltaSpec) and m.heads % m.kv_heads:
-                raise ValueError("layer %d: heads must be a multiple of kv_heads" % i)
+            for part in (m.left, m.right) if isinstance(m, ParallelSpec) else (m,):
+                if isinstance(part, (DeltaSpec, GroupedAttentionSpec)) \
+                        and part.heads % part.kv_heads:
+                    raise ValueError("layer %d: heads must be a multiple of kv_heads" % i)
+            if isinstance(m, ParallelSpec):
+                t = m.left
+                if t.rot_dims % 2 or not 0 <= t.rot_dims <= t.dim:
+                    raise ValueError("layer %d: rotary positions on %d of %d dimensions"
+                                     % (i, t.rot_dims, t.dim))
+                if t.chunk is not None and t.chunk < 1:
+                    raise ValueError("layer %d: chunks of %d positions" % (i, t.chunk))
             if isinstance(m, RGLRUSpec) and m.width % m.blocks:
                 raise ValueError("layer %d: width must be a multiple of blocks" % i)
             if isinstance(layer.mlp, MoESpec):
@@ -230,32 +294,91 @@ class HybridConfig:
                     raise ValueError("layer %d: %d experts in %d groups, %d kept, top %d"
                                      % (i, r.experts, r.groups, r.keep, r.top))
 
-    MIXERS = {"latent_attention": LatentAttentionSpec, "rglru": RGLRUSpec, "delta": DeltaSpec}
+    def runs(self):
+        """(layer, pass) in the order of execution; pass t >= 0 marks the run that begins pass t
+        of the loop, -1 every other run."""
+        k, n = self.loop, len(self.layers)
+        if k is None:
+            return [(i, -1) for i in range(n)]
+        return ([(i, -1) for i in range(k.start)]
+                + [(i, t if i == k.start else -1) for t in range(k.times)
+                   for i in range(k.start, k.stop)]
+                + [(i, -1) for i in range(k.stop, n)])
+
+    # what a config.json's "architecture" fixes: its layer types, its dense feed-forward, and the
+    # flags of the class
+    DESIGNS = {
+        "Sinulorn": dict(mixers=("latent_attention", "rglru", "delta"), dense=DenseSpec),
+        "Nomalorn": dict(mixers=("parallel",), dense=SquaredReluSpec, post_norms=False,
+                         sinusoidal=False, tied=True),
+    }
+    MIXERS = {"latent_attention": LatentAttentionSpec, "rglru": RGLRUSpec, "delta": DeltaSpec,
+              "parallel": ParallelSpec}
 
     @classmethod
     def from_json(cls, obj):
         """The configuration of a config.json (already parsed)."""
+        design = dict(cls.DESIGNS[obj.get("architecture", "Sinulorn")])
+        mixers, dense = design.pop("mixers"), design.pop("dense")
         layers = []
         for i, entry in enumerate(obj["layers"]):
             where = "layer %d" % i
             kind = entry["type"]
-            if kind not in cls.MIXERS:
+            if kind not in mixers:
                 raise NotImplementedError("config.json: %s: unknown mixer %r" % (where, kind))
-            mixer = _take(entry["mixer"], where + " mixer", cls.MIXERS[kind])
+            if kind == "parallel":
+                mixer = cls._parallel(dict(entry["mixer"]), where + " mixer")
+            else:
+                mixer = _take(entry["mixer"], where + " mixer", cls.MIXERS[kind])
             mlp = entry.get("mlp")
             if mlp is not None:
-                mlp = cls._mlp(dict(mlp), where + " mlp")
+                mlp = cls._mlp(dict(mlp), where + " mlp", dense)
             layers.append(HybridLayerSpec(mixer, mlp))
         special = {k: obj[k] for k in ("padding_idx", "eos_idx", "max_target_positions")
                    if k in obj}
+        if obj.get("loop"):
+            special["loop"] = _take(obj["loop"], "loop", LoopSpec)
         return cls(width=obj["width"], vocab_size=obj["vocab"], layers=layers,
-                   norm_eps=obj["norm"]["eps"], embed_scale=obj["embedding"]["scale"], **special)
+                   norm_eps=obj["norm"]["eps"],
+                   embed_scale=(obj.get("embedding") or {}).get("scale", 1.0), **special, **design)
 
     @staticmethod
-    def _mlp(mlp, where):
+    def _parallel(mixer, where):
+        left, right = dict(mixer.pop("left")), dict(mixer.pop("right"))
+        if mixer:
+            logger.warning("config.json: %s: unknown keys %s are ignored", where,
+                           ", ".join(sorted(mixer)))
+        rot, mask = left.pop("rot", None) or {}, left.pop("mask", None) or {}
+        for section, known, name in ((rot, {"base", "dims"}, "rot"), (mask, {"size"}, "mask")):
+            if set(section) - known:
+                logger.warning("config.json: %s left %s: unknown keys %s are ignored", where, name,
+                               ", ".join(sorted(set(section) - known)))
+        return ParallelSpec(
+            _take(left, where + " left", GroupedAttentionSpec, rot_base=rot.get("base", 1.0),
+                  rot_dims=rot.get("dims", 0), chunk=mask.get("size")),
+            _take(right, where + " right", ChannelDeltaSpec))
+
+    def with_shapes(self, shapes):
+        """The configuration completed by what only the weights' shapes (name -> shape) say."""
+        layers = []
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if isinstance(m, ParallelSpec):
+                ranks = {}
+                for field, name in (("decay_rank", "a1"), ("gate_rank", "g1")):
+                    shape = shapes.get("l%d.mix.right.%s" % (i, name))
+                    if getattr(m.right, field) is None and shape is not None:
+                        ranks[field] = int(shape[0])
+                if ranks:
+                    layer = replace(layer, mixer=replace(m, right=replace(m.right, **ranks)))
+            layers.append(layer)
+        return replace(self, layers=layers)
+
+    @staticmethod
+    def _mlp(mlp, where, dense=DenseSpec):
         kind = mlp.pop("kind")
         if kind == "dense":
-            return _take(mlp, where, DenseSpec)
+            return _take(mlp, where, dense)
         if kind != "moe":
             raise NotImplementedError("config.json: %s: unknown kind %r" % (where, kind))
         router = dict(mlp.pop("router"))
@@ -274,9 +397,11 @@ class HybridConfig:
         """name -> shape of every tensor of a checkpoint of this model."""
         D, out = self.width, {}
         out["embed"] = (self.vocab_size, D)
+        if self.loop is not None:
+            out["loop.step"] = (self.loop.times, D)
         for i, layer in enumerate(self.layers):
             pre, m = "l%d." % i, layer.mixer
-            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if layer.mlp else ()):
+            for n in self.norm_names(layer):
                 out[pre + n] = (D,)
 
             def put(section, **shapes):
@@ -294,6 +419,19 @@ class HybridConfig:
                 put("mix", y=(W, D), y_dot_b=(W,), x=(W, D), x_dot_b=(W,), conv=(W, m.conv),
                     conv_dot_b=(W,), ra=(nb, bs, bs), ra_dot_b=(nb, bs), ri=(nb, bs, bs),
                     ri_dot_b=(nb, bs), lam=(W,), o=(D, W))
+            elif isinstance(m, ParallelSpec):
+                a, d = m.left, m.right
+                put("mix.left", q=(a.heads * a.dim, D), q_dot_b=(a.heads * a.dim,),
+                    k=(a.kv_heads * a.dim, D), k_dot_b=(a.kv_heads * a.dim,),
+                    v=(a.kv_heads * a.vdim, D), v_dot_b=(a.kv_heads * a.vdim,), g=(a.heads, D),
+                    o=(D, a.heads * a.vdim))
+                qk, v = d.kv_heads * d.dim, d.heads * d.vdim
+                put("mix.right", q=(qk, D), q_dot_conv=(qk, d.conv), k=(qk, D),
+                    k_dot_conv=(qk, d.conv), v=(v, D), v_dot_conv=(v, d.conv), b=(d.heads, D),
+                    A_log=(d.heads,), norm=(d.vdim,), a1=(d.decay_rank, D),
+                    a2=(d.heads * d.dim, d.decay_rank), dt_bias=(d.heads * d.dim,),
+                    g1=(d.gate_rank, D), g2=(v, d.gate_rank), o=(D, v))
+                put("mix", left_dot_out=(D,), right_dot_out=(D,))
             else:
                 qk, v = m.kv_heads * m.dim, m.heads * m.vdim
                 put("mix", q=(qk, D), q_dot_conv=(qk, m.conv), k=(qk, D), k_dot_conv=(qk, m.conv),
@@ -302,6 +440,9 @@ class HybridConfig:
             if isinstance(layer.mlp, DenseSpec):
                 F = layer.mlp.ff
                 put("mlp", gate=(F, D), up=(F, D), down=(D, F))
+            elif isinstance(layer.mlp, SquaredReluSpec):
+                F = layer.mlp.ff
+                put("mlp", up=(F, D), up_dot_b=(F,), down=(D, F), down_dot_b=(D,))
             elif layer.mlp is not None:
                 r, e, s = layer.mlp.router, layer.mlp.expert, layer.mlp.shared
                 put("mlp", router=(r.experts, D))
@@ -310,5 +451,11 @@ class HybridConfig:
                 if s is not None:
                     put("mlp.shared", gate=(s.ff, D), up=(s.ff, D), down=(D, s.ff), sg=(1, D))
         out["final.norm"] = (D,)
-        out["head"] = (self.vocab_size, D)
+        if not self.tied:
+            out["head"] = (self.vocab_size, D)
         return out
+
+    def norm_names(self, layer):
+        """The norms over the width that a layer has."""
+        names = ("norm1", "norm1b") + (("norm2", "norm2b") if layer.mlp else ())
+        return names if self.post_norms else tuple(n for n in names if not n.endswith("b"))

@@ -1,8 +1,8 @@
 """Builds the shared libraries for gfx950 with hipcc (no GPU needed: hipcc cross-compiles).
 
     core    libmetaseq_amd.so     OPT decoder, selection and sampling (include/metaseq_amd.h)
-    hybrid  libmetaseq_hybrid.so  hybrid decoders: latent attention, recurrent layers, routed
-                                  feed-forwards (include/metaseq_hybrid.h)
+    hybrid  libmetaseq_hybrid.so  hybrid decoders: latent and grouped attention, recurrent layers,
+                                  routed feed-forwards (include/metaseq_hybrid.h)
 
 Usage: python -m metaseq_amd.csrc.build [core|hybrid ...]
 """
@@ -19,9 +19,9 @@ SOURCES = {
     "core": ["capi.hip", "layernorm.hip", "embed.hip", "gemm.hip", "attention.hip",
              "attention_prefill.hip", "sampling.hip", "probe.hip", "decoder_step.hip"],
     "hybrid": ["capi.hip", "gemm_bf16.hip", "group_linear.hip", "moe.hip", "rmsnorm.hip",
-               "recurrent.hip", "latent_attention.hip", "hybrid_step.hip"],
+               "recurrent.hip", "latent_attention.hip", "grouped_attention.hip", "hybrid_step.hip"],
 }
-HEADERS = ["common.h", "gemm_kernels.h", os.path.join("..", "..", "include", "metaseq_amd.h"),
+HEADERS = ["common.h", "gemm_kernels.h", "attention_tiles.h", os.path.join("..", "..", "include", "metaseq_amd.h"),
            os.path.join("..", "..", "include", "metaseq_hybrid.h")]
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-fPIC", "-std=c++17", "-Wall", "-Wno-unused-function",
@@ -33,7 +33,8 @@ FLAGS = [
 # registers (their softmax reads every score; by default hipcc parks them in the accumulator bank
 # and copies each one out)
 EXTRA_FLAGS = {"attention_prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
-               "latent_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
+               "latent_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+               "grouped_attention.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]}
 
 
 def _hipcc():

@@ -31,6 +31,7 @@ int msa_launch_prefill_attention(const void* q, const void* Kc, const void* Vc,
 
 // routed products over 256-row tiles, bf16 (gemm_bf16.hip)
 bool msa_launch_group_quad(const msa_group_linear_args& a, hipStream_t stream);
+int msa_launch_linear_post(const msa_linear_args& a, hipStream_t stream);
 
 #define MSA_REQUIRE(cond, code, ...) \
   do {                               \
@@ -102,6 +103,17 @@ __device__ __forceinline__ float glu_act(int kind, float g, float u, float limit
   return g * sigmoidf(1.702f * g) * (u + 1.f);
 }
 
+// log(1 + exp(v)) in the form that neither overflows nor loses the small values
+__device__ __forceinline__ float softplus(float v) {
+  return v > 20.f ? v : log1pf(expf(v));
+}
+__device__ __forceinline__ float relu2(float z) {
+  z = fmaxf(z, 0.f);
+  return z * z;
+}
+// decay of a recurrent state from its logit
+__device__ __forceinline__ float decay_of(float z, float rate) { return expf(-rate * softplus(z)); }
+
 // (max, sum of exp(z - max)) pairs merge associatively: one pass over a row suffices
 __device__ __forceinline__ void lse_merge(float& m, float& s, float om, float os) {
   if (om > m) {
@@ -166,6 +178,23 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     t += i < nw ? r : 0.f;
   }
   return t;
+}
+
+// two sums at once; `red` is >= 32 floats
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
+  a = wave_sum(a);
+  b = wave_sum(b);
+  __syncthreads();
+  if (lane == 0) red[wave] = a, red[16 + wave] = b;
+  __syncthreads();
+  a = b = 0.f;
+#pragma unroll
+  for (int i = 0; i < 16; ++i) {
+    const float r = red[i], q = red[16 + i];
+    a += i < nw ? r : 0.f;
+    b += i < nw ? q : 0.f;
+  }
 }
 
 __device__ __forceinline__ float block_max(float v, float* red) {

@@ -36,12 +36,13 @@
 
 namespace {
 
-enum { MODE_PLAIN = 0, MODE_QKV = 1, MODE_SELECT = 2, MODE_BF = 3, MODE_BF_GLU = 4 };
+enum { MODE_PLAIN = 0, MODE_QKV = 1, MODE_SELECT = 2, MODE_BF = 3, MODE_BF_GLU = 4, MODE_BF_POST = 5 };
 // The bf16 modes: operands are bf16 bit patterns (the kernels only move them; what differs is the
 // MFMA instruction and the epilogue).  Columns below Epilogue::n32 are stored as bf16, the columns
-// from there on as fp32; MODE_BF_GLU stores act(gate, up) of the (gate, up) column pairs below n32.
+// from there on as fp32; MODE_BF_GLU stores act(gate, up) of the (gate, up) column pairs below n32;
+// MODE_BF_POST is MODE_BF with a bias, an activation and a second output (post4).
 template <int MODE>
-constexpr bool is_bf = MODE == MODE_BF || MODE == MODE_BF_GLU;
+constexpr bool is_bf = MODE == MODE_BF || MODE == MODE_BF_GLU || MODE == MODE_BF_POST;
 
 struct Epilogue {
   const half_t* bias;
@@ -72,7 +73,27 @@ struct Epilogue {
   int n32, ldy;
   int glu;      // MSA_GLU_*
   float limit;  // of MSA_GLU_CLAMPED
+  // MODE_BF_POST
+  const float* bias32;      // [N] or null
+  const float* decay_rate;  // [N - n32] or null: the fp32 columns leave as exp(-rate softplus(z))
+  bf16_t* y2;               // bf16 columns from n2 on: row-major with stride ld2, or packed (out2_mb)
+  int act, n2, ld2, out2_mb;
 };
+
+// what MODE_BF_POST does to the sums of columns n .. n + 3
+__device__ __forceinline__ float4_t post4(const Epilogue& e, int n, float4_t v) {
+  if (e.bias32) v += *reinterpret_cast<const float4_t*>(e.bias32 + n);
+  if (n < e.n32) {
+    if (e.act == MSA_ACT_RELU2) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = relu2(v[i]);
+    }
+  } else if (e.decay_rate) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = decay_of(v[i], e.decay_rate[n - e.n32 + i]);
+  }
+  return v;
+}
 
 // operand fragments of any 16-bit format travel as half8_t
 template <int MODE>
@@ -155,10 +176,17 @@ __device__ __forceinline__ void select_merge(SelectState& a, float om, float os,
 template <int MODE>
 __device__ __forceinline__ void epilogue4(const Epilogue& e, int64_t m, int n, float4_t acc) {
   if constexpr (is_bf<MODE>) {
+    if constexpr (MODE == MODE_BF_POST) acc = post4(e, n, acc);
     if (n >= e.n32) {
       *reinterpret_cast<float4_t*>(e.y32 + m * (e.N - e.n32) + (n - e.n32)) = acc;
-    } else if constexpr (MODE == MODE_BF) {
+    } else if constexpr (MODE != MODE_BF_GLU) {
       const bf16x4_t o = {(bf16_t)acc[0], (bf16_t)acc[1], (bf16_t)acc[2], (bf16_t)acc[3]};
+      if (MODE == MODE_BF_POST && n >= e.n2) {
+        const int c = n - e.n2;
+        *reinterpret_cast<bf16x4_t*>(e.y2 + (e.out2_mb > 0 ? packed_act_offset((int)m, c, e.out2_mb)
+                                                           : m * e.ld2 + c)) = o;
+        return;
+      }
       *reinterpret_cast<bf16x4_t*>(e.yb + (e.out_mb > 0 ? packed_act_offset((int)m, n, e.out_mb)
                                                         : m * e.ldy + n)) = o;
     } else {
@@ -1402,6 +1430,8 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
 #pragma unroll
       for (int j = 0; j < WF; ++j) {
         const int n = nw + 16 * j + 4 * lg;
+        if constexpr (MODE == MODE_BF_POST)
+          if (n < N) acc[i][j] = post4(epi, n, acc[i][j]);
         if (nw + 16 * j >= epi.n32) {  // wave-uniform: n32 is a multiple of 16
           if (mf >= m_own && mf < M && n < N)
             *reinterpret_cast<float4_t*>(epi.y32 + mf * (N - epi.n32) + (n - epi.n32)) = acc[i][j];
@@ -1423,8 +1453,10 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
         const half8_t v = *reinterpret_cast<const half8_t*>(buf + row * BRB +
                                                             ((bc ^ (row & (BCH - 1))) * 16));
         const int64_t m = m0 + wm * 128 + i * 16 + row;
-        if (bn_ok && m >= m_own && m < M)
-          *reinterpret_cast<half8_t*>(epi.yb + m * epi.ldy + bn) = v;
+        bf16_t* y = epi.yb + m * epi.ldy + bn;
+        if constexpr (MODE == MODE_BF_POST)
+          if (bn >= epi.n2) y = epi.y2 + m * epi.ld2 + (bn - epi.n2);
+        if (bn_ok && m >= m_own && m < M) *reinterpret_cast<half8_t*>(y) = v;
       }
     }
     return;

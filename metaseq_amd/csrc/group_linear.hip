@@ -185,7 +185,15 @@ void launch_bf16(const msa_group_linear_args& a, int row_tiles, hipStream_t s) {
 // ---- fp32 -----------------------------------------------------------------------------------
 // 64 rows x 64 columns per workgroup, 16-wide K stages through LDS, 4 x 4 outputs per thread.
 // n32 splits the columns between y and y32 (linear layers); glu pairs lie within a thread.
-__global__ __launch_bounds__(256) void linear_f32_kernel(msa_group_linear_args a, float* y32, int n32) {
+// `post` (linear layers only): bias, activation, second output and decays as in MODE_BF_POST.
+struct PostF32 {
+  const float *bias, *decay_rate;
+  float* y2;
+  int act, n2, used;
+};
+
+__global__ __launch_bounds__(256) void linear_f32_kernel(msa_group_linear_args a, float* y32, int n32,
+                                                         PostF32 post) {
   __shared__ float lx[16][64 + 4], lw[16][64 + 4];
   Rows rw;
   if (!find_rows(a, blockIdx.y, blockIdx.z, rw)) return;
@@ -223,7 +231,20 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(msa_group_linear_args a
   for (int i = 0; i < 4; ++i) {
     const int64_t row = rw.first + tr * 4 + i;
     if (row >= rw.end) break;
-    const float4_t v = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+    float4_t v = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+    if (post.used) {
+      if (post.bias) v += *reinterpret_cast<const float4_t*>(post.bias + n);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (n < n32)
+          v[j] = post.act == MSA_ACT_RELU2 ? relu2(v[j]) : v[j];
+        else if (post.decay_rate)
+          v[j] = decay_of(v[j], post.decay_rate[n - n32 + j]);
+      if (n < n32 && n >= post.n2) {
+        *reinterpret_cast<float4_t*>(post.y2 + row * (n32 - post.n2) + (n - post.n2)) = v;
+        continue;
+      }
+    }
     if (n >= n32)
       *reinterpret_cast<float4_t*>(y32 + row * (a.N - n32) + (n - n32)) = v;
     else if (a.glu == MSA_GLU_NONE)
@@ -269,7 +290,7 @@ extern "C" int msa_group_linear(const msa_group_linear_args* args, void* stream)
   } else if (a.dtype == MSA_F32) {
     hipLaunchKernelGGL(linear_f32_kernel, dim3((a.N + 63) / 64, (unsigned)row_tiles,
                                                routed ? 1 : a.groups),
-                       dim3(256), 0, s, a, (float*)nullptr, a.N);
+                       dim3(256), 0, s, a, (float*)nullptr, a.N, PostF32{});
   } else if (rows <= 16) {
     launch_bf16<1, 2, 4, 4>(a, (int)row_tiles, s);
   } else if (rows <= 32) {
@@ -308,7 +329,45 @@ extern "C" int msa_linear_f32(const float* x, const float* W, float* y, float* y
   a.M = M;
   a.tile_rows = 64;
   hipLaunchKernelGGL(linear_f32_kernel, dim3((N + 63) / 64, (unsigned)((M + 63) / 64), 1), dim3(256),
-                     0, (hipStream_t)stream, a, y32, n32);
+                     0, (hipStream_t)stream, a, y32, n32, PostF32{});
+  MSA_CHECK_LAUNCH(name);
+  return MSA_OK;
+}
+
+extern "C" int msa_linear(const msa_linear_args* args, void* stream) {
+  const char* name = "msa_linear";
+  MSA_REQUIRE(args && args->x && args->W, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  const msa_linear_args& p = *args;
+  MSA_REQUIRE(p.dtype == MSA_BF16 || p.dtype == MSA_F32, MSA_ERR_INVALID_ARG, "%s: dtype", name);
+  MSA_REQUIRE(p.M >= 0 && p.N > 0 && p.N % 16 == 0 && p.K > 0 && p.K % 64 == 0 && p.n32 >= 0 &&
+                  p.n32 <= p.N && p.n32 % 16 == 0 && (p.M + 63) / 64 <= 65535 &&
+                  (!p.y2 || (p.n2 >= 0 && p.n2 <= p.n32 && p.n2 % 16 == 0)),
+              MSA_ERR_INVALID_ARG, "%s: M=%lld N=%d K=%d n32=%d n2=%d", name, (long long)p.M, p.N, p.K,
+              p.n32, p.n2);
+  const int n2 = p.y2 ? p.n2 : p.n32;
+  MSA_REQUIRE((p.y || n2 == 0) && (p.y32 || p.n32 == p.N), MSA_ERR_INVALID_ARG, "%s: null output", name);
+  MSA_REQUIRE(p.act == MSA_ACT_NONE || p.act == MSA_ACT_RELU2, MSA_ERR_INVALID_ARG, "%s: act=%d", name,
+              p.act);
+  if (p.M == 0) return MSA_OK;
+  if (p.dtype == MSA_BF16) return msa_launch_linear_post(p, (hipStream_t)stream);
+  MSA_REQUIRE(p.flags == 0, MSA_ERR_INVALID_ARG, "%s: fp32 activations are row-major", name);
+  msa_group_linear_args a{};
+  a.dtype = MSA_F32;
+  a.x = p.x;
+  a.ldx = p.K;
+  a.W = p.W;
+  a.y = p.y;
+  a.ldy = n2;
+  a.y_f32 = 1;
+  a.N = p.N;
+  a.K = p.K;
+  a.groups = 1;
+  a.glu = MSA_GLU_NONE;
+  a.M = p.M;
+  a.tile_rows = 64;
+  const PostF32 post{p.bias, p.decay_rate, (float*)p.y2, p.act, n2, 1};
+  hipLaunchKernelGGL(linear_f32_kernel, dim3((p.N + 63) / 64, (unsigned)((p.M + 63) / 64), 1), dim3(256),
+                     0, (hipStream_t)stream, a, p.y32, p.n32, post);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }

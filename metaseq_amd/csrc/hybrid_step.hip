@@ -13,9 +13,22 @@
 
 #include "common.h"
 
+namespace {
+
+// one run of a layer (a layer of a loop runs several times)
+struct LayerRun {
+  int layer;
+  int pass;   // >= 0: this run begins that pass of a loop
+  int owner;  // run whose latent it attends to (latent attention)
+};
+
+}  // namespace
+
 struct msa_hybrid {
   msa_hybrid_config cfg;
   msa_hybrid_layer* layers;
+  LayerRun* runs;
+  bool adds_embedding;  // some pass of a loop begins with the embedding
 };
 
 namespace {
@@ -81,12 +94,43 @@ struct Run {
     return msa_zero_columns(d->cfg.dtype, y.p, M, y.ld, mb, used, y.ld, stream);
   }
 
-  int latent(int li, const Act& h, Act& out);
+  // y, y2 (activation format; y row-major), y32 = a linear layer with bias, activation, decays
+  int linear_post(const Act& x, const void* W, int N, int n32, const float* bias, int act,
+                  const float* rate, void* y, bool y_act, const Act* y2, float* y32) {
+    if (dry) return MSA_OK;
+    msa_linear_args l{};
+    l.dtype = d->cfg.dtype;
+    l.x = x.p;
+    l.W = W;
+    l.M = M;
+    l.N = N;
+    l.K = x.ld;
+    l.n32 = n32;
+    l.bias = bias;
+    l.act = act;
+    l.decay_rate = rate;
+    l.y = y;
+    l.y32 = y32;
+    l.flags = in_flags() | (y_act && mb > 0 ? MSA_OUT_PACKED : 0u);
+    if (y2) {
+      l.y2 = y2->p;
+      l.n2 = n32 - y2->ld;
+      if (mb > 0) l.flags |= MSA_OUT2_PACKED;
+    }
+    return msa_linear(&l, stream);
+  }
+
+  int latent(int ri, const Act& h, Act& out);
   int latent_rows(const msa_hybrid_layer& l, void* cache, void* q, Act& out, int r0, int r1);
   int latent_segment(const msa_hybrid_layer& l, void* cache, void* q, Act& out, int seg);
-  int rglru(int li, const Act& h, Act& out);
-  int delta(int li, const Act& h, Act& out);
-  int feed_forward(int li, Act& h, float* x, const float* next);
+  int rglru(int ri, const Act& h, Act& out);
+  int delta(int ri, const Act& h, Act& out);
+  int delta_core(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in, int64_t ld,
+                 msa_delta_args& t, Act& out);
+  int grouped(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in, int64_t ld,
+              const float* gate, int ld_gate, Act& out);
+  int parallel(int ri, const Act& h, Act& left, Act& right);
+  int feed_forward(const msa_hybrid_layer& l, msa_tail_args& t);
   int tail(const msa_tail_args& t) { return dry ? MSA_OK : msa_residual_rmsnorm_tail(&t, stream); }
   int go();
 };
@@ -151,11 +195,11 @@ int Run::latent_segment(const msa_hybrid_layer& l, void* cache, void* q, Act& ou
   return MSA_OK;
 }
 
-int Run::latent(int li, const Act& h, Act& out) {
-  const msa_hybrid_layer& l = d->layers[li];
+int Run::latent(int ri, const Act& h, Act& out) {
+  const msa_hybrid_layer& l = d->layers[d->runs[ri].layer];
   const msa_batch& b = a->batch;
   const bool owner = l.kv_from < 0;
-  void* cache = dry ? nullptr : a->state[owner ? li : l.kv_from].latent;
+  void* cache = dry ? nullptr : a->state[d->runs[ri].owner].latent;
   int S, rc;
   float* part = partial(h, l.w_in, l.n_in, S, rc);
   HY(rc);
@@ -188,8 +232,8 @@ int Run::latent(int li, const Act& h, Act& out) {
   return zero_tail(out, nq);
 }
 
-int Run::rglru(int li, const Act& h, Act& out) {
-  const msa_hybrid_layer& l = d->layers[li];
+int Run::rglru(int ri, const Act& h, Act& out) {
+  const msa_hybrid_layer& l = d->layers[d->runs[ri].layer];
   const msa_batch& b = a->batch;
   const int C = l.channels, bs = C / l.blocks, chunks = msa_rglru_chunks(b.max_count);
   char* yx = (char*)alloc((int64_t)M * l.n_in * es);  // y, then the convolution's input
@@ -198,7 +242,7 @@ int Run::rglru(int li, const Act& h, Act& out) {
   float* gates = (float*)alloc((int64_t)M * 2 * C * 4);
   float* carry = (float*)alloc((int64_t)b.nseg * chunks * 2 * C * 4);
   if (!dry) {
-    const msa_hybrid_state& st = a->state[li];
+    const msa_hybrid_state& st = a->state[ri];
     char* raw = yx + (int64_t)C * es;
     HY(msa_short_conv(d->cfg.dtype, raw, l.n_in, C, l.taps, l.in_bias, l.conv_w, l.conv_b, 0, u, C,
                       st.conv, &b, stream));
@@ -225,56 +269,155 @@ int Run::rglru(int li, const Act& h, Act& out) {
   return zero_tail(out, C);
 }
 
-int Run::delta(int li, const Act& h, Act& out) {
-  const msa_hybrid_layer& l = d->layers[li];
+// The delta rule behind its projections: `in` holds q, k, v (row-major, stride ld); t comes with the
+// gate, the beta logits and the decays.
+int Run::delta_core(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in, int64_t ld,
+                    msa_delta_args& t, Act& out) {
   const msa_batch& b = a->batch;
-  const int C = 2 * l.kv_heads * l.dp + l.heads * l.vp, n32 = C + l.heads * l.vp;
-  char* in = (char*)alloc((int64_t)M * n32 * es);  // q, k, v, gate
-  float* ba = (float*)alloc((int64_t)M * (l.n_in - n32) * 4);
-  HY(linear(h, l.w_in, in, false, ba, l.n_in, n32, MSA_GLU_NONE, 0.f));
+  const int C = 2 * l.kv_heads * l.dp + l.heads * l.vp;
   void* qkv = alloc((int64_t)M * C * es);
   const bool step = b.max_count == 1;
-  float* o = step ? nullptr : (float*)alloc((int64_t)M * l.heads * l.vp * 4);
+  t.o = step ? nullptr : (float*)alloc((int64_t)M * l.heads * l.vp * 4);
   if (!dry) {
-    const msa_hybrid_state& st = a->state[li];
-    HY(msa_short_conv(d->cfg.dtype, in, n32, C, l.taps, nullptr, l.conv_w, nullptr, 1, qkv, C, st.conv,
-                      &b, stream));
-    HY(msa_conv_state(d->cfg.dtype, in, n32, C, l.taps, st.conv, &b, stream));
-    const char* gate = in + (int64_t)C * es;
+    HY(msa_short_conv(d->cfg.dtype, in, ld, C, l.taps, nullptr, l.conv_w, nullptr, 1, qkv, C, st.conv, &b,
+                      stream));
+    HY(msa_conv_state(d->cfg.dtype, in, ld, C, l.taps, st.conv, &b, stream));
+    t.dtype = d->cfg.dtype;
+    t.heads = l.heads;
+    t.kv_heads = l.kv_heads;
+    t.dim = l.dim;
+    t.dp = l.dp;
+    t.vdim = l.vdim;
+    t.vp = l.vp;
+    t.qkv = qkv;
+    t.ld = C;
+    t.state = st.rec;
+    t.w = l.o_norm;
+    t.eps = d->cfg.eps;
+    t.out = out.p;
+    t.ld_out = out.ld;
+    t.out_mb = mb;
     if (step) {
-      HY(msa_delta_step(d->cfg.dtype, qkv, C, ba, l.n_in - n32, l.decay_rate, l.dt_bias, l.heads,
-                        l.kv_heads, l.dim, l.dp, l.vdim, l.vp, st.rec, gate, n32, l.o_norm, d->cfg.eps,
-                        out.p, out.ld, mb, &b, stream));
-      return zero_tail(out, l.heads * l.vp);
+      HY(msa_delta_step(&t, &b, stream));
+    } else {
+      HY(msa_delta_scan(&t, &b, stream));
+      HY(msa_delta_output(&t, M, stream));
     }
-    HY(msa_delta_scan(d->cfg.dtype, qkv, C, ba, l.n_in - n32, l.decay_rate, l.dt_bias, l.heads,
-                      l.kv_heads, l.dim, l.dp, l.vp, st.rec, o, &b, stream));
-    HY(msa_delta_output(d->cfg.dtype, o, gate, n32, l.o_norm, l.heads, l.vdim, l.vp,
-                        d->cfg.eps, out.p, out.ld, mb, M, stream));
   }
   return zero_tail(out, l.heads * l.vp);
 }
 
-int Run::feed_forward(int li, Act& h, float* x, const float* next) {
-  const msa_hybrid_layer& l = d->layers[li];
+int Run::delta(int ri, const Act& h, Act& out) {
+  const msa_hybrid_layer& l = d->layers[d->runs[ri].layer];
+  const int C = 2 * l.kv_heads * l.dp + l.heads * l.vp, n32 = C + l.heads * l.vp;
+  char* in = (char*)alloc((int64_t)M * n32 * es);  // q, k, v, gate
+  float* ba = (float*)alloc((int64_t)M * (l.n_in - n32) * 4);
+  HY(linear(h, l.w_in, in, false, ba, l.n_in, n32, MSA_GLU_NONE, 0.f));
+  msa_delta_args t{};
+  t.ba = ba;
+  t.ldba = l.n_in - n32;
+  t.decay_rate = l.decay_rate;
+  t.dt_bias = l.dt_bias;
+  t.gate_act = MSA_GATE_SILU;
+  t.gate = in + (int64_t)C * es;
+  t.ld_gate = n32;
+  return delta_core(l, dry ? msa_hybrid_state{} : a->state[ri], in, n32, t, out);
+}
+
+// Grouped attention behind its projections: `in` holds q, k, v.  Runs of segments of one token each and of
+// longer segments have kernels of their own.
+int Run::grouped(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in, int64_t ld,
+                 const float* gate, int ld_gate, Act& out) {
+  const msa_attention_layer& t = l.att;
+  const msa_batch& b = a->batch;
+  msa_grouped_args g{};
+  g.dtype = d->cfg.dtype;
+  g.heads = t.heads;
+  g.kv_heads = t.kv_heads;
+  g.hd = t.hd;
+  g.vd = t.vd;
+  g.chunk = t.chunk;
+  g.rot_dims = t.rot_dims;
+  g.rows = st.kv_rows;
+  g.scale = t.scale;
+  g.inv_freq = t.inv_freq;
+  g.q = in;
+  g.k = in + (int64_t)t.heads * t.hd * es;
+  g.v = (char*)g.k + (int64_t)t.kv_heads * t.hd * es;
+  g.ld = ld;
+  g.k_cache = st.keys;
+  g.v_cache = st.values;
+  g.gate = gate;
+  g.ld_gate = ld_gate;
+  g.out = out.p;
+  g.ldo = out.ld;
+  g.out_mb = mb;
+  if (!dry) HY(msa_grouped_rotate(&g, &b, stream));
+  for (int s = 0; s < b.nseg;) {
+    auto count = [&](int i) { return b.max_count == 1 ? 1 : b.host_start[i + 1] - b.host_start[i]; };
+    const bool single = count(s) == 1;
+    int e = b.max_count == 1 ? b.nseg : s + 1, longest = count(s);
+    while (e < b.nseg && (count(e) == 1) == single) {
+      longest = count(e) > longest ? count(e) : longest;
+      ++e;
+    }
+    const int64_t save = off;
+    g.splits = single ? msa_grouped_attention_splits(&g, e - s, b.key_bound) : 1;
+    g.partial = g.splits > 1 ? (float*)alloc((int64_t)(e - s) * t.heads * g.splits * (t.vd + 4) * 4)
+                             : nullptr;
+    if (!dry) HY(msa_grouped_attention(&g, &b, s, e, longest, stream));
+    off = save;
+    s = e;
+  }
+  if (!dry) HY(msa_grouped_append(&g, &b, stream));
+  return zero_tail(out, t.heads * t.vd);
+}
+
+int Run::parallel(int ri, const Act& h, Act& left, Act& right) {
+  const msa_hybrid_layer& l = d->layers[d->runs[ri].layer];
+  const msa_attention_layer& t = l.att;
+  const int n_att = (t.heads + t.kv_heads) * t.hd + t.kv_heads * t.vd;
+  const int C = 2 * l.kv_heads * l.dp + l.heads * l.vp, n2 = n_att + C, n32 = n2 + l.lr;
+  const int n_gate = l.heads * l.vp, n_decay = l.heads * l.dp;
+  char* in = (char*)alloc((int64_t)M * n2 * es);
+  Act low = act(l.lr);
+  float* z = (float*)alloc((int64_t)M * (l.n_in - n32) * 4);
+  HY(linear_post(h, l.w_in, l.n_in, n32, l.in_bias, MSA_ACT_NONE, nullptr, in, false, &low, z));
+  char* gate = (char*)alloc((int64_t)M * n_gate * es);
+  float* decay = (float*)alloc((int64_t)M * n_decay * 4);
+  HY(linear_post(low, l.w_lr, n_gate + n_decay, n_gate, l.lr_bias, MSA_ACT_NONE, l.lr_rate, gate, false,
+                 nullptr, decay));
+  const msa_hybrid_state st = dry ? msa_hybrid_state{} : a->state[ri];
+  HY(grouped(l, st, in, n2, z, l.n_in - n32, left));
+  msa_delta_args g{};
+  g.ba = z + t.heads;
+  g.ldba = l.n_in - n32;
+  g.decay = decay;
+  g.gate_act = MSA_GATE_SIGMOID;
+  g.gate = gate;
+  g.ld_gate = n_gate;
+  return delta_core(l, st, in + (int64_t)n_att * es, n2, g, right);
+}
+
+// t arrives with everything that does not depend on the feed-forward
+int Run::feed_forward(const msa_hybrid_layer& l, msa_tail_args& t) {
   const msa_hybrid_config& c = d->cfg;
-  msa_tail_args t{};
-  t.dtype = c.dtype;
-  t.M = M;
-  t.D = c.D;
-  t.Dp = c.Dp;
-  t.eps = c.eps;
-  t.x = x;
-  t.h = h.p;
-  t.h_mb = mb;
-  t.w_post = l.norm2b;
-  t.w_next = next;
+  const Act h{t.h, c.Dp};
   int rc;
   if (l.ff_kind == MSA_FF_DENSE) {
     Act u = act(l.ff);
     HY(linear(h, l.w_ff_in, u.p, true, nullptr, l.n_ff_in, l.n_ff_in, MSA_GLU_GELU, 0.f));
     t.part = partial(u, l.w_ff_down, c.Dp, t.S, rc);
     HY(rc);
+    return tail(t);
+  }
+  if (l.ff_kind == MSA_FF_RELU2) {
+    Act u = act(l.ff);
+    HY(linear_post(h, l.w_ff_in, l.n_ff_in, l.n_ff_in, l.ff_bias, MSA_ACT_RELU2, nullptr, u.p, true,
+                   nullptr, nullptr));
+    t.part = partial(u, l.w_ff_down, c.Dp, t.S, rc);
+    HY(rc);
+    t.bias = l.ff_down_bias;
     return tail(t);
   }
   const int n32 = 2 * l.ff_shared, ldz = l.n_ff_in - n32, E = l.experts, P = M * l.top;
@@ -353,40 +496,61 @@ int Run::go() {
   const msa_hybrid_config& c = d->cfg;
   const msa_batch& b = a->batch;
   float* x = (float*)alloc((int64_t)M * c.Dp * 4);
+  float* e = d->adds_embedding ? (float*)alloc((int64_t)M * c.Dp * 4) : nullptr;
   Act h = act(c.Dp);
+  auto step = [&](int pass) { return pass >= 0 ? c.loop_step + (int64_t)pass * c.Dp : nullptr; };
   if (!dry)
     HY(msa_embed_rmsnorm(c.dtype, a->tokens, b.tok_pos, M, c.embed, c.vocab, c.embed_scale, c.inv_freq,
-                         c.D, c.Dp, c.eps, x, d->layers[0].norm1, h.p, mb, stream));
+                         c.D, c.Dp, c.eps, step(d->runs[0].pass), e, x,
+                         d->layers[d->runs[0].layer].norm1, h.p, mb, stream));
   const int64_t layer_base = off;
-  for (int i = 0; i < c.layers; ++i) {
-    const msa_hybrid_layer& l = d->layers[i];
-    const float* after = i + 1 < c.layers ? d->layers[i + 1].norm1 : c.final_norm;
-    const bool ff = l.ff_kind != MSA_FF_NONE;
+  for (int i = 0; i < c.n_runs; ++i) {
+    const msa_hybrid_layer& l = d->layers[d->runs[i].layer];
+    const bool last = i + 1 == c.n_runs, ff = l.ff_kind != MSA_FF_NONE;
+    // what ends the run: its output, what the loop adds, the next run's norm
+    msa_tail_args end{};
+    end.w_next = last ? c.final_norm : d->layers[d->runs[i + 1].layer].norm1;
+    end.probe = a->probe ? a->probe + (int64_t)i * M * c.Dp : nullptr;
+    const int pass = last ? -1 : d->runs[i + 1].pass;
+    end.step = step(pass);
+    end.add = pass > 0 ? e : nullptr;
+    msa_tail_args t = ff ? msa_tail_args{} : end;
+    if (ff) t.w_next = l.norm2;
+    for (msa_tail_args* k : {&t, &end}) {
+      k->dtype = c.dtype;
+      k->M = M;
+      k->D = c.D;
+      k->Dp = c.Dp;
+      k->eps = c.eps;
+      k->x = x;
+      k->h = h.p;
+      k->h_mb = mb;
+    }
     off = layer_base;
-    Act o = act(l.ko);
-    HY(l.kind == MSA_MIX_LATENT ? latent(i, h, o) : l.kind == MSA_MIX_RGLRU ? rglru(i, h, o)
-                                                                            : delta(i, h, o));
-    msa_tail_args t{};
-    t.dtype = c.dtype;
-    t.M = M;
-    t.D = c.D;
-    t.Dp = c.Dp;
-    t.eps = c.eps;
-    t.x = x;
-    t.h = h.p;
-    t.h_mb = mb;
+    Act o = act(l.ko), o2{};
     t.w_post = l.norm1b;
-    t.w_next = ff ? l.norm2 : after;
+    if (l.kind == MSA_MIX_PARALLEL) {
+      o2 = act(l.att.ko);
+      HY(parallel(i, h, o2, o));
+      t.w_post = l.out_norm;
+      t.w_post2 = l.att.out_norm;
+    } else {
+      HY(l.kind == MSA_MIX_LATENT ? latent(i, h, o) : l.kind == MSA_MIX_RGLRU ? rglru(i, h, o)
+                                                                              : delta(i, h, o));
+    }
     int rc;
     t.part = partial(o, l.w_out, c.Dp, t.S, rc);
     HY(rc);
+    if (l.kind == MSA_MIX_PARALLEL) {
+      t.part2 = partial(o2, l.att.w_out, c.Dp, t.S2, rc);
+      HY(rc);
+    }
     HY(tail(t));
     off = layer_base;
-    if (ff) HY(feed_forward(i, h, x, after));
-    if (!dry && a->probe)
-      MSA_REQUIRE(hipMemcpyAsync(a->probe + (int64_t)i * M * c.Dp, x, (size_t)M * c.Dp * 4,
-                                 hipMemcpyDeviceToDevice, (hipStream_t)stream) == hipSuccess,
-                  MSA_ERR_HIP, "msa_hybrid_step: copy of layer %d's output failed", i);
+    if (ff) {
+      end.w_post = l.norm2b;
+      HY(feed_forward(l, end));
+    }
   }
   off = layer_base;
   if (!a->logits) return MSA_OK;
@@ -455,12 +619,12 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
                   cfg->D <= cfg->Dp && cfg->Dp % 64 == 0 && cfg->Dp >= 128 && cfg->Dp <= 16384 &&
                   cfg->vocab > 0 && cfg->Vp % 16 == 0 && cfg->vocab <= cfg->Vp,
               MSA_ERR_INVALID_ARG, "%s: bad configuration", name);
-  MSA_REQUIRE(cfg->embed && cfg->inv_freq && cfg->final_norm && cfg->head, MSA_ERR_INVALID_ARG,
+  MSA_REQUIRE(cfg->embed && cfg->final_norm && cfg->head, MSA_ERR_INVALID_ARG,
               "%s: null pointer in the configuration", name);
   auto k_ok = [](int k) { return k >= 128 && k % 64 == 0; };
   for (int i = 0; i < cfg->layers; ++i) {
     const msa_hybrid_layer& l = layers[i];
-    MSA_REQUIRE(l.w_in && l.w_out && l.norm1 && l.norm1b && k_ok(l.ko) && l.n_in % 16 == 0,
+    MSA_REQUIRE(l.w_in && l.w_out && l.norm1 && k_ok(l.ko) && l.n_in % 16 == 0,
                 MSA_ERR_INVALID_ARG, "%s: layer %d: mixer projections", name, i);
     if (l.kind == MSA_MIX_LATENT) {
       MSA_REQUIRE(k_ok(l.qp) && k_ok(l.rp) && l.rp <= 2048 && l.hd % 32 == 0 && l.heads > 0 &&
@@ -478,6 +642,19 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
                       l.n_in == 2 * l.channels && l.ko >= l.channels && l.w_gates && l.conv_w &&
                       l.gate_bias && l.lam && l.y_bias,
                   MSA_ERR_INVALID_ARG, "%s: layer %d: gated linear recurrent unit", name, i);
+    } else if (l.kind == MSA_MIX_PARALLEL) {
+      const msa_attention_layer& t = l.att;
+      MSA_REQUIRE(t.heads > 0 && t.kv_heads > 0 && t.heads % t.kv_heads == 0 && t.hd > 0 &&
+                      t.hd % 16 == 0 && t.vd > 0 && t.vd % 16 == 0 && t.chunk >= 0 && t.scale > 0.f &&
+                      (t.rot_dims == 0 || t.inv_freq) && t.w_out && t.out_norm && k_ok(t.ko) &&
+                      t.ko >= t.heads * t.vd,
+                  MSA_ERR_INVALID_ARG, "%s: layer %d: grouped attention", name, i);
+      MSA_REQUIRE(l.heads > 0 && l.kv_heads > 0 && l.heads % l.kv_heads == 0 && l.conv_w && l.o_norm &&
+                      l.ko >= l.heads * l.vp && l.vp <= 512 && k_ok(l.lr) && l.w_lr && l.lr_bias &&
+                      l.lr_rate && l.out_norm && l.in_bias &&
+                      l.n_in >= (t.heads + t.kv_heads) * t.hd + t.kv_heads * t.vd +
+                                    2 * l.kv_heads * l.dp + l.heads * l.vp + l.lr + t.heads + l.heads,
+                  MSA_ERR_INVALID_ARG, "%s: layer %d: delta rule beside attention", name, i);
     } else {
       MSA_REQUIRE(l.kind == MSA_MIX_DELTA && l.heads > 0 && l.kv_heads > 0 &&
                       l.heads % l.kv_heads == 0 && l.conv_w && l.decay_rate && l.dt_bias && l.o_norm &&
@@ -486,26 +663,58 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
                   MSA_ERR_INVALID_ARG, "%s: layer %d: gated delta rule", name, i);
     }
     if (l.ff_kind == MSA_FF_DENSE)
-      MSA_REQUIRE(k_ok(l.ff) && l.n_ff_in == 2 * l.ff && l.w_ff_in && l.w_ff_down && l.norm2 && l.norm2b,
+      MSA_REQUIRE(k_ok(l.ff) && l.n_ff_in == 2 * l.ff && l.w_ff_in && l.w_ff_down && l.norm2,
+                  MSA_ERR_INVALID_ARG, "%s: layer %d: feed-forward", name, i);
+    else if (l.ff_kind == MSA_FF_RELU2)
+      MSA_REQUIRE(k_ok(l.ff) && l.n_ff_in == l.ff && l.w_ff_in && l.w_ff_down && l.norm2,
                   MSA_ERR_INVALID_ARG, "%s: layer %d: feed-forward", name, i);
     else if (l.ff_kind == MSA_FF_MOE)
       MSA_REQUIRE(l.experts > 0 && l.top > 0 && k_ok(l.ff_expert) && l.w_ff_in &&
-                      l.w_e_in && l.w_e_down && l.norm2 && l.norm2b && l.n_groups > 0 &&
+                      l.w_e_in && l.w_e_down && l.norm2 && l.n_groups > 0 &&
                       (l.ff_shared == 0 || (k_ok(l.ff_shared) && l.w_ff_down)) &&
                       l.n_ff_in >= 2 * l.ff_shared + l.experts + (l.ff_shared > 0 ? 1 : 0),
                   MSA_ERR_INVALID_ARG, "%s: layer %d: routed feed-forward", name, i);
   }
+  const int n_runs = cfg->n_runs > 0 ? cfg->n_runs : cfg->layers;
+  MSA_REQUIRE(cfg->n_runs <= 0 || (cfg->run_layer && cfg->run_pass), MSA_ERR_INVALID_ARG,
+              "%s: runs without tables", name);
   msa_hybrid* d = new (std::nothrow) msa_hybrid();
   msa_hybrid_layer* lw = (msa_hybrid_layer*)malloc(sizeof(msa_hybrid_layer) * (size_t)cfg->layers);
-  if (!d || !lw) {
+  LayerRun* runs = (LayerRun*)malloc(sizeof(LayerRun) * (size_t)n_runs);
+  auto drop = [&] {
     delete d;
     free(lw);
+    free(runs);
+  };
+  if (!d || !lw || !runs) {
+    drop();
     msa_set_error("%s: out of host memory", name);
     return MSA_ERR_INVALID_ARG;
+  }
+  for (int i = 0; i < n_runs; ++i) {
+    LayerRun& r = runs[i];
+    r.layer = cfg->n_runs > 0 ? cfg->run_layer[i] : i;
+    r.pass = cfg->n_runs > 0 ? cfg->run_pass[i] : -1;
+    r.owner = i;
+    bool ok = r.layer >= 0 && r.layer < cfg->layers && (r.pass < 0 || cfg->loop_step);
+    if (ok && layers[r.layer].kind == MSA_MIX_LATENT && layers[r.layer].kv_from >= 0) {
+      // the latest run of the layer that owns the latent
+      for (r.owner = i - 1; r.owner >= 0 && runs[r.owner].layer != layers[r.layer].kv_from;) --r.owner;
+      ok = r.owner >= 0;
+    }
+    if (!ok) {
+      drop();
+      msa_set_error("%s: run %d", name, i);
+      return MSA_ERR_INVALID_ARG;
+    }
+    if (r.pass > 0) d->adds_embedding = true;
   }
   memcpy(lw, layers, sizeof(msa_hybrid_layer) * (size_t)cfg->layers);
   d->cfg = *cfg;
   d->layers = lw;
+  d->runs = runs;
+  d->cfg.n_runs = n_runs;
+  d->cfg.run_layer = d->cfg.run_pass = nullptr;
   *out = d;
   return MSA_OK;
 }
@@ -513,6 +722,7 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
 extern "C" void msa_hybrid_destroy(msa_hybrid* d) {
   if (!d) return;
   free(d->layers);
+  free(d->runs);
   delete d;
 }
 
@@ -534,12 +744,15 @@ extern "C" int msa_hybrid_step(const msa_hybrid* d, const msa_hybrid_step_args* 
               MSA_ERR_INVALID_ARG, "%s: null pointer in the step's arguments", name);
   MSA_REQUIRE(a->workspace_bytes >= need, MSA_ERR_CAPACITY, "%s: workspace of %lld bytes, %lld needed",
               name, (long long)a->workspace_bytes, (long long)need);
-  for (int i = 0; i < d->cfg.layers; ++i) {
-    const msa_hybrid_layer& l = d->layers[i];
+  for (int i = 0; i < d->cfg.n_runs; ++i) {
+    const msa_hybrid_layer& l = d->layers[d->runs[i].layer];
     const msa_hybrid_state& st = a->state[i];
     MSA_REQUIRE(l.kind == MSA_MIX_LATENT ? (l.kv_from >= 0 || st.latent)
                                          : (st.rec && (st.conv || l.taps == 1)),
-                MSA_ERR_INVALID_ARG, "%s: layer %d has no cache or state", name, i);
+                MSA_ERR_INVALID_ARG, "%s: run %d has no cache or state", name, i);
+    const int rows = l.att.chunk > 0 && l.att.chunk < a->capacity ? l.att.chunk : a->capacity;
+    MSA_REQUIRE(l.kind != MSA_MIX_PARALLEL || (st.keys && st.values && st.kv_rows >= rows),
+                MSA_ERR_INVALID_ARG, "%s: run %d keeps %d positions of %d", name, i, st.kv_rows, rows);
   }
   HY(start(r, d, a, stream, false));
   return r.go();

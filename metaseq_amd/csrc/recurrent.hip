@@ -13,10 +13,9 @@ struct Vec8 {
 };
 
 __device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
-__device__ __forceinline__ float softplus(float v) {
-  return v > 20.f ? v : log1pf(expf(v));
+__device__ __forceinline__ float gate_of(float v, int act) {
+  return (act == MSA_GATE_SIGMOID ? 1.f : v) / (1.f + expf(-v));
 }
-
 // ---- short convolution ----------------------------------------------------------------------
 constexpr int SC_TOK = 8;      // tokens per workgroup
 constexpr int SC_MAX_TAPS = 8;
@@ -206,6 +205,7 @@ __global__ __launch_bounds__(256) void rglru_state_kernel(
 // prompt over the chip; 8 need fewer instructions per column where there are segments enough.  With S the state before the
 // token's decay, one pass over it yields both products the token needs:
 //   u = beta (v - g S^T k),   o = S_new^T q = g S^T q + u (k . q),   S_new = g S + k u^T.
+// CH: one decay per key channel (a row of S), taken from `decay`; S is decayed before the pass.
 // Tokens are taken DR_TOK at a time: the next chunk's rows are fetched into registers while the
 // current chunk runs out of LDS, where k and q arrive as unit vectors.
 constexpr int DR_TOK = 16;
@@ -227,15 +227,16 @@ __device__ __forceinline__ float lanes_sum(float v) {  // over LPC = 8 or 16 nei
   return v;
 }
 
-template <typename T, int DP, int LPC>
+template <typename T, int DP, int LPC, bool CH>
 __global__ __launch_bounds__(256) void delta_scan_kernel(
     const T* __restrict__ qkv, int64_t ld, const float* __restrict__ ba, int ldba,
-    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias, int heads, int kv_heads,
-    float q_scale, int vp, float* __restrict__ state, float* __restrict__ o,
+    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias,
+    const float* __restrict__ decay, int heads, int kv_heads, float q_scale, int vp, float* __restrict__ state, float* __restrict__ o,
     const int32_t* __restrict__ seg_start, const int32_t* __restrict__ seg_slot,
     const int32_t* __restrict__ seg_pos) {
   constexpr int R = DP / LPC, CW = 256 / LPC, R16 = DP / 16;
-  __shared__ __attribute__((aligned(16))) float lk[DR_TOK][DP], lq[DR_TOK][DP];
+  __shared__ __attribute__((aligned(16))) float lk[DR_TOK][DP], lq[DR_TOK][DP],
+      ld_[CH ? DR_TOK : 1][CH ? DP : 4];
   __shared__ float lv[DR_TOK][CW], lo[DR_TOK][CW], lg[DR_TOK], lb[DR_TOK], lkq[DR_TOK];
   const int s = blockIdx.z, h = blockIdx.y, col0 = blockIdx.x * CW;
   const int tid = threadIdx.x;
@@ -252,14 +253,16 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
   float S[R];
 #pragma unroll
   for (int i = 0; i < R; ++i) S[i] = pos > 0 ? st[i] : 0.f;
-  const float rate = decay_rate[h], dtb = dt_bias[h];
+  const float rate = CH ? 0.f : decay_rate[h], dtb = CH ? 0.f : dt_bias[h];
 
   // staging: vector x = tid / 8 (tokens 0 .. 15 of q, then of k), elements EV * (tid % 8) ..
   constexpr int EV = DP / 8, VPT = DR_TOK * CW / 256;  // q or k elements, v elements per thread
+  constexpr int GV = CH ? (DR_TOK * DP + 1023) / 1024 : 0;  // decays per thread, four at a time
   const int sv = tid >> 3, stok = sv & 15, sel = (tid & 7) * EV;
   const bool is_k = sv >= 16;
   T raw[EV];
   float rv[VPT], rb = 0.f, rg = 0.f;
+  float4_t rd[GV > 0 ? GV : 1];
   auto fetch = [&](int t0) {
     const int t = min(t0 + stok, n - 1);
     const T* p = qkv + (int64_t)(first + t) * ld + (is_k ? k_at : q_at) + sel;
@@ -278,7 +281,13 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     if (tid < DR_TOK) {
       const float* z = ba + (int64_t)(first + min(t0 + tid, n - 1)) * ldba;
       rb = z[h];
-      rg = z[heads + h];
+      if (!CH) rg = z[heads + h];
+    }
+#pragma unroll
+    for (int i = 0; i < GV; ++i) {
+      const int e = min((tid + 256 * i) * 4, DR_TOK * DP - 4), t = min(t0 + e / DP, n - 1);
+      rd[i] = *reinterpret_cast<const float4_t*>(decay + ((int64_t)(first + t) * heads + h) * DP +
+                                                 e % DP);
     }
   };
   fetch(0);
@@ -299,8 +308,12 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       for (int i = 0; i < VPT; ++i) (&lv[0][0])[tid + 256 * i] = rv[i];
       if (tid < DR_TOK) {
         lb[tid] = sigmoidf(rb);
-        lg[tid] = expf(-rate * softplus(rg + dtb));
+        if (!CH) lg[tid] = decay_of(rg + dtb, rate);
       }
+#pragma unroll
+      for (int i = 0; i < GV; ++i)
+        if ((tid + 256 * i) * 4 < DR_TOK * DP)
+          *reinterpret_cast<float4_t*>(&ld_[0][0] + (tid + 256 * i) * 4) = rd[i];
     }
     lds_barrier();
     {
@@ -315,16 +328,24 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     lds_barrier();
     // operands of the current and the next token: one set is fetched while the other is used
     struct Token {
-      float k[R], q[R], g, beta, v, kq;
+      float k[R], q[R], d[CH ? R : 1], g, beta, v, kq;
     } a, b;
     auto read = [&](Token& x, int t) {
       t = min(t, DR_TOK - 1);
 #pragma unroll
       for (int i = 0; i < R; ++i) x.k[i] = lk[t][rl * R + i], x.q[i] = lq[t][rl * R + i];
-      x.g = lg[t], x.beta = lb[t], x.v = lv[t][cl], x.kq = lkq[t];
+      if constexpr (CH) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) x.d[i] = ld_[t][rl * R + i];
+      }
+      x.g = CH ? 1.f : lg[t], x.beta = lb[t], x.v = lv[t][cl], x.kq = lkq[t];
     };
     auto advance = [&](const Token& x, int t) {
       float d1 = 0.f, d2 = 0.f, e1 = 0.f, e2 = 0.f;
+      if constexpr (CH) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) S[i] *= x.d[i];
+      }
 #pragma unroll
       for (int i = 0; i < R; i += 2) {
         d1 = fmaf(S[i], x.k[i], d1);
@@ -334,10 +355,10 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
       }
       d1 = lanes_sum<LPC>(d1 + e1);
       d2 = lanes_sum<LPC>(d2 + e2);
-      const float u = x.beta * (x.v - x.g * d1);
+      const float u = x.beta * (x.v - (CH ? d1 : x.g * d1));
 #pragma unroll
-      for (int i = 0; i < R; ++i) S[i] = fmaf(x.k[i], u, x.g * S[i]);
-      if (rl == 0) lo[t][cl] = fmaf(u, x.kq, x.g * d2);
+      for (int i = 0; i < R; ++i) S[i] = fmaf(x.k[i], u, CH ? S[i] : x.g * S[i]);
+      if (rl == 0) lo[t][cl] = fmaf(u, x.kq, CH ? d2 : x.g * d2);
     };
     read(a, 0);
     for (int t = 0; t < nt; t += 2) {
@@ -357,12 +378,12 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
 // One token per segment (a decode step): a workgroup owns one segment and one head with all its
 // columns, 4 CG of them per wave and pass, requests the whole pass's state at once and finishes the
 // head's output (norm over the columns, gate) itself.  Lanes and arithmetic as above.
-template <typename T, int R, int CG>
+template <typename T, int R, int CG, bool CH>
 __global__ __launch_bounds__(256) void delta_step_kernel(
     const T* __restrict__ qkv, int64_t ld, const float* __restrict__ ba, int ldba,
-    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias, int heads, int kv_heads,
-    float q_scale, int vdim, int vp, float* __restrict__ state, const T* __restrict__ gate,
-    int64_t ld_gate, const float* __restrict__ w, float eps, T* __restrict__ out, int64_t ld_out,
+    const float* __restrict__ decay_rate, const float* __restrict__ dt_bias,
+    const float* __restrict__ decay, int heads, int kv_heads, float q_scale, int vdim, int vp,
+    float* __restrict__ state, const T* __restrict__ gate, int64_t ld_gate, int gate_act, const float* __restrict__ w, float eps, T* __restrict__ out, int64_t ld_out,
     int out_mb, const int32_t* __restrict__ seg_slot, const int32_t* __restrict__ seg_pos) {
   constexpr int DP = 16 * R;
   __shared__ __attribute__((aligned(16))) float lk[DP], lq[DP];
@@ -408,7 +429,13 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
   }
   const float* z = ba + (int64_t)m * ldba;
   const float bt = sigmoidf(z[h]);
-  const float g = expf(-decay_rate[h] * softplus(z[heads + h] + dt_bias[h]));
+  const float g = CH ? 1.f : decay_of(z[heads + h] + dt_bias[h], decay_rate[h]);
+  float gr[CH ? R : 1];  // decays of the lane's rows
+  if constexpr (CH) {
+    const float* p = decay + ((int64_t)m * heads + h) * DP + rl * R;
+#pragma unroll
+    for (int i = 0; i < R; ++i) gr[i] = p[i];
+  }
   lds_barrier();
   float k[R], q[R], kq = 0.f;
 #pragma unroll
@@ -428,6 +455,10 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
         for (int i = 0; i < R; ++i) S[c][i] = 0.f;
       }
       float d1 = 0.f, d2 = 0.f;
+      if constexpr (CH) {
+#pragma unroll
+        for (int i = 0; i < R; ++i) S[c][i] *= gr[i];
+      }
 #pragma unroll
       for (int i = 0; i < R; ++i) {
         d1 = fmaf(S[c][i], k[i], d1);
@@ -452,7 +483,7 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
   const float rms = 1.f / sqrtf(ss / (float)vdim + eps);
   for (int c = tid; c < vp; c += 256) {
     const int at = h * vp + c;
-    const float y = lo[c] * rms * w[c] * silu((float)gate[(int64_t)m * ld_gate + at]);
+    const float y = lo[c] * rms * w[c] * gate_of((float)gate[(int64_t)m * ld_gate + at], gate_act);
     out[out_mb > 0 ? packed_act_offset(m, at, out_mb) : (int64_t)m * ld_out + at] = (T)y;
   }
 }
@@ -460,7 +491,7 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
 // one wave per (token, head)
 template <typename T>
 __global__ __launch_bounds__(256) void delta_output_kernel(
-    const float* __restrict__ o, const T* __restrict__ gate, int64_t ld_gate,
+    const float* __restrict__ o, const T* __restrict__ gate, int64_t ld_gate, int gate_act,
     const float* __restrict__ w, int heads, int vdim, int vp, float eps, T* __restrict__ out,
     int64_t ld_out, int out_mb, int M) {
   const int64_t idx = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -482,99 +513,94 @@ __global__ __launch_bounds__(256) void delta_output_kernel(
     const int c = lane + 64 * i;
     if (c < vp) {
       const int at = h * vp + c;
-      const float y = v[i] * r * w[c] * silu((float)gate[(int64_t)m * ld_gate + at]);
+      const float y = v[i] * r * w[c] * gate_of((float)gate[(int64_t)m * ld_gate + at], gate_act);
       out[out_mb > 0 ? packed_act_offset(m, at, out_mb) : (int64_t)m * ld_out + at] = (T)y;
     }
   }
 }
 
-template <typename T, int LPC>
-void run_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
-               const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vp, float* state,
-               float* o, const msa_batch* b, hipStream_t s) {
-  const dim3 grid(vp / (256 / LPC), heads, b->nseg);
-  const float q_scale = (float)pow((double)dim, -0.5);
-#define DR_CASE(DP)                                                                                 \
-  case DP:                                                                                          \
-    hipLaunchKernelGGL((delta_scan_kernel<T, DP, LPC>), grid, dim3(256), 0, s, (const T*)qkv, ld,   \
-                       ba, ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vp, state, o,       \
-                       b->seg_start, b->seg_slot, b->seg_pos);                                      \
-    break;
-  switch (dp) {
-    DR_CASE(32)
-    DR_CASE(64)
-    DR_CASE(96)
-    DR_CASE(128)
-    DR_CASE(192)
-    DR_CASE(256)
-  }
-#undef DR_CASE
+template <typename T, int DP, int LPC>
+void run_delta(const msa_delta_args& a, const msa_batch* b, hipStream_t s) {
+  const dim3 grid(a.vp / (256 / LPC), a.heads, b->nseg);
+  const float q_scale = (float)pow((double)a.dim, -0.5);
+#define DR_RUN(CH)                                                                                 \
+  hipLaunchKernelGGL((delta_scan_kernel<T, DP, LPC, CH>), grid, dim3(256), 0, s, (const T*)a.qkv,  \
+                     a.ld, a.ba, a.ldba, a.decay_rate, a.dt_bias, a.decay, a.heads, a.kv_heads,    \
+                     q_scale, a.vp, a.state, a.o, b->seg_start, b->seg_slot, b->seg_pos)
+  if (a.decay) DR_RUN(true);
+  else DR_RUN(false);
+#undef DR_RUN
 }
 
-template <typename T>
-void pick_delta(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
-                const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vp, float* state,
-                float* o, const msa_batch* b, hipStream_t s) {
+template <typename T, int DP>
+void pick_delta(const msa_delta_args& a, const msa_batch* b, hipStream_t s) {
   // eight lanes per column from two waves per SIMD on (of 1024)
-  if (vp % 32 == 0 && (int64_t)b->nseg * heads * (vp / 32) * 4 >= 2048)
-    run_delta<T, 8>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b, s);
+  if (a.vp % 32 == 0 && (int64_t)b->nseg * a.heads * (a.vp / 32) * 4 >= 2048)
+    run_delta<T, DP, 8>(a, b, s);
   else
-    run_delta<T, 16>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
-                     s);
+    run_delta<T, DP, 16>(a, b, s);
+}
+
+template <typename T, int R, int CG>
+void run_delta_step(const msa_delta_args& a, const msa_batch* b, hipStream_t s) {
+  const dim3 grid(a.heads, b->nseg);
+  const float q_scale = (float)pow((double)a.dim, -0.5);
+#define DR_RUN(CH)                                                                                 \
+  hipLaunchKernelGGL((delta_step_kernel<T, R, CG, CH>), grid, dim3(256), 0, s, (const T*)a.qkv,    \
+                     a.ld, a.ba, a.ldba, a.decay_rate, a.dt_bias, a.decay, a.heads, a.kv_heads,    \
+                     q_scale, a.vdim, a.vp, a.state, (const T*)a.gate, a.ld_gate, a.gate_act, a.w, \
+                     a.eps, (T*)a.out, a.ld_out, a.out_mb, b->seg_slot, b->seg_pos)
+  if (a.decay) DR_RUN(true);
+  else DR_RUN(false);
+#undef DR_RUN
 }
 
 template <typename T>
-void run_delta_step(const void* qkv, int64_t ld, const float* ba, int ldba, const float* decay_rate,
-                    const float* dt_bias, int heads, int kv_heads, int dim, int dp, int vdim, int vp,
-                    float* state, const void* gate, int64_t ld_gate, const float* w, float eps,
-                    void* out, int64_t ld_out, int out_mb, const msa_batch* b, hipStream_t s) {
-  const dim3 grid(heads, b->nseg);
-  const float q_scale = (float)pow((double)dim, -0.5);
-#define DR_CASE(RR, CG)                                                                             \
-  case 16 * RR:                                                                                     \
-    hipLaunchKernelGGL((delta_step_kernel<T, RR, CG>), grid, dim3(256), 0, s, (const T*)qkv, ld, ba, \
-                       ldba, decay_rate, dt_bias, heads, kv_heads, q_scale, vdim, vp, state,        \
-                       (const T*)gate, ld_gate, w, eps, (T*)out, ld_out, out_mb, b->seg_slot,       \
-                       b->seg_pos);                                                                 \
+void dispatch_delta(const msa_delta_args& a, const msa_batch* b, bool step, hipStream_t s) {
+#define DR_CASE(DP, CG)                              \
+  case DP:                                           \
+    if (step) run_delta_step<T, DP / 16, CG>(a, b, s); \
+    else pick_delta<T, DP>(a, b, s);                 \
     break;
-  switch (dp) {
-    DR_CASE(2, 8)
-    DR_CASE(4, 8)
-    DR_CASE(6, 8)
-    DR_CASE(8, 8)
-    DR_CASE(12, 4)
-    DR_CASE(16, 4)
+  switch (a.dp) {
+    DR_CASE(32, 8)
+    DR_CASE(64, 8)
+    DR_CASE(96, 8)
+    DR_CASE(128, 8)
+    DR_CASE(192, 4)
+    DR_CASE(256, 4)
   }
 #undef DR_CASE
 }
 
-bool delta_sizes_ok(int heads, int kv_heads, int dim, int dp, int vp, int ldba, int64_t ld,
-                    const msa_batch* b) {
-  return (dp == 32 || dp == 64 || dp == 96 || dp == 128 || dp == 192 || dp == 256) && dim <= dp &&
-         vp > 0 && vp % 16 == 0 && kv_heads > 0 && heads % kv_heads == 0 && ldba >= 2 * heads &&
-         ld % 8 == 0 && heads <= 65535 && b->nseg > 0 && b->nseg <= 65535;
+int check_delta(const char* name, const msa_delta_args* a, const msa_batch* b) {
+  MSA_REQUIRE(a && b && a->qkv && a->ba && a->state && (a->decay || (a->decay_rate && a->dt_bias)),
+              MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  const int dp = a->dp;
+  MSA_REQUIRE((dp == 32 || dp == 64 || dp == 96 || dp == 128 || dp == 192 || dp == 256) &&
+                  a->dim > 0 && a->dim <= dp && a->vp > 0 && a->vp % 16 == 0 && a->heads > 0 &&
+                  a->kv_heads > 0 && a->heads % a->kv_heads == 0 &&
+                  a->ldba >= (a->decay ? 1 : 2) * a->heads && a->ld % 8 == 0 && a->heads <= 65535 &&
+                  b->nseg > 0 && b->nseg <= 65535,
+              MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, a->heads,
+              a->kv_heads, a->dim, dp, a->vp);
+  return MSA_OK;
 }
 
 }  // namespace
 
-extern "C" int msa_delta_step(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
-                              const float* decay_rate, const float* dt_bias, int heads, int kv_heads,
-                              int dim, int dp, int vdim, int vp, float* state, const void* gate,
-                              int64_t ld_gate, const float* w, float eps, void* out, int64_t ld_out,
-                              int out_mb, const msa_batch* b, void* stream) {
+extern "C" int msa_delta_step(const msa_delta_args* a, const msa_batch* b, void* stream) {
   const char* name = "msa_delta_step";
-  MSA_REQUIRE(qkv && ba && decay_rate && dt_bias && state && gate && w && out && b,
-              MSA_ERR_INVALID_ARG, "%s: null pointer", name);
-  MSA_REQUIRE(delta_sizes_ok(heads, kv_heads, dim, dp, vp, ldba, ld, b) && vdim <= vp && vp <= 512 &&
-                  b->max_count == 1 && b->M == b->nseg,
-              MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
-              kv_heads, dim, dp, vp);
-  if (dtype == MSA_BF16)
-    run_delta_step<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vdim, vp,
-                           state, gate, ld_gate, w, eps, out, ld_out, out_mb, b, (hipStream_t)stream);
+  int rc = check_delta(name, a, b);
+  if (rc) return rc;
+  MSA_REQUIRE(a->gate && a->w && a->out, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  MSA_REQUIRE(a->vdim <= a->vp && a->vp <= 512 && b->max_count == 1 && b->M == b->nseg,
+              MSA_ERR_INVALID_ARG, "%s: vdim=%d vp=%d, %d tokens in %d segments", name, a->vdim, a->vp,
+              b->M, b->nseg);
+  if (a->dtype == MSA_BF16)
+    dispatch_delta<bf16_t>(*a, b, true, (hipStream_t)stream);
   else
-    run_delta_step<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vdim, vp,
-                          state, gate, ld_gate, w, eps, out, ld_out, 0, b, (hipStream_t)stream);
+    dispatch_delta<float>(*a, b, true, (hipStream_t)stream);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }
@@ -670,40 +696,34 @@ extern "C" int msa_rglru_scan(int dtype, float* gates, const float* gate_bias, c
   return MSA_OK;
 }
 
-extern "C" int msa_delta_scan(int dtype, const void* qkv, int64_t ld, const float* ba, int ldba,
-                              const float* decay_rate, const float* dt_bias, int heads, int kv_heads,
-                              int dim, int dp, int vp, float* state, float* o, const msa_batch* b,
-                              void* stream) {
+extern "C" int msa_delta_scan(const msa_delta_args* a, const msa_batch* b, void* stream) {
   const char* name = "msa_delta_scan";
-  MSA_REQUIRE(qkv && ba && decay_rate && dt_bias && state && o && b, MSA_ERR_INVALID_ARG,
-              "%s: null pointer", name);
-  MSA_REQUIRE(delta_sizes_ok(heads, kv_heads, dim, dp, vp, ldba, ld, b),
-              MSA_ERR_INVALID_ARG, "%s: heads=%d kv_heads=%d dim=%d dp=%d vp=%d", name, heads,
-              kv_heads, dim, dp, vp);
-  if (dtype == MSA_BF16)
-    pick_delta<bf16_t>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o,
-                      b, (hipStream_t)stream);
+  int rc = check_delta(name, a, b);
+  if (rc) return rc;
+  MSA_REQUIRE(a->o, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
+  if (a->dtype == MSA_BF16)
+    dispatch_delta<bf16_t>(*a, b, false, (hipStream_t)stream);
   else
-    pick_delta<float>(qkv, ld, ba, ldba, decay_rate, dt_bias, heads, kv_heads, dim, dp, vp, state, o, b,
-                     (hipStream_t)stream);
+    dispatch_delta<float>(*a, b, false, (hipStream_t)stream);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }
 
-extern "C" int msa_delta_output(int dtype, const float* o, const void* gate, int64_t ld_gate,
-                                const float* w, int heads, int vdim, int vp, float eps, void* out,
-                                int64_t ld_out, int out_mb, int M, void* stream) {
+extern "C" int msa_delta_output(const msa_delta_args* a, int M, void* stream) {
   const char* name = "msa_delta_output";
-  MSA_REQUIRE(o && gate && w && out && M > 0 && heads > 0 && vp > 0 && vp <= 512 && vdim <= vp,
-              MSA_ERR_INVALID_ARG, "%s: bad arguments (vp=%d)", name, vp);
-  const dim3 grid((unsigned)(((int64_t)M * heads + 3) / 4));
-  if (dtype == MSA_BF16)
-    hipLaunchKernelGGL(delta_output_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, o,
-                       (const bf16_t*)gate, ld_gate, w, heads, vdim, vp, eps, (bf16_t*)out, ld_out,
-                       out_mb, M);
+  MSA_REQUIRE(a && a->o && a->gate && a->w && a->out && M > 0 && a->heads > 0 && a->vp > 0 &&
+                  a->vp <= 512 && a->vdim <= a->vp,
+              MSA_ERR_INVALID_ARG, "%s: bad arguments", name);
+  const dim3 grid((unsigned)(((int64_t)M * a->heads + 3) / 4));
+  hipStream_t s = (hipStream_t)stream;
+  if (a->dtype == MSA_BF16)
+    hipLaunchKernelGGL(delta_output_kernel<bf16_t>, grid, dim3(256), 0, s, a->o, (const bf16_t*)a->gate,
+                       a->ld_gate, a->gate_act, a->w, a->heads, a->vdim, a->vp, a->eps,
+                       (bf16_t*)a->out, a->ld_out, a->out_mb, M);
   else
-    hipLaunchKernelGGL(delta_output_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, o,
-                       (const float*)gate, ld_gate, w, heads, vdim, vp, eps, (float*)out, ld_out, 0, M);
+    hipLaunchKernelGGL(delta_output_kernel<float>, grid, dim3(256), 0, s, a->o, (const float*)a->gate,
+                       a->ld_gate, a->gate_act, a->w, a->heads, a->vdim, a->vp, a->eps,
+                       (float*)a->out, a->ld_out, 0, M);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }

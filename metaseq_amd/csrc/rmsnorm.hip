@@ -50,7 +50,8 @@ template <typename T, int NV, int NT>
 __global__ __launch_bounds__(NT) void embed_kernel(
     const int64_t* __restrict__ tokens, const int32_t* __restrict__ tok_pos,
     const bf16_t* __restrict__ table, int vocab, float scale, const double* __restrict__ inv_freq,
-    int D, int Dp, float eps, float* __restrict__ x, const float* __restrict__ w, void* h, int mb) {
+    int D, int Dp, float eps, const float* __restrict__ step, float* __restrict__ e_out,
+    float* __restrict__ x, const float* __restrict__ w, void* h, int mb) {
   __shared__ float red[16];
   const int64_t m = blockIdx.x;
   int64_t t = tokens[m];
@@ -66,7 +67,7 @@ __global__ __launch_bounds__(NT) void embed_kernel(
 #pragma unroll
     for (int j = 0; j < 4; j += 2) {
       float sn = 0.f, cs = 0.f;
-      if (c + j < D) {
+      if (inv_freq && c + j < D) {
         // the angle in turns, reduced to [-1/2, 1/2] in double; sine and cosine of pi * (2 turns)
         double turns = pos * inv_freq[(c + j) >> 1] * 0.15915494309189535;
         turns -= rint(turns);
@@ -75,14 +76,40 @@ __global__ __launch_bounds__(NT) void embed_kernel(
       v[i][j] = (float)e[j] * scale + sn;
       v[i][j + 1] = (float)e[j + 1] * scale + (c + j + 1 < D ? cs : 0.f);
     }
+    if (e_out) *reinterpret_cast<float4_t*>(e_out + m * Dp + c) = v[i];
+    if (step) v[i] += *reinterpret_cast<const float4_t*>(step + c);
     *reinterpret_cast<float4_t*>(x + m * Dp + c) = v[i];
   }
   if (w) norm_out<T, NV, NT>(v, m, D, Dp, eps, w, h, mb, red);
 }
 
-template <typename T, int NV, int NT>
+// b += the sum of S slices of row m; four slices at a time, their loads in flight together
+template <int NV, int NT>
+__device__ __forceinline__ void sum_slices(const float* part, int S, int M, int64_t m, int Dp,
+                                           float4_t (&b)[NV]) {
+  for (int s0 = 0; s0 < S; s0 += 4) {
+    float4_t v[4][NV];
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const float* p = part + ((int64_t)min(s0 + s, S - 1) * M + m) * Dp;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + i * NT) * 4;
+        v[s][i] = c < Dp && s0 + s < S ? *reinterpret_cast<const float4_t*>(p + c)
+                                       : float4_t{0.f, 0.f, 0.f, 0.f};
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < 4; ++s)
+#pragma unroll
+      for (int i = 0; i < NV; ++i) b[i] += v[s][i];
+  }
+}
+
+// TWO: a second sublayer beside the first (part2)
+template <typename T, int NV, int NT, bool TWO>
 __global__ __launch_bounds__(NT) void tail_kernel(msa_tail_args a) {
-  __shared__ float red[16];
+  __shared__ float red[32];
   const int64_t m = blockIdx.x;
   const int D = a.D, Dp = a.Dp;
   float4_t b[NV], x[NV];
@@ -93,28 +120,18 @@ __global__ __launch_bounds__(NT) void tail_kernel(msa_tail_args a) {
     if (c < Dp) x[i] = *reinterpret_cast<const float4_t*>(a.x + m * Dp + c);
   }
   if (a.part) {
-    // four slices at a time, their loads in flight together
-    for (int s0 = 0; s0 < a.S; s0 += 4) {
-      float4_t v[4][NV];
-#pragma unroll
-      for (int s = 0; s < 4; ++s) {
-        const float* p = a.part + ((int64_t)min(s0 + s, a.S - 1) * a.M + m) * Dp;
-#pragma unroll
-        for (int i = 0; i < NV; ++i) {
-          const int c = (threadIdx.x + i * NT) * 4;
-          v[s][i] = c < Dp && s0 + s < a.S ? *reinterpret_cast<const float4_t*>(p + c)
-                                           : float4_t{0.f, 0.f, 0.f, 0.f};
-        }
-      }
-#pragma unroll
-      for (int s = 0; s < 4; ++s)
-#pragma unroll
-        for (int i = 0; i < NV; ++i) b[i] += v[s][i];
-    }
+    sum_slices<NV, NT>(a.part, a.S, a.M, m, Dp, b);
     if (a.gate) {
       const float g = a.gate[m];
 #pragma unroll
       for (int i = 0; i < NV; ++i) b[i] = b[i] * g;
+    }
+    if (a.bias) {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (threadIdx.x + i * NT) * 4;
+        if (c < Dp) b[i] += *reinterpret_cast<const float4_t*>(a.bias + c);
+      }
     }
   }
   if (a.pair_y) {
@@ -148,7 +165,23 @@ __global__ __launch_bounds__(NT) void tail_kernel(msa_tail_args a) {
       if ((threadIdx.x + i * NT) * 4 >= Dp) b[i] = float4_t{0.f, 0.f, 0.f, 0.f};
   }
   float r = 1.f;
-  if (a.w_post) {
+  if constexpr (TWO) {
+    float4_t b2[NV];
+    float ss = 0.f, ss2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) b2[i] = float4_t{0.f, 0.f, 0.f, 0.f};
+    sum_slices<NV, NT>(a.part2, a.S2, a.M, m, Dp, b2);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss += dot4(b[i]), ss2 += dot4(b2[i]);
+    block_sum2(ss, ss2, red);
+    r = 1.f / sqrtf(ss / (float)D + a.eps);
+    const float r2 = 1.f / sqrtf(ss2 / (float)D + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = (threadIdx.x + i * NT) * 4;
+      if (c < Dp) x[i] += b2[i] * r2 * *reinterpret_cast<const float4_t*>(a.w_post2 + c);
+    }
+  } else if (a.w_post) {
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) ss += dot4(b[i]);
@@ -164,6 +197,9 @@ __global__ __launch_bounds__(NT) void tail_kernel(msa_tail_args a) {
         b[i] = b[i] * r * wv;
       }
       x[i] += b[i];
+      if (a.probe) *reinterpret_cast<float4_t*>(a.probe + m * Dp + c) = x[i];
+      if (a.add) x[i] += *reinterpret_cast<const float4_t*>(a.add + m * Dp + c);
+      if (a.step) x[i] += *reinterpret_cast<const float4_t*>(a.step + c);
       *reinterpret_cast<float4_t*>(a.x + m * Dp + c) = x[i];
     }
   }
@@ -253,6 +289,10 @@ constexpr int RN_MAX_WIDTH = 16384;
 // one row per workgroup of NT threads with NV float4 each
 #define RN_RUN(KERNEL, T, NV, NT, M, ...) \
   hipLaunchKernelGGL((KERNEL<T, NV, NT>), dim3(M), dim3(NT), 0, (hipStream_t)stream, __VA_ARGS__)
+template <typename T, int NV, int NT>
+constexpr auto tail_one = tail_kernel<T, NV, NT, false>;
+template <typename T, int NV, int NT>
+constexpr auto tail_two = tail_kernel<T, NV, NT, true>;
 #define RN_DISPATCH(KERNEL, T, M, Dp, ...)                                                  \
   do {                                                                                      \
     const int q_ = (Dp) / 4;                                                                \
@@ -272,19 +312,20 @@ constexpr int RN_MAX_WIDTH = 16384;
 
 extern "C" int msa_embed_rmsnorm(int dtype, const int64_t* tokens, const int32_t* tok_pos, int M,
                                  const void* table, int vocab, float scale, const double* inv_freq,
-                                 int D, int Dp, float eps, float* x, const float* w, void* h, int h_mb,
-                                 void* stream) {
+                                 int D, int Dp, float eps, const float* step, float* e, float* x,
+                                 const float* w, void* h, int h_mb, void* stream) {
   const char* name = "msa_embed_rmsnorm";
-  MSA_REQUIRE(tokens && tok_pos && table && inv_freq && x && (!w || h), MSA_ERR_INVALID_ARG,
+  MSA_REQUIRE(tokens && tok_pos && table && x && (!w || h), MSA_ERR_INVALID_ARG,
               "%s: null pointer", name);
   MSA_REQUIRE(M > 0 && vocab > 0 && D > 0 && D <= Dp && Dp % 4 == 0 && Dp <= RN_MAX_WIDTH, MSA_ERR_INVALID_ARG,
               "%s: M=%d vocab=%d D=%d Dp=%d", name, M, vocab, D, Dp);
   if (dtype == MSA_BF16)
     RN_DISPATCH(embed_kernel, bf16_t, M, Dp, tokens,
-                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, h_mb);
+                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, step, e, x, w, h,
+                h_mb);
   else
     RN_DISPATCH(embed_kernel, float, M, Dp, tokens,
-                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, x, w, h, 0);
+                tok_pos, (const bf16_t*)table, vocab, scale, inv_freq, D, Dp, eps, step, e, x, w, h, 0);
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }
@@ -298,10 +339,19 @@ extern "C" int msa_residual_rmsnorm_tail(const msa_tail_args* a, void* stream) {
   MSA_REQUIRE(a->M > 0 && a->D > 0 && a->D <= a->Dp && a->Dp % 4 == 0 && a->Dp <= RN_MAX_WIDTH &&
                   (!a->part || a->S > 0),
               MSA_ERR_INVALID_ARG, "%s: M=%d D=%d Dp=%d S=%d", name, a->M, a->D, a->Dp, a->S);
-  if (a->dtype == MSA_BF16)
-    RN_DISPATCH(tail_kernel, bf16_t, a->M, a->Dp, *a);
-  else
-    RN_DISPATCH(tail_kernel, float, a->M, a->Dp, *a);
+  MSA_REQUIRE(!a->part2 || (a->part && a->w_post && a->w_post2 && a->S2 > 0), MSA_ERR_INVALID_ARG,
+              "%s: a second sublayer beside none, or without norms", name);
+  MSA_REQUIRE(!a->bias || a->part, MSA_ERR_INVALID_ARG, "%s: a bias without a product", name);
+  if (a->part2) {
+    if (a->dtype == MSA_BF16)
+      RN_DISPATCH(tail_two, bf16_t, a->M, a->Dp, *a);
+    else
+      RN_DISPATCH(tail_two, float, a->M, a->Dp, *a);
+  } else if (a->dtype == MSA_BF16) {
+    RN_DISPATCH(tail_one, bf16_t, a->M, a->Dp, *a);
+  } else {
+    RN_DISPATCH(tail_one, float, a->M, a->Dp, *a);
+  }
   MSA_CHECK_LAUNCH(name);
   return MSA_OK;
 }

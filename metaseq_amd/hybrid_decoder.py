@@ -1,5 +1,6 @@
-"""Hybrid decoders on gfx950: attention over a cached latent, gated linear recurrent units and the
-gated delta rule, with dense or routed feed-forwards, behind the same interface as
+"""Hybrid decoders on gfx950: attention over a cached latent, grouped attention within chunks, gated
+linear recurrent units and the gated delta rule, alone or side by side, with dense or routed
+feed-forwards and layers that may run in a loop, behind the same interface as
 ``TransformerDecoder`` (``forward`` with a caller-owned ``incremental_state``, and the slot
 interface of the serving loop).
 
@@ -16,7 +17,8 @@ import torch
 
 from . import _capi
 from ._capi import check, ptr
-from .config import DenseSpec, HybridConfig, LatentAttentionSpec, RGLRUSpec
+from .config import (DenseSpec, HybridConfig, LatentAttentionSpec, ParallelSpec, RGLRUSpec,
+                     SquaredReluSpec)
 from .decoder_base import IncrementalDecoder, upload
 from .kv_cache import HybridCache
 
@@ -38,6 +40,7 @@ def _fit(n, sizes, what):
 
 
 HEAD_SIZES = (32, 64, 96, 128, 192, 256)     # flash attention and delta-rule key sizes
+GROUPED_SIZES = (64, 128, 192, 256)          # grouped attention on the matrix cores
 LATENT_SIZES = (128, 192, 256, 384, 512)     # latent sizes of the matrix-core decode attention
 
 
@@ -77,10 +80,19 @@ class _LayerPlan:
             self.n_in = 2 * self.channels
             self.ko = _k(self.channels)
             self.keep = {"conv": (m.conv - 1, self.channels), "rec": (self.channels,)}
+        elif isinstance(m, ParallelSpec):
+            a, d = m.left, m.right
+            self.hd, self.vd = self._grouped_sizes(a)
+            self.att = (a.heads + a.kv_heads) * self.hd + a.kv_heads * self.vd
+            self._delta_sizes(d)
+            self.lr = _k((d.gate_rank or 0) + (d.decay_rank or 0))
+            self.n_in = self.att + self.qkv + self.lr + _up(a.heads + d.heads, 16)
+            self.ko, self.kl = _k(d.heads * self.vp), _k(a.heads * self.vd)
+            self.keep = {"keys": self.hd, "values": self.vd, "kv_heads": a.kv_heads,
+                         "chunk": a.chunk, "conv": (d.conv - 1, self.qkv),
+                         "rec": (d.heads, self.vp, self.dp)}
         else:
-            self.dp = _fit(m.dim, HEAD_SIZES, "delta-rule key size")
-            self.vp = _up(m.vdim, 16)
-            self.qkv = 2 * m.kv_heads * self.dp + m.heads * self.vp
+            self._delta_sizes(m)
             self.n_in = self.qkv + m.heads * self.vp + _up(2 * m.heads, 16)
             self.ko = _k(m.heads * self.vp)
             self.keep = {"conv": (m.conv - 1, self.qkv), "rec": (m.heads, self.vp, self.dp)}
@@ -88,10 +100,24 @@ class _LayerPlan:
         if isinstance(f, DenseSpec):
             self.ff = _k(f.ff)
             self.n_ff = 2 * self.ff
+        elif isinstance(f, SquaredReluSpec):
+            self.n_ff = self.ff = _k(f.ff)
         elif f is not None:
             self.ffe = _k(f.expert.ff)
             self.ffs = _k(f.shared.ff) if f.shared is not None else 0
             self.n_ff = 2 * self.ffs + _up(f.router.experts + (1 if self.ffs else 0), 16)
+
+
+    def _delta_sizes(self, m):
+        self.dp = _fit(m.dim, HEAD_SIZES, "delta-rule key size")
+        self.vp = _up(m.vdim, 16)
+        self.qkv = 2 * m.kv_heads * self.dp + m.heads * self.vp
+
+    @staticmethod
+    def _grouped_sizes(m):
+        if max(m.dim, m.vdim) <= GROUPED_SIZES[-1]:
+            return tuple(_fit(n, GROUPED_SIZES, "attention head size") for n in (m.dim, m.vdim))
+        return _up(m.dim, 16), _up(m.vdim, 16)     # on the vector ALU
 
 
 class HybridDecoder(IncrementalDecoder):
@@ -113,11 +139,11 @@ class HybridDecoder(IncrementalDecoder):
         self.padding_idx = cfg.padding_idx
         self.max_target_positions = cfg.max_target_positions
         self.inference = True
-        self.layer_probe = None  # called as layer_probe(i, x) after every layer of an extend()
+        self.layer_probe = None  # called as layer_probe(i, x) for every run of a layer, per step
         self.kv_cache_capacity: Optional[int] = None
         self._state_key = str(uuid.uuid4()) + ".hybrid_cache"
         self.Dp, self.Vp = _k(cfg.width), _up(cfg.vocab_size, 16)
-        self.plans = [_LayerPlan(spec, self.Dp) for spec in cfg.layers]
+        self._plan()
         self._raw: Optional[Dict[str, torch.Tensor]] = None
         self._handle = None
         self._weights: List[Any] = []
@@ -127,12 +153,17 @@ class HybridDecoder(IncrementalDecoder):
         if state_dict is not None:
             self.load_state_dict(state_dict)
 
+    def _plan(self):
+        self.plans = [_LayerPlan(spec, self.Dp) for spec in self.cfg.layers]
+        self.runs = self.cfg.runs()
+
     # ------------------------------------------------------------------ weights
     def load_state_dict(self, state_dict, strict=True, **kw):
         """Takes a checkpoint's tensors by name (``HybridConfig.tensor_shapes``)."""
-        shapes = self.cfg.tensor_shapes()
         sd = {k[len("decoder."):] if k.startswith("decoder.") else k: v
               for k, v in state_dict.items()}
+        cfg = self.cfg.with_shapes({k: tuple(v.shape) for k, v in sd.items()})
+        shapes = cfg.tensor_shapes()
         missing = [n for n in shapes if n not in sd]
         unexpected = [n for n in sd if n not in shapes]
         if missing or (strict and unexpected):
@@ -142,6 +173,8 @@ class HybridDecoder(IncrementalDecoder):
             if tuple(sd[n].shape) != tuple(shape):
                 raise ValueError("shape of %s: expected %s, got %s" % (n, shape, tuple(sd[n].shape)))
         self._drop()
+        self.cfg = self.args = cfg
+        self._plan()
         self._raw = {n: sd[n].detach() for n in shapes}
         return self
 
@@ -234,20 +267,66 @@ class HybridDecoder(IncrementalDecoder):
             t.w_gates = self._mat(gates.view(2 * nb * bp, bp), 2 * nb * bp, bp)
             t.gate_bias = self._hold(torch.cat([vec("mix.ra.b"), vec("mix.ri.b")]))
             t.w_out = self._mat(self._head_columns(w("mix.o"), nb, bs, bp), self.Dp, plan.ko)
+        elif isinstance(m, ParallelSpec):
+            self._fill_parallel(t, m, plan, w)
         else:
             H, Hk, dp, vp = m.heads, m.kv_heads, plan.dp, plan.vp
             t.kind, t.heads, t.kv_heads, t.taps = _capi.MSA_MIX_DELTA, H, Hk, m.conv
             t.dim, t.dp, t.vdim, t.vp = m.dim, dp, m.vdim, vp
-            split = [("mix.q", Hk, m.dim, dp), ("mix.k", Hk, m.dim, dp), ("mix.v", H, m.vdim, vp)]
-            rows = [self._heads(w(n), h, s, p) for n, h, s, p in split]
+            rows, conv = self._delta_rows(m, plan, w, "mix.")
             rows += [self._heads(w("mix.g"), H, m.vdim, vp)]
             rows += [w("mix.b").to(self.device), w("mix.a").to(self.device)]
             t.w_in = self._mat(torch.cat(rows), plan.n_in, self.Dp)
-            conv = torch.cat([self._heads(w(n + ".conv"), h, s, p) for n, h, s, p in split])
-            t.conv_w = self._hold(conv.float().t())
+            t.conv_w = self._hold(conv)
             t.decay_rate = self._hold(torch.exp(w("mix.A_log").to(self.device).float()))
             t.dt_bias, t.o_norm = self._vec(w("mix.dt_bias")), self._vec(w("mix.norm"), vp)
             t.w_out = self._mat(self._head_columns(w("mix.o"), H, m.vdim, vp), self.Dp, plan.ko)
+
+    def _delta_rows(self, m, plan, w, pre):
+        """q, k and v rows of a delta rule and its convolution's taps [taps, channels]."""
+        split = [("q", m.kv_heads, m.dim, plan.dp), ("k", m.kv_heads, m.dim, plan.dp),
+                 ("v", m.heads, m.vdim, plan.vp)]
+        conv = torch.cat([self._heads(w(pre + n + ".conv"), h, s, p) for n, h, s, p in split])
+        return [self._heads(w(pre + n), h, s, p) for n, h, s, p in split], conv.float().t()
+
+    def _fill_parallel(self, t, m, plan, w):
+        a, d, Dp = m.left, m.right, self.Dp
+        dev = lambda name: w("mix." + name).to(self.device)
+        t.kind, at = _capi.MSA_MIX_PARALLEL, t.att
+        at.heads, at.kv_heads, at.hd, at.vd = a.heads, a.kv_heads, plan.hd, plan.vd
+        at.chunk, at.rot_dims, at.ko, at.scale = a.chunk or 0, a.rot_dims, plan.kl, a.scale
+        i = torch.arange(a.rot_dims // 2, dtype=torch.float64)
+        if a.rot_dims:
+            at.inv_freq = self._hold(float(a.rot_base) ** (-2.0 * i / a.rot_dims))
+        at.w_out = self._mat(self._head_columns(dev("left.o"), a.heads, a.vdim, plan.vd), Dp, plan.kl)
+        t.heads, t.kv_heads, t.taps = d.heads, d.kv_heads, d.conv
+        t.dim, t.dp, t.vdim, t.vp = d.dim, plan.dp, d.vdim, plan.vp
+        # the inputs of every projection of the layer's input, in one matrix
+        split = [("left.q", a.heads, a.dim, plan.hd), ("left.k", a.kv_heads, a.dim, plan.hd),
+                 ("left.v", a.kv_heads, a.vdim, plan.vd)]
+        rows = [self._heads(dev(n), h, s, p) for n, h, s, p in split]
+        column = lambda name: dev(name).float().view(-1, 1)
+        bias = [self._heads(column(n + ".b"), h, s, p).view(-1) for n, h, s, p in split]
+        delta, conv = self._delta_rows(d, plan, w, "mix.right.")
+        low = torch.cat([dev("right.g1"), dev("right.a1")])
+        rows += delta + [_pad(low, plan.lr, low.shape[1]), dev("left.g"), dev("right.b")]
+        t.w_in = self._mat(torch.cat(rows), plan.n_in, Dp)
+        t.in_bias, t.conv_w = self._vec(torch.cat(bias), plan.n_in), self._hold(conv)
+        # gate and decays from the low-rank inputs, block-diagonal
+        H, dp, vp, rg, ra = d.heads, plan.dp, plan.vp, d.gate_rank, d.decay_rank
+        lr = torch.zeros(H * (vp + dp), plan.lr, dtype=dev("right.g2").dtype, device=self.device)
+        lr[:H * vp, :rg] = self._heads(dev("right.g2"), H, d.vdim, vp)
+        lr[H * vp:, rg:rg + ra] = self._heads(dev("right.a2"), H, d.dim, dp)
+        t.lr, t.w_lr = plan.lr, self._mat(lr, H * (vp + dp), plan.lr)
+        dt = self._heads(column("right.dt_bias"), H, d.dim, dp).view(-1)
+        t.lr_bias = self._hold(torch.cat([torch.zeros(H * vp, device=self.device), dt]))
+        rate = torch.exp(dev("right.A_log").float()).view(H, 1).expand(H, d.dim)
+        t.lr_rate = self._vec(rate, H, dp)
+        t.o_norm = self._vec(w("mix.right.norm"), vp)
+        t.w_out = self._mat(self._head_columns(dev("right.o"), H, d.vdim, vp), Dp, plan.ko)
+        # half of each side
+        at.out_norm = self._vec(0.5 * dev("left.out").float(), Dp)
+        t.out_norm = self._vec(0.5 * dev("right.out").float(), Dp)
 
     def _fill_feed_forward(self, t, spec, plan, w):
         f, Dp = spec.mlp, self.Dp
@@ -260,6 +339,12 @@ class HybridDecoder(IncrementalDecoder):
             t.ff_kind, t.ff = _capi.MSA_FF_DENSE, plan.ff
             t.w_ff_in = self._mat(self._pairs(dev("gate"), dev("up"), plan.ff), plan.n_ff, Dp)
             t.w_ff_down = self._mat(dev("down"), Dp, plan.ff)
+            return
+        if isinstance(f, SquaredReluSpec):
+            t.ff_kind, t.ff = _capi.MSA_FF_RELU2, plan.ff
+            t.w_ff_in, t.w_ff_down = self._mat(dev("up"), plan.ff, Dp), self._mat(dev("down"), Dp,
+                                                                                  plan.ff)
+            t.ff_bias, t.ff_down_bias = self._vec(dev("up.b"), plan.ff), self._vec(dev("down.b"), Dp)
             return
         r = f.router
         t.ff_kind, t.experts, t.top = _capi.MSA_FF_MOE, r.experts, r.top
@@ -304,7 +389,7 @@ class HybridDecoder(IncrementalDecoder):
             w = lambda name, pre="l%d." % i: raw[pre + name]
             self._fill_mixer(t, spec, plan, w)
             self._fill_feed_forward(t, spec, plan, w)
-            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if spec.mlp else ()):
+            for n in cfg.norm_names(spec):
                 setattr(t, n, self._vec(w(n), Dp))
         c = _capi.HybridConfigC()
         c.dtype = _capi.MSA_F32 if self.dtype == torch.float32 else _capi.MSA_BF16
@@ -313,10 +398,15 @@ class HybridDecoder(IncrementalDecoder):
         c.eps, c.embed_scale = cfg.norm_eps, cfg.embed_scale
         c.embed = self._hold(_pad(raw["embed"].to(self.device).to(torch.bfloat16),
                                   cfg.vocab_size, Dp))
-        i = torch.arange((D + 1) // 2, dtype=torch.float64)
-        c.inv_freq = self._hold(10000.0 ** (-2.0 * i / D))
+        if cfg.sinusoidal:
+            i = torch.arange((D + 1) // 2, dtype=torch.float64)
+            c.inv_freq = self._hold(10000.0 ** (-2.0 * i / D))
         c.final_norm = self._vec(raw["final.norm"], Dp)
-        c.head = self._mat(raw["head"], self.Vp, Dp)
+        c.head = self._mat(raw["embed" if cfg.tied else "head"], self.Vp, Dp)
+        tables = [(ctypes.c_int32 * len(self.runs))(*x) for x in zip(*self.runs)]
+        c.n_runs, (c.run_layer, c.run_pass) = len(self.runs), tables
+        if cfg.loop is not None:
+            c.loop_step = self._vec(raw["loop.step"], cfg.loop.times, Dp)
         handle = ctypes.c_void_p()
         check(lib.msa_hybrid_create(ctypes.byref(c), table, ctypes.byref(handle)), lib)
         self._handle = handle
@@ -327,7 +417,7 @@ class HybridDecoder(IncrementalDecoder):
         return self.max_target_positions
 
     def _new_cache(self, slots, capacity):
-        return HybridCache([p.keep for p in self.plans], slots, capacity, self.dtype, self.device)
+        return HybridCache([self.plans[i].keep for i, _ in self.runs], slots, capacity, self.dtype, self.device)
 
     def new_slot_cache(self, slots: int, capacity: int, device=None) -> HybridCache:
         """An empty cache of ``slots`` rows and ``capacity`` positions each."""
@@ -344,6 +434,8 @@ class HybridDecoder(IncrementalDecoder):
             table = (_capi.HybridState * len(cache.layers))()
             for s, t in zip(table, cache.layers):
                 s.latent, s.conv, s.rec = ptr(t.get("latent")), ptr(t.get("conv")), ptr(t.get("rec"))
+                if "keys" in t:
+                    s.keys, s.values, s.kv_rows = ptr(t["keys"]), ptr(t["values"]), t["keys"].shape[2]
             kept = cache._table = (key, table)
         return kept[1]
 
@@ -361,7 +453,7 @@ class HybridDecoder(IncrementalDecoder):
             logits = torch.empty(n, self.Vp, dtype=torch.float32, device=self.device)
             a.rows, a.n_rows, a.logits = ptr(rows), n_rows, logits.data_ptr()
         if self.layer_probe is not None:
-            probe = torch.empty(len(self.plans), batch.M, self.Dp, dtype=torch.float32,
+            probe = torch.empty(len(self.runs), batch.M, self.Dp, dtype=torch.float32,
                                 device=self.device)
             a.probe = probe.data_ptr()
         need = lib.msa_hybrid_workspace_bytes(self._handle, ctypes.byref(a))
@@ -372,7 +464,7 @@ class HybridDecoder(IncrementalDecoder):
         a.workspace, a.workspace_bytes = self._workspace.data_ptr(), self._workspace.numel()
         check(lib.msa_hybrid_step(self._handle, ctypes.byref(a), _capi.stream_ptr()), lib)
         if probe is not None:
-            for i in range(len(self.plans)):
+            for i in range(len(self.runs)):
                 self.layer_probe(i, probe[i, :, :self.cfg.width])
         return None if logits is None else logits[:, :self.cfg.vocab_size]
 

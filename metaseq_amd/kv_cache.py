@@ -91,8 +91,12 @@ class HybridCache:
     """What the layers of a hybrid decoder keep per slot (a row of a batch, or a serving slot):
 
     * attention layers that own a latent: ``latent`` [slots, capacity, rank], activation format;
+    * attention layers with keys and values: ``keys`` and ``values`` [slots, kv_heads, rows, size],
+      activation format; rows is the capacity, or one chunk where attention stays within chunks;
     * recurrent layers: ``conv`` [slots, taps - 1, channels], the short convolution's last inputs
       (activation format), and ``rec``, the fp32 recurrent state.
+
+    A layer that runs several times keeps that much for each of its runs.
 
     ``lens`` (int32 [slots] on the device): positions each slot holds, negative = empty slot;
     ``host_lens``: the same on the host where the caller of the slot interface knows it.  Nothing
@@ -103,8 +107,9 @@ class HybridCache:
     ragged = True
 
     def __init__(self, layout, slots, capacity, dtype, device):
-        """``layout``: per layer {"latent": rank} and / or {"conv": (taps - 1, channels), "rec":
-        shape} (what the layer keeps; an empty dict: nothing)."""
+        """``layout``: per run of a layer {"latent": rank}, {"keys": size, "values": size,
+        "kv_heads": n, "chunk": positions or None}, {"conv": (taps - 1, channels), "rec": shape}
+        or several of them (what the layer keeps; an empty dict: nothing)."""
         self.layout, self.batch, self.capacity = layout, int(slots), int(capacity)
         self.dtype, self.device = dtype, device
         self.length = 0
@@ -116,6 +121,11 @@ class HybridCache:
             if "latent" in keep:
                 t["latent"] = torch.zeros(self.batch, self.capacity, keep["latent"], dtype=dtype,
                                           device=device)
+            for name in ("keys", "values"):
+                if name in keep:
+                    t[name] = torch.zeros(self.batch, keep["kv_heads"],
+                                          self.kept_rows(keep, self.capacity), keep[name],
+                                          dtype=dtype, device=device)
             if "rec" in keep:
                 t["rec"] = torch.zeros((self.batch,) + tuple(keep["rec"]), dtype=torch.float32,
                                        device=device)
@@ -124,12 +134,26 @@ class HybridCache:
                                         device=device)
             self.layers.append(t)
 
+    @staticmethod
+    def kept_rows(keep, capacity):
+        """Positions whose keys and values a slot of that capacity keeps."""
+        return min(capacity, keep["chunk"]) if keep.get("chunk") else capacity
+
     def grow(self, new_capacity):
-        """Re-allocates the latents to ``new_capacity`` positions per slot."""
+        """Re-allocates latents, keys and values to ``new_capacity`` positions per slot."""
         new_capacity = int(new_capacity)
         if new_capacity <= self.capacity:
             return
-        for t in self.layers:
+        for keep, t in zip(self.layout, self.layers):
+            for name in ("keys", "values"):
+                if name not in t or self.kept_rows(keep, new_capacity) == t[name].shape[2]:
+                    continue
+                old = t[name]
+                new = torch.zeros(old.shape[:2] + (self.kept_rows(keep, new_capacity),
+                                                   old.shape[3]), dtype=self.dtype,
+                                  device=self.device)
+                new[:, :, :old.shape[2]].copy_(old)
+                t[name] = new
             if "latent" in t:
                 old = t["latent"]
                 new = torch.zeros(self.batch, new_capacity, old.shape[2], dtype=self.dtype,
@@ -144,6 +168,8 @@ class HybridCache:
             for name, x in t.items():
                 if name == "latent":
                     x[dst, :n].copy_(x[src, :n])
+                elif name in ("keys", "values"):
+                    x[dst, :, :n].copy_(x[src, :, :n])
                 else:
                     x[dst].copy_(x[src])
         self.host_lens[dst] = n

@@ -29,6 +29,8 @@ ARCHITECTURES: Dict[str, Architecture] = {
     "OPT": Architecture(OPTConfig, _opt_config, TransformerDecoder, (torch.float16,)),
     "Sinulorn": Architecture(HybridConfig, HybridConfig.from_json, HybridDecoder,
                              (torch.bfloat16, torch.float32)),
+    "Nomalorn": Architecture(HybridConfig, HybridConfig.from_json, HybridDecoder,
+                             (torch.bfloat16, torch.float32)),
 }
 
 

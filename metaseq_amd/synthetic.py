@@ -84,7 +84,7 @@ def random_hybrid_state_dict(cfg: HybridConfig, seed: int = 1234, dtype=torch.bf
     for name, shape in cfg.tensor_shapes().items():
         t = torch.empty(*shape, dtype=torch.float32, device=device)
         last = name.rsplit(".", 1)[-1]
-        if last.startswith("norm"):
+        if last.startswith("norm") or last == "out":
             t.normal_(1.0, 0.1, generator=gen)
         elif last == "embed":
             t.normal_(0.0, 1.0, generator=gen)
@@ -94,7 +94,9 @@ def random_hybrid_state_dict(cfg: HybridConfig, seed: int = 1234, dtype=torch.bf
             t.uniform_(-3.0, 0.5, generator=gen)
         elif last == "conv":
             t.normal_(0.0, shape[-1] ** -0.5, generator=gen)
-        elif last == "b" and len(shape) < 3 and not name.endswith("mix.b"):
+        elif last == "step":
+            t.normal_(0.0, 0.3, generator=gen)
+        elif last == "b" and len(shape) < 3 and not name.endswith(("mix.b", "right.b")):
             t.normal_(0.0, 0.3, generator=gen)
         else:
             t.normal_(0.0, shape[-1] ** -0.5, generator=gen)

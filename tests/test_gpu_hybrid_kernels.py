@@ -254,13 +254,16 @@ def _batch(segments, M):
 @pytest.mark.parametrize("heads,kv_heads,dim,dp,vp,counts", [
     (4, 2, 30, 32, 48, (5, 1, 40)), (3, 3, 128, 128, 64, (17, 16)), (2, 1, 250, 256, 32, (33,)),
     (32, 8, 64, 64, 64, (9, 2, 1, 30, 16, 17, 3, 4)),      # eight lanes per column
-    (64, 64, 128, 128, 32, (7, 20, 1, 2, 1, 1, 1, 1)), (32, 16, 96, 96, 64, (5,) * 8)])
+    (64, 64, 128, 128, 32, (7, 20, 1, 2, 1, 1, 1, 1)), (32, 16, 96, 96, 64, (5,) * 8),
+    (6, 3, 90, 96, 80, (1, 1, 1)), (3, 1, 128, 128, 208, (1,) * 5)])
+@pytest.mark.parametrize("channels", [False, True], ids=["head decays", "channel decays"])
 @pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
-def test_delta_scan(heads, kv_heads, dim, dp, vp, counts, dtype):
+def test_delta_scan(heads, kv_heads, dim, dp, vp, counts, dtype, channels):
     """Several segments, one of them continuing its slot's state and (with three or more) one
-    inactive; outputs and the states left behind."""
+    inactive; outputs and the states left behind.  Segments of one token each also through the
+    one-launch step."""
     lib = _capi.load_hybrid()
-    print("delta_scan", heads, kv_heads, dim, dp, vp, counts, flush=True)
+    print("delta_scan", heads, kv_heads, dim, dp, vp, counts, channels, flush=True)
     g = gen(heads + dp)
     M, slots = sum(counts), len(counts) + 1
     C = 2 * kv_heads * dp + heads * vp
@@ -269,6 +272,7 @@ def test_delta_scan(heads, kv_heads, dim, dp, vp, counts, dtype):
     qkv = qkv.to(dtype)
     ba = torch.randn(M, 2 * heads + 3, generator=g)
     rate, dtb = torch.rand(heads, generator=g) * 0.3, torch.randn(heads, generator=g)
+    decays = torch.rand(M, heads, dp, generator=g) ** 0.25
     state = torch.randn(slots, heads, vp, dp, generator=g)
     state[..., dim:] = 0
     segs = [(slots - 1 - i, 0 if i else 12, n) for i, n in enumerate(counts)]
@@ -290,18 +294,40 @@ def test_delta_scan(heads, kv_heads, dim, dp, vp, counts, dtype):
                 beta = torch.sigmoid(z[:heads])
                 decay = torch.exp(-rate.double() * torch.nn.functional.softplus(
                     z[heads:2 * heads] + dtb.double()))
-                s = s * decay.view(-1, 1, 1)
+                s = s * (decays[m].double().unsqueeze(1) if channels else decay.view(-1, 1, 1))
                 u = beta.view(-1, 1) * (v - torch.einsum("hvd,hd->hv", s, k))
                 s = s + u.unsqueeze(2) * k.unsqueeze(1)
                 want[m] = torch.einsum("hvd,hd->hv", s, q)
             S[slot] = s
         at += n
     b, alive = _batch(segs, M)
-    qd, bd, rd, td, sd = (t.cuda() for t in (qkv, ba, rate, dtb, state))
+    qd, bd, rd, td, sd, dd = (t.cuda() for t in (qkv, ba, rate, dtb, state, decays))
     o = torch.full((M, heads * vp), 7.0, device="cuda")
-    check(lib.msa_delta_scan(0 if dtype == BF16 else 1, ptr(qd), C, ptr(bd), 2 * heads + 3, ptr(rd),
-                             ptr(td), heads, kv_heads, dim, dp, vp, ptr(sd), ptr(o), ctypes.byref(b),
-                             _capi.stream_ptr()), lib)
+    a = _capi.DeltaArgs()
+    a.dtype, a.heads, a.kv_heads, a.dim, a.dp, a.vp = int(dtype == F32), heads, kv_heads, dim, dp, vp
+    a.qkv, a.ld, a.ba, a.ldba, a.state, a.o = ptr(qd), C, ptr(bd), 2 * heads + 3, ptr(sd), ptr(o)
+    if channels:
+        a.decay = ptr(dd)
+    else:
+        a.decay_rate, a.dt_bias = ptr(rd), ptr(td)
+    if b.max_count == 1:
+        step = state.cuda()
+        out = torch.zeros(M, heads * vp, dtype=dtype, device="cuda")
+        gate, w = torch.randn(M, heads * vp, generator=g).to(dtype), torch.randn(vp, generator=g)
+        gd, wd = gate.cuda(), w.cuda()
+        a.state, a.vdim, a.gate, a.ld_gate, a.w = ptr(step), vp, ptr(gd), heads * vp, ptr(wd)
+        a.out, a.ld_out, a.eps = ptr(out), heads * vp, 1e-5
+        for act, f in ((_capi.MSA_GATE_SILU, torch.nn.functional.silu),
+                       (_capi.MSA_GATE_SIGMOID, torch.sigmoid)):
+            step.copy_(state)
+            a.gate_act = act
+            check(lib.msa_delta_step(ctypes.byref(a), ctypes.byref(b), _capi.stream_ptr()), lib)
+            normed = O.rms(want, 1e-5, w.double()) * f(gate.double()).view(M, heads, vp)
+            on = [m for m in range(M) if segs[m][1] >= 0]
+            close(out.view(M, heads, vp)[on], normed[on], 2e-5 if dtype == F32 else 6e-3, "step")
+            close(step, S, 2e-5, "states of the step")
+        a.state = ptr(sd)
+    check(lib.msa_delta_scan(ctypes.byref(a), ctypes.byref(b), _capi.stream_ptr()), lib)
     close(o.view(M, heads, vp), want, 2e-5, "outputs")
     close(sd, S, 2e-5, "states")
     del alive

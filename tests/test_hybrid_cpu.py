@@ -211,7 +211,9 @@ def test_hybrid_library_exports_and_binding_match_the_header():
 @pytest.mark.skipif(shutil.which("gcc") is None, reason="needs a C compiler")
 def test_structures_match_the_header(tmp_path):
     pairs = {"msa_batch": _capi.Batch, "msa_group_linear_args": _capi.GroupLinearArgs,
-             "msa_tail_args": _capi.TailArgs, "msa_hybrid_layer": _capi.HybridLayer,
+             "msa_tail_args": _capi.TailArgs, "msa_linear_args": _capi.LinearArgs,
+             "msa_delta_args": _capi.DeltaArgs, "msa_grouped_args": _capi.GroupedArgs,
+             "msa_attention_layer": _capi.AttentionLayer, "msa_hybrid_layer": _capi.HybridLayer,
              "msa_hybrid_config": _capi.HybridConfigC, "msa_hybrid_state": _capi.HybridState,
              "msa_hybrid_step_args": _capi.HybridStepArgs}
     lines, want = [], []
@@ -244,8 +246,27 @@ def test_arguments_are_checked_before_anything_is_launched():
     a = _capi.GroupLinearArgs()
     assert lib.msa_group_linear(ctypes.byref(a), None) == -1
     b = _capi.Batch()
-    assert lib.msa_delta_scan(0, one, 64, one, 8, one, one, 4, 3, 32, 32, 32, one, one,
-                              ctypes.byref(b), None) == -1
+    b.M = b.nseg = b.max_count = 1
+    d = _capi.DeltaArgs()
+    d.qkv = d.ba = d.decay_rate = d.dt_bias = d.state = d.o = 4096
+    d.ld, d.ldba, d.heads, d.kv_heads, d.dim, d.dp, d.vp = 64, 8, 4, 3, 32, 32, 32
+    assert lib.msa_delta_scan(ctypes.byref(d), ctypes.byref(b), None) == -1
+    assert b"kv_heads=3" in lib.msa_last_error()
+    g = _capi.GroupedArgs()
+    g.q = g.k = g.v = g.k_cache = g.v_cache = g.out = 4096
+    g.ld, g.heads, g.kv_heads, g.hd, g.vd, g.rows, g.scale, g.splits = 256, 2, 1, 64, 64, 8, 1.0, 1
+    for field, bad in (("rot_dims", 3), ("rot_dims", 66), ("rows", 0), ("hd", 60), ("kv_heads", 3)):
+        kept = getattr(g, field)
+        setattr(g, field, bad)
+        assert lib.msa_grouped_append(ctypes.byref(g), ctypes.byref(b), None) == -1, field
+        setattr(g, field, kept)
+    for seg0, seg1, longest in ((0, 0, 1), (0, 2, 1), (0, 1, 2), (-1, 1, 1)):
+        assert lib.msa_grouped_attention(ctypes.byref(g), ctypes.byref(b), seg0, seg1, longest,
+                                         None) == -1
+    x = _capi.LinearArgs()
+    x.x = x.W = x.y = 4096
+    x.M, x.N, x.K, x.n32, x.act = 4, 64, 128, 64, 7
+    assert lib.msa_linear(ctypes.byref(x), None) == -1
     cfg = _capi.HybridConfigC()
     h = ctypes.c_void_p()
     table = (_capi.HybridLayer * 1)()
