@@ -394,13 +394,16 @@ HYBRID_STACKS = {
     "delta + dense": [("delta", "dense")] * 4,
     "latent + moe": [("latent", "moe")] * 4,
     "mixed": [("rglru", "dense"), ("latent", "moe"), ("delta", "dense"), ("latent-borrowed", "moe")],
+    # three layers, the middle one twice
+    "parallel + relu2 (Nomalorn)": [("parallel", "relu2")] * 3,
 }
 
 
 def hybrid_config(width, stack, vocab=50272):
     """A hybrid decoder of a real model's layer sizes at this width: heads of 128, a latent of
-    512, gate blocks of 256, 64 experts of which 8 run, and a dense feed-forward of as many
-    weights as OPT's 4 x width."""
+    512, gate blocks of 256, 64 experts of which 8 run, a dense feed-forward of as many weights as
+    OPT's 4 x width; beside the delta rule, attention with four query heads per key/value head
+    within chunks of 8192 positions."""
     from metaseq_amd import HybridConfig
     heads = width // 128
 
@@ -411,11 +414,19 @@ def hybrid_config(width, stack, vocab=50272):
             if kind.endswith("borrowed"):
                 m["kv_from"] = 1
             return "latent_attention", m
+        if kind == "parallel":
+            left = dict(heads=heads, kv_heads=max(1, heads // 4), dim=128, vdim=128,
+                        scale=128 ** -0.5, rot=dict(base=500000.0, dims=64), mask=dict(size=8192))
+            right = dict(heads=heads, kv_heads=heads // 2, dim=128, vdim=128, conv=4,
+                         decay_rank=128, gate_rank=128)
+            return kind, dict(left=left, right=right)
         if kind == "rglru":
             return kind, dict(width=width, blocks=width // 256, conv=4)
         return kind, dict(heads=heads, kv_heads=heads // 2, dim=128, vdim=128, conv=4)
 
     def mlp(kind):
+        if kind == "relu2":
+            return dict(kind="dense", ff=4 * width)
         if kind == "dense":
             return dict(kind=kind, ff=(8 * width // 3 + 63) // 64 * 64)
         ff = 11 * width // 32 // 64 * 64
@@ -425,12 +436,14 @@ def hybrid_config(width, stack, vocab=50272):
     for i, (m, f) in enumerate(HYBRID_STACKS[stack]):
         kind, sizes = mixer(m, i)
         layers.append(dict(type=kind, mixer=sizes, mlp=mlp(f)))
+    looped = HYBRID_STACKS[stack][0][0] == "parallel"
+    design = dict(architecture="Nomalorn", loop=dict(start=1, stop=2, times=2)) if looped else {}
     return HybridConfig.from_json(dict(width=width, vocab=vocab, layers=layers,
-                                       norm=dict(eps=1e-6), embedding=dict(scale=1.0)))
+                                       norm=dict(eps=1e-6), **design))
 
 
 def hybrid_throughput(width, only=None, prompt=1024, steps=20, warmup=5):
-    """Prefill and decode throughput of hybrid decoders (random weights, bf16) of four layers at
+    """Prefill and decode throughput of hybrid decoders (random weights, bf16) of four layer runs at
     one width, beside OPT layers of that width and number of weights (fp16), all driven through
     the slot interface: a prefill of 8 prompts in one step, decode steps of 1, 32 and 128 rows
     that each hold the prompt."""

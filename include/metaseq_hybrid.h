@@ -201,14 +201,18 @@ typedef struct {
   void* out; int64_t ldo; int out_mb;
   float* partial;         /* splits > 1: [M][heads][splits][vd + 4] */
   int splits;
+  int fused;              /* the attention kernel rotates and appends (msa_grouped_fuses) */
 } msa_grouped_args;
 /* rotates q and k in place; where every segment holds one token, also appends keys and values */
 int msa_grouped_rotate(const msa_grouped_args* a, const msa_batch* b, void* stream);
 /* appends the keys and values of every segment's last chunk (nothing where msa_grouped_rotate did) */
 int msa_grouped_append(const msa_grouped_args* a, const msa_batch* b, void* stream);
 int msa_grouped_attention_splits(const msa_grouped_args* a, int M, int key_bound);
+/* whether msa_grouped_attention can take rotation and appending over for this batch: with `fused` set, the
+ * other two calls fall away */
+int msa_grouped_fuses(const msa_grouped_args* a, const msa_batch* b);
 /* The outputs of segments seg0 .. seg1 - 1: all of them of one token each (longest == 1), or of any size up
- * to `longest`, after msa_grouped_rotate and before msa_grouped_append.  Head sizes: fp32, and bf16 beyond
+ * to `longest`, after msa_grouped_rotate and before msa_grouped_append (unless fused).  Head sizes: fp32, and bf16 beyond
  * 256, up to 1024; bf16 64, 128, 192 or 256. */
 int msa_grouped_attention(const msa_grouped_args* a, const msa_batch* b, int seg0, int seg1, int longest,
                           void* stream);
@@ -252,7 +256,8 @@ typedef struct {
   int heads, kv_heads, hd, vd, chunk, rot_dims, ko;
   float scale;
   const double* inv_freq; /* device, [rot_dims / 2] */
-  const void* w_out;      /* [Dp, ko] */
+  const void* w_out;      /* [Dp, ko]; NULL where both sides' ko are equal: the layer's w_out is
+                             [Dp, 2 ko], this side's columns behind the delta rule's */
   const float* out_norm;  /* [Dp] */
 } msa_attention_layer;
 

@@ -151,7 +151,7 @@ GroupedArgs = _struct(
     "GroupedArgs", "msa_grouped_args", (c_int, "dtype heads kv_heads hd vd chunk rot_dims rows"),
     (c_float, "scale"), (c_void_p, "inv_freq q k v"), (c_int64, "ld"),
     (c_void_p, "k_cache v_cache gate"), (c_int, "ld_gate"), (c_void_p, "out"), (c_int64, "ldo"),
-    (c_int, "out_mb"), (c_void_p, "partial"), (c_int, "splits"))
+    (c_int, "out_mb"), (c_void_p, "partial"), (c_int, "splits fused"))
 AttentionLayer = _struct(
     "AttentionLayer", "msa_attention_layer", (c_int, "heads kv_heads hd vd chunk rot_dims ko"),
     (c_float, "scale"), (c_void_p, "inv_freq w_out out_norm"))
@@ -202,6 +202,7 @@ HYBRID_SIGNATURES = {
     "msa_grouped_rotate": [ctypes.POINTER(GroupedArgs), _BP, _P],
     "msa_grouped_append": [ctypes.POINTER(GroupedArgs), _BP, _P],
     "msa_grouped_attention_splits": [ctypes.POINTER(GroupedArgs), c_int, c_int],
+    "msa_grouped_fuses": [ctypes.POINTER(GroupedArgs), _BP],
     "msa_grouped_attention": [ctypes.POINTER(GroupedArgs), _BP, c_int, c_int, c_int, _P],
     "msa_latent_norm": [c_int, _P, c_int, c_int, c_int, c_int, c_int, _P, c_int, c_int, _P,
                         c_float, _P, c_int, _P, c_int, _BP, _P],

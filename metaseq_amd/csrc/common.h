@@ -111,8 +111,15 @@ __device__ __forceinline__ float relu2(float z) {
   z = fmaxf(z, 0.f);
   return z * z;
 }
-// decay of a recurrent state from its logit
-__device__ __forceinline__ float decay_of(float z, float rate) { return expf(-rate * softplus(z)); }
+// Decay of a recurrent state from its logit, exp(-rate softplus(z)), on the hardware's exponential and
+// logarithm: softplus(z) = max(z, 0) + log(1 + t), t = exp(-|z|) <= 1, and log(1 + t) = t log(u) / (u - 1) with
+// the rounded u = 1 + t, which keeps the small values' relative accuracy.
+__device__ __forceinline__ float decay_of(float z, float rate) {
+  constexpr float LN2 = 0.6931471805599453f, L2E = 1.4426950408889634f;
+  const float t = __builtin_amdgcn_exp2f(-fabsf(z) * L2E), u = 1.f + t, d = u - 1.f;
+  const float l = d > 0.f ? __builtin_amdgcn_logf(u) * LN2 * t * __builtin_amdgcn_rcpf(d) : t;
+  return __builtin_amdgcn_exp2f(-rate * (fmaxf(z, 0.f) + l) * L2E);
+}
 
 // (max, sum of exp(z - max)) pairs merge associatively: one pass over a row suffices
 __device__ __forceinline__ void lse_merge(float& m, float& s, float om, float os) {

@@ -6,7 +6,8 @@
 //    several chunks and overwrite the one that its first tokens still needed.
 //  * One new token per sequence (decode): the heads of a group are the columns of the MFMA tiles, a
 //    wave owns 32 keys at a time straight from memory, and the four waves of a workgroup (and its
-//    splits) merge their sums at the end.  Bound: the keys and values from HBM, once per 16 heads.
+//    splits) merge their sums at the end.  Rotation and appending are part of it.  Bound: the keys and
+//    values from HBM, once per 16 heads.
 //  * Several: 128 queries of one head per workgroup over key tiles of 64, one pass (see
 //    flash_attention_kernel, which this follows, in latent_attention.hip).
 //  * fp32, and heads of more than 256: one workgroup per (token, head) on the vector ALU.
@@ -31,6 +32,13 @@ struct Vec8 {
   typedef T type __attribute__((ext_vector_type(8), aligned(16)));
 };
 
+// sine and cosine of pos * inv_freq; the angle in turns, reduced to [-1/2, 1/2] in double
+__device__ __forceinline__ void rotary_angle(int pos, double inv_freq, float& s, float& c) {
+  double turns = (double)pos * inv_freq * 0.15915494309189535;
+  turns -= rint(turns);
+  sincospif(2.f * (float)turns, &s, &c);
+}
+
 // ---- rotary positions, appending ---------------------------------------------------------------
 // One workgroup per token; V pairs of a head per thread.
 template <typename T, int V>
@@ -44,12 +52,7 @@ __global__ __launch_bounds__(256) void rotate_kernel(msa_grouped_args a,
   T* q = (T*)a.q + m * a.ld;
   T* k = (T*)a.k + m * a.ld;
   if (half > 0) {
-    for (int i = tid; i < half; i += 256) {
-      // the angle in turns, reduced to [-1/2, 1/2] in double
-      double turns = (double)pos * a.inv_freq[i] * 0.15915494309189535;
-      turns -= rint(turns);
-      sincospif(2.f * (float)turns, &sn[i], &cs[i]);
-    }
+    for (int i = tid; i < half; i += 256) rotary_angle(pos, a.inv_freq[i], sn[i], cs[i]);
     __syncthreads();
     typedef T tv __attribute__((ext_vector_type(V), aligned(V * sizeof(T) < 16 ? V * sizeof(T) : 16)));
     const int per = half / V, total = (a.heads + a.kv_heads) * per;
@@ -118,17 +121,23 @@ __global__ __launch_bounds__(256) void append_kernel(msa_grouped_args a,
 // ---- one new token per sequence, bf16 -----------------------------------------------------------
 template <int VD>
 constexpr int gd_pitch = VD * 2 + 16;
-template <int VD>
-constexpr int gd_lds_bytes = 4 * 32 * gd_pitch<VD>;
-
+template <int HD>
+constexpr int gd_row = HD + 8;  // elements between two staged heads
 template <int HD, int VD>
+constexpr int gd_lds_bytes = 4 * 32 * gd_pitch<VD> + 17 * gd_row<HD> * 2;
+
+// FUSED: q and k come as the projection left them; the workgroup rotates its heads, and the first
+// of a group's workgroups appends.
+template <int HD, int VD, bool FUSED>
 __global__ __launch_bounds__(256) void grouped_decode_kernel(msa_grouped_args a, int r0, int M,
                                                              const int32_t* __restrict__ tok_slot,
                                                              const int32_t* __restrict__ tok_pos,
                                                              float scale_log2) {
   constexpr int KS = HD / 32, DW = VD / 16, PITCH = gd_pitch<VD>, CH = VD / 8, VL = 32 * CH / 64;
+  constexpr int ROW = gd_row<HD>, QCH = HD / 8, QL = (17 * QCH + 255) / 256;
   extern __shared__ __attribute__((aligned(16))) char lds[];  // per wave: values of 32 keys; sums
-  __shared__ float sm[4][16], sl[4][16];
+  __shared__ float sm[4][16], sl[4][16], cs[HD / 2], sn[HD / 2];
+  bf16_t* lq = reinterpret_cast<bf16_t*>(lds + 4 * 32 * PITCH);  // 16 heads, the own key
   const int per = a.heads / a.kv_heads, HB = (per + 15) / 16;
   int idx = blockIdx.x;
   const int split = idx % a.splits;
@@ -140,17 +149,23 @@ __global__ __launch_bounds__(256) void grouped_decode_kernel(msa_grouped_args a,
   const int64_t m = r0 + mr;
   const int tid = threadIdx.x, lane = tid & 63, hc = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int head = g * per + min(hb * 16 + hc, per - 1);
+  const bf16_t* own_k = (const bf16_t*)a.k + m * a.ld + g * HD;
+  const bf16_t* own_v = (const bf16_t*)a.v + m * a.ld + g * VD;
+  half8_t qr[QL];  // the heads' and the own key's elements on their way to LDS
+#pragma unroll
+  for (int i = 0; i < QL; ++i) {
+    const int e = min(tid + 256 * i, 17 * QCH - 1), r = e / QCH;
+    const bf16_t* p = r == 16 ? own_k
+                              : (const bf16_t*)a.q + m * a.ld + (g * per + min(hb * 16 + r, per - 1)) * HD;
+    qr[i] = *reinterpret_cast<const half8_t*>(p + (e % QCH) * 8);
+  }
   const int pos = tok_pos[m];
-  const int n_keys = pos < 0 ? 0 : pos - chunk_start(pos, a.chunk) + 1;
+  const int n_keys = pos < 0 ? 0 : pos - chunk_start(pos, a.chunk);  // in the cache
   const int len = split_keys(n_keys, a.splits);
   const int k_begin = split * len, k_end = min(n_keys, k_begin + len);
   const int64_t slot = (int64_t)tok_slot[m] * a.kv_heads + g;
-  const bf16_t* kc = (const bf16_t*)a.k_cache + slot * a.rows * HD;
-  const bf16_t* vc = (const bf16_t*)a.v_cache + slot * a.rows * VD;
-  // the token's own key and value are the last
-  const bf16_t* own_k = (const bf16_t*)a.k + m * a.ld + g * HD;
-  const bf16_t* own_v = (const bf16_t*)a.v + m * a.ld + g * VD;
+  bf16_t* kc = (bf16_t*)a.k_cache + slot * a.rows * HD;
+  bf16_t* vc = (bf16_t*)a.v_cache + slot * a.rows * VD;
 
   struct Tile {
     bf16x8_t k[2][KS];
@@ -159,35 +174,75 @@ __global__ __launch_bounds__(256) void grouped_decode_kernel(msa_grouped_args a,
   auto fetch = [&](Tile& t, int base) {
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-      const int i = min(base + 16 * b + hc, n_keys - 1);
-      const bf16_t* p = (i == n_keys - 1 ? own_k : kc + (int64_t)i * HD) + lg * 8;
+      const bf16_t* p = kc + (int64_t)min(base + 16 * b + hc, n_keys - 1) * HD + lg * 8;
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) t.k[b][ks] = *reinterpret_cast<const bf16x8_t*>(p + ks * 32);
     }
 #pragma unroll
     for (int j = 0; j < VL; ++j) {
-      const int c = lane + 64 * j, i = min(base + c / CH, n_keys - 1);
-      const bf16_t* p = i == n_keys - 1 ? own_v : vc + (int64_t)i * VD;
-      t.v[j] = *reinterpret_cast<const half8_t*>(p + (c % CH) * 8);
+      const int c = lane + 64 * j;
+      t.v[j] = __builtin_nontemporal_load(reinterpret_cast<const half8_t*>(
+          vc + (int64_t)min(base + c / CH, n_keys - 1) * VD + (c % CH) * 8));
     }
   };
-  bf16x8_t qf[KS];
-  {
-    const bf16_t* p = (const bf16_t*)a.q + m * a.ld + head * HD + lg * 8;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8_t*>(p + ks * 32);
-  }
   int base = k_begin + 32 * wave;  // the wave's tiles are 128 keys apart
+#pragma unroll
+  for (int i = 0; i < QL; ++i)
+    if (tid + 256 * i < 17 * QCH)
+      *reinterpret_cast<half8_t*>(lq + (tid + 256 * i) / QCH * ROW + (tid + 256 * i) % QCH * 8) = qr[i];
   if (base < k_end) {
     fetch(t0, base);
     fetch(t1, base + 128);  // past the end: the last key again
   }
+  if constexpr (FUSED) {
+    const int half = a.rot_dims / 2;
+    for (int i = tid; i < half; i += 256) rotary_angle(pos, a.inv_freq[i], sn[i], cs[i]);
+    lds_barrier();
+    for (int e = tid; e < 17 * half; e += 256) {
+      const int r = e / half, i = e - r * half;
+      bf16_t* p = lq + r * ROW + i;
+      const float x = (float)p[0], y = (float)p[half];
+      p[0] = (bf16_t)(x * cs[i] - y * sn[i]);
+      p[half] = (bf16_t)(y * cs[i] + x * sn[i]);
+    }
+  }
+  lds_barrier();
+  bf16x8_t qf[KS];
 #pragma unroll
-  for (int ks = 0; ks < KS; ++ks) asm volatile("" : "+v"(qf[ks]));  // arrived in front of the loop
+  for (int ks = 0; ks < KS; ++ks)
+    qf[ks] = *reinterpret_cast<const bf16x8_t*>(lq + hc * ROW + ks * 32 + lg * 8);
+  if (FUSED && split == 0 && hb == 0 && pos >= 0 && n_keys < a.rows) {
+    for (int e = tid; e < QCH + CH; e += 256)
+      if (e < QCH)
+        *reinterpret_cast<half8_t*>(kc + (int64_t)n_keys * HD + e * 8) =
+            *reinterpret_cast<const half8_t*>(lq + 16 * ROW + e * 8);
+      else
+        *reinterpret_cast<half8_t*>(vc + (int64_t)n_keys * VD + (e - QCH) * 8) =
+            *reinterpret_cast<const half8_t*>(own_v + (e - QCH) * 8);
+  }
   float4_t o[DW];
 #pragma unroll
   for (int d = 0; d < DW; ++d) o[d] = float4_t{0.f, 0.f, 0.f, 0.f};
   float mx = -INFINITY, l = 0.f;
+  if (split == 0 && wave == 0 && pos >= 0) {  // the token's own key, which every head sees
+    float s = 0.f;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bf16x8_t k = *reinterpret_cast<const bf16x8_t*>(lq + 16 * ROW + ks * 32 + lg * 8);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s = fmaf((float)k[i], (float)qf[ks][i], s);
+    }
+    s += __shfl_xor(s, 16, MSA_WAVE);
+    s += __shfl_xor(s, 32, MSA_WAVE);
+    mx = s * scale_log2;
+    l = lg == 0 ? 1.f : 0.f;  // the lane groups are summed at the end
+#pragma unroll
+    for (int d = 0; d < DW; ++d) {
+      const bf16x4_t v = *reinterpret_cast<const bf16x4_t*>(own_v + 16 * d + 4 * lg);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[d][r] = (float)v[r];
+    }
+  }
   char* mine = lds + wave * 32 * PITCH;
   const char* tr = mine + (4 * lg + (hc >> 2)) * PITCH + (hc & 3) * 8;
   auto tile = [&](Tile& t, int k0) {
@@ -284,30 +339,40 @@ __global__ __launch_bounds__(256) void grouped_decode_kernel(msa_grouped_args a,
   }
 }
 
-// sums the splits of one (token, head)
+// sums the splits (at most 64) of one (token, head): lane s weighs split s
 __global__ __launch_bounds__(64) void grouped_combine_kernel(msa_grouped_args a, int r0) {
   const int64_t row = blockIdx.x;
   const int64_t m = r0 + row / a.heads;
-  const int h = (int)(row % a.heads), vd = a.vd;
+  const int h = (int)(row % a.heads), vd = a.vd, lane = threadIdx.x;
   const float* p = a.partial + row * a.splits * (vd + 4);
-  float mx = -INFINITY, l = 0.f;
-  for (int s = 0; s < a.splits; ++s) mx = fmaxf(mx, p[(int64_t)s * (vd + 4) + vd]);
-  for (int s = 0; s < a.splits; ++s) {
-    const float* q = p + (int64_t)s * (vd + 4) + vd;
-    if (q[0] > -INFINITY) l += __builtin_amdgcn_exp2f(q[0] - mx) * q[1];
-  }
-  const float f = l > 0.f ? head_gate(a, m, h) / l : 0.f;
-  for (int c = threadIdx.x * 4; c < vd; c += 256) {
+  const float* mine = p + (int64_t)min(lane, a.splits - 1) * (vd + 4) + vd;
+  const float pm = lane < a.splits ? mine[0] : -INFINITY, pl = mine[1];
+  const float gate = head_gate(a, m, h);
+  const float mx = wave_max(pm);
+  const float w = pm > -INFINITY ? __builtin_amdgcn_exp2f(pm - mx) : 0.f;
+  const float l = wave_sum(w * pl);
+  const float f = l > 0.f ? gate * w / l : 0.f;  // the split's weight in the output
+  for (int c0 = 0; c0 < vd; c0 += 256) {
+    const int c = c0 + lane * 4;
     float4_t v = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < a.splits; ++s) {
-      const float* q = p + (int64_t)s * (vd + 4);
-      if (q[vd] > -INFINITY)
-        v += __builtin_amdgcn_exp2f(q[vd] - mx) * *reinterpret_cast<const float4_t*>(q + c);
+    for (int s0 = 0; s0 < a.splits; s0 += 8) {
+      float4_t x[8];
+#pragma unroll
+      for (int s = 0; s < 8; ++s)
+        x[s] = *reinterpret_cast<const float4_t*>(p + (int64_t)min(s0 + s, a.splits - 1) * (vd + 4) +
+                                                  min(c, vd - 4));
+#pragma unroll
+      for (int s = 0; s < 8; ++s) {
+        const float ws = __shfl(f, min(s0 + s, 63), MSA_WAVE);
+        if (ws != 0.f) v += ws * x[s];  // lanes past the splits weigh nothing
+      }
     }
     const int at = h * vd + c;
-    *reinterpret_cast<bf16x4_t*>((bf16_t*)a.out + (a.out_mb > 0 ? packed_act_offset((int)m, at, a.out_mb)
-                                                                : m * a.ldo + at)) =
-        bf16x4_t{(bf16_t)(v[0] * f), (bf16_t)(v[1] * f), (bf16_t)(v[2] * f), (bf16_t)(v[3] * f)};
+    if (c < vd)
+      *reinterpret_cast<bf16x4_t*>((bf16_t*)a.out + (a.out_mb > 0
+                                                         ? packed_act_offset((int)m, at, a.out_mb)
+                                                         : m * a.ldo + at)) =
+          bf16x4_t{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
   }
 }
 
@@ -557,16 +622,25 @@ bool has_tiles(const msa_grouped_args& a) {
   return a.dtype == MSA_BF16 && tile_size(a.hd) && tile_size(a.vd);
 }
 
+template <int HD, int VD, bool FUSED>
+bool run_decode(const msa_grouped_args& a, const msa_batch* b, int r0, int segs, hipStream_t s) {
+  static std::atomic<uint64_t> raised{0};
+  constexpr int bytes = gd_lds_bytes<HD, VD>;
+  if (!raise_lds((const void*)grouped_decode_kernel<HD, VD, FUSED>, bytes, raised)) return false;
+  const int HB = (a.heads / a.kv_heads + 15) / 16;
+  hipLaunchKernelGGL((grouped_decode_kernel<HD, VD, FUSED>),
+                     dim3((unsigned)(segs * a.kv_heads * HB * a.splits)), dim3(256), bytes, s, a, r0, segs,
+                     b->tok_slot, b->tok_pos, a.scale * LOG2E);
+  return true;
+}
+
 template <int HD, int VD>
 bool run_tiles(const msa_grouped_args& a, const msa_batch* b, int r0, int seg0, int segs, int longest,
                hipStream_t s) {
   if (longest == 1) {
-    static std::atomic<uint64_t> raised{0};
-    if (!raise_lds((const void*)grouped_decode_kernel<HD, VD>, gd_lds_bytes<VD>, raised)) return false;
-    const int HB = (a.heads / a.kv_heads + 15) / 16;
-    hipLaunchKernelGGL((grouped_decode_kernel<HD, VD>), dim3((unsigned)(segs * a.kv_heads * HB * a.splits)),
-                       dim3(256), gd_lds_bytes<VD>, s, a, r0, segs, b->tok_slot, b->tok_pos,
-                       a.scale * LOG2E);
+    const bool ok = a.fused ? run_decode<HD, VD, true>(a, b, r0, segs, s)
+                            : run_decode<HD, VD, false>(a, b, r0, segs, s);
+    if (!ok) return false;
     if (a.splits > 1)
       hipLaunchKernelGGL(grouped_combine_kernel, dim3((unsigned)(segs * a.heads)), dim3(64), 0, s, a, r0);
     return true;
@@ -654,9 +728,13 @@ extern "C" int msa_grouped_attention_splits(const msa_grouped_args* a, int M, in
   const int64_t groups = (int64_t)M * a->kv_heads * ((per + 15) / 16);
   const int keys = a->chunk > 0 && a->chunk < key_bound ? a->chunk : key_bound;
   int s = 1;
-  // about two workgroups per CU, at least 128 keys (a tile per wave) each
-  while (s < 64 && groups * s < 512 && (int64_t)keys >= 256 * s) s *= 2;
+  // up to a workgroup per CU, at least 128 keys (a tile per wave) each
+  while (s < 64 && groups * s * 2 <= 256 && (int64_t)keys >= 256 * s) s *= 2;
   return s;
+}
+
+extern "C" int msa_grouped_fuses(const msa_grouped_args* a, const msa_batch* b) {
+  return a && b && b->max_count == 1 && has_tiles(*a);
 }
 
 extern "C" int msa_grouped_attention(const msa_grouped_args* a, const msa_batch* b, int seg0, int seg1,
@@ -671,6 +749,7 @@ extern "C" int msa_grouped_attention(const msa_grouped_args* a, const msa_batch*
                   (a->splits == 1 || (a->partial && longest == 1 && has_tiles(*a))),
               MSA_ERR_INVALID_ARG, "%s: splits=%d scale=%g", name, a->splits, (double)a->scale);
   MSA_REQUIRE(b->max_count == 1 || b->host_start, MSA_ERR_INVALID_ARG, "%s: no host tables", name);
+  MSA_REQUIRE(!a->fused || msa_grouped_fuses(a, b), MSA_ERR_INVALID_ARG, "%s: nothing to fuse with", name);
   hipStream_t s = (hipStream_t)stream;
   const int r0 = b->max_count == 1 ? seg0 : b->host_start[seg0];
   const int r1 = b->max_count == 1 ? seg1 : b->host_start[seg1];

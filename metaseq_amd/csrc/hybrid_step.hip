@@ -41,10 +41,10 @@ constexpr int EXPAND_FROM = 16;
     if (rc_) return rc_;      \
   } while (0)
 
-// An activation matrix [M, ld] in the step's format.
+// An activation matrix of n columns in the step's format; ld > n: some columns of a wider one.
 struct Act {
   void* p;
-  int ld;
+  int ld, n;
 };
 
 struct Run {
@@ -63,7 +63,11 @@ struct Run {
     if (off > peak) peak = off;
     return p;
   }
-  Act act(int ld) { return {alloc((int64_t)(mb > 0 ? mb * 16 : M) * ld * es), ld}; }
+  Act act(int ld) { return {alloc((int64_t)(mb > 0 ? mb * 16 : M) * ld * es), ld, ld}; }
+  // n columns of x from c on (a multiple of 32)
+  Act columns(const Act& x, int c, int n) const {
+    return {(char*)x.p + (int64_t)c * (mb > 0 ? mb * 16 : 1) * es, x.ld, n};
+  }
   unsigned in_flags() const { return mb > 0 ? MSA_IN_PACKED : 0u; }
 
   // y (row-major or, with glu, in the activation layout) = x W^T with fp32 tail columns
@@ -77,8 +81,12 @@ struct Run {
                            in_flags() | (y_act && mb > 0 ? MSA_OUT_PACKED : 0u), stream);
   }
   // fp32 sums of S slices
-  float* partial(const Act& x, const void* W, int N, int& S, int& rc) {
+  float* partial(const Act& x, const void* W, int N, int& S, int& rc, int least = 1) {
     S = f32 ? 1 : msa_linear_bf16_splits(M, N, x.ld, mb > 0);
+    if (least > 1) {  // slices that do not cross the borders of `least` equal parts of K
+      S = S > least ? S : least;
+      while (S > least && x.ld % (64 * S)) S /= 2;
+    }
     float* part = (float*)alloc((int64_t)S * M * N * 4);
     rc = MSA_OK;
     if (dry) return part;
@@ -90,8 +98,8 @@ struct Run {
     return part;
   }
   int zero_tail(const Act& y, int used) {
-    if (dry || used == y.ld) return MSA_OK;
-    return msa_zero_columns(d->cfg.dtype, y.p, M, y.ld, mb, used, y.ld, stream);
+    if (dry || used == y.n) return MSA_OK;
+    return msa_zero_columns(d->cfg.dtype, y.p, M, y.ld, mb, used, y.n, stream);
   }
 
   // y, y2 (activation format; y row-major), y32 = a linear layer with bias, activation, decays
@@ -352,7 +360,8 @@ int Run::grouped(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in
   g.out = out.p;
   g.ldo = out.ld;
   g.out_mb = mb;
-  if (!dry) HY(msa_grouped_rotate(&g, &b, stream));
+  g.fused = msa_grouped_fuses(&g, &b);
+  if (!dry && !g.fused) HY(msa_grouped_rotate(&g, &b, stream));
   for (int s = 0; s < b.nseg;) {
     auto count = [&](int i) { return b.max_count == 1 ? 1 : b.host_start[i + 1] - b.host_start[i]; };
     const bool single = count(s) == 1;
@@ -369,7 +378,7 @@ int Run::grouped(const msa_hybrid_layer& l, const msa_hybrid_state& st, char* in
     off = save;
     s = e;
   }
-  if (!dry) HY(msa_grouped_append(&g, &b, stream));
+  if (!dry && !g.fused) HY(msa_grouped_append(&g, &b, stream));
   return zero_tail(out, t.heads * t.vd);
 }
 
@@ -402,7 +411,7 @@ int Run::parallel(int ri, const Act& h, Act& left, Act& right) {
 // t arrives with everything that does not depend on the feed-forward
 int Run::feed_forward(const msa_hybrid_layer& l, msa_tail_args& t) {
   const msa_hybrid_config& c = d->cfg;
-  const Act h{t.h, c.Dp};
+  const Act h{t.h, c.Dp, c.Dp};
   int rc;
   if (l.ff_kind == MSA_FF_DENSE) {
     Act u = act(l.ff);
@@ -422,7 +431,7 @@ int Run::feed_forward(const msa_hybrid_layer& l, msa_tail_args& t) {
   }
   const int n32 = 2 * l.ff_shared, ldz = l.n_ff_in - n32, E = l.experts, P = M * l.top;
   const bool shared = l.ff_shared > 0;
-  Act u = shared ? act(l.ff_shared) : Act{nullptr, 0};
+  Act u = shared ? act(l.ff_shared) : Act{};
   float* z = (float*)alloc((int64_t)M * ldz * 4);
   // the shared expert's hidden layer, the router logits and the shared gate's logit in one product
   HY(linear(h, l.w_ff_in, u.p, true, z, l.n_ff_in, n32, shared ? MSA_GLU_CLAMPED : MSA_GLU_NONE,
@@ -527,10 +536,12 @@ int Run::go() {
       k->h_mb = mb;
     }
     off = layer_base;
-    Act o = act(l.ko), o2{};
+    const bool two = l.kind == MSA_MIX_PARALLEL, merged = two && !l.att.w_out;
+    const Act both = act(merged ? 2 * l.ko : l.ko);
+    Act o = merged ? columns(both, 0, l.ko) : both, o2{};
     t.w_post = l.norm1b;
-    if (l.kind == MSA_MIX_PARALLEL) {
-      o2 = act(l.att.ko);
+    if (two) {
+      o2 = merged ? columns(both, l.ko, l.ko) : act(l.att.ko);
       HY(parallel(i, h, o2, o));
       t.w_post = l.out_norm;
       t.w_post2 = l.att.out_norm;
@@ -539,9 +550,12 @@ int Run::go() {
                                                                               : delta(i, h, o));
     }
     int rc;
-    t.part = partial(o, l.w_out, c.Dp, t.S, rc);
+    t.part = partial(both, l.w_out, c.Dp, t.S, rc, merged ? 2 : 1);
     HY(rc);
-    if (l.kind == MSA_MIX_PARALLEL) {
+    if (merged) {
+      t.S2 = t.S /= 2;
+      t.part2 = t.part + (int64_t)t.S * M * c.Dp;
+    } else if (two) {
       t.part2 = partial(o2, l.att.w_out, c.Dp, t.S2, rc);
       HY(rc);
     }
@@ -559,7 +573,7 @@ int Run::go() {
   if (a->rows) {
     rows = a->n_rows;
     fmb = !f32 && rows <= MSA_PACKED_MAX_ROWS ? packed_row_blocks(rows) : 0;
-    f = {alloc((int64_t)(fmb > 0 ? fmb * 16 : rows) * c.Dp * es), c.Dp};
+    f = {alloc((int64_t)(fmb > 0 ? fmb * 16 : rows) * c.Dp * es), c.Dp, c.Dp};
     if (!dry) HY(msa_gather_rows(c.dtype, h.p, mb, a->rows, rows, c.Dp, f.p, fmb, stream));
   }
   if (dry || rows == 0) return MSA_OK;
@@ -646,7 +660,8 @@ extern "C" int msa_hybrid_create(const msa_hybrid_config* cfg, const msa_hybrid_
       const msa_attention_layer& t = l.att;
       MSA_REQUIRE(t.heads > 0 && t.kv_heads > 0 && t.heads % t.kv_heads == 0 && t.hd > 0 &&
                       t.hd % 16 == 0 && t.vd > 0 && t.vd % 16 == 0 && t.chunk >= 0 && t.scale > 0.f &&
-                      (t.rot_dims == 0 || t.inv_freq) && t.w_out && t.out_norm && k_ok(t.ko) &&
+                      (t.rot_dims == 0 || t.inv_freq) && t.out_norm && k_ok(t.ko) &&
+                      (t.w_out || (t.ko == l.ko && cfg->dtype == MSA_BF16)) &&
                       t.ko >= t.heads * t.vd,
                   MSA_ERR_INVALID_ARG, "%s: layer %d: grouped attention", name, i);
       MSA_REQUIRE(l.heads > 0 && l.kv_heads > 0 && l.heads % l.kv_heads == 0 && l.conv_w && l.o_norm &&

@@ -290,7 +290,7 @@ class HybridDecoder(IncrementalDecoder):
         return [self._heads(w(pre + n), h, s, p) for n, h, s, p in split], conv.float().t()
 
     def _fill_parallel(self, t, m, plan, w):
-        a, d, Dp = m.left, m.right, self.Dp
+        a, d, D, Dp = m.left, m.right, self.cfg.width, self.Dp
         dev = lambda name: w("mix." + name).to(self.device)
         t.kind, at = _capi.MSA_MIX_PARALLEL, t.att
         at.heads, at.kv_heads, at.hd, at.vd = a.heads, a.kv_heads, plan.hd, plan.vd
@@ -298,7 +298,6 @@ class HybridDecoder(IncrementalDecoder):
         i = torch.arange(a.rot_dims // 2, dtype=torch.float64)
         if a.rot_dims:
             at.inv_freq = self._hold(float(a.rot_base) ** (-2.0 * i / a.rot_dims))
-        at.w_out = self._mat(self._head_columns(dev("left.o"), a.heads, a.vdim, plan.vd), Dp, plan.kl)
         t.heads, t.kv_heads, t.taps = d.heads, d.kv_heads, d.conv
         t.dim, t.dp, t.vdim, t.vp = d.dim, plan.dp, d.vdim, plan.vp
         # the inputs of every projection of the layer's input, in one matrix
@@ -323,7 +322,13 @@ class HybridDecoder(IncrementalDecoder):
         rate = torch.exp(dev("right.A_log").float()).view(H, 1).expand(H, d.dim)
         t.lr_rate = self._vec(rate, H, dp)
         t.o_norm = self._vec(w("mix.right.norm"), vp)
-        t.w_out = self._mat(self._head_columns(dev("right.o"), H, d.vdim, vp), Dp, plan.ko)
+        left = self._head_columns(dev("left.o"), a.heads, a.vdim, plan.vd)
+        right = self._head_columns(dev("right.o"), H, d.vdim, vp)
+        if plan.kl == plan.ko and self.dtype == torch.bfloat16:     # one product for both sides
+            sides = [_pad(x, D, plan.ko) for x in (right, left)]
+            t.w_out = self._mat(torch.cat(sides, dim=1), Dp, 2 * plan.ko)
+        else:
+            t.w_out, at.w_out = self._mat(right, Dp, plan.ko), self._mat(left, Dp, plan.kl)
         # half of each side
         at.out_norm = self._vec(0.5 * dev("left.out").float(), Dp)
         t.out_norm = self._vec(0.5 * dev("right.out").float(), Dp)
