@@ -80,9 +80,18 @@ struct Epilogue {
   int act, n2, ld2, out2_mb;
 };
 
-// what MODE_BF_POST does to the sums of columns n .. n + 3
-__device__ __forceinline__ float4_t post4(const Epilogue& e, int n, float4_t v) {
-  if (e.bias32) v += *reinterpret_cast<const float4_t*>(e.bias32 + n);
+// what MODE_BF_POST does to the sums of columns n .. n + 3, and the vectors it takes for them
+struct PostVectors {
+  float4_t bias, rate;
+};
+__device__ __forceinline__ PostVectors post_vectors(const Epilogue& e, int n) {
+  PostVectors p{{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  if (e.bias32) p.bias = *reinterpret_cast<const float4_t*>(e.bias32 + n);
+  if (n >= e.n32 && e.decay_rate) p.rate = *reinterpret_cast<const float4_t*>(e.decay_rate + n - e.n32);
+  return p;
+}
+__device__ __forceinline__ float4_t post4(const Epilogue& e, int n, float4_t v, const PostVectors& p) {
+  v += p.bias;
   if (n < e.n32) {
     if (e.act == MSA_ACT_RELU2) {
 #pragma unroll
@@ -90,7 +99,7 @@ __device__ __forceinline__ float4_t post4(const Epilogue& e, int n, float4_t v) 
     }
   } else if (e.decay_rate) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = decay_of(v[i], e.decay_rate[n - e.n32 + i]);
+    for (int i = 0; i < 4; ++i) v[i] = decay_of(v[i], p.rate[i]);
   }
   return v;
 }
@@ -176,7 +185,7 @@ __device__ __forceinline__ void select_merge(SelectState& a, float om, float os,
 template <int MODE>
 __device__ __forceinline__ void epilogue4(const Epilogue& e, int64_t m, int n, float4_t acc) {
   if constexpr (is_bf<MODE>) {
-    if constexpr (MODE == MODE_BF_POST) acc = post4(e, n, acc);
+    if constexpr (MODE == MODE_BF_POST) acc = post4(e, n, acc, post_vectors(e, n));
     if (n >= e.n32) {
       *reinterpret_cast<float4_t*>(e.y32 + m * (e.N - e.n32) + (n - e.n32)) = acc;
     } else if constexpr (MODE != MODE_BF_GLU) {
@@ -1423,6 +1432,12 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
     const int nw = n0 + wn * (16 * WF);      // first column of the wave
     const int bn = GLU ? (nw >> 1) + bc * 8 : nw + bc * 8;  // first output column of the lane
     const bool bn_ok = bn < (GLU ? epi.n32 >> 1 : epi.n32);
+    // (read once: behind the first store the compiler may no longer keep them)
+    PostVectors post[MODE == MODE_BF_POST ? WF : 1];
+    if constexpr (MODE == MODE_BF_POST) {
+#pragma unroll
+      for (int j = 0; j < WF; ++j) post[j] = post_vectors(epi, min(nw + 16 * j, N - 16) + 4 * lg);
+    }
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       char* buf = stage + (i & 1) * 4096;
@@ -1430,8 +1445,7 @@ __global__ __launch_bounds__(TQ_THREADS) void linear_quad_kernel(
 #pragma unroll
       for (int j = 0; j < WF; ++j) {
         const int n = nw + 16 * j + 4 * lg;
-        if constexpr (MODE == MODE_BF_POST)
-          if (n < N) acc[i][j] = post4(epi, n, acc[i][j]);
+        if constexpr (MODE == MODE_BF_POST) acc[i][j] = post4(epi, nw + 16 * j, acc[i][j], post[j]);
         if (nw + 16 * j >= epi.n32) {  // wave-uniform: n32 is a multiple of 16
           if (mf >= m_own && mf < M && n < N)
             *reinterpret_cast<float4_t*>(epi.y32 + mf * (N - epi.n32) + (n - epi.n32)) = acc[i][j];
