@@ -1,4 +1,5 @@
 """Small hybrid configurations, their weights and comparisons with the plain oracle."""
+import copy
 import json
 
 import torch
@@ -27,6 +28,20 @@ def delta(heads=6, kv_heads=2, dim=20, vdim=24, conv=4):
     return "delta", dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=conv)
 
 
+def parallel(heads=6, kv_heads=2, dim=24, vdim=40, chunk=37, rot=(10000.0, 12), scale=0.25,
+             delta_heads=4, delta_kv_heads=2, delta_dim=20, delta_vdim=28, conv=3, ranks=(18, 10)):
+    """Grouped attention beside a delta rule with channel decays; ``ranks``: of the read-out gate's
+    and the decays' low-rank projections."""
+    left = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale)
+    if rot:
+        left["rot"] = dict(base=rot[0], dims=rot[1])
+    if chunk:
+        left["mask"] = dict(size=chunk)
+    right = dict(heads=delta_heads, kv_heads=delta_kv_heads, dim=delta_dim, vdim=delta_vdim,
+                 conv=conv, gate_rank=ranks[0], decay_rank=ranks[1])
+    return "parallel", dict(left=left, right=right)
+
+
 def dense(ff=136):
     return dict(kind="dense", ff=ff)
 
@@ -48,6 +63,37 @@ def config(layers, width=72, vocab=101, eps=1e-5, scale=2.0):
                 layers=[dict(type=t, mixer=m, mlp=f) for (t, m), f in layers])
 
 
+def looped(layers, loop=None, width=72, vocab=101, eps=1e-5):
+    """The same for the design whose layers run in a loop; ``loop``: (start, stop, times)."""
+    out = dict(architecture="Nomalorn", width=width, vocab=vocab, norm=dict(eps=eps),
+               layers=[dict(type=t, mixer=m, mlp=f) for (t, m), f in layers])
+    if loop:
+        out["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return out
+
+
+def looped_mixed(width=72):
+    """Unequal layers, a loop over two of them, a layer without a feed-forward, a chunk shorter
+    than most portions beside one longer than most sequences."""
+    return looped([(parallel(), dense()),
+                   (parallel(heads=4, kv_heads=4, dim=36, vdim=16, chunk=100, rot=(500.0, 36),
+                             delta_heads=3, delta_kv_heads=3, delta_dim=36, delta_vdim=16, conv=4,
+                             ranks=(7, 30)), None),
+                   (parallel(heads=18, kv_heads=1, dim=16, vdim=20, chunk=64, rot=(1e5, 6),
+                             delta_heads=6, delta_kv_heads=1, ranks=(5, 5)), dense(90)),
+                   (parallel(chunk=1000, conv=2), dense(200))], loop=(1, 3, 2), width=width)
+
+
+def published(cfg):
+    """The configuration as a model folder has it: the ranks are left to the weights' shapes."""
+    cfg = copy.deepcopy(cfg)
+    for layer in cfg["layers"]:
+        if layer["type"] == "parallel":
+            for rank in ("gate_rank", "decay_rank"):
+                layer["mixer"]["right"].pop(rank, None)
+    return cfg
+
+
 def mixed(dtype=torch.float32, width=72):
     """Every mechanism once, a borrowed latent, an expert layer without groups, a layer without a
     feed-forward.  With random weights some token's choice of experts is always so close that bf16
@@ -63,7 +109,15 @@ def mixed(dtype=torch.float32, width=72):
 
 def no_specials(state):
     """Logits of the special ids 0 .. 3 are never the largest (a record ends at one)."""
-    state["head"][:4] = 0
+    state.get("head", state["embed"])[:4] = 0
+
+
+def steady(state):
+    """Keys of the delta rules close to their queries.  A first token's read-out is (k . q) v, normed:
+    with random weights k . q is sometimes so small that bf16 rounding decides its sign."""
+    for name in [n for n in state if ".right.k" in n]:
+        q = state[name.replace(".right.k", ".right.q")]
+        state[name] = (0.8 * q.float() + 0.6 * state[name].float()).to(q.dtype)
 
 
 def write_safetensors(path, tensors):
@@ -82,7 +136,7 @@ def write_safetensors(path, tensors):
 def model_folder(path, cfg, state):
     """A model folder as the registry reads it."""
     write_safetensors(path / "model.safetensors", state)
-    (path / "config.json").write_text(json.dumps(cfg))
+    (path / "config.json").write_text(json.dumps(published(cfg)))
     return str(path)
 
 
@@ -96,7 +150,9 @@ class Case:
         if tweak is not None:
             tweak(self.state)
         self.W = {k: v.double() for k, v in self.state.items()}
-        self.decoder = HybridDecoder(self.cfg, self.state, device=device, dtype=dtype)
+        self.decoder = HybridDecoder(HybridConfig.from_json(published(cfg)), self.state,
+                                     device=device, dtype=dtype)
+        self.cfg = self.decoder.cfg
 
     def tokens(self, n, seed=0):
         g = torch.Generator().manual_seed(seed)

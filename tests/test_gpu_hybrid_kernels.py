@@ -116,6 +116,213 @@ def test_linear_f32(M, N, K):
 
 
 @pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+@pytest.mark.parametrize("M,N,K", SHAPES)
+def test_linear_with_bias_activation_and_decays(M, N, K, dtype):
+    """Every kernel behind msa_linear: a bias, relu^2, a second output, fp32 columns as they are and
+    as decays (logits far out on both sides among them)."""
+    lib = _capi.load_hybrid()
+    if dtype == F32 and N * M > 1 << 21:
+        pytest.skip("one fp32 kernel serves every shape")
+    print("linear", M, N, K, flush=True)
+    g = gen(M + N + K)
+    x = torch.randn(M, K, generator=g).to(dtype)
+    w = (torch.randn(N, K, generator=g) * K ** -0.5).to(dtype)
+    bias = torch.randn(N, generator=g)
+    bias[-8:-4], bias[-4:] = -16.0, 30.0
+    ref = x.double() @ w.double().T + bias.double()
+    packed = M <= 128 and dtype == BF16
+    xd = (pack_rows(x) if packed else x).cuda()
+    wd = (pack_tiles(w) if dtype == BF16 else w).cuda()
+    bd = bias.cuda()
+    MB = (M + 15) // 16 if M <= 64 else 8
+    tol = 6e-3 if dtype == BF16 else 2e-6
+    for n2, n32, act, decays in ((N, N, 1, 0), (N // 64 * 32, N // 32 * 32, 0, 0),
+                                 (0, N // 32 * 32 - 32, 0, 1), (16, N - 16, 1, 1), (N - 16, N - 16, 0, 1),
+                                 (0, 0, 0, 1)):
+        rate = torch.rand(N - n32, generator=g) * 3
+        rd = rate.cuda()
+        out2_packed = packed and (n32 - n2) % 32 == 0
+        y = torch.zeros(M, n2, dtype=dtype, device="cuda")
+        y2 = torch.zeros((MB * 16 if out2_packed else M) * (n32 - n2), dtype=dtype, device="cuda")
+        y32 = torch.zeros(M, N - n32, device="cuda")
+        a = _capi.LinearArgs()
+        a.dtype, a.x, a.W, a.M, a.N, a.K = int(dtype == F32), ptr(xd), ptr(wd), M, N, K
+        a.n32, a.n2, a.act, a.bias = n32, n2, act, ptr(bd)
+        a.decay_rate = ptr(rd) if decays and n32 < N else None
+        a.flags = (_capi.MSA_IN_PACKED if packed else 0) | (_capi.MSA_OUT2_PACKED if out2_packed else 0)
+        a.y, a.y32 = ptr(y) if n2 else None, ptr(y32) if n32 < N else None
+        if n2 < n32:
+            a.y2 = ptr(y2)
+        check(lib.msa_linear(ctypes.byref(a), _capi.stream_ptr()), lib)
+        want = torch.relu(ref) ** 2 if act else ref
+        what = "n2=%d n32=%d act=%d" % (n2, n32, act)
+        if n2:
+            close(y, want[:, :n2], tol, what)
+        if n2 < n32:
+            got = unpack_rows(y2.cpu(), M, n32 - n2) if out2_packed else y2.view(M, n32 - n2)
+            close(got, want[:, n2:n32], tol, "second output, " + what)
+        if n32 < N:
+            z = ref[:, n32:]
+            if decays:
+                z = torch.exp(-rate.double() * torch.nn.functional.softplus(z))
+            close(y32, z, 1e-5 if dtype == BF16 else 3e-6, "fp32 columns, " + what)
+            if decays:   # next to 1 the distance from 1 counts
+                slow = z > 0.999
+                off = ((1 - y32.cpu().double()) - (1 - z)).abs()[slow]
+                assert off.numel() == 0 or float(off.max()) < 3e-7, what
+
+
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+@pytest.mark.parametrize("M,D", [(1, 72), (5, 4096), (40, 1000), (130, 2100), (1100, 300),
+                                 (1030, 5000), (3, 9000)])
+def test_tail_of_two_sides_with_loop_terms(M, D, dtype):
+    """Both sides' sums and norms, a bias, what a loop adds, the probe and the next norm."""
+    lib = _capi.load_hybrid()
+    g = gen(M + D)
+    Dp, eps = (D + 63) // 64 * 64, 1e-3
+
+    def wide(*shape):
+        t = torch.zeros(*shape, Dp)
+        t[..., :D] = torch.randn(*shape, D, generator=g)
+        return t
+    for S, S2, two, extra in ((1, 1, True, True), (3, 5, True, False), (2, 0, False, True)):
+        x, part, part2 = wide(M), wide(S, M), wide(max(1, S2), M)
+        bias, w, w2, add, step, nxt = wide(), wide(), wide(), wide(M), wide(), wide()
+        b = part.double().sum(0) + (bias.double() if extra else 0)
+        want = x.double()
+        want = want + (O.rms(b[:, :D], eps, w[:D].double()) if two else b[:, :D]) \
+            if Dp == D else want.clone()
+        if Dp != D:
+            want[:, :D] += O.rms(b[:, :D], eps, w[:D].double()) if two else b[:, :D]
+        if two:
+            want[:, :D] += O.rms(part2.double().sum(0)[:, :D], eps, w2[:D].double())
+        probe = want.clone()
+        if extra:
+            want = want + add.double() + step.double()
+        h = O.rms(want[:, :D], eps, nxt[:D].double())
+        dev = [t.cuda() for t in (x, part, part2, bias, w, w2, add, step, nxt)]
+        hd = torch.zeros(M, Dp, dtype=dtype, device="cuda")
+        pd = torch.zeros(M, Dp, device="cuda")
+        a = _capi.TailArgs()
+        a.dtype, a.M, a.D, a.Dp, a.S, a.eps = int(dtype == F32), M, D, Dp, S, eps
+        a.x, a.part, a.h, a.w_next, a.probe = ptr(dev[0]), ptr(dev[1]), ptr(hd), ptr(dev[8]), ptr(pd)
+        if two:
+            a.part2, a.S2, a.w_post, a.w_post2 = ptr(dev[2]), S2, ptr(dev[4]), ptr(dev[5])
+        if extra:
+            a.bias, a.add, a.step = ptr(dev[3]), ptr(dev[6]), ptr(dev[7])
+        check(lib.msa_residual_rmsnorm_tail(ctypes.byref(a), _capi.stream_ptr()), lib)
+        close(dev[0], want, 2e-6, "stream")
+        close(pd, probe, 2e-6, "probe")
+        close(hd[:, :D], h, 6e-3 if dtype == BF16 else 3e-6, "normed")
+
+
+def _grouped(lib, dtype, heads, kv_heads, hd, vd, chunk, rot, segments, capacity, seed, fused=None):
+    """One step of grouped attention over ``segments`` ((slot, first position, tokens)) through the
+    three calls; returns its outputs and the caches with what they should be."""
+    g = gen(seed)
+    M = sum(n for _, _, n in segments)
+    slots = 1 + max(s for s, _, _ in segments)
+    rows = min(capacity, chunk) if chunk else capacity
+    ld = (heads + kv_heads) * hd + kv_heads * vd + 16
+    x = torch.randn(M, ld, generator=g).to(dtype)
+    kc = torch.randn(slots, kv_heads, rows, hd, generator=g).to(dtype)
+    vc = torch.randn(slots, kv_heads, rows, vd, generator=g).to(dtype)
+    gate = torch.randn(M, heads + 3, generator=g)
+    inv = 100.0 ** (-2.0 * torch.arange(rot // 2, dtype=torch.float64) / max(1, rot))
+    scale = 1.5 * hd ** -0.5
+    want, kw, vw = torch.zeros(M, heads, vd, dtype=torch.float64), kc.clone(), vc.clone()
+    at = 0
+    for slot, pos, n in segments:
+        if pos >= 0:
+            own = x[at:at + n].double()
+            q = own[:, :heads * hd].view(n, heads, hd)
+            k = own[:, heads * hd:(heads + kv_heads) * hd].view(n, kv_heads, hd)
+            v = own[:, (heads + kv_heads) * hd:-16].view(n, kv_heads, vd)
+            p = torch.arange(pos, pos + n)
+            if rot:
+                q, k = (O.rotate_half(t, p, 100.0, rot).to(dtype).double() for t in (q, k))
+            c0 = pos // chunk * chunk if chunk else 0
+            keys = torch.cat([kc[slot, :, :pos - c0].double().transpose(0, 1), k])
+            vals = torch.cat([vc[slot, :, :pos - c0].double().transpose(0, 1), v])
+            where = torch.arange(c0, pos + n)
+            for h in range(heads):
+                j = h // (heads // kv_heads)
+                s = q[:, h] @ keys[:, j].T * scale
+                first = p // chunk * chunk if chunk else torch.zeros_like(p)
+                sees = (where <= p[:, None]) & (where >= first[:, None])
+                s = s.masked_fill(~sees, float("-inf"))
+                want[at:at + n, h] = torch.softmax(s, -1) @ vals[:, j] * torch.sigmoid(
+                    gate[at:at + n, h:h + 1].double())
+            last = (pos + n - 1) // chunk * chunk if chunk else 0
+            for i in range(max(0, last - pos), n):
+                kw[slot, :, pos + i - last] = k[i].to(dtype)
+                vw[slot, :, pos + i - last] = v[i].to(dtype)
+        at += n
+    b, alive = _batch(segments, M)
+    b.key_bound = max(max(p + n for _, p, n in segments), 1)
+    xd, kd, vd_, gd, fd = x.cuda(), kc.cuda(), vc.cuda(), gate.cuda(), inv.cuda()
+    out = torch.full((M, heads * vd), 7.0, dtype=dtype, device="cuda")
+    a = _capi.GroupedArgs()
+    a.dtype, a.heads, a.kv_heads, a.hd, a.vd = int(dtype == F32), heads, kv_heads, hd, vd
+    a.chunk, a.rot_dims, a.rows, a.scale = chunk, rot, rows, scale
+    a.inv_freq = ptr(fd) if rot else None
+    es = x.element_size()
+    a.q, a.k = xd.data_ptr(), xd.data_ptr() + heads * hd * es
+    a.v, a.ld = a.k + kv_heads * hd * es, ld
+    a.k_cache, a.v_cache, a.gate, a.ld_gate = ptr(kd), ptr(vd_), ptr(gd), heads + 3
+    a.out, a.ldo = ptr(out), heads * vd
+    a.fused = lib.msa_grouped_fuses(ctypes.byref(a), ctypes.byref(b)) if fused is None else fused
+    part = torch.zeros(M * heads * 64 * (vd + 4), device="cuda")
+    a.partial, s = ptr(part), _capi.stream_ptr()
+    ref = (ctypes.byref(a), ctypes.byref(b))
+    if not a.fused:
+        check(lib.msa_grouped_rotate(*ref, s), lib)
+    seg = 0
+    counts = [n for _, _, n in segments]
+    while seg < len(counts):
+        end = seg + 1
+        while end < len(counts) and (counts[end] == 1) == (counts[seg] == 1):
+            end += 1
+        a.splits = 1
+        if counts[seg] == 1:
+            a.splits = lib.msa_grouped_attention_splits(ctypes.byref(a), end - seg, b.key_bound)
+        check(lib.msa_grouped_attention(*ref, seg, end, max(counts[seg:end]), s), lib)
+        seg = end
+    if not a.fused:
+        check(lib.msa_grouped_append(*ref, s), lib)
+    tol = 2e-5 if dtype == F32 else 1.5e-2
+    on = torch.cat([torch.full((n,), p >= 0) for _, p, n in segments])
+    close(out.view(M, heads, vd)[on.cuda()], want[on], tol, "outputs, splits=%d" % a.splits)
+    # rotated keys in another order of operations: the last bit may differ
+    close(kd, kw, 1e-6 if dtype == F32 else 8e-3, "keys kept")
+    assert torch.equal(vd_.cpu(), vw), "values kept"
+
+
+GROUPED = [(4, 2, 64, 64, 40), (8, 8, 128, 128, 128), (34, 2, 64, 128, 10), (3, 1, 192, 64, 0),
+           (4, 1, 256, 256, 64), (2, 2, 128, 192, 126), (5, 5, 192, 256, 34), (16, 8, 256, 64, 2),
+           (17, 1, 64, 192, 64), (3, 3, 80, 272, 16), (8, 8, 64, 256, 62), (2, 1, 128, 64, 0)]
+
+
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
+@pytest.mark.parametrize("heads,kv_heads,hd,vd,rot", GROUPED)
+def test_grouped_attention(heads, kv_heads, hd, vd, rot, dtype):
+    """Decode steps (fused and not, with and without splits), portions over several chunks, mixed
+    batches with inactive segments, with and without chunks."""
+    lib = _capi.load_hybrid()
+    size = (heads, kv_heads, hd, vd)
+    print("grouped", size, rot, flush=True)
+    decode = [(2, 700, 1), (0, 0, 1), (1, -1, 1), (4, 255, 1), (3, 129, 1), (5, 511, 1)]
+    mix = [(1, 250, 1), (0, 90, 70), (2, 5, 1), (3, -1, 1), (4, 0, 150), (5, 127, 2), (6, -1, 3),
+           (7, 64, 64)]
+    for chunk in (0, 100, 128, 1000):
+        _grouped(lib, dtype, *size, chunk, rot, decode, 800, heads)
+        _grouped(lib, dtype, *size, chunk, rot, decode, 800, heads, fused=0)
+        _grouped(lib, dtype, *size, chunk, rot, mix, 300, heads + 1)
+    _grouped(lib, dtype, *size, 7, rot, [(0, 3, 40), (1, 6, 1), (2, 0, 7), (3, 13, 2)], 300, hd)
+    _grouped(lib, dtype, *size, 0, rot, [(0, 1500, 1)], 1600, hd)          # splits
+
+
+@pytest.mark.parametrize("dtype", [BF16, F32], ids=["bf16", "f32"])
 @pytest.mark.parametrize("M", [1, 16, 20, 64, 150])
 def test_group_linear_dense(M, dtype):
     """Per-group columns (a head, a diagonal block), also with the groups' inputs shared."""
