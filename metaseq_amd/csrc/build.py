@@ -18,10 +18,12 @@ LIB = LIBS["core"]
 SOURCES = {
     "core": ["capi.hip", "layernorm.hip", "embed.hip", "gemm.hip", "attention.hip",
              "attention_prefill.hip", "sampling.hip", "probe.hip", "decoder_step.hip"],
-    "hybrid": ["capi.hip", "gemm_bf16.hip", "group_linear.hip", "moe.hip", "rmsnorm.hip",
-               "recurrent.hip", "latent_attention.hip", "grouped_attention.hip", "hybrid_step.hip"],
+    "hybrid": ["capi.hip", "gemm_bf16.hip", "gemm_bf16_post.hip", "group_linear.hip", "moe.hip",
+               "rmsnorm.hip", "recurrent.hip", "latent_attention.hip", "grouped_attention.hip",
+               "hybrid_step.hip"],
 }
-HEADERS = ["common.h", "gemm_kernels.h", "attention_tiles.h", os.path.join("..", "..", "include", "metaseq_amd.h"),
+HEADERS = ["common.h", "gemm_kernels.h", "attention_tiles.h",
+           os.path.join("..", "..", "include", "metaseq_amd.h"),
            os.path.join("..", "..", "include", "metaseq_hybrid.h")]
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-fPIC", "-std=c++17", "-Wall", "-Wno-unused-function",

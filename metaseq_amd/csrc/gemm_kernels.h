@@ -1891,6 +1891,15 @@ void launch_tiled(const void* x, const void* W, const void* scales, int64_t M, i
                      (const half_t*)x, W, (const half_t*)scales, M, N, K, epi);
 }
 
+template <int MODE>
+void run_linear(const void* x, const void* W, const Epilogue& e, int64_t M, int N, int K,
+                unsigned flags, hipStream_t s) {
+  if (flags & MSA_IN_PACKED)
+    launch_stream<false, MODE>(x, W, nullptr, nullptr, 1, (int)M, N, K, e, s);
+  else
+    launch_tiled<false, MODE>(x, W, nullptr, M, N, K, e, s);
+}
+
 int check_linear_args(const char* name, const void* x, const void* W, const void* y, int64_t M,
                       int N, int K, bool w8, unsigned flags, unsigned allowed) {
   MSA_REQUIRE(x && W && y, MSA_ERR_INVALID_ARG, "%s: null pointer", name);
