@@ -1,7 +1,8 @@
 /*
  * metaseq_hybrid.h - C ABI of libmetaseq_hybrid.so: gfx950 kernels and the step function of hybrid
- * decoders, i.e. models whose layers mix attention over a cached latent with recurrent layers
- * (gated linear recurrent units, gated delta rule) and dense or routed feed-forwards.
+ * decoders, i.e. models whose layers mix attention (over a cached latent, or grouped within chunks)
+ * with recurrent layers (gated linear recurrent units, gated delta rule), one after the other or side
+ * by side, and dense or routed feed-forwards.
  *
  * Conventions are those of metaseq_amd.h (device pointers, a hipStream_t as `stream`, 0 or a negative
  * msa_status, nothing allocates or synchronises).  In addition:

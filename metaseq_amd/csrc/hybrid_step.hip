@@ -4,7 +4,7 @@
 //
 // Up to 128 tokens the matrix products run on the weight-streaming kernels with packed activations
 // (split-K sums finished by the norm tail), beyond on the MFMA tile kernels with row-major ones.
-// Attention segments of more than EXPAND_FROM new tokens expand keys and values per head, shorter
+// Latent attention: segments of more than EXPAND_FROM new tokens expand keys and values per head, shorter
 // ones attend in the latent space.
 #include <stdlib.h>
 #include <string.h>

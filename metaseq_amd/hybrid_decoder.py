@@ -107,7 +107,6 @@ class _LayerPlan:
             self.ffs = _k(f.shared.ff) if f.shared is not None else 0
             self.n_ff = 2 * self.ffs + _up(f.router.experts + (1 if self.ffs else 0), 16)
 
-
     def _delta_sizes(self, m):
         self.dp = _fit(m.dim, HEAD_SIZES, "delta-rule key size")
         self.vp = _up(m.vdim, 16)
